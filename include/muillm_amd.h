@@ -44,6 +44,7 @@ extern "C" {
 
 #define MUI_DTYPE_F16 0
 #define MUI_DTYPE_BF16 1
+#define MUI_DTYPE_F32 2 /* only where an entry point says so */
 
 /* largest token batch of the weight-streaming decode kernels (and of mui_decoder_stack_step); the
  * linear entry points take more tokens than this through their tiled GEMM */
@@ -515,6 +516,124 @@ int mui_decoder_stack_step(mui_stream_t stream, const mui_decoder_stack_t* model
  * [n_tokens, dim]. */
 int mui_embedding(mui_stream_t stream, int dtype, const void* table, long row_pitch,
                   const void* ids, int ids_are_int32, void* out, int n_tokens, int dim, int vocab);
+
+/* ------------------------------------------------------------------------------------
+ * Decoders with an fp32 residual stream and a norm on both sides of every sublayer, latent
+ * attention, recurrent (matrix-memory) layers and mixtures of experts. No counterpart in the
+ * reference. Every entry point of this section also takes MUI_DTYPE_F32: activations and weights are
+ * then fp32 ("activations' type" below is the type `dtype` names).
+ * ---------------------------------------------------------------------------------- */
+
+/* Between two sublayers, per row of k elements:
+ *   x = residual_in + (post_gain ? post_gain * y * rsqrt(mean((y_scale y)^2) + epsilon) * y_scale : y_scale * y)
+ *   residual_out = x;   h = next_gain * x * rsqrt(mean(x^2) + epsilon)
+ * residual_in (NULL: 0) and residual_out (may be residual_in) are fp32 [rows, k]; y, the gains and h are
+ * in the activations' type; next_gain and h are both NULL or both given. Any k. */
+int mui_residual_norm(mui_stream_t stream, int dtype, const float* residual_in, const void* y, float y_scale,
+                      const void* post_gain, const void* next_gain, float epsilon, float* residual_out,
+                      void* h, int rows, int k);
+
+/* The same with y[r] = sum_j weight[r, j] * (expert[r, j] < n_experts ? pair_out[r * top + j] : identity_in[r]):
+ * the end of a mixture of experts (mui_moe_down's output, the block's own input for identity experts). */
+int mui_moe_residual_norm(mui_stream_t stream, int dtype, const float* residual_in, const void* pair_out,
+                          const void* identity_in, const int32_t* expert, const float* weight, int n_experts,
+                          int top, const void* post_gain, const void* next_gain, float epsilon,
+                          float* residual_out, void* h, int rows, int k);
+
+/* y[t, n] = W[n, :] . x[t, :] + bias[n] with fp32 outputs: router logits, recurrence gates. W [n_out, k_in],
+ * x [tokens, k_in] and bias [n_out] (may be NULL) in the activations' type. Any sizes. */
+int mui_linear_f32(mui_stream_t stream, int dtype, const void* weights, const void* x, const void* bias,
+                   float* y, int n_out, int k_in, int tokens);
+
+/* Routing: s = softmax(logits[t, :]) over n_experts + n_identity outputs; the `top` outputs with the largest
+ * s + correction (activations' type, may be NULL) are chosen (lowest index on ties), expert[t, j] and
+ * weight[t, j] = s of the j-th. With tile_pairs = mui_moe_tile_pairs(...) != 0 the pairs t * top + j of real
+ * experts are also sorted by expert into `pairs` (int32 [tokens * top]) and cut into tiles
+ * ((mui_moe_max_tiles(...) + 1) * 16 bytes), as mui_moe_gateup / mui_moe_down want them.
+ * n_experts + n_identity <= 1024. */
+int mui_moe_tile_pairs(int dtype, int tokens, int top, int n_experts, int width, int ff);
+int mui_moe_max_tiles(int tokens, int top, int n_experts, int tile_pairs);
+int mui_moe_route(mui_stream_t stream, int dtype, const float* logits, const void* correction, int n_experts,
+                  int n_identity, int top, int tokens, int tile_pairs, int32_t* expert, float* weight,
+                  int32_t* pairs, void* tiles);
+
+/* act[t * top + j, :] = g sigmoid(1.702 g) (u + 1), g = min(G_e x_t, limit), u = clamp(U_e x_t, -limit, limit)
+ * for the chosen experts e = expert[t, j] < n_experts (other rows of act are not written). gate / up: [n_experts,
+ * n_inter, k_in], expert_stride elements between experts. tile_pairs 0 (expert only), or what mui_moe_route
+ * was given, with its pairs and tiles. */
+int mui_moe_gateup(mui_stream_t stream, int dtype, const void* gate, const void* up, long expert_stride,
+                   const void* x, float limit, const int32_t* expert, const int32_t* pairs,
+                   const void* tiles, int tile_pairs, void* act, int n_experts, int n_inter, int k_in,
+                   int top, int tokens);
+
+/* out[pair, :] = D_e act[pair, :]; down: [n_experts, n_out, k_in]. */
+int mui_moe_down(mui_stream_t stream, int dtype, const void* down, long expert_stride, const void* act,
+                 const int32_t* expert, const int32_t* pairs, const void* tiles, int tile_pairs, void* out,
+                 int n_experts, int n_out, int k_in, int top, int tokens);
+
+/* Latent attention, after the down projections. down rows (down_pitch elements apart, batch * t of them) are
+ * [q_rank query latent | kv_rank latent | rot_dim rotated key part], the last two only where kv_gain != NULL.
+ *   q_latent[tok] = q_gain * rmsnorm(query latent)
+ *   c_cache[b, slot] = kv_gain * rmsnorm(latent), r_cache[b, slot] = rotate(key part, slot - row_start[b])
+ *   cos_sin[tok] = [cos | sin] of the token's rot_dim / 2 angles
+ * slot = cache_position[t] (device); rows of the caches are kv_rank / rot_dim elements; slots outside
+ * [0, max_cache_len) are skipped. inv_freq: double [rot_dim / 2]; pairs are (i, i + rot_dim / 2). */
+int mui_latent_prepare(mui_stream_t stream, int dtype, const void* down, long down_pitch, const void* q_gain,
+                       const void* kv_gain, float epsilon, const double* inv_freq,
+                       const int64_t* cache_position, const int64_t* row_start, void* q_latent,
+                       float* cos_sin, void* c_cache, long c_batch_stride, void* r_cache,
+                       long r_batch_stride, int batch, int t, int q_rank, int kv_rank, int rot_dim,
+                       int max_cache_len);
+
+/* Which kernels serve a call: PLAIN (one workgroup per query and head: fp32, odd sizes), DECODE (attention
+ * over the latent rows themselves), PREFILL (mui_latent_prefill_attention). `tokens`: per batch row. */
+#define MUI_LATENT_PLAIN 0
+#define MUI_LATENT_DECODE 1
+#define MUI_LATENT_PREFILL 2
+int mui_latent_attention_route(int dtype, int tokens, int heads, int dim, int rot_dim, int vdim, int kv_rank);
+size_t mui_latent_decode_scratch_bytes(int batch, int t, int heads, int kv_rank, int rot_dim, int span);
+
+/* out[tok, h, :] = Wuv_h sum_s p_s c_s, p = softmax over the visible slots s of
+ * (q[tok, h, :dim] . Wuk_h c_s + rotate(q[tok, h, dim:]) . r_s) * scale; visible: row_start[b] <= s <= slot,
+ * and s > slot - window where window > 0. The caches already hold the new rows. route PLAIN (scratch NULL)
+ * or DECODE: span = the largest number of visible keys (the window, or the cache's capacity), scratch
+ * mui_latent_decode_scratch_bytes() bytes, 256-byte aligned. */
+int mui_latent_attention(mui_stream_t stream, int dtype, int route, const void* q, const float* cos_sin,
+                         const void* w_uk, const void* w_uv, const void* c_cache, long c_batch_stride,
+                         const void* r_cache, long r_batch_stride, const int64_t* cache_position,
+                         const int64_t* row_start, float scale, int window, void* scratch, int span,
+                         void* out, int batch, int t, int heads, int dim, int rot_dim, int vdim, int kv_rank,
+                         int max_cache_len);
+
+/* The same for t tokens in slots q_first ... of ONE batch row with keys and values made beforehand:
+ * kv [kv_rows, heads * dim | heads * vdim] holds Wuk c and Wuv c of slots kv_first ... (kv_first + kv_rows =
+ * q_first + t; everything visible must be inside). q, cos_sin and out are those of the whole batch. 16-bit
+ * types, dim + rot_dim <= 256, vdim <= 256. */
+int mui_latent_prefill_attention(mui_stream_t stream, int dtype, const void* q, const float* cos_sin,
+                                 const void* kv, int kv_first, int kv_rows, const void* r_cache,
+                                 long r_batch_stride, const int64_t* row_start, float scale, int window,
+                                 int q_first, void* out, int batch_row, int t, int heads, int dim, int rot_dim,
+                                 int vdim);
+
+/* Matrix-memory recurrence over t tokens per batch row, from and to the state S [batch, heads, dk, dv],
+ * n [batch, heads, slices, dk], m [batch, heads, slices] (fp32; slices = mui_mlstm_slices(dv) equal copies; all
+ * zero: a fresh sequence):
+ *   i = cap tanh(gates[tok, h] / cap), f = logsigmoid(cap tanh(gates[tok, heads + h] / cap))
+ *   m' = max(f + m, i);  S' = e^{f + m - m'} S + e^{i - m'} k v^T;  n' = e^{f + m - m'} n + e^{i - m'} k
+ *   o[tok, h, :] = S'^T q / (max(|n' . q|, e^{-m'}) + 1e-6)
+ * q (multiplied by q_scale in fp32), k, v: token rows token_pitch elements apart, heads dense. gates, o: fp32.
+ * Tokens with cache_position[t] < row_start[b] (row_start may be NULL) leave the state alone. workspace:
+ * mui_mlstm_workspace_bytes() bytes (0 up to MUI_MAX_TOKENS tokens). */
+int mui_mlstm_slices(int dv);
+size_t mui_mlstm_workspace_bytes(int batch, int t, int heads, int dk, int dv);
+int mui_mlstm(mui_stream_t stream, int dtype, const void* q, const void* k, const void* v, long token_pitch,
+              const float* gates, float q_scale, float gate_cap, float* state_s, float* state_n,
+              float* state_m, const int64_t* cache_position, const int64_t* row_start, float* o,
+              void* workspace, int batch, int t, int heads, int dk, int dv);
+
+/* y[tok, h, :] = o[tok, h, :] * rsqrt(mean over the head + epsilon) * gain[h, :] * sigmoid(gate[tok, h, :]) */
+int mui_mlstm_output(mui_stream_t stream, int dtype, const float* o, const void* gain, const void* gate,
+                     long gate_pitch, float epsilon, void* y, int tokens, int heads, int dv);
 
 #ifdef __cplusplus
 }

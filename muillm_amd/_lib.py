@@ -20,7 +20,9 @@ TUNE_HEADER_PATH = os.path.join(os.path.dirname(_HERE), "include", "muillm_amd_t
 MUI_OK = 0
 MUI_DTYPE_F16 = 0
 MUI_DTYPE_BF16 = 1
+MUI_DTYPE_F32 = 2
 MUI_MAX_TOKENS = 16
+MUI_LATENT_PLAIN, MUI_LATENT_DECODE, MUI_LATENT_PREFILL = 0, 1, 2
 
 
 class MuiDeviceInfo(ctypes.Structure):
@@ -95,6 +97,29 @@ _SIGNATURES = {
     "mui_embedding": (c_int, [_P, c_int, _P, c_long, _P, c_int, _P, c_int, c_int, c_int]),
     "mui_decoder_stack_workspace_bytes": (ctypes.c_size_t, [_P, c_int, c_int]),
     "mui_decoder_stack_step": (c_int, [_P, _P, c_int, _P, _P, _P, c_long, _P, c_int, _P, c_long, c_int, _P]),
+    "mui_residual_norm": (c_int, [_P, c_int, _P, _P, c_float, _P, _P, c_float, _P, _P, c_int, c_int]),
+    "mui_moe_residual_norm": (c_int, [_P, c_int, _P, _P, _P, _P, _P, c_int, c_int, _P, _P, c_float, _P, _P, c_int,
+                                      c_int]),
+    "mui_linear_f32": (c_int, [_P, c_int, _P, _P, _P, _P, c_int, c_int, c_int]),
+    "mui_moe_tile_pairs": (c_int, [c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mui_moe_max_tiles": (c_int, [c_int, c_int, c_int, c_int]),
+    "mui_moe_route": (c_int, [_P, c_int, _P, _P, c_int, c_int, c_int, c_int, c_int, _P, _P, _P, _P]),
+    "mui_moe_gateup": (c_int, [_P, c_int, _P, _P, c_long, _P, c_float, _P, _P, _P, c_int, _P, c_int, c_int, c_int,
+                               c_int, c_int]),
+    "mui_moe_down": (c_int, [_P, c_int, _P, c_long, _P, _P, _P, _P, c_int, _P, c_int, c_int, c_int, c_int, c_int]),
+    "mui_latent_prepare": (c_int, [_P, c_int, _P, c_long, _P, _P, c_float, _P, _P, _P, _P, _P, _P, c_long, _P, c_long,
+                                   c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mui_latent_attention_route": (c_int, [c_int, c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mui_latent_decode_scratch_bytes": (ctypes.c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mui_latent_attention": (c_int, [_P, c_int, c_int, _P, _P, _P, _P, _P, c_long, _P, c_long, _P, _P, c_float, c_int,
+                                     _P, c_int, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mui_latent_prefill_attention": (c_int, [_P, c_int, _P, _P, _P, c_int, c_int, _P, c_long, _P, c_float, c_int,
+                                             c_int, _P, c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mui_mlstm_slices": (c_int, [c_int]),
+    "mui_mlstm_workspace_bytes": (ctypes.c_size_t, [c_int, c_int, c_int, c_int, c_int]),
+    "mui_mlstm": (c_int, [_P, c_int, _P, _P, _P, c_long, _P, c_float, c_float, _P, _P, _P, _P, _P, _P, _P, c_int,
+                          c_int, c_int, c_int, c_int]),
+    "mui_mlstm_output": (c_int, [_P, c_int, _P, _P, _P, c_long, c_float, _P, c_int, c_int, c_int]),
     "mui_probe_read": (c_int, [_P, _P, ctypes.c_uint64, _P]),
     "mui_tune_lock": (c_int, []),
     "mui_tune_gemv": (c_int, [c_int, c_int]),

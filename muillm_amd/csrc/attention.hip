@@ -485,7 +485,6 @@ __global__ void __launch_bounds__(NW * kWave) attn_decode_kernel(
 // ---------------------------------------------------------------------------------------
 typedef _Float16 af16x8 __attribute__((ext_vector_type(8)));
 typedef __bf16 abf16x8 __attribute__((ext_vector_type(8)));
-typedef short ai16x4 __attribute__((ext_vector_type(4)));
 
 template <typename T>
 __device__ __forceinline__ f32x4 attn_mfma(u32x4 a, u32x4 b, f32x4 c);
@@ -496,12 +495,6 @@ __device__ __forceinline__ f32x4 attn_mfma<F16>(u32x4 a, u32x4 b, f32x4 c) {
 template <>
 __device__ __forceinline__ f32x4 attn_mfma<BF16>(u32x4 a, u32x4 b, f32x4 c) {
   return __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(abf16x8, a), __builtin_bit_cast(abf16x8, b), c, 0, 0, 0);
-}
-
-__device__ __forceinline__ u32x2 lds_read_tr16(const uint16_t* lds_ptr) {
-  typedef ai16x4 __attribute__((address_space(3))) * lds_v4;
-  const ai16x4 r = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4)lds_ptr);
-  return __builtin_bit_cast(u32x2, r);
 }
 
 constexpr int kMfTok = 32;        // tokens per wave block

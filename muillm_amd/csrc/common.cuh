@@ -24,6 +24,7 @@ typedef float f32x4 __attribute__((ext_vector_type(4)));
 // ---------------------------------------------------------------------------------------
 struct F16 {
   static constexpr int kDtype = MUI_DTYPE_F16;
+  typedef uint16_t storage;
   // low / high half of a packed 32-bit word -> fp32
   static __device__ __forceinline__ float lo(uint32_t w) {
     return (float)__builtin_bit_cast(f16x2, w).x;
@@ -48,6 +49,7 @@ struct F16 {
 
 struct BF16 {
   static constexpr int kDtype = MUI_DTYPE_BF16;
+  typedef uint16_t storage;
   static __device__ __forceinline__ float lo(uint32_t w) {
     return __builtin_bit_cast(float, w << 16);
   }
@@ -67,6 +69,15 @@ struct BF16 {
     const f32x2_t v = {a, b};
     return __builtin_bit_cast(uint32_t, __builtin_convertvector(v, bf16x2_t));
   }
+};
+
+// 32-bit storage: models that run in fp32 take the same kernels where those are written against
+// one() / pack() and `storage` (none of the packed-word helpers applies)
+struct F32 {
+  static constexpr int kDtype = MUI_DTYPE_F32;
+  typedef float storage;
+  static __device__ __forceinline__ float one(float v) { return v; }
+  static __device__ __forceinline__ float pack(float v) { return v; }
 };
 
 template <typename T>
@@ -115,6 +126,38 @@ __device__ __forceinline__ uint16_t ld2(const void* p) {
 template <bool STREAM>
 __device__ __forceinline__ u32x4 ld16_sel(const void* p) {
   if constexpr (STREAM) return ld16_stream(p); else return ld16(p);
+}
+
+// 8 consecutive elements as fp32 (16-byte aligned 16-bit storage, or 32-byte runs of fp32)
+template <typename T>
+__device__ __forceinline__ void load8(const typename T::storage* p, float (&f)[8]) {
+  if constexpr (T::kDtype == MUI_DTYPE_F32) {
+    const u32x4 a = ld16(p), b = ld16(p + 4);
+    const uint32_t w[8] = {a.x, a.y, a.z, a.w, b.x, b.y, b.z, b.w};
+#pragma unroll
+    for (int i = 0; i < 8; ++i) f[i] = __builtin_bit_cast(float, w[i]);
+  } else {
+    unpack8<T>(ld16(p), f);
+  }
+}
+template <typename T>
+__device__ __forceinline__ void store8(typename T::storage* p, const float (&f)[8]) {
+  if constexpr (T::kDtype == MUI_DTYPE_F32) {
+    *(f32x4*)p = f32x4{f[0], f[1], f[2], f[3]};
+    *(f32x4*)(p + 4) = f32x4{f[4], f[5], f[6], f[7]};
+  } else {
+    *(u32x4*)p = pack8<T>(f);
+  }
+}
+
+// A 4 x 16 block of 16-bit elements read transposed from LDS: within a group of 16 lanes, lane i
+// receives element i % 4 of the 8-byte rows addressed by lanes i / 4, i / 4 + 4, i / 4 + 8 and
+// i / 4 + 12 -- four rows of column i when lane i points at row i / 4, columns 4 (i % 4) .. + 3.
+__device__ __forceinline__ u32x2 lds_read_tr16(const uint16_t* lds_ptr) {
+  typedef short i16x4_t __attribute__((ext_vector_type(4)));
+  typedef i16x4_t __attribute__((address_space(3))) * lds_v4;
+  const i16x4_t r = __builtin_amdgcn_ds_read_tr16_b64_v4i16((lds_v4)lds_ptr);
+  return __builtin_bit_cast(u32x2, r);
 }
 
 // ---------------------------------------------------------------------------------------
@@ -269,6 +312,18 @@ static inline int balanced_grid(int n_items, int per_cu) {
 static inline int launch_status() {
   hipError_t e = hipGetLastError();
   return e == hipSuccess ? MUI_OK : MUI_ERR_LAUNCH;
+}
+
+// Launch with `lds` bytes of dynamic LDS; a kernel that also declares static LDS, or asks for more than
+// the default limit, has its limit raised first.
+template <typename Kernel, typename Params>
+static int launch_with_lds(Kernel kernel, dim3 grid, dim3 block, size_t lds, hipStream_t s, const Params& p) {
+  if (lds > 160 * 1024) return MUI_ERR_UNSUPPORTED;
+  if (lds > 48 * 1024 &&
+      hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
+    return MUI_ERR_LAUNCH;
+  hipLaunchKernelGGL(kernel, grid, block, lds, s, p);
+  return launch_status();
 }
 
 }  // namespace mui

@@ -1,0 +1,647 @@
+// Mixture-of-experts feed-forward: routing, grouping of the chosen (token, expert) pairs by expert, and
+// the experts' two matrix products over the groups.
+//
+//   logits   fp32 [tokens, outputs]  (linear_f32 below; also the gates of recurrent layers)
+//   route    s = softmax(logits); the `top` outputs with the largest s + correction are chosen, weighted
+//            by their s. Outputs >= n_experts are identity experts: they take part in the choice and are
+//            added by mui_moe_residual_norm, no product is computed for them.
+//   group    pairs sorted by expert, cut into tiles of at most `tile_pairs` pairs of ONE expert
+//   gateup   act[pair] = a(G_e x, U_e x), a(g, u) = g' sigmoid(1.702 g') (u' + 1) with g' = min(g, limit),
+//            u' = clamp(u, -limit, limit)
+//   down     out[pair] = D_e act[pair]
+//
+// Everything stays on the device (no counts travel to the host): the grids cover the largest possible
+// number of tiles and workgroups without one leave at once, so a captured decode step replays whatever
+// the routing does.
+//
+// Products, wave64 v_mfma_f32_16x16x32 (weights = A rows, pairs = B columns):
+//   tile 16   up to 16 pairs of an expert: 16 gate + 16 up rows (or 32 rows) per workgroup, K dealt out to
+//             its four waves, operands straight from global memory in matrix order. Decode and short
+//             prompts: every chosen expert's weights are streamed once.
+//   tile 128  128 pairs x 128 rows, both operands through swizzled LDS stages filled by LDS-direct loads.
+// fp32 models and sizes that are no multiple of 8 take a plain one-wave-per-output kernel.
+#include "skinny.cuh"
+
+namespace mui {
+
+enum { MOE_GATEUP = 0, MOE_DOWN = 1, MOE_F32 = 2 };
+
+struct MoeTile { int expert, first, count, pad; };
+
+__device__ __forceinline__ float moe_act(float g, float u, float limit) {
+  g = fminf(g, limit);
+  u = fminf(fmaxf(u, -limit), limit);
+  return g / (1.0f + __expf(-1.702f * g)) * (u + 1.0f);
+}
+
+// ---------------------------------------------------------------------------------------
+// fp32 outputs of a small matrix: y[t, n] = W[n, :] . x[t, :] + bias[n], one wave per row
+// ---------------------------------------------------------------------------------------
+template <typename T, bool VEC>
+__global__ void __launch_bounds__(256) linear_f32_rows_kernel(const typename T::storage* w, const typename T::storage* x,
+                                                              const typename T::storage* bias, float* y, int n, int k,
+                                                              int tokens) {
+  constexpr int TB = 4;  // tokens per pass over a row
+  const int lane = threadIdx.x & (kWave - 1);
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (row >= n) return;
+  const float b = bias ? T::one(bias[row]) : 0.f;
+  const typename T::storage* wr = w + (long)row * k;
+  for (int t0 = blockIdx.y * TB; t0 < tokens; t0 += gridDim.y * TB) {
+    float acc[TB];
+#pragma unroll
+    for (int j = 0; j < TB; ++j) acc[j] = 0.f;
+    if constexpr (VEC) {
+#pragma unroll 4
+      for (int c = lane * 8; c < k; c += kWave * 8) {
+        float wf[8];
+        load8<T>(wr + c, wf);
+#pragma unroll
+        for (int j = 0; j < TB; ++j) {
+          const int t = t0 + j < tokens ? t0 + j : tokens - 1;
+          float xf[8];
+          load8<T>(x + (long)t * k + c, xf);
+#pragma unroll
+          for (int i = 0; i < 8; ++i) acc[j] = fmaf(wf[i], xf[i], acc[j]);
+        }
+      }
+    } else {
+      for (int c = lane; c < k; c += kWave) {
+        const float wf = T::one(wr[c]);
+#pragma unroll
+        for (int j = 0; j < TB; ++j) {
+          const int t = t0 + j < tokens ? t0 + j : tokens - 1;
+          acc[j] = fmaf(wf, T::one(x[(long)t * k + c]), acc[j]);
+        }
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < TB; ++j) {
+      const float s = wave_sum(acc[j]);
+      if (lane == 0 && t0 + j < tokens) y[(long)(t0 + j) * n + row] = s + b;
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------
+// routing
+// ---------------------------------------------------------------------------------------
+constexpr int kMaxRouter = 1024;   // router outputs
+constexpr int kRouteThreads = 1024;
+constexpr int kRouterPerLane = kMaxRouter / kWave;
+
+// one token by one wave
+template <typename T>
+__device__ __forceinline__ void route_token(const float* lg, const typename T::storage* corr, int n_out, int top,
+                                            int lane, int32_t* expert, float* weight) {
+  float s[kRouterPerLane], choice[kRouterPerLane];
+  float mx = -INFINITY;
+#pragma unroll
+  for (int i = 0; i < kRouterPerLane; ++i) {
+    const int e = lane + kWave * i;
+    s[i] = e < n_out ? lg[e] : -INFINITY;
+    mx = fmaxf(mx, s[i]);
+    if (kWave * (i + 1) >= n_out) break;
+  }
+  mx = wave_max(mx);
+  float sum = 0.f;
+#pragma unroll
+  for (int i = 0; i < kRouterPerLane; ++i) {
+    s[i] = expf(s[i] - mx);
+    sum += s[i];
+    if (kWave * (i + 1) >= n_out) break;
+  }
+  sum = wave_sum(sum);
+#pragma unroll
+  for (int i = 0; i < kRouterPerLane; ++i) {
+    const int e = lane + kWave * i;
+    s[i] = s[i] / sum;
+    choice[i] = e < n_out ? s[i] + (corr ? T::one(corr[e]) : 0.f) : -INFINITY;
+    if (kWave * (i + 1) >= n_out) break;
+  }
+  for (int j = 0; j < top; ++j) {
+    float best = -INFINITY, bs = 0.f;
+    int bi = 0x7fffffff;
+#pragma unroll
+    for (int i = 0; i < kRouterPerLane; ++i) {
+      const int e = lane + kWave * i;
+      if (choice[i] > best) { best = choice[i]; bi = e; bs = s[i]; }
+      if (kWave * (i + 1) >= n_out) break;
+    }
+#pragma unroll
+    for (int d = 1; d < kWave; d <<= 1) {
+      const float ob = __shfl_xor(best, d), os = __shfl_xor(bs, d);
+      const int oi = __shfl_xor(bi, d);
+      if (ob > best || (ob == best && oi < bi)) { best = ob; bi = oi; bs = os; }
+    }
+    if (bi >= n_out) bi = 0;  // nothing left to choose (NaN logits): stays in range
+#pragma unroll
+    for (int i = 0; i < kRouterPerLane; ++i) {
+      if (lane + kWave * i == bi) choice[i] = -INFINITY;
+      if (kWave * (i + 1) >= n_out) break;
+    }
+    if (lane == 0) {
+      expert[j] = bi;
+      weight[j] = bs;
+    }
+  }
+}
+
+template <typename T>
+__global__ void __launch_bounds__(256) moe_route_kernel(const float* logits, const typename T::storage* corr, int n_out,
+                                                        int top, int tokens, int32_t* expert, float* weight) {
+  const int t = blockIdx.x * 4 + (threadIdx.x >> 6);
+  if (t < tokens)
+    route_token<T>(logits + (long)t * n_out, corr, n_out, top, threadIdx.x & (kWave - 1), expert + (long)t * top,
+                   weight + (long)t * top);
+}
+
+// One workgroup: (ROUTE: the routing of all tokens, then) count per expert, cut into tiles, scatter.
+// tiles[0].count = number of tiles, tiles[1 + i] the i-th tile; unused entries up to max_tiles get count 0.
+template <typename T, bool ROUTE>
+__global__ void __launch_bounds__(kRouteThreads) moe_group_kernel(const float* logits, const typename T::storage* corr,
+                                                                  int n_out, int n_experts, int top, int tokens,
+                                                                  int tile_pairs, int max_tiles, int32_t* expert,
+                                                                  float* weight, int32_t* pairs, MoeTile* tiles) {
+  __shared__ int count[kMaxRouter], cursor[kMaxRouter], first_tile[kMaxRouter];
+  __shared__ int n_tiles_s;
+  const int t = threadIdx.x;
+  const int n_pairs = tokens * top;
+  for (int e = t; e < n_experts; e += kRouteThreads) count[e] = 0;
+  if constexpr (ROUTE) {
+    for (int tk = t >> 6; tk < tokens; tk += kRouteThreads / kWave)
+      route_token<T>(logits + (long)tk * n_out, corr, n_out, top, t & (kWave - 1), expert + (long)tk * top,
+                     weight + (long)tk * top);
+    __threadfence_block();
+  }
+  __syncthreads();
+  for (int i = t; i < n_pairs; i += kRouteThreads) {
+    const int e = expert[i];
+    if (e < n_experts) atomicAdd(&count[e], 1);
+  }
+  __syncthreads();
+  if (t < kWave) {  // exclusive sums over experts: 64 at a time by one wave
+    int pair_base = 0, tile_base = 0;
+    for (int e0 = 0; e0 < n_experts; e0 += kWave) {
+      const int e = e0 + t;
+      const int c = e < n_experts ? count[e] : 0;
+      const int nt = (c + tile_pairs - 1) / tile_pairs;
+      int sc = c, st = nt;
+#pragma unroll
+      for (int d = 1; d < kWave; d <<= 1) {
+        const int oc = __shfl_up(sc, d), ot = __shfl_up(st, d);
+        if (t >= d) { sc += oc; st += ot; }
+      }
+      if (e < n_experts) {
+        cursor[e] = pair_base + sc - c;
+        first_tile[e] = tile_base + st - nt;
+      }
+      pair_base += __shfl(sc, kWave - 1);
+      tile_base += __shfl(st, kWave - 1);
+    }
+    if (t == 0) n_tiles_s = tile_base < max_tiles ? tile_base : max_tiles;
+  }
+  __syncthreads();
+  const int n_tiles = n_tiles_s;
+  for (int e = t; e < n_experts; e += kRouteThreads) {
+    const int c = count[e], base = cursor[e], ft = first_tile[e];
+    for (int i = 0; i * tile_pairs < c && ft + i < max_tiles; ++i) {
+      const int left = c - i * tile_pairs;
+      tiles[1 + ft + i] = MoeTile{e, base + i * tile_pairs, left < tile_pairs ? left : tile_pairs, 0};
+    }
+  }
+  for (int i = n_tiles + t; i < max_tiles; i += kRouteThreads) tiles[1 + i] = MoeTile{0, 0, 0, 0};
+  if (t == 0) tiles[0] = MoeTile{0, 0, n_tiles, 0};
+  __syncthreads();  // cursors are read above before they move
+  for (int i = t; i < n_pairs; i += kRouteThreads) {
+    const int e = expert[i];
+    if (e < n_experts) pairs[atomicAdd(&cursor[e], 1)] = i;
+  }
+}
+
+// ---------------------------------------------------------------------------------------
+// products
+// ---------------------------------------------------------------------------------------
+struct MoeGemmParams {
+  const uint16_t* w0;   // gate / down / matrix: [experts, n, k]
+  const uint16_t* w1;   // up
+  long expert_stride;   // elements between experts (w0 and w1)
+  const uint16_t* x;    // gateup, f32: [tokens, k]; down: [pairs, k]
+  const uint16_t* bias; // f32: [n] or null
+  void* y;              // gateup: [pairs, n] 16-bit; down: [pairs, n] 16-bit; f32: [tokens, n] fp32
+  const int32_t* pairs; // sorted pairs, null: pair i is i (f32)
+  const MoeTile* tiles;
+  int n, k, top, tokens;
+  float limit;
+  int max_tiles;
+};
+
+__device__ __forceinline__ MoeTile moe_tile_at(const MoeGemmParams& p, int i, int tile_pairs) {
+  if (p.tiles) return p.tiles[1 + i];
+  const int first = i * tile_pairs, left = p.tokens - first;
+  return MoeTile{0, first, left < 0 ? 0 : (left < tile_pairs ? left : tile_pairs), 0};
+}
+
+template <typename T, int EPI>
+__global__ void __launch_bounds__(256) moe_tile16_kernel(const MoeGemmParams p) {
+  constexpr int ROWS = EPI == MOE_GATEUP ? 16 : 32;  // outputs per workgroup
+  constexpr int UNR = 4;
+  __shared__ float red[4][2][16][17];
+  __shared__ int prow[16];
+  const MoeTile tile = moe_tile_at(p, blockIdx.y, 16);
+  if (tile.count <= 0) return;
+  const int t = threadIdx.x, lane = t & (kWave - 1), wave = t >> 6;
+  const int r16 = lane & 15, g = lane >> 4;
+  const int o0 = blockIdx.x * ROWS;
+  if (t < 16) {
+    const int i = tile.first + (t < tile.count ? t : 0);
+    prow[t] = p.pairs ? p.pairs[i] : i;
+  }
+  const int mine = tile.first + (r16 < tile.count ? r16 : 0);
+  const int pair = p.pairs ? p.pairs[mine] : mine;
+  const uint16_t* xr = p.x + (long)(EPI == MOE_GATEUP ? pair / p.top : pair) * p.k;
+  const long eb = (long)tile.expert * p.expert_stride;
+  const int ra = o0 + r16 < p.n ? o0 + r16 : p.n - 1;
+  const int rb = EPI == MOE_GATEUP ? ra : (o0 + 16 + r16 < p.n ? o0 + 16 + r16 : p.n - 1);
+  const uint16_t* wa = p.w0 + eb + (long)ra * p.k;
+  const uint16_t* wb = (EPI == MOE_GATEUP ? p.w1 : p.w0) + eb + (long)rb * p.k;
+  f32x4 acc0 = {0.f, 0.f, 0.f, 0.f}, acc1 = {0.f, 0.f, 0.f, 0.f};
+  const int steps = (p.k + 31) >> 5;
+  const u32x4 zero = {0u, 0u, 0u, 0u};
+  for (int s0 = wave; s0 < steps; s0 += 4 * UNR) {
+    u32x4 a[UNR], b[UNR], x[UNR];
+#pragma unroll
+    for (int u = 0; u < UNR; ++u) {
+      const int kk = (s0 + 4 * u) * 32 + g * 8;
+      const int off = kk < p.k ? kk : 0;  // chunks past the row read its start and meet x = 0
+      a[u] = ld16_stream(wa + off);
+      b[u] = ld16_stream(wb + off);
+      x[u] = ld16(xr + off);
+    }
+#pragma unroll
+    for (int u = 0; u < UNR; ++u) {
+      const int kk = (s0 + 4 * u) * 32 + g * 8;
+      const bool live = kk < p.k;
+      const u32x4 xv = live ? x[u] : zero;
+      acc0 = mfma16x16x32<T>(live ? a[u] : zero, xv, acc0);
+      acc1 = mfma16x16x32<T>(live ? b[u] : zero, xv, acc1);
+    }
+  }
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    red[wave][0][4 * g + r][r16] = acc0[r];
+    red[wave][1][4 * g + r][r16] = acc1[r];
+  }
+  __syncthreads();
+  const int row = t & 15, col = t >> 4;
+  float v0 = 0.f, v1 = 0.f;
+#pragma unroll
+  for (int w = 0; w < 4; ++w) { v0 += red[w][0][row][col]; v1 += red[w][1][row][col]; }
+  if (col >= tile.count) return;
+  const long out = (long)prow[col] * p.n;
+  if constexpr (EPI == MOE_GATEUP) {
+    if (o0 + row < p.n) ((uint16_t*)p.y)[out + o0 + row] = T::pack(moe_act(v0, v1, p.limit));
+  } else if constexpr (EPI == MOE_DOWN) {
+    if (o0 + row < p.n) ((uint16_t*)p.y)[out + o0 + row] = T::pack(v0);
+    if (o0 + 16 + row < p.n) ((uint16_t*)p.y)[out + o0 + 16 + row] = T::pack(v1);
+  } else {
+    const int n0 = o0 + row, n1 = o0 + 16 + row;
+    if (n0 < p.n) ((float*)p.y)[out + n0] = v0 + (p.bias ? T::one(p.bias[n0]) : 0.f);
+    if (n1 < p.n) ((float*)p.y)[out + n1] = v1 + (p.bias ? T::one(p.bias[n1]) : 0.f);
+  }
+}
+
+// 128 rows (gate/up: 64 outputs, each wave 32 gate rows and the 32 up rows of the same outputs) x 128
+// pairs, 64 k-values per step, four waves of 64 x 64. LDS rows are 128 bytes; 16-byte chunk c of row r
+// lives at chunk c ^ ((r >> 1) & 7). DMA (k % 64 == 0): LDS-direct loads, lane i of a wave instruction
+// fills slot i of eight consecutive rows, the swizzle applied to the source chunk. Otherwise the chunks
+// go through registers and those past the end of a row are zeroed.
+constexpr int kMgTile = 128, kMgK = 64;
+extern __shared__ __align__(16) unsigned char moe_smem[];
+
+template <typename T, int EPI, bool DMA>
+__global__ void __launch_bounds__(256, 2) moe_tile128_kernel(const MoeGemmParams p) {
+  constexpr int OUT = EPI == MOE_GATEUP ? kMgTile / 2 : kMgTile;
+  typedef uint16_t Stage[kMgTile * kMgK];
+  Stage* w_lds = (Stage*)moe_smem;
+  Stage* x_lds = (Stage*)(moe_smem + 2 * sizeof(Stage));
+  __shared__ int prow[kMgTile];
+
+  // tile order: four pair tiles (of one expert, mostly) fastest, then row tiles, so that the workgroups
+  // an XCD runs at a time share weight rows and token rows; the tiles are dealt to the XCDs in
+  // contiguous shares of what there really is
+  const int n_tiles = p.tiles[0].count;
+  const int r_tiles = (p.n + OUT - 1) / OUT;
+  const int total = ((n_tiles + 3) / 4) * 4 * r_tiles;
+  const int share = (total + 7) / 8;
+  const int slot = blockIdx.x >> 3, id = (blockIdx.x & 7) * share + slot;
+  if (slot >= share || id >= total) return;
+  const int sup = id / (4 * r_tiles), in_sup = id - sup * 4 * r_tiles;
+  const int ti = sup * 4 + (in_sup & 3);
+  if (ti >= n_tiles) return;
+  const MoeTile tile = p.tiles[1 + ti];
+  const int o0 = (in_sup >> 2) * OUT;
+
+  const int t = threadIdx.x, lane = t & (kWave - 1), wave = t >> 6;
+  const int wr = wave >> 1, wt = wave & 1;
+  if (t < kMgTile) prow[t] = p.pairs[tile.first + (t < tile.count ? t : 0)];
+  __syncthreads();
+  const long eb = (long)tile.expert * p.expert_stride;
+  // tile row r -> weight row
+  auto wrow = [&](int r) -> const uint16_t* {
+    if constexpr (EPI == MOE_GATEUP) {
+      const int h = r >> 6, in = r & 63;
+      int o = o0 + h * 32 + (in & 31);
+      o = o < p.n ? o : p.n - 1;
+      return (in >= 32 ? p.w1 : p.w0) + eb + (long)o * p.k;
+    } else {
+      int o = o0 + r;
+      o = o < p.n ? o : p.n - 1;
+      return p.w0 + eb + (long)o * p.k;
+    }
+  };
+  const int sr = lane >> 3, sc = lane & 7;
+  const uint16_t *wsrc[4], *xsrc[4];  // this lane's source rows: tile row (q * 4 + wave) * 8 + sr
+  int chunk[4];
+#pragma unroll
+  for (int q = 0; q < 4; ++q) {
+    const int r = (q * 4 + wave) * 8 + sr;
+    const int pr = prow[r];
+    wsrc[q] = wrow(r);
+    xsrc[q] = p.x + (long)(EPI == MOE_GATEUP ? pr / p.top : pr) * p.k;
+    chunk[q] = (sc ^ ((r >> 1) & 7)) * 8;
+  }
+  const int steps = (p.k + kMgK - 1) / kMgK;
+  auto dma = [&](int s, int buf) {
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int base = (q * 4 + wave) * 8 * kMgK;
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(wsrc[q] + s * kMgK + chunk[q]),
+                                       (__attribute__((address_space(3))) void*)&w_lds[buf][base], 16, 0, 0);
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(xsrc[q] + s * kMgK + chunk[q]),
+                                       (__attribute__((address_space(3))) void*)&x_lds[buf][base], 16, 0, 0);
+    }
+  };
+  u32x4 rw[4], rx[4];
+  auto fetch = [&](int s) {
+    const u32x4 zero = {0u, 0u, 0u, 0u};
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int kk = s * kMgK + chunk[q];
+      const bool live = kk < p.k;
+      const u32x4 a = ld16(wsrc[q] + (live ? kk : 0)), b = ld16(xsrc[q] + (live ? kk : 0));
+      rw[q] = live ? a : zero;
+      rx[q] = live ? b : zero;
+    }
+  };
+  auto put = [&](int buf) {
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      const int at = (q * 4 + wave) * 8 * kMgK + lane * 8;
+      *(u32x4*)&w_lds[buf][at] = rw[q];
+      *(u32x4*)&x_lds[buf][at] = rx[q];
+    }
+  };
+  f32x4 acc[4][4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i)
+#pragma unroll
+    for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const int r16 = lane & 15, lg = lane >> 4, lsw = (r16 >> 1) & 7;
+  const int a_base = (wr * 64 + r16) * kMgK, b_base = (wt * 64 + r16) * kMgK;
+
+  if constexpr (DMA) {
+    dma(0, 0);
+  } else {
+    fetch(0);
+    put(0);
+  }
+  for (int s = 0; s < steps; ++s) {
+    const int buf = s & 1;
+    const bool more = s + 1 < steps;
+    if constexpr (DMA) __builtin_amdgcn_s_waitcnt(0x0F70);  // this wave's blocks of step s have landed
+    __syncthreads();  // ... and everybody's; everybody is done with the other stage
+    if (more) {
+      if constexpr (DMA) dma(s + 1, buf ^ 1);
+      else fetch(s + 1);
+    }
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) {
+      u32x4 a[4], b[4];
+#pragma unroll
+      for (int j = 0; j < 4; ++j) b[j] = *(const u32x4*)&x_lds[buf][b_base + j * 16 * kMgK + (((kk * 4 + lg) ^ lsw) * 8)];
+#pragma unroll
+      for (int i = 0; i < 4; ++i) a[i] = *(const u32x4*)&w_lds[buf][a_base + i * 16 * kMgK + (((kk * 4 + lg) ^ lsw) * 8)];
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = mfma16x16x32<T>(a[i], b[j], acc[i][j]);
+    }
+    if constexpr (!DMA) {
+      if (more) put(buf ^ 1);
+    }
+  }
+  // lane: pair column r16, rows 4 lg + r of every 16-row tile
+#pragma unroll
+  for (int j = 0; j < 4; ++j) {
+    const int c = wt * 64 + j * 16 + r16;
+    if (c >= tile.count) continue;
+    uint16_t* yr = (uint16_t*)p.y + (long)prow[c] * p.n;
+    if constexpr (EPI == MOE_GATEUP) {
+#pragma unroll
+      for (int i = 0; i < 2; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int o = o0 + wr * 32 + i * 16 + 4 * lg + r;
+          if (o < p.n) yr[o] = T::pack(moe_act(acc[i][j][r], acc[i + 2][j][r], p.limit));
+        }
+    } else {
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int o = o0 + wr * 64 + i * 16 + 4 * lg + r;
+          if (o < p.n) yr[o] = T::pack(acc[i][j][r]);
+        }
+    }
+  }
+}
+
+// one wave per output of a pair: fp32 storage, and sizes that are no multiple of 8
+template <typename T, int EPI>
+__global__ void __launch_bounds__(256) moe_rows_kernel(const typename T::storage* w0, const typename T::storage* w1,
+                                                       long expert_stride, const typename T::storage* x,
+                                                       typename T::storage* y, const int32_t* expert, int n_experts,
+                                                       int n, int k, int top, float limit) {
+  const int lane = threadIdx.x & (kWave - 1);
+  const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
+  const long pair = blockIdx.y + (long)blockIdx.z * 65535;
+  if (row >= n) return;
+  const int e = expert[pair];
+  if (e >= n_experts) return;
+  const typename T::storage* xr = x + (EPI == MOE_GATEUP ? pair / top : pair) * k;
+  const typename T::storage* a = w0 + e * expert_stride + (long)row * k;
+  float s0 = 0.f, s1 = 0.f;
+  for (int c = lane; c < k; c += kWave) {
+    const float xv = T::one(xr[c]);
+    s0 = fmaf(T::one(a[c]), xv, s0);
+    if constexpr (EPI == MOE_GATEUP) s1 = fmaf(T::one(w1[e * expert_stride + (long)row * k + c]), xv, s1);
+  }
+  s0 = wave_sum(s0);
+  if constexpr (EPI == MOE_GATEUP) {
+    s1 = wave_sum(s1);
+    s0 = moe_act(s0, s1, limit);
+  }
+  if (lane == 0) y[pair * n + row] = T::pack(s0);
+}
+
+template <typename T, int EPI>
+static int launch_moe_product(hipStream_t s, const MoeGemmParams& p, const int32_t* expert, int n_experts, int n_pairs,
+                              int tile_pairs) {
+  typedef typename T::storage S;
+  bool rows = T::kDtype == MUI_DTYPE_F32 || p.k % 8 != 0 || tile_pairs == 0;
+  rows = rows || !aligned16(p.w0) || (p.w1 && !aligned16(p.w1)) || !aligned16(p.x) || p.expert_stride % 8 != 0;
+  if (rows) {
+    const int z = ceil_div(n_pairs, 65535);
+    // the last z slice must not run past the pairs: one launch per slice of at most 65535
+    for (int i = 0; i < z; ++i) {
+      const int first = i * 65535, cnt = n_pairs - first < 65535 ? n_pairs - first : 65535;
+      const long xrow = EPI == MOE_GATEUP ? first / p.top : first;
+      if (EPI == MOE_GATEUP && first % p.top) return MUI_ERR_UNSUPPORTED;
+      hipLaunchKernelGGL((moe_rows_kernel<T, EPI>), dim3(ceil_div(p.n, 4), cnt), dim3(256), 0, s, (const S*)p.w0,
+                         (const S*)p.w1, p.expert_stride, (const S*)p.x + xrow * p.k, (S*)p.y + (long)first * p.n,
+                         expert + first, n_experts, p.n, p.k, p.top, p.limit);
+    }
+    return launch_status();
+  }
+  if constexpr (T::kDtype != MUI_DTYPE_F32) {
+    if (tile_pairs == 16) {
+      if (p.max_tiles > 65535) return MUI_ERR_UNSUPPORTED;
+      hipLaunchKernelGGL((moe_tile16_kernel<T, EPI>), dim3(ceil_div(p.n, EPI == MOE_GATEUP ? 16 : 32), p.max_tiles),
+                         dim3(256), 0, s, p);
+      return launch_status();
+    }
+    if (tile_pairs != kMgTile) return MUI_ERR_INVALID_ARG;
+    const int r_tiles = ceil_div(p.n, EPI == MOE_GATEUP ? kMgTile / 2 : kMgTile);
+    const long total = (long)ceil_div(p.max_tiles, 4) * 4 * r_tiles;
+    const int blocks = (int)((total + 7) / 8 * 8);
+    const size_t lds = 4 * (size_t)kMgTile * kMgK * 2;
+    if (p.k % kMgK == 0) return launch_with_lds(moe_tile128_kernel<T, EPI, true>, dim3(blocks), dim3(256), lds, s, p);
+    return launch_with_lds(moe_tile128_kernel<T, EPI, false>, dim3(blocks), dim3(256), lds, s, p);
+  }
+  return MUI_ERR_UNSUPPORTED;
+}
+
+template <typename T>
+static int launch_linear_f32(hipStream_t s, const void* w, const void* x, const void* bias, float* y, int n, int k,
+                             int tokens) {
+  typedef typename T::storage S;
+  const bool vec = k % 8 == 0 && aligned16(w) && aligned16(x);
+  if constexpr (T::kDtype != MUI_DTYPE_F32) {
+    if (vec && tokens > MUI_MAX_TOKENS) {
+      MoeGemmParams p = {};
+      p.w0 = (const uint16_t*)w; p.x = (const uint16_t*)x; p.bias = (const uint16_t*)bias; p.y = y; p.n = n; p.k = k;
+      p.top = 1; p.tokens = tokens;
+      const int tiles = ceil_div(tokens, 16);
+      if (tiles > 65535) return MUI_ERR_UNSUPPORTED;
+      hipLaunchKernelGGL((moe_tile16_kernel<T, MOE_F32>), dim3(ceil_div(n, 32), tiles), dim3(256), 0, s, p);
+      return launch_status();
+    }
+  }
+  int ty = ceil_div(tokens, 4);
+  if (ty > 4096) ty = 4096;
+  const dim3 grid(ceil_div(n, 4), ty);
+  if (vec)
+    hipLaunchKernelGGL((linear_f32_rows_kernel<T, true>), grid, dim3(256), 0, s, (const S*)w, (const S*)x, (const S*)bias, y, n, k, tokens);
+  else
+    hipLaunchKernelGGL((linear_f32_rows_kernel<T, false>), grid, dim3(256), 0, s, (const S*)w, (const S*)x, (const S*)bias, y, n, k, tokens);
+  return launch_status();
+}
+
+template <typename T>
+static int launch_route(hipStream_t s, const float* logits, const void* corr, int n_out, int n_experts, int top,
+                        int tokens, int tile_pairs, int max_tiles, int32_t* expert, float* weight, int32_t* pairs,
+                        MoeTile* tiles) {
+  typedef typename T::storage S;
+  const bool one = tokens <= 64 && tile_pairs;
+  if (!one)
+    hipLaunchKernelGGL((moe_route_kernel<T>), dim3(ceil_div(tokens, 4)), dim3(256), 0, s, logits, (const S*)corr, n_out,
+                       top, tokens, expert, weight);
+  if (!tile_pairs) return launch_status();
+  if (one)
+    hipLaunchKernelGGL((moe_group_kernel<T, true>), dim3(1), dim3(kRouteThreads), 0, s, logits, (const S*)corr, n_out,
+                       n_experts, top, tokens, tile_pairs, max_tiles, expert, weight, pairs, tiles);
+  else
+    hipLaunchKernelGGL((moe_group_kernel<T, false>), dim3(1), dim3(kRouteThreads), 0, s, logits, (const S*)corr, n_out,
+                       n_experts, top, tokens, tile_pairs, max_tiles, expert, weight, pairs, tiles);
+  return launch_status();
+}
+
+}  // namespace mui
+
+using namespace mui;
+
+#define MUI_BY_DTYPE(call)                                  \
+  do {                                                      \
+    if (dtype == MUI_DTYPE_F16) { typedef F16 TT; return call; }   \
+    if (dtype == MUI_DTYPE_BF16) { typedef BF16 TT; return call; } \
+    if (dtype == MUI_DTYPE_F32) { typedef F32 TT; return call; }   \
+    return MUI_ERR_INVALID_ARG;                             \
+  } while (0)
+
+extern "C" int mui_linear_f32(mui_stream_t stream, int dtype, const void* weights, const void* x, const void* bias,
+                              float* y, int n_out, int k_in, int tokens) {
+  MUI_CHECK_ARG(weights && x && y && n_out > 0 && k_in > 0 && tokens > 0);
+  MUI_BY_DTYPE((launch_linear_f32<TT>((hipStream_t)stream, weights, x, bias, y, n_out, k_in, tokens)));
+}
+
+extern "C" int mui_moe_tile_pairs(int dtype, int tokens, int top, int n_experts, int width, int ff) {
+  if (dtype == MUI_DTYPE_F32 || width % 8 || ff % 8 || n_experts < 1) return 0;
+  // 128-pair tiles once the experts have enough pairs each to fill a good part of one
+  return (long)tokens * top >= 40L * n_experts ? kMgTile : 16;
+}
+
+extern "C" int mui_moe_max_tiles(int tokens, int top, int n_experts, int tile_pairs) {
+  if (tile_pairs < 1) return 0;
+  const long pairs = (long)tokens * top;
+  return (int)(pairs / tile_pairs + (pairs < n_experts ? pairs : n_experts));
+}
+
+extern "C" int mui_moe_route(mui_stream_t stream, int dtype, const float* logits, const void* correction, int n_experts,
+                             int n_identity, int top, int tokens, int tile_pairs, int32_t* expert, float* weight,
+                             int32_t* pairs, void* tiles) {
+  MUI_CHECK_ARG(logits && expert && weight && tokens > 0 && n_experts >= 0 && n_identity >= 0);
+  const int n_out = n_experts + n_identity;
+  MUI_CHECK_ARG(n_out > 0 && top > 0 && top <= n_out);
+  MUI_CHECK_ARG(tile_pairs == 0 || tile_pairs == 16 || tile_pairs == kMgTile);
+  MUI_CHECK_ARG(tile_pairs == 0 || (pairs && tiles));
+  if (n_out > kMaxRouter || (long)tokens * top > (1L << 30)) return MUI_ERR_UNSUPPORTED;
+  const int mt = mui_moe_max_tiles(tokens, top, n_experts, tile_pairs);
+  MUI_BY_DTYPE((launch_route<TT>((hipStream_t)stream, logits, correction, n_out, n_experts, top, tokens, tile_pairs, mt,
+                                 expert, weight, pairs, (MoeTile*)tiles)));
+}
+
+extern "C" int mui_moe_gateup(mui_stream_t stream, int dtype, const void* gate, const void* up, long expert_stride,
+                              const void* x, float limit, const int32_t* expert, const int32_t* pairs,
+                              const void* tiles, int tile_pairs, void* act, int n_experts, int n_inter, int k_in,
+                              int top, int tokens) {
+  MUI_CHECK_ARG(gate && up && x && expert && act && n_experts > 0 && n_inter > 0 && k_in > 0 && top > 0 && tokens > 0);
+  MUI_CHECK_ARG(tile_pairs == 0 || (pairs && tiles));
+  MoeGemmParams p = {};
+  p.w0 = (const uint16_t*)gate; p.w1 = (const uint16_t*)up; p.expert_stride = expert_stride; p.x = (const uint16_t*)x;
+  p.y = act; p.pairs = pairs; p.tiles = (const MoeTile*)tiles; p.n = n_inter; p.k = k_in; p.top = top; p.tokens = tokens;
+  p.limit = limit; p.max_tiles = mui_moe_max_tiles(tokens, top, n_experts, tile_pairs);
+  MUI_BY_DTYPE((launch_moe_product<TT, MOE_GATEUP>((hipStream_t)stream, p, expert, n_experts, tokens * top, tile_pairs)));
+}
+
+extern "C" int mui_moe_down(mui_stream_t stream, int dtype, const void* down, long expert_stride, const void* act,
+                            const int32_t* expert, const int32_t* pairs, const void* tiles, int tile_pairs, void* out,
+                            int n_experts, int n_out, int k_in, int top, int tokens) {
+  MUI_CHECK_ARG(down && act && expert && out && n_experts > 0 && n_out > 0 && k_in > 0 && top > 0 && tokens > 0);
+  MUI_CHECK_ARG(tile_pairs == 0 || (pairs && tiles));
+  MoeGemmParams p = {};
+  p.w0 = (const uint16_t*)down; p.expert_stride = expert_stride; p.x = (const uint16_t*)act; p.y = out; p.pairs = pairs;
+  p.tiles = (const MoeTile*)tiles; p.n = n_out; p.k = k_in; p.top = top; p.tokens = tokens;
+  p.max_tiles = mui_moe_max_tiles(tokens, top, n_experts, tile_pairs);
+  MUI_BY_DTYPE((launch_moe_product<TT, MOE_DOWN>((hipStream_t)stream, p, expert, n_experts, tokens * top, tile_pairs)));
+}

@@ -20,8 +20,24 @@ def _get_num_key_value_heads(config) -> int:
 
 
 class MuiCache:
+    """What the decode loop asks of a cache, whatever its layers keep."""
+
     def sync_back(self):
         pass
+
+    def tensors(self) -> List[torch.Tensor]:
+        """Every device tensor a captured decode step holds by address."""
+        return []
+
+    def step_state(self) -> List[torch.Tensor]:
+        """The tensors that a step changes other than by writing its own slot (recurrent state): they
+        have to be put back after a step that is not to count."""
+        return []
+
+    def set_seen_tokens(self, n: int) -> None:
+        self._seen_tokens = n
+        if getattr(self, "cpp_module", None) is not None:
+            self.cpp_module.seen_tokens = n
 
 
 class MuiStaticCache(MuiCache):
@@ -68,6 +84,9 @@ class MuiStaticCache(MuiCache):
 
     def __len__(self):
         return len(self.key_cache)
+
+    def tensors(self) -> List[torch.Tensor]:
+        return list(self.key_cache) + list(self.value_cache)
 
     def _kernel_ok(self, t: torch.Tensor) -> bool:
         return t.is_cuda and t.dtype in (torch.float16, torch.bfloat16) and self.head_dim == 128

@@ -16,7 +16,7 @@ from typing import Optional
 import torch
 
 from ... import muillm_ext
-from ..kvcache.cache_utils import MuiStaticCache, _next_pow2, create_static_cache
+from ..kvcache.cache_utils import MuiCache, _next_pow2
 
 
 class MuiGraphDecoder:
@@ -56,7 +56,7 @@ class MuiGraphDecoder:
         self.graph = None
         self.graph_multi = None  # STEPS_PER_REPLAY steps in one graph, captured on first use
         self._graph_key = None  # what the captured graph has baked in (see _capture_key)
-        self.cache: Optional[MuiStaticCache] = None
+        self.cache: Optional[MuiCache] = None
         self.owns_cache = False  # True when prefill() created self.cache itself
         self._window = 0  # sliding window kept in mask4d by every step (0: none)
         self._embed_table = None
@@ -148,15 +148,15 @@ class MuiGraphDecoder:
         # the weights a captured step reads (the embedding table of the folded gather included): a
         # model moved with .to() or quantised again after the first generate() must be captured anew
         weights = hash(tuple(t.data_ptr() for t in self.lm.parameters()) + tuple(t.data_ptr() for t in self.lm.buffers()))
-        return (id(c), self._batch, c.max_cache_len, tuple(t.data_ptr() for t in c.key_cache),
-                tuple(t.data_ptr() for t in c.value_cache),
+        return (id(c), self._batch, c.max_cache_len, tuple(t.data_ptr() for t in c.tensors()),
                 None if self.mask4d is None else self.mask4d.data_ptr(), self._window, weights,
                 None if self._embed_table is None else self._embed_table.data_ptr())
 
     def _capture(self):
         self.cache.device_length_mode = True
         seen = self.cache._seen_tokens
-        # warm up on a side stream (allocator, lazy module state), then restore the cache counters
+        # warm up on a side stream (allocator, lazy module state), then restore the cache counters and
+        # whatever else the step moved on (recurrent state)
         saved = [t.clone() for t in self._step_state()]
         side = torch.cuda.Stream()
         side.wait_stream(torch.cuda.current_stream())
@@ -172,9 +172,7 @@ class MuiGraphDecoder:
         self.graph_multi = None
         self._graph_key = self._capture_key()
         # capture does not execute: the device state is as restored; the host counter moved once
-        self.cache._seen_tokens = seen
-        if self.cache.cpp_module is not None:
-            self.cache.cpp_module.seen_tokens = seen
+        self.cache.set_seen_tokens(seen)
 
     def _capture_multi(self):
         """STEPS_PER_REPLAY steps as one graph (the one-step graph has been captured and warmed up
@@ -186,26 +184,22 @@ class MuiGraphDecoder:
             for _ in range(self.STEPS_PER_REPLAY):
                 self._multi_logits = self._step()  # the last step's
         self.graph_multi = g
-        self.cache._seen_tokens = seen
-        if self.cache.cpp_module is not None:
-            self.cache.cpp_module.seen_tokens = seen
+        self.cache.set_seen_tokens(seen)
 
     def _step_state(self):
         """The device tensors a decode step changes (besides the cache slot it writes)."""
         state = [self.ids, self.pos, self.cpos, self.step, self.out_tokens, self.unfinished]
         if self._embed_table is not None:
             state.append(self.hidden)
-        return state
+        return state + self.cache.step_state()
 
     def _restore(self, saved, seen):
         for dst, src in zip(self._step_state(), saved):
             dst.copy_(src)
-        self.cache._seen_tokens = seen
-        if self.cache.cpp_module is not None:
-            self.cache.cpp_module.seen_tokens = seen
+        self.cache.set_seen_tokens(seen)
 
     @torch.no_grad()
-    def prefill(self, input_ids: torch.LongTensor, max_new_tokens: int, cache: Optional[MuiStaticCache] = None,
+    def prefill(self, input_ids: torch.LongTensor, max_new_tokens: int, cache: Optional[MuiCache] = None,
                 attention_mask: Optional[torch.Tensor] = None):
         """attention_mask [B, prompt_len] of 0/1 marks LEFT padding (0 = pad): padded slots stay
         masked for the whole generation and every row counts its rotary positions from its own
@@ -222,18 +216,18 @@ class MuiGraphDecoder:
         total = past + prompt_len + max_new_tokens
         window = getattr(lm.config, "sliding_window", None)
         windowed = bool(window) and total > int(window)  # decided for the whole generation: a captured step keeps its mask
-        max_pos = lm.model.rotary_emb.max_seq_len_cached
-        if total > max_pos:
+        max_pos = lm.max_positions()  # None: no table of positions to run past
+        if max_pos is not None and total > max_pos:
             raise ValueError(f"cached tokens + prompt + max_new_tokens = {total} exceeds the {max_pos} rotary "
                              "positions of this model (max_position_embeddings)")
         self.owns_cache = cache is None or (cache is self.cache and self.owns_cache)
         if cache is None:
-            cache = create_static_cache(lm.engine_config, lm.config, batch, total, device, lm.model.mdtype)
+            cache = lm.create_cache(batch, total)
         else:
             if batch > cache.max_batch_size:
                 raise ValueError(f"batch {batch} exceeds the cache's max_batch_size {cache.max_batch_size}")
             if cache.max_cache_len < total:
-                cache.grow_cache(total, max(lm.config.max_position_embeddings, _next_pow2(total)))
+                cache.grow_cache(total, max(max_pos or 0, _next_pow2(total)))
         self.cache = cache
         cache.device_length_mode = False
         if padded:
@@ -249,7 +243,7 @@ class MuiGraphDecoder:
         if self._batch != batch or getattr(self, "_max_new", 0) < max_new_tokens:
             self._alloc_state(batch, max_new_tokens, device)
             self.graph = None
-        if padded or windowed:
+        if (padded and not lm.pads_in_cache) or windowed:
             mdtype = lm.model.mdtype
             if self.mask4d is None or self.mask4d.shape[-1] != cache.max_cache_len or self.mask4d.shape[0] != batch:
                 self.mask4d = torch.zeros((batch, 1, 1, cache.max_cache_len), dtype=mdtype, device=device)
@@ -329,13 +323,11 @@ class MuiGraphDecoder:
                 ev.record()
                 pending = (ev, self._stop_host)
         if self.use_graph:
-            self.cache._seen_tokens += done
-            if self.cache.cpp_module is not None:
-                self.cache.cpp_module.seen_tokens = self.cache._seen_tokens
+            self.cache.set_seen_tokens(self.cache._seen_tokens + done)
         return logits_hist
 
     @torch.no_grad()
-    def generate(self, input_ids: torch.LongTensor, max_new_tokens: int, cache: Optional[MuiStaticCache] = None,
+    def generate(self, input_ids: torch.LongTensor, max_new_tokens: int, cache: Optional[MuiCache] = None,
                  return_logits: bool = False, attention_mask: Optional[torch.Tensor] = None,
                  stop_check_every: int = 0):
         first_logits = self.prefill(input_ids, max_new_tokens, cache, attention_mask=attention_mask)

@@ -37,6 +37,7 @@ from ...linear import MuiLinear
 from ...module import MuiModule
 from ...multilinear import MuiMultiLinear
 from ...norm.rmsnorm import MuiRMSNorm
+from ..generation import MuiGenerationMixin
 
 
 @dataclass
@@ -305,9 +306,9 @@ class MuiLlamaModel(MuiModule):
                               hidden_states=all_hidden_states, attentions=all_self_attns)
 
 
-class MuiLlamaForCausalLM(MuiModule):
+class MuiLlamaForCausalLM(MuiGenerationMixin, MuiModule):
     def __init__(self, engine_config: MuiEngineConfig, config, model: MuiLlamaModel, lm_head: MuiLinear):
-        super().__init__(engine_config=engine_config)
+        MuiModule.__init__(self, engine_config=engine_config)
         self.config = config
         self.model = model
         self.vocab_size = config.vocab_size
@@ -369,6 +370,15 @@ class MuiLlamaForCausalLM(MuiModule):
         setattr(lm, "muillm_config", engine_config)
         return lm
 
+    # ---- what the decode loop asks of a causal LM ---------------------------------------------
+    pads_in_cache = False  # left padding travels as an additive mask with every step
+
+    def create_cache(self, batch_size: int, seq_len: int) -> MuiStaticCache:
+        return create_static_cache(self.engine_config, self.config, batch_size, seq_len, self.model.mdevice, self.model.mdtype)
+
+    def max_positions(self) -> Optional[int]:
+        return self.model.rotary_emb.max_seq_len_cached
+
     def get_input_embeddings(self):
         return self.model.embed_tokens
 
@@ -380,7 +390,10 @@ class MuiLlamaForCausalLM(MuiModule):
                 inputs_embeds: Optional[torch.Tensor] = None, labels=None, use_cache: Optional[bool] = None,
                 output_attentions: Optional[bool] = None, output_hidden_states: Optional[bool] = None,
                 return_dict: Optional[bool] = None, cache_position: Optional[torch.LongTensor] = None,
-                all_ones_mask: Optional[bool] = None, num_logits_to_keep: int = 0, float_logits: bool = True):
+                all_ones_mask: Optional[bool] = None, num_logits_to_keep: int = 0, float_logits: bool = True,
+                logits_positions: Union[None, list, torch.Tensor] = None):
+        """logits_positions: the places among the tokens whose logits are wanted (default all;
+        num_logits_to_keep: the last ones)."""
         if labels is not None:
             raise NotImplementedError("inference only: labels/loss are not supported")
         shape = input_ids.shape if input_ids is not None else inputs_embeds.shape
@@ -394,7 +407,9 @@ class MuiLlamaForCausalLM(MuiModule):
             output_attentions=output_attentions, output_hidden_states=output_hidden_states,
             cache_position=cache_position, all_ones_mask=all_ones_mask, skip_final_norm=fuse_norm)
         hidden_states = outputs.last_hidden_state
-        if num_logits_to_keep:
+        if logits_positions is not None:
+            hidden_states = hidden_states[:, logits_positions, :]
+        elif num_logits_to_keep:
             hidden_states = hidden_states[:, -num_logits_to_keep:, :]
         if fuse_norm and hidden_states.is_cuda:
             logits = muillm_ext.muillm_linear_forward(self.engine_config.cpp_engine, hidden_states, head.weight, norm.weight, norm.variance_epsilon,
@@ -407,72 +422,6 @@ class MuiLlamaForCausalLM(MuiModule):
             logits = logits.float()
         return MuiCausalLMOutput(logits=logits, past_key_values=outputs.past_key_values,
                                  hidden_states=outputs.hidden_states, attentions=outputs.attentions)
-
-    @torch.no_grad()
-    def generate_greedy(self, input_ids: torch.LongTensor, max_new_tokens: int, use_graph: Optional[bool] = None,
-                        cache: Optional[MuiStaticCache] = None, return_logits: bool = False):
-        """Prefill on the prompt, then max_new_tokens greedy decode steps at the prompt's batch
-        size. Returns int64 [B, prompt + max_new_tokens] (and, optionally, the per-step fp16
-        logits of the decode steps).
-
-        use_graph=True captures the decode step (model forward, argmax, position bookkeeping,
-        all on the device) into a HIP graph and replays it; False enqueues the same step on the
-        stream every time; None (default) lets the decoder choose (MuiGraphDecoder: stream launches
-        when the layer stack is one library call, graph replay otherwise)."""
-        dec = self._decoder_for(use_graph=use_graph)
-        cache = self._reusable_cache(dec, cache, input_ids)
-        return dec.generate(input_ids, max_new_tokens, cache=cache, return_logits=return_logits)
-
-    def _decoder_for(self, **options):
-        """The MuiGraphDecoder for these options; the last one is kept, so that repeated generate()
-        calls replay the graph captured by the first instead of warming up and capturing again."""
-        from ..graphdecoder import MuiGraphDecoder
-
-        key = tuple(sorted((k, tuple(v) if isinstance(v, (list, tuple)) else v) for k, v in options.items()))
-        if self._graph_decoder is None or self._graph_decoder[0] != key:
-            self._graph_decoder = (key, MuiGraphDecoder(self, **options))
-        return self._graph_decoder[1]
-
-    @staticmethod
-    def _reusable_cache(dec, cache, input_ids):
-        """Without a cache from the caller, a kept decoder starts again on its own (emptied) cache
-        when the batch size fits: same buffers, so its captured graph stays valid. A cache that a
-        caller handed to an earlier call is the caller's (multi-turn state) and is never touched."""
-        if cache is None and dec.cache is not None and dec.owns_cache \
-                and dec.cache.max_batch_size == input_ids.shape[0] \
-                and dec.cache.key_cache[0].device == input_ids.device:
-            dec.cache.reset()
-            return dec.cache
-        return cache
-
-    @torch.no_grad()
-    def generate(self, input_ids: torch.LongTensor = None, attention_mask: Optional[torch.Tensor] = None,
-                 max_new_tokens: int = 20, do_sample: bool = False, temperature: float = 1.0,
-                 top_k: Optional[int] = None, top_p: Optional[float] = None,
-                 eos_token_id=None, pad_token_id: Optional[int] = None, seed: int = 0, use_graph: Optional[bool] = None,
-                 cache: Optional[MuiStaticCache] = None, **unused):
-        """HuggingFace-style entry point over the device-resident decode loop (the reference routes
-        generate() through its MuiGenerationMixin._sample, muillm/sampling/generation.py:77-408).
-        Greedy (do_sample=False) or temperature sampling; left-padded batches via attention_mask;
-        rows stop at eos_token_id (int or list) and are filled with pad_token_id afterwards.
-        Returns int64 [B, prompt_len + max_new_tokens]. top_k / top_p filter the logits with torch
-        ops in front of the sampling kernel (the loop then runs eagerly instead of from the HIP
-        graph); other logit processors (penalties, ...) are not part of this loop."""
-        dropped = {k: v for k, v in unused.items() if v is not None and k in ("repetition_penalty", "num_beams")}
-        if dropped:
-            raise NotImplementedError(f"generate(): unsupported options {sorted(dropped)}")
-        eos = None
-        if eos_token_id is not None:
-            eos = [int(eos_token_id)] if isinstance(eos_token_id, int) else [int(e) for e in eos_token_id]
-        if pad_token_id is None:
-            pad_token_id = eos[0] if eos else 0
-        dec = self._decoder_for(use_graph=use_graph, eos_token_ids=eos, pad_token_id=pad_token_id,
-                                do_sample=do_sample, temperature=temperature, seed=seed,
-                                top_k=top_k if do_sample else None, top_p=top_p if do_sample else None)
-        cache = self._reusable_cache(dec, cache, input_ids)
-        # with an eos criterion the loop polls, without blocking, whether every row has finished
-        return dec.generate(input_ids, max_new_tokens, cache=cache, attention_mask=attention_mask,
-                            stop_check_every=8 if eos else 0)
 
 
 # Mistral shares the Llama implementation; config.sliding_window, where set, goes into the attention
