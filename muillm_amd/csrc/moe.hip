@@ -475,7 +475,7 @@ __global__ void __launch_bounds__(256) moe_rows_kernel(const typename T::storage
                                                        int n, int k, int top, float limit) {
   const int lane = threadIdx.x & (kWave - 1);
   const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
-  const long pair = blockIdx.y + (long)blockIdx.z * 65535;
+  const long pair = blockIdx.y;
   if (row >= n) return;
   const int e = expert[pair];
   if (e >= n_experts) return;
@@ -502,12 +502,12 @@ static int launch_moe_product(hipStream_t s, const MoeGemmParams& p, const int32
   bool rows = T::kDtype == MUI_DTYPE_F32 || p.k % 8 != 0 || tile_pairs == 0;
   rows = rows || !aligned16(p.w0) || (p.w1 && !aligned16(p.w1)) || !aligned16(p.x) || p.expert_stride % 8 != 0;
   if (rows) {
-    const int z = ceil_div(n_pairs, 65535);
-    // the last z slice must not run past the pairs: one launch per slice of at most 65535
-    for (int i = 0; i < z; ++i) {
-      const int first = i * 65535, cnt = n_pairs - first < 65535 ? n_pairs - first : 65535;
+    // pairs are one dimension of the grid: whole tokens' worth of them per launch
+    const int step = 65535 / p.top * p.top;
+    if (step < 1) return MUI_ERR_UNSUPPORTED;
+    for (int first = 0; first < n_pairs; first += step) {
+      const int cnt = n_pairs - first < step ? n_pairs - first : step;
       const long xrow = EPI == MOE_GATEUP ? first / p.top : first;
-      if (EPI == MOE_GATEUP && first % p.top) return MUI_ERR_UNSUPPORTED;
       hipLaunchKernelGGL((moe_rows_kernel<T, EPI>), dim3(ceil_div(p.n, 4), cnt), dim3(256), 0, s, (const S*)p.w0,
                          (const S*)p.w1, p.expert_stride, (const S*)p.x + xrow * p.k, (S*)p.y + (long)first * p.n,
                          expert + first, n_experts, p.n, p.k, p.top, p.limit);

@@ -1,7 +1,8 @@
-"""Configuration of a Salepel decoder, read from its config.json: every size and constant comes from there,
-keys that this build does not know are refused."""
+"""Configuration of a Salepel decoder, read from its config.json: every size and constant comes from there;
+a key that this build does not know is reported."""
 import json
 import os
+import warnings
 from dataclasses import dataclass, field
 from typing import Any, Dict, List, Optional, Union
 
@@ -13,11 +14,12 @@ ARCHITECTURE = "Salepel"
 
 
 def _take(section: Dict[str, Any], where: str, required, optional=()) -> Dict[str, Any]:
-    unknown = sorted(set(section) - set(required) - set(optional))
     missing = sorted(set(required) - set(section))
-    if unknown or missing:
-        raise ValueError(f"{where}: " + "; ".join(([f"unknown keys {unknown}"] if unknown else []) +
-                                                   ([f"missing keys {missing}"] if missing else [])))
+    if missing:
+        raise ValueError(f"{where}: missing keys {missing}")
+    unknown = sorted(set(section) - set(required) - set(optional))
+    if unknown:
+        warnings.warn(f"{where}: unknown keys {unknown} are ignored")
     return section
 
 
