@@ -1154,6 +1154,102 @@ def _cpu_model():
     return platform.processor() or platform.machine()
 
 
+# --------------------------------------------------------------------------------------
+# the Salepel decoder beside the Llama-shaped one
+# --------------------------------------------------------------------------------------
+# layer sizes of real models' order; the Llama-shaped twin has the same width and, as its MLP, as many
+# features as a token's chosen experts have together
+SALEPEL_SIZES = {
+    "width4096": dict(width=4096, heads=32, q_rank=1536, window=4096, lstm_heads=8, experts=64, identity=8, top=8, ff=1792),
+    "width2048": dict(width=2048, heads=16, q_rank=768, window=1024, lstm_heads=4, experts=64, identity=8, top=6, ff=1408),
+}
+SALEPEL_VOCAB = 32768
+
+
+def _salepel_config(z):
+    """Eight layers: latent attention with rows of its own, over those rows, with rows of its own, and a
+    matrix memory, twice; a mixture of experts in each."""
+    from muillm_amd.modules.attention.latentattention import MuiLatentAttentionConfig
+    from muillm_amd.modules.models.salepel.config import MuiSalepelConfig, MuiSalepelLayerConfig
+    from muillm_amd.modules.moe import MuiMoEConfig
+    from muillm_amd.modules.recurrent.mlstm import MuiMLstmConfig
+
+    def latent(source=None):
+        return MuiLatentAttentionConfig(heads=z["heads"], dim=128, rot_dim=64, vdim=128, q_rank=z["q_rank"], kv_rank=512,
+                                        scale=192 ** -0.5, rot_base=10000.0, window=z["window"], kv_source=source)
+
+    mem = MuiMLstmConfig(heads=z["lstm_heads"], dim=256, vdim=512, gate_cap=15.0)
+    ff = MuiMoEConfig(experts=z["experts"], identity=z["identity"], top=z["top"], ff=z["ff"], limit=7.0)
+    mixers = [latent(), latent(0), latent(), mem, latent(), latent(4), latent(), mem]
+    return MuiSalepelConfig(vocab_size=SALEPEL_VOCAB, hidden_size=z["width"], rms_norm_eps=1e-5, embedding_scale=1.0,
+                            layers=[MuiSalepelLayerConfig(m, ff) for m in mixers])
+
+
+def _salepel_models(z, which=("salepel", "llama")):
+    import torch
+
+    from muillm_amd.engineconfig import MuiEngineConfig
+    from muillm_amd.modules.models.llama.model import MuiDecoderConfig, MuiLlamaForCausalLM
+    from muillm_amd.modules.models.salepel.model import MuiSalepelForCausalLM
+
+    for name in which:
+        if name == "salepel":
+            yield name, MuiSalepelForCausalLM.from_config(MuiEngineConfig(), _salepel_config(z), dtype=torch.bfloat16)
+        else:
+            cfg = MuiDecoderConfig(hidden_size=z["width"], intermediate_size=z["top"] * z["ff"], num_hidden_layers=8,
+                                   num_attention_heads=z["width"] // 128, num_key_value_heads=z["width"] // 512,
+                                   vocab_size=SALEPEL_VOCAB, max_position_embeddings=8192)
+            yield name, MuiLlamaForCausalLM.from_config(MuiEngineConfig(), cfg, dtype=torch.bfloat16, device="cuda", seed=0)
+
+
+def bench_salepel(steps=64, sizes=None):
+    """Prefill and decode throughput of both models at every size; prints one JSON line."""
+    import torch
+
+    out = {}
+    for size, z in SALEPEL_SIZES.items():
+        if sizes and size not in sizes:
+            continue
+        out[size] = {}
+        for name, lm in _salepel_models(z):
+            r = out[size][name] = {}
+            for tokens in (512, 2048, 4096):
+                ids = torch.randint(0, SALEPEL_VOCAB, (1, tokens), generator=torch.Generator().manual_seed(1)).to("cuda")
+                with torch.no_grad():
+                    us = _event_time_us(lambda i: lm(input_ids=ids, num_logits_to_keep=1), 5, 2)
+                r[f"prefill_{tokens}_tokens_ms"] = round(us / 1e3, 3)
+                r[f"prefill_{tokens}_tokens_per_s"] = round(tokens / us * 1e6)
+            for batch in (1, 8):
+                for ctx in (64, 2048):
+                    times, _ = bench_decode(lm, steps, 16, prompt_len=ctx, batch=batch, windows=3)
+                    r[f"decode_batch{batch}_context{ctx}_tokens_per_s"] = round(batch * steps / _median(times), 1)
+            _progress(f"{size} {name}: {r}")
+            del lm
+            torch.cuda.empty_cache()
+    print(json.dumps({"salepel": out, "dtype": "bf16", "layers": 8, "data": "random weights and tokens"}))
+
+
+def trace_salepel(spec):
+    """SIZE:MODEL:prefill=TOKENS or SIZE:MODEL:decode=BATCH -- a few passes for rocprofv3 --kernel-trace."""
+    import torch
+
+    size, name, what = spec.split(":")
+    mode, n = what.split("=")
+    (_, lm), = _salepel_models(SALEPEL_SIZES[size], (name,))
+    ids = torch.randint(0, SALEPEL_VOCAB, (1 if mode == "prefill" else int(n), int(n) if mode == "prefill" else 2048)).to("cuda")
+    with torch.no_grad():
+        if mode == "prefill":
+            for _ in range(4):
+                lm(input_ids=ids, num_logits_to_keep=1)
+        else:
+            cache = lm.create_cache(int(n), 4096)
+            lm(input_ids=ids, past_key_values=cache, num_logits_to_keep=1)
+            for _ in range(32):
+                lm(input_ids=ids[:, :1], past_key_values=cache)
+    torch.cuda.synchronize()
+    print("traced", spec)
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
@@ -1212,6 +1308,10 @@ def main():
     ap.add_argument("--pmc-probe-prompt", action="store_true",
                     help="launch the gate/up prompt GEMM (2048 tokens) and prompt attention (4096) three times and exit "
                          "(for rocprofv3 --pmc)")
+    ap.add_argument("--salepel", nargs="?", const="", default=None, metavar="SIZES",
+                    help="prefill and decode throughput of the Salepel decoder beside the Llama-shaped model at equal size, and exit")
+    ap.add_argument("--trace-salepel", default=None, metavar="SIZE:MODEL:MODE=N",
+                    help="a few passes of one of those models (MODE prefill=TOKENS or decode=BATCH) for rocprofv3 --kernel-trace, and exit")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build drives exactly one GPU (no tensor parallelism, no collectives); "
@@ -1224,6 +1324,12 @@ def main():
     from muillm_amd.modules.models.llama.model import MuiDecoderConfig, MuiLlamaForCausalLM
 
     assert torch.cuda.is_available(), "bench.py needs a GPU"
+    if args.salepel is not None:
+        bench_salepel(sizes=[v for v in args.salepel.split(",") if v])
+        return
+    if args.trace_salepel:
+        trace_salepel(args.trace_salepel)
+        return
     if args.pmc_probe:
         pmc_probe()
         return

@@ -282,10 +282,12 @@ __global__ void __launch_bounds__(256) latent_decode_kernel(const LatentParams p
   s_end = s_end < hi + 1 ? s_end : hi + 1;
   const int cpr = p.kp >> 3;
   const u32x4 zero = {0u, 0u, 0u, 0u};
-  for (int c = t; c < 16 * cpr; c += 256) {
-    const int r = c / cpr, k = (c - r * cpr) * 8;
-    *(u32x4*)&ql[r * pitch + k] =
-        h0 + r < p.heads ? ld16((const uint16_t*)p.q_abs + ((long)tok * p.heads + h0 + r) * p.kp + k) : zero;
+  {
+    const int r = t >> 4;  // 16 threads per head
+    const int hh = h0 + r < p.heads ? h0 + r : p.heads - 1;
+    const uint16_t* src = (const uint16_t*)p.q_abs + ((long)tok * p.heads + hh) * p.kp;
+#pragma unroll 5
+    for (int c = t & 15; c < cpr; c += 16) *(u32x4*)&ql[r * pitch + c * 8] = ld16(src + c * 8);
   }
   const uint16_t* cc = (const uint16_t*)p.c_cache + b * p.c_batch;
   const uint16_t* rc = (const uint16_t*)p.r_cache + b * p.r_batch;
@@ -297,29 +299,45 @@ __global__ void __launch_bounds__(256) latent_decode_kernel(const LatentParams p
   const float sc = p.scale * 1.4426950408889634f;
   for (long s0 = s_begin; s0 < s_end; s0 += 64) {
     __syncthreads();  // the previous block is done with
-    for (int c = t; c < 64 * cpr; c += 256) {
-      const int r = c / cpr, k = (c - r * cpr) * 8;
-      long s = s0 + r;
-      const bool live = s < s_end;
-      s = live ? s : s_end - 1;
-      u32x4 v = zero;
-      if (k + 8 <= p.kv_rank) v = ld16(cc + s * p.kv_rank + k);
-      else if (rot8) {
-        if (k < p.kv_rank + p.rot) v = ld16(rc + s * p.rot + (k - p.kv_rank));
-      } else {
-        uint16_t e[8];
+    // eight threads per key, keys t / 8 and t / 8 + 32; up to ten loads requested together
+    const int kr = t >> 3;
+    long key[2];
+    bool live[2];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) {
-          const int q = k + j - p.kv_rank;
-          e[j] = q < p.rot ? rc[s * p.rot + q] : (uint16_t)0;
+    for (int u = 0; u < 2; ++u) {
+      key[u] = s0 + kr + 32 * u;
+      live[u] = key[u] < s_end;
+      key[u] = live[u] ? key[u] : s_end - 1;
+    }
+    for (int c0 = t & 7; c0 < cpr; c0 += 8 * 5) {
+      u32x4 v[5][2];
+#pragma unroll
+      for (int j = 0; j < 5; ++j) {
+        const int k = (c0 + 8 * j) * 8;
+        const bool in_c = k + 8 <= p.kv_rank, in_r = rot8 && !in_c && k < p.kv_rank + p.rot;
+#pragma unroll
+        for (int u = 0; u < 2; ++u) {
+          const uint16_t* src = in_r ? rc + key[u] * p.rot + (k - p.kv_rank) : cc + key[u] * p.kv_rank + (in_c ? k : 0);
+          v[j][u] = ld16(src);
+          v[j][u] = live[u] && (in_c || in_r) ? v[j][u] : zero;
         }
-        v = u32x4{(uint32_t)e[0] | ((uint32_t)e[1] << 16), (uint32_t)e[2] | ((uint32_t)e[3] << 16),
-                  (uint32_t)e[4] | ((uint32_t)e[5] << 16), (uint32_t)e[6] | ((uint32_t)e[7] << 16)};
       }
-      *(u32x4*)&cl[r * pitch + k] = live ? v : zero;
+#pragma unroll
+      for (int j = 0; j < 5; ++j)
+        if (c0 + 8 * j < cpr)
+#pragma unroll
+          for (int u = 0; u < 2; ++u) *(u32x4*)&cl[(kr + 32 * u) * pitch + (c0 + 8 * j) * 8] = v[j][u];
+    }
+    if (!rot8) {
+      __syncthreads();
+      for (int c = t; c < 64 * p.rot; c += 256) {
+        const int r = c / p.rot, e = c - r * p.rot;
+        if (s0 + r < s_end) cl[r * pitch + p.kv_rank + e] = rc[(s0 + r) * p.rot + e];
+      }
     }
     __syncthreads();
     f32x4 s4 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll 6
     for (int k = 0; k < p.kp; k += 32) {
       const u32x4 a = *(const u32x4*)&cl[(16 * wave + i16) * pitch + k + 8 * g];
       const u32x4 q = *(const u32x4*)&ql[i16 * pitch + k + 8 * g];
@@ -382,53 +400,66 @@ __global__ void __launch_bounds__(256) latent_decode_kernel(const LatentParams p
   }
 }
 
-// Grid (heads, blocks of 16 value rows, tokens): merges the splits of a head, then Wuv_h times the result;
-// 16 lanes per value row
+// Grid (heads, blocks of 32 value rows, tokens): merges the splits of a head, then Wuv_h times the result;
+// eight lanes per value row
+constexpr int kMaxSplits = 64;
 template <typename T>
 __global__ void __launch_bounds__(256) latent_output_kernel(const LatentParams p) {
+  __shared__ float ws[kMaxSplits];
   float* o = (float*)la_smem;  // kv_rank
   const int h = blockIdx.x, tok = blockIdx.z, t = threadIdx.x;
   const long stride = p.kv_rank + 2;
   const float* part = p.part + ((long)tok * p.heads + h) * p.splits * stride;
-  float m = -1e30f, l = 0.f;
-  for (int s = 0; s < p.splits; ++s) m = fmaxf(m, part[s * stride + p.kv_rank]);
-  for (int s = 0; s < p.splits; ++s) l = fmaf(exp2f(part[s * stride + p.kv_rank] - m), part[s * stride + p.kv_rank + 1], l);
-  const float inv = l > 0.f ? 1.f / l : 0.f;
-  for (int r = t; r < p.kv_rank; r += 256) {
-    float a = 0.f;
-    for (int s = 0; s < p.splits; ++s) a = fmaf(exp2f(part[s * stride + p.kv_rank] - m), part[s * stride + r], a);
-    o[r] = a * inv;
+  if (t < kWave) {  // the splits' shares, one per lane
+    const bool in = t < p.splits;
+    const float mm = in ? part[t * stride + p.kv_rank] : -1e30f, ll = in ? part[t * stride + p.kv_rank + 1] : 0.f;
+    const float e = exp2f(mm - wave_max(mm));
+    const float l = wave_sum(e * ll);
+    if (in) ws[t] = ll > 0.f ? e / l : 0.f;
   }
   __syncthreads();
-  const int v = blockIdx.y * 16 + (t >> 4);
+  for (int r = t; r < p.kv_rank; r += 256) {
+    float a = 0.f;
+#pragma unroll 8
+    for (int s = 0; s < p.splits; ++s) a = fmaf(ws[s], part[s * stride + r], a);
+    o[r] = a;
+  }
+  __syncthreads();
+  const int v = blockIdx.y * 32 + (t >> 3);
   const int vc = v < p.vdim ? v : p.vdim - 1;
   const uint16_t* w = (const uint16_t*)p.w_uv + ((long)h * p.vdim + vc) * p.kv_rank;
   float a = 0.f;
-#pragma unroll 4
-  for (int c = (t & 15) * 8; c < p.kv_rank; c += 128) {
+#pragma unroll 8
+  for (int c = (t & 7) * 8; c < p.kv_rank; c += 64) {
     float f[8];
     unpack8<T>(ld16_stream(w + c), f);
 #pragma unroll
     for (int i = 0; i < 8; ++i) a = fmaf(f[i], o[c + i], a);
   }
-  a = row16_sum(a);
-  if ((t & 15) == 0 && v < p.vdim) ((uint16_t*)p.out)[((long)tok * p.heads + h) * p.vdim + v] = T::pack(a);
+  a += dpp_f32<kDppXor1>(a);
+  a += dpp_f32<kDppXor2>(a);
+  a += dpp_f32<kDppHalfMirror>(a);
+  if ((t & 7) == 0 && v < p.vdim) ((uint16_t*)p.out)[((long)tok * p.heads + h) * p.vdim + v] = T::pack(a);
 }
 
 // ---------------------------------------------------------------------------------------
-// prefill: grid (heads, tiles of 128 queries) of one batch row; four waves of 32 queries
+// prefill: grid (heads, tiles of 32 NW queries, longest first) of one batch row; NW waves of 32 queries,
+// two LDS stages of 64 keys: the next block's loads are in flight while one is attended to
 // ---------------------------------------------------------------------------------------
-template <typename T, int DKC, int DVT>
-__global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(const LatentParams p) {
+template <typename T, int DKC, int DVT, int NW>
+__global__ void __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) latent_prefill_kernel(const LatentParams p) {
   constexpr int KPITCH = DKC * 32 + 8, VPITCH = DVT * 16 + 16;  // elements per LDS row
-  uint16_t* kl = (uint16_t*)la_smem;  // [64][KPITCH]; before that the 128 queries
-  uint16_t* vl = kl + 64 * KPITCH;    // [64][VPITCH]
+  constexpr int THREADS = 64 * NW, QT = 32 * NW;
+  constexpr int KCH = 64 * DKC * 4, VCH = 64 * DVT * 2;  // 16-byte chunks per block
+  constexpr int KI = (KCH + THREADS - 1) / THREADS, VI = (VCH + THREADS - 1) / THREADS;
+  constexpr int STAGE = 64 * (KPITCH + VPITCH);
+  uint16_t* smem = (uint16_t*)la_smem;  // first the queries, [QT][KPITCH], then two stages of K | V rows
   const int t = threadIdx.x, lane = t & 63, wave = t >> 6, g = lane >> 4, i16 = lane & 15;
-  const int h = blockIdx.x, qt0 = blockIdx.y * 128;
+  const int h = blockIdx.x, qt0 = ((int)gridDim.y - 1 - (int)blockIdx.y) * QT;
   const int hd = p.dim + p.rot, dk = hd;
   const long first_row = p.row_start ? p.row_start[p.b0] : 0;
   // queries: rotated, rounded, through LDS into operand registers (column i16, k-chunk g)
-  for (int c = t; c < 128 * DKC * 4; c += 256) {
+  for (int c = t; c < QT * DKC * 4; c += THREADS) {
     const int r = c / (DKC * 4), e0 = (c - r * DKC * 4) * 8;
     uint16_t v[8];
     const int tq = qt0 + r;
@@ -437,15 +468,16 @@ __global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(co
 #pragma unroll
     for (int j = 0; j < 8; ++j)
       v[j] = e0 + j < dk ? T::pack(rotated_q<T>(qh, p.cos_sin + tok * p.rot, p.dim, p.rot, e0 + j)) : (uint16_t)0;
-    *(u32x4*)&kl[r * KPITCH + e0] = u32x4{(uint32_t)v[0] | ((uint32_t)v[1] << 16), (uint32_t)v[2] | ((uint32_t)v[3] << 16),
-                                          (uint32_t)v[4] | ((uint32_t)v[5] << 16), (uint32_t)v[6] | ((uint32_t)v[7] << 16)};
+    *(u32x4*)&smem[r * KPITCH + e0] = u32x4{(uint32_t)v[0] | ((uint32_t)v[1] << 16), (uint32_t)v[2] | ((uint32_t)v[3] << 16),
+                                            (uint32_t)v[4] | ((uint32_t)v[5] << 16), (uint32_t)v[6] | ((uint32_t)v[7] << 16)};
   }
   __syncthreads();
   u32x4 q[2][DKC];
 #pragma unroll
   for (int qt = 0; qt < 2; ++qt)
 #pragma unroll
-    for (int c = 0; c < DKC; ++c) q[qt][c] = *(const u32x4*)&kl[(wave * 32 + qt * 16 + i16) * KPITCH + c * 32 + 8 * g];
+    for (int c = 0; c < DKC; ++c) q[qt][c] = *(const u32x4*)&smem[(wave * 32 + qt * 16 + i16) * KPITCH + c * 32 + 8 * g];
+  __syncthreads();
   f32x4 acc[2][DVT];
   float m[2] = {-1e30f, -1e30f}, l[2] = {0.f, 0.f};
 #pragma unroll
@@ -453,58 +485,69 @@ __global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(co
 #pragma unroll
     for (int j = 0; j < DVT; ++j) acc[qt][j] = f32x4{0.f, 0.f, 0.f, 0.f};
   const float sc = p.scale * 1.4426950408889634f;
-  const int q_last = (qt0 + 128 < p.t ? qt0 + 128 : p.t) - 1;
+  const int q_last = (qt0 + QT < p.t ? qt0 + QT : p.t) - 1;
   const long hi = (long)p.q_first + q_last;
   long lo = p.window > 0 ? (long)p.q_first + qt0 - p.window + 1 : 0;
   lo = lo > first_row ? lo : first_row;
   lo = lo > p.kv_first ? lo : p.kv_first;
-  const long kvp = (long)p.heads * (p.dim + p.vdim);
-  const uint16_t* kbase = (const uint16_t*)p.kv + (long)h * p.dim;
-  const uint16_t* vbase = (const uint16_t*)p.kv + (long)p.heads * p.dim + (long)h * p.vdim;
-  const uint16_t* rc = (const uint16_t*)p.r_cache + p.b0 * p.r_batch;
-  const bool k8 = p.dim % 8 == 0 && p.rot % 8 == 0 && kvp % 8 == 0;  // 16-byte chunks stay aligned
-  const bool v8 = p.vdim % 8 == 0 && p.dim % 8 == 0;
+  const int kvp = p.heads * (p.dim + p.vdim);
+  // key / value rows counted from lo
+  const uint16_t* kbase = (const uint16_t*)p.kv + (lo - p.kv_first) * kvp + (long)h * p.dim;
+  const uint16_t* vbase = (const uint16_t*)p.kv + (lo - p.kv_first) * kvp + (long)p.heads * p.dim + (long)h * p.vdim;
+  const uint16_t* rc = (const uint16_t*)p.r_cache + p.b0 * p.r_batch + lo * p.rot;
+  const int n_keys = hi >= lo ? (int)(hi - lo + 1) : 0;
+  const bool v8 = p.dim % 8 == 0 && p.rot % 8 == 0 && p.vdim % 8 == 0;  // 16-byte chunks stay aligned
   const u32x4 zero = {0u, 0u, 0u, 0u};
-  // wave's own span of slots: steps outside it are skipped
-  const long wq0 = (long)p.q_first + qt0 + wave * 32, wq1 = wq0 + 31;
-  for (long s0 = lo; s0 <= hi; s0 += 64) {
-    __syncthreads();
-    for (int c = t; c < 64 * DKC * 4; c += 256) {
-      const int r = c / (DKC * 4), e0 = (c - r * DKC * 4) * 8;
-      const long s = s0 + r <= hi ? s0 + r : hi;
-      const long row = s - p.kv_first;
-      u32x4 v = zero;
-      if (k8) {
-        if (e0 < p.dim) v = ld16(kbase + row * kvp + e0);
-        else if (e0 < dk) v = ld16(rc + s * p.rot + (e0 - p.dim));
-      } else {
-        uint16_t e[8];
+  u32x4 rk[KI], rv[VI];
+  auto fetch = [&](int s0) {
+    if (v8) {
 #pragma unroll
-        for (int j = 0; j < 8; ++j)
-          e[j] = e0 + j < p.dim ? kbase[row * kvp + e0 + j] : (e0 + j < dk ? rc[s * p.rot + e0 + j - p.dim] : (uint16_t)0);
-        v = u32x4{(uint32_t)e[0] | ((uint32_t)e[1] << 16), (uint32_t)e[2] | ((uint32_t)e[3] << 16),
-                  (uint32_t)e[4] | ((uint32_t)e[5] << 16), (uint32_t)e[6] | ((uint32_t)e[7] << 16)};
+      for (int i = 0; i < KI; ++i) {
+        const int c = t + THREADS * i, r = c / (DKC * 4), e0 = (c - r * DKC * 4) * 8;
+        const long row = s0 + r < n_keys ? s0 + r : n_keys - 1;
+        const uint16_t* src = e0 < p.dim ? kbase + row * kvp + e0 : rc + row * p.rot + (e0 < dk ? e0 - p.dim : 0);
+        rk[i] = ld16(src);
+        rk[i] = e0 < dk ? rk[i] : zero;
       }
-      *(u32x4*)&kl[r * KPITCH + e0] = v;
-    }
-    for (int c = t; c < 64 * DVT * 2; c += 256) {
-      const int r = c / (DVT * 2), e0 = (c - r * DVT * 2) * 8;
-      const long s = s0 + r <= hi ? s0 + r : hi;
-      const long row = s - p.kv_first;
-      u32x4 v = zero;
-      if (v8) {
-        if (e0 < p.vdim) v = ld16(vbase + row * kvp + e0);
-      } else {
-        uint16_t e[8];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) e[j] = e0 + j < p.vdim ? vbase[row * kvp + e0 + j] : (uint16_t)0;
-        v = u32x4{(uint32_t)e[0] | ((uint32_t)e[1] << 16), (uint32_t)e[2] | ((uint32_t)e[3] << 16),
-                  (uint32_t)e[4] | ((uint32_t)e[5] << 16), (uint32_t)e[6] | ((uint32_t)e[7] << 16)};
+      for (int i = 0; i < VI; ++i) {
+        const int c = t + THREADS * i, r = c / (DVT * 2), e0 = (c - r * DVT * 2) * 8;
+        const long row = s0 + r < n_keys ? s0 + r : n_keys - 1;
+        rv[i] = ld16(vbase + row * kvp + (e0 < p.vdim ? e0 : 0));
+        rv[i] = e0 < p.vdim ? rv[i] : zero;
       }
-      *(u32x4*)&vl[r * VPITCH + e0] = v;
     }
-    __syncthreads();
-    if (s0 > wq1 || (p.window > 0 && s0 + 63 < wq0 - p.window + 1)) continue;  // uniform per wave; barriers are at the top
+  };
+  auto put = [&](int s0, int buf) {
+    uint16_t *kl = smem + buf * STAGE, *vl = kl + 64 * KPITCH;
+    if (v8) {
+#pragma unroll
+      for (int i = 0; i < KI; ++i) {
+        const int c = t + THREADS * i, r = c / (DKC * 4), e0 = (c - r * DKC * 4) * 8;
+        if (KCH % THREADS == 0 || c < KCH) *(u32x4*)&kl[r * KPITCH + e0] = rk[i];
+      }
+#pragma unroll
+      for (int i = 0; i < VI; ++i) {
+        const int c = t + THREADS * i, r = c / (DVT * 2), e0 = (c - r * DVT * 2) * 8;
+        if (VCH % THREADS == 0 || c < VCH) *(u32x4*)&vl[r * VPITCH + e0] = rv[i];
+      }
+    } else {  // rows whose parts are no multiples of 16 bytes: element by element
+      for (int c = t; c < 64 * DKC * 32; c += THREADS) {
+        const int r = c / (DKC * 32), e = c - r * DKC * 32;
+        const long row = s0 + r < n_keys ? s0 + r : n_keys - 1;
+        kl[r * KPITCH + e] = e < p.dim ? kbase[row * kvp + e] : (e < dk ? rc[row * p.rot + e - p.dim] : (uint16_t)0);
+      }
+      for (int c = t; c < 64 * DVT * 16; c += THREADS) {
+        const int r = c / (DVT * 16), e = c - r * DVT * 16;
+        const long row = s0 + r < n_keys ? s0 + r : n_keys - 1;
+        vl[r * VPITCH + e] = e < p.vdim ? vbase[row * kvp + e] : (uint16_t)0;
+      }
+    }
+  };
+  // this wave's queries, as positions counted from lo
+  const int wq0 = (int)((long)p.q_first + qt0 + wave * 32 - lo), wq1 = wq0 + 31;
+  auto attend = [&](int s0, int buf) {
+    const uint16_t *kl = smem + buf * STAGE, *vl = kl + 64 * KPITCH;
     f32x4 s4[2][4];
 #pragma unroll
     for (int kt = 0; kt < 4; ++kt) {
@@ -517,11 +560,11 @@ __global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(co
         for (int qt = 0; qt < 2; ++qt) s4[qt][kt] = mfma16x16x32<T>(a, q[qt][c], s4[qt][kt]);
       }
     }
-    const bool full = s0 + 63 <= wq0 && s0 >= first_row && (p.window <= 0 || s0 >= wq1 - p.window + 1);
+    const bool full = s0 + 63 <= wq0 && (p.window <= 0 || s0 >= wq1 - p.window + 1);
     u32x4 pb[2][2];
 #pragma unroll
     for (int qt = 0; qt < 2; ++qt) {
-      const long qp = wq0 + qt * 16 + i16;
+      const int qp = wq0 + qt * 16 + i16;
       float mx = -INFINITY;
 #pragma unroll
       for (int kt = 0; kt < 4; ++kt)
@@ -529,8 +572,8 @@ __global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(co
         for (int r = 0; r < 4; ++r) {
           float v = s4[qt][kt][r] * sc;
           if (!full) {
-            const long s = s0 + kt * 16 + 4 * g + r;
-            if (s > qp || s < first_row || (p.window > 0 && s <= qp - p.window)) v = -INFINITY;
+            const int s = s0 + kt * 16 + 4 * g + r;
+            if (s > qp || (p.window > 0 && s <= qp - p.window)) v = -INFINITY;
           }
           s4[qt][kt][r] = v;
           mx = fmaxf(mx, v);
@@ -567,6 +610,18 @@ __global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(co
 #pragma unroll
         for (int qt = 0; qt < 2; ++qt) acc[qt][j] = mfma16x16x32<T>(va, pb[qt][kk], acc[qt][j]);
       }
+  };
+  if (n_keys > 0) {
+    fetch(0);
+    put(0, 0);
+  }
+  for (int s0 = 0, buf = 0; s0 < n_keys; s0 += 64, buf ^= 1) {
+    __syncthreads();  // block s0 is in its stage; everybody is done with the other one
+    const bool more = s0 + 64 < n_keys;
+    if (more) fetch(s0 + 64);
+    // (blocks that none of the wave's queries sees are skipped)
+    if (s0 <= wq1 && (p.window <= 0 || s0 + 63 > wq0 - p.window)) attend(s0, buf);
+    if (more) put(s0 + 64, buf ^ 1);
   }
 #pragma unroll
   for (int qt = 0; qt < 2; ++qt) {
@@ -611,16 +666,23 @@ static int launch_latent_decode(hipStream_t s, const LatentParams& p) {
   else if (p.kv_rank <= 512) st = launch_with_lds(latent_decode_kernel<T, 8>, grid, dim3(256), lds, s, p);
   else st = launch_with_lds(latent_decode_kernel<T, 16>, grid, dim3(256), lds, s, p);
   if (st != MUI_OK) return st;
-  return launch_with_lds(latent_output_kernel<T>, dim3(p.heads, ceil_div(p.vdim, 16), tokens), dim3(256),
+  return launch_with_lds(latent_output_kernel<T>, dim3(p.heads, ceil_div(p.vdim, 32), tokens), dim3(256),
                          (size_t)p.kv_rank * 4, s, p);
+}
+
+template <typename T, int DKC, int DVT, int NW>
+static int launch_latent_prefill_w(hipStream_t s, const LatentParams& p) {
+  constexpr size_t kv = (size_t)2 * 64 * (DKC * 32 + 8 + DVT * 16 + 16) * 2, q = (size_t)32 * NW * (DKC * 32 + 8) * 2;
+  const int tiles = ceil_div(p.t, 32 * NW);
+  if (tiles > 65535) return MUI_ERR_UNSUPPORTED;
+  return launch_with_lds(latent_prefill_kernel<T, DKC, DVT, NW>, dim3(p.heads, tiles), dim3(64 * NW), kv > q ? kv : q, s, p);
 }
 
 template <typename T, int DKC, int DVT>
 static int launch_latent_prefill_t(hipStream_t s, const LatentParams& p) {
-  constexpr size_t kv = (size_t)64 * (DKC * 32 + 8 + DVT * 16 + 16) * 2, q = (size_t)128 * (DKC * 32 + 8) * 2;
-  const int tiles = ceil_div(p.t, 128);
-  if (tiles > 65535) return MUI_ERR_UNSUPPORTED;
-  return launch_with_lds(latent_prefill_kernel<T, DKC, DVT>, dim3(p.heads, tiles), dim3(256), kv > q ? kv : q, s, p);
+  // 256 queries per workgroup once that leaves most of the chip something to do
+  if (p.heads * ceil_div(p.t, 256) * 2 >= device_cus()) return launch_latent_prefill_w<T, DKC, DVT, 8>(s, p);
+  return launch_latent_prefill_w<T, DKC, DVT, 4>(s, p);
 }
 
 static bool prefill_covers(int dk, int vdim) { return dk <= 256 && vdim <= 256; }
@@ -632,7 +694,7 @@ static int launch_latent_prefill(hipStream_t s, const LatentParams& p) {
   if (dk <= 96 && p.vdim <= 64) return launch_latent_prefill_t<T, 3, 4>(s, p);
   if (dk <= 128 && p.vdim <= 128) return launch_latent_prefill_t<T, 4, 8>(s, p);
   if (dk <= 192 && p.vdim <= 128) return launch_latent_prefill_t<T, 6, 8>(s, p);
-  if (prefill_covers(dk, p.vdim)) return launch_latent_prefill_t<T, 8, 16>(s, p);
+  if (prefill_covers(dk, p.vdim)) return launch_latent_prefill_w<T, 8, 16, 4>(s, p);
   return MUI_ERR_UNSUPPORTED;
 }
 
@@ -670,9 +732,10 @@ static int latent_kp(int kv_rank, int rot_dim) { return (kv_rank + rot_dim + 31)
 static void latent_split(int batch, int t, int heads, int span, int* splits, int* split_keys) {
   const int groups = batch * t * ceil_div(heads, 16);
   int want = device_cus() * 2 / (groups > 0 ? groups : 1);
-  want = want < 1 ? 1 : (want > 64 ? 64 : want);
+  want = want < 1 ? 1 : (want > kMaxSplits ? kMaxSplits : want);
   const int blocks = ceil_div(span, 64);
-  const int per = ceil_div(blocks, want);
+  int per = ceil_div(blocks, want);
+  if (per < 2 && blocks > 8) per = 2;  // merging costs a split's partial result per head
   *split_keys = per * 64;
   *splits = ceil_div(blocks, per);
 }

@@ -18,7 +18,8 @@
 //   tile 16   up to 16 pairs of an expert: 16 gate + 16 up rows (or 32 rows) per workgroup, K dealt out to
 //             its four waves, operands straight from global memory in matrix order. Decode and short
 //             prompts: every chosen expert's weights are streamed once.
-//   tile 128  128 pairs x 128 rows, both operands through swizzled LDS stages filled by LDS-direct loads.
+//   tile 128 / 256   as many pairs x as many rows, waves of 64 x 64, both operands through swizzled LDS
+//             stages filled by LDS-direct loads.
 // fp32 models and sizes that are no multiple of 8 take a plain one-wave-per-output kernel.
 #include "skinny.cuh"
 
@@ -35,51 +36,52 @@ __device__ __forceinline__ float moe_act(float g, float u, float limit) {
 }
 
 // ---------------------------------------------------------------------------------------
-// fp32 outputs of a small matrix: y[t, n] = W[n, :] . x[t, :] + bias[n], one wave per row
+// fp32 outputs of a small matrix: y[t, n] = W[n, :] . x[t, :] + bias[n], one workgroup per row
 // ---------------------------------------------------------------------------------------
-template <typename T, bool VEC>
+template <typename T, bool VEC, int TB>  // TB tokens per pass over a row
 __global__ void __launch_bounds__(256) linear_f32_rows_kernel(const typename T::storage* w, const typename T::storage* x,
                                                               const typename T::storage* bias, float* y, int n, int k,
                                                               int tokens) {
-  constexpr int TB = 4;  // tokens per pass over a row
-  const int lane = threadIdx.x & (kWave - 1);
-  const int row = blockIdx.x * 4 + (threadIdx.x >> 6);
-  if (row >= n) return;
-  const float b = bias ? T::one(bias[row]) : 0.f;
+  __shared__ float red[4][TB];
+  const int t = threadIdx.x, row = blockIdx.x;
   const typename T::storage* wr = w + (long)row * k;
   for (int t0 = blockIdx.y * TB; t0 < tokens; t0 += gridDim.y * TB) {
     float acc[TB];
 #pragma unroll
     for (int j = 0; j < TB; ++j) acc[j] = 0.f;
     if constexpr (VEC) {
-#pragma unroll 4
-      for (int c = lane * 8; c < k; c += kWave * 8) {
+#pragma unroll 2
+      for (int c = t * 8; c < k; c += 256 * 8) {
         float wf[8];
         load8<T>(wr + c, wf);
 #pragma unroll
         for (int j = 0; j < TB; ++j) {
-          const int t = t0 + j < tokens ? t0 + j : tokens - 1;
+          const int tk = t0 + j < tokens ? t0 + j : tokens - 1;
           float xf[8];
-          load8<T>(x + (long)t * k + c, xf);
+          load8<T>(x + (long)tk * k + c, xf);
 #pragma unroll
           for (int i = 0; i < 8; ++i) acc[j] = fmaf(wf[i], xf[i], acc[j]);
         }
       }
     } else {
-      for (int c = lane; c < k; c += kWave) {
+      for (int c = t; c < k; c += 256) {
         const float wf = T::one(wr[c]);
 #pragma unroll
         for (int j = 0; j < TB; ++j) {
-          const int t = t0 + j < tokens ? t0 + j : tokens - 1;
-          acc[j] = fmaf(wf, T::one(x[(long)t * k + c]), acc[j]);
+          const int tk = t0 + j < tokens ? t0 + j : tokens - 1;
+          acc[j] = fmaf(wf, T::one(x[(long)tk * k + c]), acc[j]);
         }
       }
     }
 #pragma unroll
     for (int j = 0; j < TB; ++j) {
       const float s = wave_sum(acc[j]);
-      if (lane == 0 && t0 + j < tokens) y[(long)(t0 + j) * n + row] = s + b;
+      if ((t & 63) == 0) red[t >> 6][j] = s;
     }
+    __syncthreads();
+    if (t < TB && t0 + t < tokens)
+      y[(long)(t0 + t) * n + row] = ((red[0][t] + red[1][t]) + (red[2][t] + red[3][t])) + (bias ? T::one(bias[row]) : 0.f);
+    __syncthreads();
   }
 }
 
@@ -128,13 +130,22 @@ __device__ __forceinline__ void route_token(const float* lg, const typename T::s
       if (choice[i] > best) { best = choice[i]; bi = e; bs = s[i]; }
       if (kWave * (i + 1) >= n_out) break;
     }
-#pragma unroll
-    for (int d = 1; d < kWave; d <<= 1) {
-      const float ob = __shfl_xor(best, d), os = __shfl_xor(bs, d);
-      const int oi = __shfl_xor(bi, d);
-      if (ob > best || (ob == best && oi < bi)) { best = ob; bi = oi; bs = os; }
+    // the wave's largest, the lowest index where several lanes hold it
+    const float top_v = wave_max(best);
+    uint64_t holders = __ballot(best == top_v && bi < n_out);
+    int win = 0x7fffffff;
+    float win_s = 0.f;
+    while (holders) {
+      const int l = __ffsll((unsigned long long)holders) - 1;
+      const int li = __builtin_amdgcn_readlane(bi, l);
+      if (li < win) {
+        win = li;
+        win_s = readlane_f32(bs, l);
+      }
+      holders &= holders - 1;
     }
-    if (bi >= n_out) bi = 0;  // nothing left to choose (NaN logits): stays in range
+    bi = win < n_out ? win : 0;  // nothing left to choose (NaN logits): stays in range
+    bs = win_s;
 #pragma unroll
     for (int i = 0; i < kRouterPerLane; ++i) {
       if (lane + kWave * i == bi) choice[i] = -INFINITY;
@@ -268,23 +279,36 @@ __global__ void __launch_bounds__(256) moe_tile16_kernel(const MoeGemmParams p) 
   f32x4 acc0 = {0.f, 0.f, 0.f, 0.f}, acc1 = {0.f, 0.f, 0.f, 0.f};
   const int steps = (p.k + 31) >> 5;
   const u32x4 zero = {0u, 0u, 0u, 0u};
-  for (int s0 = wave; s0 < steps; s0 += 4 * UNR) {
-    u32x4 a[UNR], b[UNR], x[UNR];
+  // two register sets: the next batch of loads is in flight while one is multiplied. Chunks past the row
+  // (or past this wave's steps) read its start and are multiplied as zeros.
+  struct Batch { u32x4 a[UNR], b[UNR], x[UNR]; };
+  auto load = [&](int s0, Batch& v) {
 #pragma unroll
     for (int u = 0; u < UNR; ++u) {
       const int kk = (s0 + 4 * u) * 32 + g * 8;
-      const int off = kk < p.k ? kk : 0;  // chunks past the row read its start and meet x = 0
-      a[u] = ld16_stream(wa + off);
-      b[u] = ld16_stream(wb + off);
-      x[u] = ld16(xr + off);
+      const int off = kk < p.k ? kk : 0;
+      v.a[u] = ld16_stream(wa + off);
+      v.b[u] = ld16_stream(wb + off);
+      v.x[u] = ld16(xr + off);
     }
+  };
+  auto multiply = [&](int s0, const Batch& v) {
 #pragma unroll
     for (int u = 0; u < UNR; ++u) {
-      const int kk = (s0 + 4 * u) * 32 + g * 8;
-      const bool live = kk < p.k;
-      const u32x4 xv = live ? x[u] : zero;
-      acc0 = mfma16x16x32<T>(live ? a[u] : zero, xv, acc0);
-      acc1 = mfma16x16x32<T>(live ? b[u] : zero, xv, acc1);
+      const bool live = (s0 + 4 * u) * 32 + g * 8 < p.k;
+      const u32x4 xv = live ? v.x[u] : zero;
+      acc0 = mfma16x16x32<T>(live ? v.a[u] : zero, xv, acc0);
+      acc1 = mfma16x16x32<T>(live ? v.b[u] : zero, xv, acc1);
+    }
+  };
+  Batch b0, b1;
+  if (wave < steps) {
+    load(wave, b0);
+    for (int s0 = wave; s0 < steps; s0 += 8 * UNR) {
+      load(s0 + 4 * UNR, b1);
+      multiply(s0, b0);
+      load(s0 + 8 * UNR, b0);
+      multiply(s0 + 4 * UNR, b1);
     }
   }
 #pragma unroll
@@ -311,40 +335,43 @@ __global__ void __launch_bounds__(256) moe_tile16_kernel(const MoeGemmParams p) 
   }
 }
 
-// 128 rows (gate/up: 64 outputs, each wave 32 gate rows and the 32 up rows of the same outputs) x 128
-// pairs, 64 k-values per step, four waves of 64 x 64. LDS rows are 128 bytes; 16-byte chunk c of row r
-// lives at chunk c ^ ((r >> 1) & 7). DMA (k % 64 == 0): LDS-direct loads, lane i of a wave instruction
-// fills slot i of eight consecutive rows, the swizzle applied to the source chunk. Otherwise the chunks
-// go through registers and those past the end of a row are zeroed.
-constexpr int kMgTile = 128, kMgK = 64;
+// NWR x NWT waves of 64 rows x 64 pairs each (gate/up: a wave's rows are 32 gate rows and the 32 up rows of the
+// same outputs), 64 k-values per step. LDS rows are 128 bytes; 16-byte chunk c of row r lives at chunk
+// c ^ ((r >> 1) & 7). DMA (k % 64 == 0): LDS-direct loads, lane i of a wave instruction fills slot i of eight
+// consecutive rows, the swizzle applied to the source chunk. Otherwise the chunks go through registers and
+// those past the end of a row are zeroed.
+constexpr int kMgK = 64;
 extern __shared__ __align__(16) unsigned char moe_smem[];
 
-template <typename T, int EPI, bool DMA>
-__global__ void __launch_bounds__(256, 2) moe_tile128_kernel(const MoeGemmParams p) {
-  constexpr int OUT = EPI == MOE_GATEUP ? kMgTile / 2 : kMgTile;
-  typedef uint16_t Stage[kMgTile * kMgK];
-  Stage* w_lds = (Stage*)moe_smem;
-  Stage* x_lds = (Stage*)(moe_smem + 2 * sizeof(Stage));
-  __shared__ int prow[kMgTile];
+template <typename T, int EPI, bool DMA, int NWR, int NWT>
+__global__ void __launch_bounds__(64 * NWR * NWT, NWR * NWT == 4 ? 2 : 1) moe_tile_kernel(const MoeGemmParams p) {
+  constexpr int NW = NWR * NWT, ROWS = 64 * NWR, PAIRS = 64 * NWT, OUT = EPI == MOE_GATEUP ? ROWS / 2 : ROWS;
+  constexpr int WQ = 8 / NWT, XQ = 8 / NWR;  // load instructions (eight rows each) per wave and step
+  typedef uint16_t WStage[ROWS * kMgK];
+  typedef uint16_t XStage[PAIRS * kMgK];
+  WStage* w_lds = (WStage*)moe_smem;
+  XStage* x_lds = (XStage*)(moe_smem + 2 * sizeof(WStage));
+  __shared__ int prow[PAIRS];
 
-  // tile order: four pair tiles (of one expert, mostly) fastest, then row tiles, so that the workgroups
+  // tile order: a few pair tiles (of one expert, mostly) fastest, then row tiles, so that the workgroups
   // an XCD runs at a time share weight rows and token rows; the tiles are dealt to the XCDs in
   // contiguous shares of what there really is
+  constexpr int SUP = PAIRS == 128 ? 4 : 2;
   const int n_tiles = p.tiles[0].count;
   const int r_tiles = (p.n + OUT - 1) / OUT;
-  const int total = ((n_tiles + 3) / 4) * 4 * r_tiles;
+  const int total = ((n_tiles + SUP - 1) / SUP) * SUP * r_tiles;
   const int share = (total + 7) / 8;
   const int slot = blockIdx.x >> 3, id = (blockIdx.x & 7) * share + slot;
   if (slot >= share || id >= total) return;
-  const int sup = id / (4 * r_tiles), in_sup = id - sup * 4 * r_tiles;
-  const int ti = sup * 4 + (in_sup & 3);
+  const int sup = id / (SUP * r_tiles), in_sup = id - sup * SUP * r_tiles;
+  const int ti = sup * SUP + in_sup % SUP;
   if (ti >= n_tiles) return;
   const MoeTile tile = p.tiles[1 + ti];
-  const int o0 = (in_sup >> 2) * OUT;
+  const int o0 = (in_sup / SUP) * OUT;
 
   const int t = threadIdx.x, lane = t & (kWave - 1), wave = t >> 6;
-  const int wr = wave >> 1, wt = wave & 1;
-  if (t < kMgTile) prow[t] = p.pairs[tile.first + (t < tile.count ? t : 0)];
+  const int wr = wave / NWT, wt = wave % NWT;
+  if (t < PAIRS) prow[t] = p.pairs[tile.first + (t < tile.count ? t : 0)];
   __syncthreads();
   const long eb = (long)tile.expert * p.expert_stride;
   // tile row r -> weight row
@@ -360,47 +387,45 @@ __global__ void __launch_bounds__(256, 2) moe_tile128_kernel(const MoeGemmParams
       return p.w0 + eb + (long)o * p.k;
     }
   };
+  // instruction q of this wave covers tile rows (q NW + wave) * 8 ..; the swizzled chunk of a row depends on
+  // the lane (and the wave's parity) only
   const int sr = lane >> 3, sc = lane & 7;
-  const uint16_t *wsrc[4], *xsrc[4];  // this lane's source rows: tile row (q * 4 + wave) * 8 + sr
-  int chunk[4];
+  const int chunk = (sc ^ (((wave * 8 + sr) >> 1) & 7)) * 8;
+  static_assert(NW % 2 == 0, "rows q NW * 8 apart share their swizzle");
+  const uint16_t *wsrc[WQ], *xsrc[XQ];
 #pragma unroll
-  for (int q = 0; q < 4; ++q) {
-    const int r = (q * 4 + wave) * 8 + sr;
-    const int pr = prow[r];
-    wsrc[q] = wrow(r);
-    xsrc[q] = p.x + (long)(EPI == MOE_GATEUP ? pr / p.top : pr) * p.k;
-    chunk[q] = (sc ^ ((r >> 1) & 7)) * 8;
+  for (int q = 0; q < WQ; ++q) wsrc[q] = wrow((q * NW + wave) * 8 + sr) + chunk;
+#pragma unroll
+  for (int q = 0; q < XQ; ++q) {
+    const int pr = prow[(q * NW + wave) * 8 + sr];
+    xsrc[q] = p.x + (long)(EPI == MOE_GATEUP ? pr / p.top : pr) * p.k + chunk;
   }
   const int steps = (p.k + kMgK - 1) / kMgK;
   auto dma = [&](int s, int buf) {
 #pragma unroll
-    for (int q = 0; q < 4; ++q) {
-      const int base = (q * 4 + wave) * 8 * kMgK;
-      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(wsrc[q] + s * kMgK + chunk[q]),
-                                       (__attribute__((address_space(3))) void*)&w_lds[buf][base], 16, 0, 0);
-      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(xsrc[q] + s * kMgK + chunk[q]),
-                                       (__attribute__((address_space(3))) void*)&x_lds[buf][base], 16, 0, 0);
-    }
+    for (int q = 0; q < WQ; ++q)
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(wsrc[q] + s * kMgK),
+                                       (__attribute__((address_space(3))) void*)&w_lds[buf][(q * NW + wave) * 8 * kMgK], 16, 0, 0);
+#pragma unroll
+    for (int q = 0; q < XQ; ++q)
+      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(xsrc[q] + s * kMgK),
+                                       (__attribute__((address_space(3))) void*)&x_lds[buf][(q * NW + wave) * 8 * kMgK], 16, 0, 0);
   };
-  u32x4 rw[4], rx[4];
+  u32x4 rw[WQ], rx[XQ];
   auto fetch = [&](int s) {
     const u32x4 zero = {0u, 0u, 0u, 0u};
+    const bool live = s * kMgK + chunk < p.k;
+    const int off = live ? s * kMgK : -chunk;
 #pragma unroll
-    for (int q = 0; q < 4; ++q) {
-      const int kk = s * kMgK + chunk[q];
-      const bool live = kk < p.k;
-      const u32x4 a = ld16(wsrc[q] + (live ? kk : 0)), b = ld16(xsrc[q] + (live ? kk : 0));
-      rw[q] = live ? a : zero;
-      rx[q] = live ? b : zero;
-    }
+    for (int q = 0; q < WQ; ++q) { rw[q] = ld16(wsrc[q] + off); rw[q] = live ? rw[q] : zero; }
+#pragma unroll
+    for (int q = 0; q < XQ; ++q) { rx[q] = ld16(xsrc[q] + off); rx[q] = live ? rx[q] : zero; }
   };
   auto put = [&](int buf) {
 #pragma unroll
-    for (int q = 0; q < 4; ++q) {
-      const int at = (q * 4 + wave) * 8 * kMgK + lane * 8;
-      *(u32x4*)&w_lds[buf][at] = rw[q];
-      *(u32x4*)&x_lds[buf][at] = rx[q];
-    }
+    for (int q = 0; q < WQ; ++q) *(u32x4*)&w_lds[buf][(q * NW + wave) * 8 * kMgK + lane * 8] = rw[q];
+#pragma unroll
+    for (int q = 0; q < XQ; ++q) *(u32x4*)&x_lds[buf][(q * NW + wave) * 8 * kMgK + lane * 8] = rx[q];
   };
   f32x4 acc[4][4];
 #pragma unroll
@@ -442,27 +467,36 @@ __global__ void __launch_bounds__(256, 2) moe_tile128_kernel(const MoeGemmParams
     }
   }
   // lane: pair column r16, rows 4 lg + r of every 16-row tile
+  const bool n4 = (p.n & 3) == 0;
+  auto store4 = [&](uint16_t* yr, int o, const float (&v)[4]) {
+    if (n4 && o + 4 <= p.n) {
+      *(u32x2*)&yr[o] = u32x2{T::pack2(v[0], v[1]), T::pack2(v[2], v[3])};
+    } else {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (o + r < p.n) yr[o + r] = T::pack(v[r]);
+    }
+  };
 #pragma unroll
   for (int j = 0; j < 4; ++j) {
     const int c = wt * 64 + j * 16 + r16;
     if (c >= tile.count) continue;
     uint16_t* yr = (uint16_t*)p.y + (long)prow[c] * p.n;
+    float v[4];
     if constexpr (EPI == MOE_GATEUP) {
 #pragma unroll
-      for (int i = 0; i < 2; ++i)
+      for (int i = 0; i < 2; ++i) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int o = o0 + wr * 32 + i * 16 + 4 * lg + r;
-          if (o < p.n) yr[o] = T::pack(moe_act(acc[i][j][r], acc[i + 2][j][r], p.limit));
-        }
+        for (int r = 0; r < 4; ++r) v[r] = moe_act(acc[i][j][r], acc[i + 2][j][r], p.limit);
+        store4(yr, o0 + wr * 32 + i * 16 + 4 * lg, v);
+      }
     } else {
 #pragma unroll
-      for (int i = 0; i < 4; ++i)
+      for (int i = 0; i < 4; ++i) {
 #pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          const int o = o0 + wr * 64 + i * 16 + 4 * lg + r;
-          if (o < p.n) yr[o] = T::pack(acc[i][j][r]);
-        }
+        for (int r = 0; r < 4; ++r) v[r] = acc[i][j][r];
+        store4(yr, o0 + wr * 64 + i * 16 + 4 * lg, v);
+      }
     }
   }
 }
@@ -495,6 +529,17 @@ __global__ void __launch_bounds__(256) moe_rows_kernel(const typename T::storage
   if (lane == 0) y[pair * n + row] = T::pack(s0);
 }
 
+template <typename T, int EPI, int NWR, int NWT>
+static int launch_moe_tile(hipStream_t s, const MoeGemmParams& p) {
+  constexpr int OUT = (EPI == MOE_GATEUP ? 32 : 64) * NWR, SUP = NWT == 2 ? 4 : 2;
+  const long total = (long)ceil_div(p.max_tiles, SUP) * SUP * ceil_div(p.n, OUT);
+  if (total > (1L << 30)) return MUI_ERR_UNSUPPORTED;
+  const dim3 grid((unsigned)((total + 7) / 8 * 8)), block(64 * NWR * NWT);
+  const size_t lds = (size_t)2 * 64 * (NWR + NWT) * kMgK * 2;
+  if (p.k % kMgK == 0) return launch_with_lds(moe_tile_kernel<T, EPI, true, NWR, NWT>, grid, block, lds, s, p);
+  return launch_with_lds(moe_tile_kernel<T, EPI, false, NWR, NWT>, grid, block, lds, s, p);
+}
+
 template <typename T, int EPI>
 static int launch_moe_product(hipStream_t s, const MoeGemmParams& p, const int32_t* expert, int n_experts, int n_pairs,
                               int tile_pairs) {
@@ -521,13 +566,10 @@ static int launch_moe_product(hipStream_t s, const MoeGemmParams& p, const int32
                          dim3(256), 0, s, p);
       return launch_status();
     }
-    if (tile_pairs != kMgTile) return MUI_ERR_INVALID_ARG;
-    const int r_tiles = ceil_div(p.n, EPI == MOE_GATEUP ? kMgTile / 2 : kMgTile);
-    const long total = (long)ceil_div(p.max_tiles, 4) * 4 * r_tiles;
-    const int blocks = (int)((total + 7) / 8 * 8);
-    const size_t lds = 4 * (size_t)kMgTile * kMgK * 2;
-    if (p.k % kMgK == 0) return launch_with_lds(moe_tile128_kernel<T, EPI, true>, dim3(blocks), dim3(256), lds, s, p);
-    return launch_with_lds(moe_tile128_kernel<T, EPI, false>, dim3(blocks), dim3(256), lds, s, p);
+    if (((uintptr_t)p.y & 7) != 0) return MUI_ERR_ALIGNMENT;
+    if (tile_pairs == 128) return launch_moe_tile<T, EPI, 2, 2>(s, p);
+    if (tile_pairs == 256) return launch_moe_tile<T, EPI, 4, 4>(s, p);
+    return MUI_ERR_INVALID_ARG;
   }
   return MUI_ERR_UNSUPPORTED;
 }
@@ -548,14 +590,15 @@ static int launch_linear_f32(hipStream_t s, const void* w, const void* x, const 
       return launch_status();
     }
   }
-  int ty = ceil_div(tokens, 4);
-  if (ty > 4096) ty = 4096;
-  const dim3 grid(ceil_div(n, 4), ty);
-  if (vec)
-    hipLaunchKernelGGL((linear_f32_rows_kernel<T, true>), grid, dim3(256), 0, s, (const S*)w, (const S*)x, (const S*)bias, y, n, k, tokens);
-  else
-    hipLaunchKernelGGL((linear_f32_rows_kernel<T, false>), grid, dim3(256), 0, s, (const S*)w, (const S*)x, (const S*)bias, y, n, k, tokens);
-  return launch_status();
+  auto launch = [&](auto kernel, int tb) {
+    int ty = ceil_div(tokens, tb);
+    if (ty > 4096) ty = 4096;
+    hipLaunchKernelGGL(kernel, dim3(n, ty), dim3(256), 0, s, (const S*)w, (const S*)x, (const S*)bias, y, n, k, tokens);
+    return launch_status();
+  };
+  if (!vec) return launch(linear_f32_rows_kernel<T, false, 4>, 4);
+  if (tokens == 1) return launch(linear_f32_rows_kernel<T, true, 1>, 1);
+  return launch(linear_f32_rows_kernel<T, true, 4>, 4);
 }
 
 template <typename T>
@@ -597,8 +640,11 @@ extern "C" int mui_linear_f32(mui_stream_t stream, int dtype, const void* weight
 
 extern "C" int mui_moe_tile_pairs(int dtype, int tokens, int top, int n_experts, int width, int ff) {
   if (dtype == MUI_DTYPE_F32 || width % 8 || ff % 8 || n_experts < 1) return 0;
-  // 128-pair tiles once the experts have enough pairs each to fill a good part of one
-  return (long)tokens * top >= 40L * n_experts ? kMgTile : 16;
+  // wide tiles once the experts have enough pairs each to fill a good part of one; of the two widths the one
+  // whose tiles cost less (a 256-pair tile about 1.3 times as much as a 128-pair one)
+  const long per = (long)tokens * top / n_experts;
+  if (per < 40) return 16;
+  return 13 * ((per + 255) / 256) < 10 * ((per + 127) / 128) ? 256 : 128;
 }
 
 extern "C" int mui_moe_max_tiles(int tokens, int top, int n_experts, int tile_pairs) {
@@ -613,7 +659,7 @@ extern "C" int mui_moe_route(mui_stream_t stream, int dtype, const float* logits
   MUI_CHECK_ARG(logits && expert && weight && tokens > 0 && n_experts >= 0 && n_identity >= 0);
   const int n_out = n_experts + n_identity;
   MUI_CHECK_ARG(n_out > 0 && top > 0 && top <= n_out);
-  MUI_CHECK_ARG(tile_pairs == 0 || tile_pairs == 16 || tile_pairs == kMgTile);
+  MUI_CHECK_ARG(tile_pairs == 0 || tile_pairs == 16 || tile_pairs == 128 || tile_pairs == 256);
   MUI_CHECK_ARG(tile_pairs == 0 || (pairs && tiles));
   if (n_out > kMaxRouter || (long)tokens * top > (1L << 30)) return MUI_ERR_UNSUPPORTED;
   const int mt = mui_moe_max_tiles(tokens, top, n_experts, tile_pairs);

@@ -67,18 +67,28 @@ __global__ void __launch_bounds__(kRnThreads) residual_norm_vec_kernel(const Res
     }
   }
   if constexpr (MOE) {
-    for (int s = 0; s < p.top; ++s) {
-      const int e = p.expert[row * p.top + s];
-      const float w = p.weight[row * p.top + s];
-      const S* src = e < p.n_experts ? (const S*)p.pairs + (row * p.top + s) * p.k : (const S*)p.identity + base;
+    // four experts' rows requested together
+    for (int s0 = 0; s0 < p.top; s0 += 4) {
+      const S* src[4];
+      float w[4];
+#pragma unroll
+      for (int u = 0; u < 4; ++u) {
+        const int s = s0 + u < p.top ? s0 + u : p.top - 1;
+        const int e = p.expert[row * p.top + s];
+        w[u] = s0 + u < p.top ? p.weight[row * p.top + s] : 0.f;
+        src[u] = e < p.n_experts ? (const S*)p.pairs + (row * p.top + s) * p.k : (const S*)p.identity + base;
+      }
 #pragma unroll
       for (int j = 0; j < CH; ++j) {
         const int c = t + kRnThreads * j;
         if (c < kc) {
-          float f[8];
-          load8<T>(src + (c << 3), f);
+          float f[4][8];
 #pragma unroll
-          for (int i = 0; i < 8; ++i) y[j][i] = fmaf(w, f[i], y[j][i]);
+          for (int u = 0; u < 4; ++u) load8<T>(src[u] + (c << 3), f[u]);
+#pragma unroll
+          for (int u = 0; u < 4; ++u)
+#pragma unroll
+            for (int i = 0; i < 8; ++i) y[j][i] = fmaf(w[u], f[u][i], y[j][i]);
         }
       }
     }

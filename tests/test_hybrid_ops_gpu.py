@@ -89,7 +89,7 @@ def test_linear_f32(dtype, tokens, n, k):
 # --------------------------------------------------------------------------------------
 @pytest.mark.parametrize("tokens,experts,identity,top", [(1, 5, 2, 3), (7, 1, 0, 1), (40, 70, 60, 9), (100, 6, 3, 9), (300, 12, 1, 2),
                                                          (9, 200, 0, 1)])
-@pytest.mark.parametrize("tile", [0, 16, 128])
+@pytest.mark.parametrize("tile", [0, 16, 128, 256])
 def test_route(tokens, experts, identity, top, tile):
     g = torch.Generator().manual_seed(tokens)
     n = experts + identity
@@ -116,7 +116,7 @@ def test_route(tokens, experts, identity, top, tile):
 @pytest.mark.parametrize("dtype", DTYPES)
 @pytest.mark.parametrize("tokens,experts,identity,top,width,ff", [
     (1, 5, 2, 3, 96, 56), (2, 3, 0, 3, 64, 40), (16, 4, 1, 2, 200, 128), (33, 9, 4, 4, 96, 24), (150, 3, 2, 4, 128, 192),
-    (401, 3, 1, 2, 96, 72), (5, 4, 1, 2, 51, 23), (90, 1, 0, 1, 64, 64)])
+    (401, 3, 1, 2, 96, 72), (620, 2, 1, 2, 128, 200), (5, 4, 1, 2, 51, 23), (90, 1, 0, 1, 64, 64)])
 def test_experts(dtype, tokens, experts, identity, top, width, ff):
     g = torch.Generator().manual_seed(tokens + width)
     x, limit = _rand(g, tokens, width).to(dtype), 0.6  # clamps in most of the places
@@ -138,7 +138,7 @@ def test_experts(dtype, tokens, experts, identity, top, width, ff):
 
 
 def test_experts_of_every_tile_size_agree():
-    """The same pairs through 16-pair and 128-pair tiles (bf16)."""
+    """The same pairs through tiles of every width (bf16)."""
     g = torch.Generator().manual_seed(3)
     tokens, experts, top, width, ff, dtype = 200, 3, 2, 160, 96, torch.bfloat16
     x = _rand(g, tokens, width).to(dtype).to(DEV)
@@ -146,10 +146,11 @@ def test_experts_of_every_tile_size_agree():
     down = _rand(g, experts, width, ff, std=0.1).to(dtype).to(DEV)
     logits = _rand(g, tokens, experts).to(DEV)
     outs = []
-    for tile in (16, 128):
+    for tile in (16, 128, 256):
         expert, _, pairs, tiles = ops.moe_route(logits, torch.zeros(experts, dtype=dtype, device=DEV), experts, top, tile)
         outs.append(ops.moe_experts(x, gate, up, down, 1.0, expert, pairs, tiles, tile).float())
-    _close(outs[0], outs[1].cpu(), 1e-2)
+    _close(outs[1], outs[0].cpu(), 1e-2)
+    _close(outs[2], outs[0].cpu(), 1e-2)
 
 
 # --------------------------------------------------------------------------------------
