@@ -150,6 +150,19 @@ __device__ __forceinline__ void store8(typename T::storage* p, const float (&f)[
   }
 }
 
+// 16 bytes per lane from global memory straight into LDS: lane i's bytes land at dst + 16 i (dst is the same
+// for the wave). Counted like any vector memory load: wait_loads<N>() before the data is read.
+__device__ __forceinline__ void load_lds16(const uint16_t* src, uint16_t* dst) {
+  __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)src,
+                                   (__attribute__((address_space(3))) void*)dst, 16, 0, 0);
+}
+// until at most N vector memory loads of this wave are outstanding (they return in order); no memory
+// access moves across it
+template <int N>
+__device__ __forceinline__ void wait_loads() {
+  asm volatile("s_waitcnt vmcnt(%0)" ::"n"(N) : "memory");
+}
+
 // A 4 x 16 block of 16-bit elements read transposed from LDS: within a group of 16 lanes, lane i
 // receives element i % 4 of the 8-byte rows addressed by lanes i / 4, i / 4 + 4, i / 4 + 8 and
 // i / 4 + 12 -- four rows of column i when lane i points at row i / 4, columns 4 (i % 4) .. + 3.

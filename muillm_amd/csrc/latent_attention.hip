@@ -70,22 +70,35 @@ __device__ __forceinline__ float block_sum256(float v, float* red) {
 template <typename T>
 __global__ void __launch_bounds__(256) latent_prepare_kernel(const LatentParams p) {
   typedef typename T::storage S;
-  __shared__ float red[4];
+  __shared__ float red[2][4];
   const int tok = blockIdx.x, b = tok / p.t, t = threadIdx.x;
   const S* row = (const S*)p.down + (long)tok * p.down_pitch;
+  const S* cr = row + p.q_rank;
+  const bool kv_here = p.kv_gain != nullptr;
   const long slot = p.cache_position[tok - b * p.t];
   const long pos = slot - (p.row_start ? p.row_start[b] : 0);
-  float ss = 0.f;
+  float sq = 0.f, sk = 0.f;
+#pragma unroll 4
   for (int i = t; i < p.q_rank; i += 256) {
     const float v = T::one(row[i]);
-    ss = fmaf(v, v, ss);
+    sq = fmaf(v, v, sq);
   }
-  float rs = rsqrtf(block_sum256(ss, red) / (float)p.q_rank + p.eps);
-  S* ql = (S*)p.q_latent + (long)tok * p.q_rank;
-  for (int i = t; i < p.q_rank; i += 256) ql[i] = T::pack(T::one(((const S*)p.q_gain)[i]) * (T::one(row[i]) * rs));
-  const bool kv = p.kv_gain != nullptr && slot >= 0 && slot < p.max_cache_len;
+  if (kv_here) {
+#pragma unroll 4
+    for (int i = t; i < p.kv_rank; i += 256) {
+      const float v = T::one(cr[i]);
+      sk = fmaf(v, v, sk);
+    }
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if ((t & 63) == 0) {
+    red[0][t >> 6] = sq;
+    red[1][t >> 6] = sk;
+  }
+  const bool kv = kv_here && slot >= 0 && slot < p.max_cache_len;
   const int half = p.rot >> 1;
-  const S* kr = row + p.q_rank + p.kv_rank;
+  const S* kr = cr + p.kv_rank;
   for (int i = t; i < half; i += 256) {
     float c, s;
     rope_angle((double)(pos > 0 ? pos : 0), p.inv_freq[i], c, s);
@@ -98,15 +111,15 @@ __global__ void __launch_bounds__(256) latent_prepare_kernel(const LatentParams 
       dst[half + i] = T::pack(v * c + u * s);
     }
   }
-  if (!kv) return;  // uniform for the workgroup
-  const S* cr = row + p.q_rank;
-  ss = 0.f;
-  for (int i = t; i < p.kv_rank; i += 256) {
-    const float v = T::one(cr[i]);
-    ss = fmaf(v, v, ss);
-  }
-  rs = rsqrtf(block_sum256(ss, red) / (float)p.kv_rank + p.eps);
+  __syncthreads();
+  float rs = rsqrtf(((red[0][0] + red[0][1]) + (red[0][2] + red[0][3])) / (float)p.q_rank + p.eps);
+  S* ql = (S*)p.q_latent + (long)tok * p.q_rank;
+#pragma unroll 4
+  for (int i = t; i < p.q_rank; i += 256) ql[i] = T::pack(T::one(((const S*)p.q_gain)[i]) * (T::one(row[i]) * rs));
+  if (!kv) return;
+  rs = rsqrtf(((red[1][0] + red[1][1]) + (red[1][2] + red[1][3])) / (float)p.kv_rank + p.eps);
   S* dst = (S*)p.c_cache + b * p.c_batch + slot * p.kv_rank;
+#pragma unroll 4
   for (int i = t; i < p.kv_rank; i += 256) dst[i] = T::pack(T::one(((const S*)p.kv_gain)[i]) * (T::one(cr[i]) * rs));
 }
 
@@ -261,99 +274,99 @@ __global__ void __launch_bounds__(256) latent_absorb_kernel(const LatentParams p
   }
 }
 
-// Grid (splits, head groups of 16, tokens); four waves. 64 keys per block in LDS, rows of kp + 8 elements.
-//   scores: wave w takes keys 16 w ..: A = key rows, B = the 16 heads' queries; lane (g, i) ends up with
-//           head i, keys 16 w + 4 g + r
+// LDS tiles filled by LDS-direct loads: blocks of 64 columns, in a block rows of 128 bytes whose 16-byte chunk c
+// lives at chunk c ^ ((row >> 1) & 7) (16 rows of one logical chunk fall into 64 different banks). A wave
+// instruction delivers eight rows of one block.
+__device__ __forceinline__ int tile_swz(int row) { return (row >> 1) & 7; }
+template <int ROWS>
+__device__ __forceinline__ int tile_at(int row, int col) {  // in elements
+  return ((col >> 6) * ROWS + row) * 64 + ((((col >> 3) & 7) ^ tile_swz(row)) << 3) + (col & 7);
+}
+
+// Grid (splits, head groups of 16, tokens); eight waves, 128 keys per block, all of a block's rows requested at
+// once.
+//   scores: wave w takes keys 16 w ..: A = key rows, B = the 16 heads' queries (registers); lane (g, i) ends up
+//           with head i, keys 16 w + 4 g + r
 //   values: O^T[rank, head] += C^T P^T, the latent rows read back transposed; wave w owns the rank
-//           tiles w, w + 4, ...; contraction slots of lane group g: keys 4 g + r and 16 + 4 g + r of 32
-template <typename T, int NT>
-__global__ void __launch_bounds__(256) latent_decode_kernel(const LatentParams p) {
-  __shared__ float mred[4][16], lred[4][16];
-  __shared__ __align__(16) uint16_t pl[16][64 + 8];
-  const int pitch = p.kp + 8;
-  uint16_t* cl = (uint16_t*)la_smem;  // [64][pitch]
-  uint16_t* ql = cl + 64 * pitch;     // [16][pitch]
-  const int t = threadIdx.x, lane = t & 63, wave = t >> 6, g = lane >> 4, i16 = lane & 15;
+//           tiles w, w + 8, ...; contraction slots of lane group g: keys 4 g + r and 16 + 4 g + r of 32
+constexpr int kDecKeys = 128;
+constexpr int kMaxDecodeWidth = 576;  // kv_rank + rot, rounded up to 64: 128 rows of it fit into LDS
+template <typename T, int NT>  // kv_rank <= 128 NT
+__global__ void __launch_bounds__(512) latent_decode_kernel(const LatentParams p) {
+  constexpr int KC = 4 * NT + 2;  // query chunks of 32 (kv_rank + rot <= 128 NT + 64)
+  __shared__ float mred[8][16], lred[8][16];
+  __shared__ __align__(16) uint16_t pl[16][kDecKeys + 8];
+  uint16_t* cl = (uint16_t*)la_smem;  // [kp / 64][128][64]
+  const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), g = lane >> 4, i16 = lane & 15;
   const int split = blockIdx.x, h0 = blockIdx.y * 16, tok = blockIdx.z, b = tok / p.t;
+  u32x4 q[KC];
+  {
+    const int hh = h0 + i16 < p.heads ? h0 + i16 : p.heads - 1;
+    const uint16_t* src = (const uint16_t*)p.q_abs + ((long)tok * p.heads + hh) * p.kp + 8 * g;
+#pragma unroll
+    for (int c = 0; c < KC; ++c) q[c] = ld16(src + (c * 32 < p.kp ? c * 32 : 0));
+  }
   long lo, hi;
   visible(p, tok, b, lo, hi);
   const long s_begin = lo + (long)split * p.split_keys;
   long s_end = s_begin + p.split_keys;  // exclusive
   s_end = s_end < hi + 1 ? s_end : hi + 1;
-  const int cpr = p.kp >> 3;
-  const u32x4 zero = {0u, 0u, 0u, 0u};
-  {
-    const int r = t >> 4;  // 16 threads per head
-    const int hh = h0 + r < p.heads ? h0 + r : p.heads - 1;
-    const uint16_t* src = (const uint16_t*)p.q_abs + ((long)tok * p.heads + hh) * p.kp;
-#pragma unroll 5
-    for (int c = t & 15; c < cpr; c += 16) *(u32x4*)&ql[r * pitch + c * 8] = ld16(src + c * 8);
-  }
   const uint16_t* cc = (const uint16_t*)p.c_cache + b * p.c_batch;
   const uint16_t* rc = (const uint16_t*)p.r_cache + b * p.r_batch;
   const bool rot8 = p.rot % 8 == 0;
+  const int lrow = lane >> 3;
+  const int width = p.kv_rank + (rot8 ? p.rot : 0);  // columns that are loaded
   f32x4 acc[NT];
 #pragma unroll
   for (int j = 0; j < NT; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
   float m = -1e30f, l = 0.f;
   const float sc = p.scale * 1.4426950408889634f;
-  for (long s0 = s_begin; s0 < s_end; s0 += 64) {
+  for (long s0 = s_begin; s0 < s_end; s0 += kDecKeys) {
     __syncthreads();  // the previous block is done with
-    // eight threads per key, keys t / 8 and t / 8 + 32; up to ten loads requested together
-    const int kr = t >> 3;
-    long key[2];
-    bool live[2];
+    // wave w delivers rows 8 w .. and 64 + 8 w ..; rows past the split repeat its last one (their scores
+    // are masked), columns past the rows' end repeat their start (the queries hold zeros there)
 #pragma unroll
     for (int u = 0; u < 2; ++u) {
-      key[u] = s0 + kr + 32 * u;
-      live[u] = key[u] < s_end;
-      key[u] = live[u] ? key[u] : s_end - 1;
-    }
-    for (int c0 = t & 7; c0 < cpr; c0 += 8 * 5) {
-      u32x4 v[5][2];
-#pragma unroll
-      for (int j = 0; j < 5; ++j) {
-        const int k = (c0 + 8 * j) * 8;
-        const bool in_c = k + 8 <= p.kv_rank, in_r = rot8 && !in_c && k < p.kv_rank + p.rot;
-#pragma unroll
-        for (int u = 0; u < 2; ++u) {
-          const uint16_t* src = in_r ? rc + key[u] * p.rot + (k - p.kv_rank) : cc + key[u] * p.kv_rank + (in_c ? k : 0);
-          v[j][u] = ld16(src);
-          v[j][u] = live[u] && (in_c || in_r) ? v[j][u] : zero;
-        }
+      const int row = (wave + 8 * u) * 8 + lrow;
+      const long s = s0 + row < s_end ? s0 + row : s_end - 1;
+      const int lc = ((lane & 7) ^ tile_swz(row)) * 8;
+      for (int c0 = 0; c0 < p.kp; c0 += 64) {
+        const int c = c0 + lc < width ? c0 + lc : 0;
+        load_lds16(c < p.kv_rank ? cc + s * p.kv_rank + c : rc + s * p.rot + (c - p.kv_rank),
+                   &cl[((c0 >> 6) * kDecKeys + (wave + 8 * u) * 8) * 64]);
       }
-#pragma unroll
-      for (int j = 0; j < 5; ++j)
-        if (c0 + 8 * j < cpr)
-#pragma unroll
-          for (int u = 0; u < 2; ++u) *(u32x4*)&cl[(kr + 32 * u) * pitch + (c0 + 8 * j) * 8] = v[j][u];
     }
-    if (!rot8) {
+    wait_loads<0>();
+    if (!rot8) {  // the rotated part element by element
       __syncthreads();
-      for (int c = t; c < 64 * p.rot; c += 256) {
+      for (int c = t; c < kDecKeys * p.rot; c += 512) {
         const int r = c / p.rot, e = c - r * p.rot;
-        if (s0 + r < s_end) cl[r * pitch + p.kv_rank + e] = rc[(s0 + r) * p.rot + e];
+        const long s = s0 + r < s_end ? s0 + r : s_end - 1;
+        cl[tile_at<kDecKeys>(r, p.kv_rank + e)] = rc[s * p.rot + e];
       }
     }
     __syncthreads();
-    f32x4 s4 = {0.f, 0.f, 0.f, 0.f};
-#pragma unroll 6
-    for (int k = 0; k < p.kp; k += 32) {
-      const u32x4 a = *(const u32x4*)&cl[(16 * wave + i16) * pitch + k + 8 * g];
-      const u32x4 q = *(const u32x4*)&ql[i16 * pitch + k + 8 * g];
-      s4 = mfma16x16x32<T>(a, q, s4);
+    f32x4 s4 = {0.f, 0.f, 0.f, 0.f}, s5 = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int c = 0; c < KC; c += 2) {
+      if (c * 32 < p.kp) {  // (kp is a multiple of 64)
+        s4 = mfma16x16x32<T>(*(const u32x4*)&cl[tile_at<kDecKeys>(16 * wave + i16, c * 32 + 8 * g)], q[c], s4);
+        s5 = mfma16x16x32<T>(*(const u32x4*)&cl[tile_at<kDecKeys>(16 * wave + i16, c * 32 + 32 + 8 * g)], q[c + 1], s5);
+      }
     }
     float mx = -INFINITY;
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
-      s4[r] = s0 + 16 * wave + 4 * g + r < s_end ? s4[r] * sc : -INFINITY;
+      s4[r] = s0 + 16 * wave + 4 * g + r < s_end ? (s4[r] + s5[r]) * sc : -INFINITY;
       mx = fmaxf(mx, s4[r]);
     }
     mx = fmaxf(mx, __shfl_xor(mx, 16));
     mx = fmaxf(mx, __shfl_xor(mx, 32));
     if (g == 0) mred[wave][i16] = mx;
     __syncthreads();
-    const float mn = fmaxf(m, fmaxf(fmaxf(mred[0][i16], mred[1][i16]), fmaxf(mred[2][i16], mred[3][i16])));
+    float mn = m;
+#pragma unroll
+    for (int w = 0; w < 8; ++w) mn = fmaxf(mn, mred[w][i16]);
     const float keep = exp2f(m - mn);
     m = mn;
     float e[4], sum = 0.f;
@@ -364,21 +377,25 @@ __global__ void __launch_bounds__(256) latent_decode_kernel(const LatentParams p
     sum += __shfl_xor(sum, 32);
     if (g == 0) lred[wave][i16] = sum;
     __syncthreads();
-    l = l * keep + ((lred[0][i16] + lred[1][i16]) + (lred[2][i16] + lred[3][i16]));
+    sum = 0.f;
+#pragma unroll
+    for (int w = 0; w < 8; ++w) sum += lred[w][i16];
+    l = l * keep + sum;
 #pragma unroll
     for (int j = 0; j < NT; ++j)
 #pragma unroll
       for (int r = 0; r < 4; ++r) acc[j][r] *= keep;
 #pragma unroll
-    for (int kk = 0; kk < 2; ++kk) {
+    for (int kk = 0; kk < kDecKeys / 32; ++kk) {
       const u32x2 plo = *(const u32x2*)&pl[i16][32 * kk + 4 * g], phi = *(const u32x2*)&pl[i16][32 * kk + 16 + 4 * g];
       const u32x4 pb = {plo.x, plo.y, phi.x, phi.y};
 #pragma unroll
       for (int j = 0; j < NT; ++j) {
-        const int col = 16 * (wave + 4 * j);
+        const int col = 16 * (wave + 8 * j);
         if (col < p.kv_rank) {  // uniform; a last tile may reach into the rotated part: never stored
-          const u32x2 a0 = lds_read_tr16(&cl[(32 * kk + 4 * g + (i16 >> 2)) * pitch + col + 4 * (i16 & 3)]);
-          const u32x2 a1 = lds_read_tr16(&cl[(32 * kk + 16 + 4 * g + (i16 >> 2)) * pitch + col + 4 * (i16 & 3)]);
+          const int row = 32 * kk + 4 * g + (i16 >> 2);
+          const u32x2 a0 = lds_read_tr16(&cl[tile_at<kDecKeys>(row, col + 4 * (i16 & 3))]);
+          const u32x2 a1 = lds_read_tr16(&cl[tile_at<kDecKeys>(row + 16, col + 4 * (i16 & 3))]);
           acc[j] = mfma16x16x32<T>(u32x4{a0.x, a0.y, a1.x, a1.y}, pb, acc[j]);
         }
       }
@@ -390,7 +407,7 @@ __global__ void __launch_bounds__(256) latent_decode_kernel(const LatentParams p
     for (int j = 0; j < NT; ++j)
 #pragma unroll
       for (int r = 0; r < 4; ++r) {
-        const int c = 16 * (wave + 4 * j) + 4 * g + r;
+        const int c = 16 * (wave + 8 * j) + 4 * g + r;
         if (c < p.kv_rank) dst[c] = acc[j][r];
       }
     if (wave == 0 && g == 0) {
@@ -443,23 +460,23 @@ __global__ void __launch_bounds__(256) latent_output_kernel(const LatentParams p
 }
 
 // ---------------------------------------------------------------------------------------
-// prefill: grid (heads, tiles of 32 NW queries, longest first) of one batch row; NW waves of 32 queries,
-// two LDS stages of 64 keys: the next block's loads are in flight while one is attended to
+// prefill: grid (heads, tiles of 128 queries, longest first) of one batch row; four waves of 32 queries, two
+// workgroups per CU. LDS holds two stages of 64 keys and one of their values: while block s is multiplied with
+// the queries, its values and the keys of block s + 1 are on their way (LDS-direct loads, no registers).
 // ---------------------------------------------------------------------------------------
-template <typename T, int DKC, int DVT, int NW>
-__global__ void __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) latent_prefill_kernel(const LatentParams p) {
-  constexpr int KPITCH = DKC * 32 + 8, VPITCH = DVT * 16 + 16;  // elements per LDS row
-  constexpr int THREADS = 64 * NW, QT = 32 * NW;
-  constexpr int KCH = 64 * DKC * 4, VCH = 64 * DVT * 2;  // 16-byte chunks per block
-  constexpr int KI = (KCH + THREADS - 1) / THREADS, VI = (VCH + THREADS - 1) / THREADS;
-  constexpr int STAGE = 64 * (KPITCH + VPITCH);
-  uint16_t* smem = (uint16_t*)la_smem;  // first the queries, [QT][KPITCH], then two stages of K | V rows
-  const int t = threadIdx.x, lane = t & 63, wave = t >> 6, g = lane >> 4, i16 = lane & 15;
+template <typename T, int DKC, int DVT>
+__global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(const LatentParams p) {
+  static_assert(DKC % 2 == 0 && DVT % 4 == 0, "tiles of 64 columns");
+  constexpr int QT = 128, KG = DKC / 2, VG = DVT / 4;  // queries per workgroup, blocks of 64 columns
+  constexpr int KSTAGE = KG * 64 * 64, VSTAGE = VG * 64 * 64;
+  uint16_t* smem = (uint16_t*)la_smem;  // first the queries, [KG][QT][64], then K, K', V
+  uint16_t* vl = smem + 2 * KSTAGE;
+  const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), g = lane >> 4, i16 = lane & 15;
   const int h = blockIdx.x, qt0 = ((int)gridDim.y - 1 - (int)blockIdx.y) * QT;
   const int hd = p.dim + p.rot, dk = hd;
   const long first_row = p.row_start ? p.row_start[p.b0] : 0;
   // queries: rotated, rounded, through LDS into operand registers (column i16, k-chunk g)
-  for (int c = t; c < QT * DKC * 4; c += THREADS) {
+  for (int c = t; c < QT * DKC * 4; c += 256) {
     const int r = c / (DKC * 4), e0 = (c - r * DKC * 4) * 8;
     uint16_t v[8];
     const int tq = qt0 + r;
@@ -468,15 +485,15 @@ __global__ void __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) latent_prefill_kerne
 #pragma unroll
     for (int j = 0; j < 8; ++j)
       v[j] = e0 + j < dk ? T::pack(rotated_q<T>(qh, p.cos_sin + tok * p.rot, p.dim, p.rot, e0 + j)) : (uint16_t)0;
-    *(u32x4*)&smem[r * KPITCH + e0] = u32x4{(uint32_t)v[0] | ((uint32_t)v[1] << 16), (uint32_t)v[2] | ((uint32_t)v[3] << 16),
-                                            (uint32_t)v[4] | ((uint32_t)v[5] << 16), (uint32_t)v[6] | ((uint32_t)v[7] << 16)};
+    *(u32x4*)&smem[tile_at<QT>(r, e0)] = u32x4{(uint32_t)v[0] | ((uint32_t)v[1] << 16), (uint32_t)v[2] | ((uint32_t)v[3] << 16),
+                                               (uint32_t)v[4] | ((uint32_t)v[5] << 16), (uint32_t)v[6] | ((uint32_t)v[7] << 16)};
   }
   __syncthreads();
   u32x4 q[2][DKC];
 #pragma unroll
   for (int qt = 0; qt < 2; ++qt)
 #pragma unroll
-    for (int c = 0; c < DKC; ++c) q[qt][c] = *(const u32x4*)&smem[(wave * 32 + qt * 16 + i16) * KPITCH + c * 32 + 8 * g];
+    for (int c = 0; c < DKC; ++c) q[qt][c] = *(const u32x4*)&smem[tile_at<QT>(wave * 32 + qt * 16 + i16, c * 32 + 8 * g)];
   __syncthreads();
   f32x4 acc[2][DVT];
   float m[2] = {-1e30f, -1e30f}, l[2] = {0.f, 0.f};
@@ -496,132 +513,142 @@ __global__ void __launch_bounds__(64 * NW, NW == 8 ? 2 : 1) latent_prefill_kerne
   const uint16_t* vbase = (const uint16_t*)p.kv + (lo - p.kv_first) * kvp + (long)p.heads * p.dim + (long)h * p.vdim;
   const uint16_t* rc = (const uint16_t*)p.r_cache + p.b0 * p.r_batch + lo * p.rot;
   const int n_keys = hi >= lo ? (int)(hi - lo + 1) : 0;
-  const bool v8 = p.dim % 8 == 0 && p.rot % 8 == 0 && p.vdim % 8 == 0;  // 16-byte chunks stay aligned
-  const u32x4 zero = {0u, 0u, 0u, 0u};
-  u32x4 rk[KI], rv[VI];
-  auto fetch = [&](int s0) {
-    if (v8) {
+  const bool vec = p.dim % 8 == 0 && p.rot % 8 == 0 && p.vdim % 8 == 0;  // 16-byte chunks stay aligned
+  // Wave w delivers rows 8 w .. and 32 + 8 w .. of a block (their swizzles agree). Rows past the last key
+  // repeat it (masked), columns past a key's end repeat its start (the queries hold zeros there), columns
+  // past a value's end are never stored.
+  const int lrow = wave * 8 + (lane >> 3), lc = ((lane & 7) ^ tile_swz(lrow)) * 8;
+  auto load_k = [&](int s0, uint16_t* dst) {
+    if (vec) {
 #pragma unroll
-      for (int i = 0; i < KI; ++i) {
-        const int c = t + THREADS * i, r = c / (DKC * 4), e0 = (c - r * DKC * 4) * 8;
-        const long row = s0 + r < n_keys ? s0 + r : n_keys - 1;
-        const uint16_t* src = e0 < p.dim ? kbase + row * kvp + e0 : rc + row * p.rot + (e0 < dk ? e0 - p.dim : 0);
-        rk[i] = ld16(src);
-        rk[i] = e0 < dk ? rk[i] : zero;
+      for (int u = 0; u < 2; ++u) {
+        const long row = s0 + lrow + 32 * u < n_keys ? s0 + lrow + 32 * u : n_keys - 1;
+#pragma unroll
+        for (int cg = 0; cg < KG; ++cg) {
+          const int c = cg * 64 + lc < dk ? cg * 64 + lc : 0;
+          load_lds16(c < p.dim ? kbase + row * kvp + c : rc + row * p.rot + (c - p.dim),
+                     &dst[(cg * 64 + wave * 8 + 32 * u) * 64]);
+        }
       }
-#pragma unroll
-      for (int i = 0; i < VI; ++i) {
-        const int c = t + THREADS * i, r = c / (DVT * 2), e0 = (c - r * DVT * 2) * 8;
+    } else {
+      for (int c = t; c < 64 * DKC * 32; c += 256) {
+        const int r = c / (DKC * 32), e = c - r * DKC * 32;
         const long row = s0 + r < n_keys ? s0 + r : n_keys - 1;
-        rv[i] = ld16(vbase + row * kvp + (e0 < p.vdim ? e0 : 0));
-        rv[i] = e0 < p.vdim ? rv[i] : zero;
+        dst[tile_at<64>(r, e)] = e < p.dim ? kbase[row * kvp + e] : (e < dk ? rc[row * p.rot + e - p.dim] : (uint16_t)0);
       }
     }
   };
-  auto put = [&](int s0, int buf) {
-    uint16_t *kl = smem + buf * STAGE, *vl = kl + 64 * KPITCH;
-    if (v8) {
+  auto load_v = [&](int s0) {
+    if (vec) {
 #pragma unroll
-      for (int i = 0; i < KI; ++i) {
-        const int c = t + THREADS * i, r = c / (DKC * 4), e0 = (c - r * DKC * 4) * 8;
-        if (KCH % THREADS == 0 || c < KCH) *(u32x4*)&kl[r * KPITCH + e0] = rk[i];
-      }
+      for (int u = 0; u < 2; ++u) {
+        const long row = s0 + lrow + 32 * u < n_keys ? s0 + lrow + 32 * u : n_keys - 1;
 #pragma unroll
-      for (int i = 0; i < VI; ++i) {
-        const int c = t + THREADS * i, r = c / (DVT * 2), e0 = (c - r * DVT * 2) * 8;
-        if (VCH % THREADS == 0 || c < VCH) *(u32x4*)&vl[r * VPITCH + e0] = rv[i];
+        for (int cg = 0; cg < VG; ++cg)
+          load_lds16(vbase + row * kvp + (cg * 64 + lc < p.vdim ? cg * 64 + lc : 0), &vl[(cg * 64 + wave * 8 + 32 * u) * 64]);
       }
-    } else {  // rows whose parts are no multiples of 16 bytes: element by element
-      for (int c = t; c < 64 * DKC * 32; c += THREADS) {
-        const int r = c / (DKC * 32), e = c - r * DKC * 32;
-        const long row = s0 + r < n_keys ? s0 + r : n_keys - 1;
-        kl[r * KPITCH + e] = e < p.dim ? kbase[row * kvp + e] : (e < dk ? rc[row * p.rot + e - p.dim] : (uint16_t)0);
-      }
-      for (int c = t; c < 64 * DVT * 16; c += THREADS) {
+    } else {
+      for (int c = t; c < 64 * DVT * 16; c += 256) {
         const int r = c / (DVT * 16), e = c - r * DVT * 16;
         const long row = s0 + r < n_keys ? s0 + r : n_keys - 1;
-        vl[r * VPITCH + e] = e < p.vdim ? vbase[row * kvp + e] : (uint16_t)0;
+        vl[tile_at<64>(r, e)] = e < p.vdim ? vbase[row * kvp + e] : (uint16_t)0;
       }
     }
   };
   // this wave's queries, as positions counted from lo
   const int wq0 = (int)((long)p.q_first + qt0 + wave * 32 - lo), wq1 = wq0 + 31;
-  auto attend = [&](int s0, int buf) {
-    const uint16_t *kl = smem + buf * STAGE, *vl = kl + 64 * KPITCH;
-    f32x4 s4[2][4];
+  if (n_keys > 0) load_k(0, smem);
+  for (int s0 = 0, buf = 0; s0 < n_keys; s0 += 64, buf ^= 1) {
+    const uint16_t* kl = smem + buf * KSTAGE;
+    const bool more = s0 + 64 < n_keys;
+    // (blocks that none of the wave's queries sees are skipped)
+    const bool mine = s0 <= wq1 && (p.window <= 0 || s0 + 63 > wq0 - p.window);
+    wait_loads<0>();  // this wave's rows of the keys have landed
+    __syncthreads();                     // ... and everybody's; everybody is done with the values and the other keys
+    load_v(s0);
+    if (more) load_k(s0 + 64, smem + (buf ^ 1) * KSTAGE);
+    u32x4 pb[2][2];
+    if (mine) {
+      f32x4 s4[2][4];
 #pragma unroll
-    for (int kt = 0; kt < 4; ++kt) {
+      for (int kt = 0; kt < 4; ++kt) {
 #pragma unroll
-      for (int qt = 0; qt < 2; ++qt) s4[qt][kt] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int qt = 0; qt < 2; ++qt) s4[qt][kt] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-      for (int c = 0; c < DKC; ++c) {
-        const u32x4 a = *(const u32x4*)&kl[(kt * 16 + i16) * KPITCH + c * 32 + 8 * g];
+        for (int c = 0; c < DKC; ++c) {
+          const u32x4 a = *(const u32x4*)&kl[tile_at<64>(kt * 16 + i16, c * 32 + 8 * g)];
 #pragma unroll
-        for (int qt = 0; qt < 2; ++qt) s4[qt][kt] = mfma16x16x32<T>(a, q[qt][c], s4[qt][kt]);
+          for (int qt = 0; qt < 2; ++qt) s4[qt][kt] = mfma16x16x32<T>(a, q[qt][c], s4[qt][kt]);
+        }
+      }
+      const bool full = s0 + 63 <= wq0 && (p.window <= 0 || s0 >= wq1 - p.window + 1);
+#pragma unroll
+      for (int qt = 0; qt < 2; ++qt) {
+        float mx = -INFINITY;
+        if (full) {
+#pragma unroll
+          for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              s4[qt][kt][r] *= sc;
+              mx = fmaxf(mx, s4[qt][kt][r]);
+            }
+        } else {
+          // keys counted from the block's start: the last one seen, and the last one in front of the window
+          const int last = wq0 + qt * 16 + i16 - s0, before = p.window > 0 ? last - p.window : -1;
+#pragma unroll
+          for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+              const int s = kt * 16 + 4 * g + r;
+              const float v = s4[qt][kt][r] * sc;
+              s4[qt][kt][r] = s <= last && s > before ? v : -INFINITY;
+              mx = fmaxf(mx, s4[qt][kt][r]);
+            }
+        }
+        mx = fmaxf(mx, __shfl_xor(mx, 16));
+        mx = fmaxf(mx, __shfl_xor(mx, 32));
+        if (__any(mx > m[qt])) {
+          const float mn = fmaxf(m[qt], mx), keep = __builtin_amdgcn_exp2f(m[qt] - mn);
+          m[qt] = mn;
+          l[qt] *= keep;
+#pragma unroll
+          for (int j = 0; j < DVT; ++j)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) acc[qt][j][r] *= keep;
+        }
+        float e[4][4], sum = 0.f;
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) {
+            e[kt][r] = __builtin_amdgcn_exp2f(s4[qt][kt][r] - m[qt]);
+            sum += e[kt][r];
+          }
+        l[qt] += sum;  // this lane's keys only; the lane groups are added up at the end
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk)
+          pb[qt][kk] = u32x4{T::pack2(e[2 * kk][0], e[2 * kk][1]), T::pack2(e[2 * kk][2], e[2 * kk][3]),
+                             T::pack2(e[2 * kk + 1][0], e[2 * kk + 1][1]), T::pack2(e[2 * kk + 1][2], e[2 * kk + 1][3])};
       }
     }
-    const bool full = s0 + 63 <= wq0 && (p.window <= 0 || s0 >= wq1 - p.window + 1);
-    u32x4 pb[2][2];
-#pragma unroll
-    for (int qt = 0; qt < 2; ++qt) {
-      const int qp = wq0 + qt * 16 + i16;
-      float mx = -INFINITY;
-#pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) {
-          float v = s4[qt][kt][r] * sc;
-          if (!full) {
-            const int s = s0 + kt * 16 + 4 * g + r;
-            if (s > qp || (p.window > 0 && s <= qp - p.window)) v = -INFINITY;
-          }
-          s4[qt][kt][r] = v;
-          mx = fmaxf(mx, v);
-        }
-      mx = fmaxf(mx, __shfl_xor(mx, 16));
-      mx = fmaxf(mx, __shfl_xor(mx, 32));
-      if (__any(mx > m[qt])) {
-        const float mn = fmaxf(m[qt], mx), keep = exp2f(m[qt] - mn);
-        m[qt] = mn;
-        l[qt] *= keep;
-#pragma unroll
-        for (int j = 0; j < DVT; ++j)
-#pragma unroll
-          for (int r = 0; r < 4; ++r) acc[qt][j][r] *= keep;
-      }
-      float e[4][4], sum = 0.f;
-#pragma unroll
-      for (int kt = 0; kt < 4; ++kt)
-#pragma unroll
-        for (int r = 0; r < 4; ++r) { e[kt][r] = exp2f(s4[qt][kt][r] - m[qt]); sum += e[kt][r]; }
-      l[qt] += sum;  // this lane's keys only; the lane groups are added up at the end
+    // the values were requested before the next keys
+    if (more) wait_loads<2 * KG>();
+    else wait_loads<0>();
+    __syncthreads();
+    if (mine) {
 #pragma unroll
       for (int kk = 0; kk < 2; ++kk)
-        pb[qt][kk] = u32x4{T::pack2(e[2 * kk][0], e[2 * kk][1]), T::pack2(e[2 * kk][2], e[2 * kk][3]),
-                           T::pack2(e[2 * kk + 1][0], e[2 * kk + 1][1]), T::pack2(e[2 * kk + 1][2], e[2 * kk + 1][3])};
+#pragma unroll
+        for (int j = 0; j < DVT; ++j) {
+          const int row = 32 * kk + 4 * g + (i16 >> 2), col = 16 * j + 4 * (i16 & 3);
+          const u32x2 a0 = lds_read_tr16(&vl[tile_at<64>(row, col)]);
+          const u32x2 a1 = lds_read_tr16(&vl[tile_at<64>(row + 16, col)]);
+          const u32x4 va = {a0.x, a0.y, a1.x, a1.y};
+#pragma unroll
+          for (int qt = 0; qt < 2; ++qt) acc[qt][j] = mfma16x16x32<T>(va, pb[qt][kk], acc[qt][j]);
+        }
     }
-#pragma unroll
-    for (int kk = 0; kk < 2; ++kk)
-#pragma unroll
-      for (int j = 0; j < DVT; ++j) {
-        const u32x2 a0 = lds_read_tr16(&vl[(32 * kk + 4 * g + (i16 >> 2)) * VPITCH + 16 * j + 4 * (i16 & 3)]);
-        const u32x2 a1 = lds_read_tr16(&vl[(32 * kk + 16 + 4 * g + (i16 >> 2)) * VPITCH + 16 * j + 4 * (i16 & 3)]);
-        const u32x4 va = {a0.x, a0.y, a1.x, a1.y};
-#pragma unroll
-        for (int qt = 0; qt < 2; ++qt) acc[qt][j] = mfma16x16x32<T>(va, pb[qt][kk], acc[qt][j]);
-      }
-  };
-  if (n_keys > 0) {
-    fetch(0);
-    put(0, 0);
-  }
-  for (int s0 = 0, buf = 0; s0 < n_keys; s0 += 64, buf ^= 1) {
-    __syncthreads();  // block s0 is in its stage; everybody is done with the other one
-    const bool more = s0 + 64 < n_keys;
-    if (more) fetch(s0 + 64);
-    // (blocks that none of the wave's queries sees are skipped)
-    if (s0 <= wq1 && (p.window <= 0 || s0 + 63 > wq0 - p.window)) attend(s0, buf);
-    if (more) put(s0 + 64, buf ^ 1);
   }
 #pragma unroll
   for (int qt = 0; qt < 2; ++qt) {
@@ -655,34 +682,26 @@ static int launch_latent_plain(hipStream_t s, const LatentParams& p) {
 template <typename T>
 static int launch_latent_decode(hipStream_t s, const LatentParams& p) {
   const int tokens = p.batch * p.t;
-  if (tokens > 65535 || p.kv_rank > 1024) return MUI_ERR_UNSUPPORTED;
+  if (tokens > 65535 || p.kp > kMaxDecodeWidth) return MUI_ERR_UNSUPPORTED;
   hipLaunchKernelGGL((latent_absorb_kernel<T>), dim3(p.heads, ceil_div(p.kv_rank, 64), ceil_div(tokens, kAbsTok)),
                      dim3(256), 0, s, p);
   const dim3 grid(p.splits, ceil_div(p.heads, 16), tokens);
-  const size_t lds = (size_t)80 * (p.kp + 8) * 2;
+  const size_t lds = (size_t)kDecKeys * p.kp * 2;
   int st;
-  if (p.kv_rank <= 128) st = launch_with_lds(latent_decode_kernel<T, 2>, grid, dim3(256), lds, s, p);
-  else if (p.kv_rank <= 256) st = launch_with_lds(latent_decode_kernel<T, 4>, grid, dim3(256), lds, s, p);
-  else if (p.kv_rank <= 512) st = launch_with_lds(latent_decode_kernel<T, 8>, grid, dim3(256), lds, s, p);
-  else st = launch_with_lds(latent_decode_kernel<T, 16>, grid, dim3(256), lds, s, p);
+  if (p.kp <= 192 && p.kv_rank <= 128) st = launch_with_lds(latent_decode_kernel<T, 1>, grid, dim3(512), lds, s, p);
+  else if (p.kp <= 320 && p.kv_rank <= 256) st = launch_with_lds(latent_decode_kernel<T, 2>, grid, dim3(512), lds, s, p);
+  else st = launch_with_lds(latent_decode_kernel<T, 4>, grid, dim3(512), lds, s, p);
   if (st != MUI_OK) return st;
   return launch_with_lds(latent_output_kernel<T>, dim3(p.heads, ceil_div(p.vdim, 32), tokens), dim3(256),
                          (size_t)p.kv_rank * 4, s, p);
 }
 
-template <typename T, int DKC, int DVT, int NW>
-static int launch_latent_prefill_w(hipStream_t s, const LatentParams& p) {
-  constexpr size_t kv = (size_t)2 * 64 * (DKC * 32 + 8 + DVT * 16 + 16) * 2, q = (size_t)32 * NW * (DKC * 32 + 8) * 2;
-  const int tiles = ceil_div(p.t, 32 * NW);
-  if (tiles > 65535) return MUI_ERR_UNSUPPORTED;
-  return launch_with_lds(latent_prefill_kernel<T, DKC, DVT, NW>, dim3(p.heads, tiles), dim3(64 * NW), kv > q ? kv : q, s, p);
-}
-
 template <typename T, int DKC, int DVT>
 static int launch_latent_prefill_t(hipStream_t s, const LatentParams& p) {
-  // 256 queries per workgroup once that leaves most of the chip something to do
-  if (p.heads * ceil_div(p.t, 256) * 2 >= device_cus()) return launch_latent_prefill_w<T, DKC, DVT, 8>(s, p);
-  return launch_latent_prefill_w<T, DKC, DVT, 4>(s, p);
+  constexpr size_t kv = (size_t)(2 * DKC * 32 + DVT * 16) * 64 * 2, q = (size_t)128 * DKC * 32 * 2;
+  const int tiles = ceil_div(p.t, 128);
+  if (tiles > 65535) return MUI_ERR_UNSUPPORTED;
+  return launch_with_lds(latent_prefill_kernel<T, DKC, DVT>, dim3(p.heads, tiles), dim3(256), kv > q ? kv : q, s, p);
 }
 
 static bool prefill_covers(int dk, int vdim) { return dk <= 256 && vdim <= 256; }
@@ -691,10 +710,9 @@ template <typename T>
 static int launch_latent_prefill(hipStream_t s, const LatentParams& p) {
   const int dk = p.dim + p.rot;
   if (dk <= 64 && p.vdim <= 64) return launch_latent_prefill_t<T, 2, 4>(s, p);
-  if (dk <= 96 && p.vdim <= 64) return launch_latent_prefill_t<T, 3, 4>(s, p);
   if (dk <= 128 && p.vdim <= 128) return launch_latent_prefill_t<T, 4, 8>(s, p);
   if (dk <= 192 && p.vdim <= 128) return launch_latent_prefill_t<T, 6, 8>(s, p);
-  if (prefill_covers(dk, p.vdim)) return launch_latent_prefill_w<T, 8, 16, 4>(s, p);
+  if (prefill_covers(dk, p.vdim)) return launch_latent_prefill_t<T, 8, 16>(s, p);
   return MUI_ERR_UNSUPPORTED;
 }
 
@@ -726,25 +744,23 @@ extern "C" int mui_latent_prepare(mui_stream_t stream, int dtype, const void* do
   return launch_status();
 }
 
-static int latent_kp(int kv_rank, int rot_dim) { return (kv_rank + rot_dim + 31) / 32 * 32; }
+static int latent_kp(int kv_rank, int rot_dim) { return (kv_rank + rot_dim + 63) / 64 * 64; }
 
 // keys per split and number of splits of the decode kernel for spans of up to `span` keys
 static void latent_split(int batch, int t, int heads, int span, int* splits, int* split_keys) {
   const int groups = batch * t * ceil_div(heads, 16);
   int want = device_cus() * 2 / (groups > 0 ? groups : 1);
   want = want < 1 ? 1 : (want > kMaxSplits ? kMaxSplits : want);
-  const int blocks = ceil_div(span, 64);
-  int per = ceil_div(blocks, want);
-  if (per < 2 && blocks > 8) per = 2;  // merging costs a split's partial result per head
-  *split_keys = per * 64;
+  const int blocks = ceil_div(span, kDecKeys);
+  const int per = ceil_div(blocks, want);
+  *split_keys = per * kDecKeys;
   *splits = ceil_div(blocks, per);
 }
 
 extern "C" int mui_latent_attention_route(int dtype, int tokens, int heads, int dim, int rot_dim, int vdim, int kv_rank) {
   if (dtype == MUI_DTYPE_F32 || kv_rank % 8) return MUI_LATENT_PLAIN;
   if (tokens > MUI_MAX_TOKENS && prefill_covers(dim + rot_dim, vdim)) return MUI_LATENT_PREFILL;
-  return kv_rank <= 1024 && (size_t)80 * (latent_kp(kv_rank, rot_dim) + 8) * 2 <= 150 * 1024 ? MUI_LATENT_DECODE
-                                                                                             : MUI_LATENT_PLAIN;
+  return latent_kp(kv_rank, rot_dim) <= kMaxDecodeWidth ? MUI_LATENT_DECODE : MUI_LATENT_PLAIN;
 }
 
 extern "C" size_t mui_latent_decode_scratch_bytes(int batch, int t, int heads, int kv_rank, int rot_dim, int span) {
@@ -776,7 +792,7 @@ extern "C" int mui_latent_attention(mui_stream_t stream, int dtype, int route, c
     return MUI_ERR_INVALID_ARG;
   }
   MUI_CHECK_ARG(route == MUI_LATENT_DECODE && scratch && span > 0);
-  if (kv_rank % 8) return MUI_ERR_UNSUPPORTED;
+  if (kv_rank % 8 || latent_kp(kv_rank, rot_dim) > kMaxDecodeWidth) return MUI_ERR_UNSUPPORTED;
   if (!aligned16(w_uk) || !aligned16(w_uv) || !aligned16(c_cache) || !aligned16(r_cache) || c_batch_stride % 8 ||
       (rot_dim % 8 == 0 && r_batch_stride % 8) || ((uintptr_t)scratch & 255))
     return MUI_ERR_ALIGNMENT;

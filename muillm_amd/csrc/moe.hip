@@ -253,15 +253,20 @@ __device__ __forceinline__ MoeTile moe_tile_at(const MoeGemmParams& p, int i, in
   return MoeTile{0, first, left < 0 ? 0 : (left < tile_pairs ? left : tile_pairs), 0};
 }
 
+// Weight rows reach LDS (a private area per wave, two stages) in runs of 256 bytes by LDS-direct loads and are
+// read back as operands: 16 rows x 128 k-values per tile and stage, rows of 256 bytes whose 16-byte chunk c
+// lives at chunk c ^ row. Loaded straight in operand order (64 bytes of 16 rows per instruction) the same
+// bytes arrive at about two thirds of the rate.
+constexpr int kT16Seg = 128;
 template <typename T, int EPI>
-__global__ void __launch_bounds__(256) moe_tile16_kernel(const MoeGemmParams p) {
+__global__ void __launch_bounds__(256, 2) moe_tile16_kernel(const MoeGemmParams p) {
   constexpr int ROWS = EPI == MOE_GATEUP ? 16 : 32;  // outputs per workgroup
-  constexpr int UNR = 4;
-  __shared__ float red[4][2][16][17];
+  // [wave][tile]; the stages are arrays of their own, so that the compiler can tell which loads a read waits for
+  __shared__ __align__(16) uint16_t wl0[4][2][16 * kT16Seg], wl1[4][2][16 * kT16Seg];
   __shared__ int prow[16];
   const MoeTile tile = moe_tile_at(p, blockIdx.y, 16);
   if (tile.count <= 0) return;
-  const int t = threadIdx.x, lane = t & (kWave - 1), wave = t >> 6;
+  const int t = threadIdx.x, lane = t & (kWave - 1), wave = __builtin_amdgcn_readfirstlane(t >> 6);
   const int r16 = lane & 15, g = lane >> 4;
   const int o0 = blockIdx.x * ROWS;
   if (t < 16) {
@@ -272,49 +277,68 @@ __global__ void __launch_bounds__(256) moe_tile16_kernel(const MoeGemmParams p) 
   const int pair = p.pairs ? p.pairs[mine] : mine;
   const uint16_t* xr = p.x + (long)(EPI == MOE_GATEUP ? pair / p.top : pair) * p.k;
   const long eb = (long)tile.expert * p.expert_stride;
-  const int ra = o0 + r16 < p.n ? o0 + r16 : p.n - 1;
-  const int rb = EPI == MOE_GATEUP ? ra : (o0 + 16 + r16 < p.n ? o0 + 16 + r16 : p.n - 1);
-  const uint16_t* wa = p.w0 + eb + (long)ra * p.k;
-  const uint16_t* wb = (EPI == MOE_GATEUP ? p.w1 : p.w0) + eb + (long)rb * p.k;
-  f32x4 acc0 = {0.f, 0.f, 0.f, 0.f}, acc1 = {0.f, 0.f, 0.f, 0.f};
-  const int steps = (p.k + 31) >> 5;
+  // load instruction q of a tile: rows 4 q + lane / 16, this lane's logical chunk of the row
+  const uint16_t* src[2][4];
+  int chunk[4];
+#pragma unroll
+  for (int q = 0; q < 4; ++q) {
+    const int r = 4 * q + g;
+    chunk[q] = (r16 ^ r) * 8;
+    const int ra = o0 + r < p.n ? o0 + r : p.n - 1;
+    const int rb = EPI == MOE_GATEUP ? ra : (o0 + 16 + r < p.n ? o0 + 16 + r : p.n - 1);
+    src[0][q] = p.w0 + eb + (long)ra * p.k;
+    src[1][q] = (EPI == MOE_GATEUP ? p.w1 : p.w0) + eb + (long)rb * p.k;
+  }
+  f32x4 acc[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+  const int segs = (p.k + kT16Seg - 1) / kT16Seg;
   const u32x4 zero = {0u, 0u, 0u, 0u};
-  // two register sets: the next batch of loads is in flight while one is multiplied. Chunks past the row
-  // (or past this wave's steps) read its start and are multiplied as zeros.
-  struct Batch { u32x4 a[UNR], b[UNR], x[UNR]; };
-  auto load = [&](int s0, Batch& v) {
+  // segment s into a stage (past the last one: the first again, into a stage nobody reads); chunks past
+  // the end of a row read its start and meet x = 0
+  auto issue = [&](int s, uint16_t (&wl)[4][2][16 * kT16Seg], u32x4 (&x)[4]) {
+    const int k0 = s < segs ? s * kT16Seg : 0;
 #pragma unroll
-    for (int u = 0; u < UNR; ++u) {
-      const int kk = (s0 + 4 * u) * 32 + g * 8;
-      const int off = kk < p.k ? kk : 0;
-      v.a[u] = ld16_stream(wa + off);
-      v.b[u] = ld16_stream(wb + off);
-      v.x[u] = ld16(xr + off);
+    for (int j = 0; j < 2; ++j)
+#pragma unroll
+      for (int q = 0; q < 4; ++q) {
+        const int kk = k0 + chunk[q];
+        load_lds16(src[j][q] + (kk < p.k ? kk : 0), &wl[wave][j][q * 4 * kT16Seg]);
+      }
+#pragma unroll
+    for (int u = 0; u < 4; ++u) {
+      const int kk = k0 + 32 * u + 8 * g;
+      x[u] = ld16(xr + (kk < p.k ? kk : 0));
     }
   };
-  auto multiply = [&](int s0, const Batch& v) {
+  auto multiply = [&](int s, const uint16_t (&wl)[4][2][16 * kT16Seg], const u32x4 (&x)[4]) {
 #pragma unroll
-    for (int u = 0; u < UNR; ++u) {
-      const bool live = (s0 + 4 * u) * 32 + g * 8 < p.k;
-      const u32x4 xv = live ? v.x[u] : zero;
-      acc0 = mfma16x16x32<T>(live ? v.a[u] : zero, xv, acc0);
-      acc1 = mfma16x16x32<T>(live ? v.b[u] : zero, xv, acc1);
+    for (int u = 0; u < 4; ++u) {
+      const u32x4 xv = s * kT16Seg + 32 * u + 8 * g < p.k ? x[u] : zero;
+#pragma unroll
+      for (int j = 0; j < 2; ++j)
+        acc[j] = mfma16x16x32<T>(*(const u32x4*)&wl[wave][j][r16 * kT16Seg + ((4 * u + g) ^ r16) * 8], xv, acc[j]);
     }
   };
-  Batch b0, b1;
-  if (wave < steps) {
-    load(wave, b0);
-    for (int s0 = wave; s0 < steps; s0 += 8 * UNR) {
-      load(s0 + 4 * UNR, b1);
-      multiply(s0, b0);
-      load(s0 + 8 * UNR, b0);
-      multiply(s0 + 4 * UNR, b1);
+  u32x4 x0[4], x1[4];
+  if (wave < segs) {
+    issue(wave, wl0, x0);
+    for (int s = wave; s < segs; s += 8) {
+      issue(s + 4, wl1, x1);
+      wait_loads<12>();  // everything but the newest segment has landed
+      multiply(s, wl0, x0);
+      if (s + 4 >= segs) break;
+      issue(s + 8, wl0, x0);
+      wait_loads<12>();
+      multiply(s + 4, wl1, x1);
     }
   }
+  wait_loads<0>();  // (no load is still on its way into LDS)
+  __syncthreads();
+  float(*red)[2][16][17] = (float(*)[2][16][17])wl0;
+  static_assert(sizeof(wl0) >= sizeof(float) * 4 * 2 * 16 * 17, "the partial tiles fit where the weights were");
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
-    red[wave][0][4 * g + r][r16] = acc0[r];
-    red[wave][1][4 * g + r][r16] = acc1[r];
+    red[wave][0][4 * g + r][r16] = acc[0][r];
+    red[wave][1][4 * g + r][r16] = acc[1][r];
   }
   __syncthreads();
   const int row = t & 15, col = t >> 4;
@@ -404,12 +428,10 @@ __global__ void __launch_bounds__(64 * NWR * NWT, NWR * NWT == 4 ? 2 : 1) moe_ti
   auto dma = [&](int s, int buf) {
 #pragma unroll
     for (int q = 0; q < WQ; ++q)
-      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(wsrc[q] + s * kMgK),
-                                       (__attribute__((address_space(3))) void*)&w_lds[buf][(q * NW + wave) * 8 * kMgK], 16, 0, 0);
+      load_lds16(wsrc[q] + s * kMgK, &w_lds[buf][(q * NW + wave) * 8 * kMgK]);
 #pragma unroll
     for (int q = 0; q < XQ; ++q)
-      __builtin_amdgcn_global_load_lds((const __attribute__((address_space(1))) void*)(xsrc[q] + s * kMgK),
-                                       (__attribute__((address_space(3))) void*)&x_lds[buf][(q * NW + wave) * 8 * kMgK], 16, 0, 0);
+      load_lds16(xsrc[q] + s * kMgK, &x_lds[buf][(q * NW + wave) * 8 * kMgK]);
   };
   u32x4 rw[WQ], rx[XQ];
   auto fetch = [&](int s) {
@@ -444,7 +466,7 @@ __global__ void __launch_bounds__(64 * NWR * NWT, NWR * NWT == 4 ? 2 : 1) moe_ti
   for (int s = 0; s < steps; ++s) {
     const int buf = s & 1;
     const bool more = s + 1 < steps;
-    if constexpr (DMA) __builtin_amdgcn_s_waitcnt(0x0F70);  // this wave's blocks of step s have landed
+    if constexpr (DMA) wait_loads<0>();  // this wave's blocks of step s have landed
     __syncthreads();  // ... and everybody's; everybody is done with the other stage
     if (more) {
       if constexpr (DMA) dma(s + 1, buf ^ 1);
