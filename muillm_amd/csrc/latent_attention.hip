@@ -15,7 +15,7 @@
 //   plain     one workgroup per query and head: fp32 models, sizes the others do not cover.
 //
 // Positions: a token's slot in the cache minus its row's first slot (left-padded batches). Angles are
-// formed in double precision (position * inv_freq, reduced modulo 2 pi) and rounded to fp32 once.
+// formed and reduced in double precision and rounded to fp32 once: no table, no longest sequence.
 #include "skinny.cuh"
 
 namespace mui {
@@ -42,18 +42,19 @@ struct LatentParams {
   void* out;  // [tokens, heads * vdim]
 
   void* q_abs;       // decode: [tokens, heads, kp] 16-bit
-  float* part;       // decode: [tokens, heads, splits, kv_rank + 2]
+  float* part;       // decode: [tokens, heads, splits, kv_rank]
+  float* part_ml;    // decode: [tokens, heads, splits, 2]: running maximum, sum
   int kp, splits, split_keys;
 
   const void* kv;    // prefill: [keys, heads * (dim + vdim)], key row 0 = slot kv_first
   int kv_first, kv_rows, q_first, b0;
 };
 
+// cos and sin of pos * inv_freq: the angle in turns, its whole turns dropped in double precision, rounded once
 __device__ __forceinline__ void rope_angle(double pos, double inv_freq, float& c, float& s) {
-  const double two_pi = 6.283185307179586476925286766559;
-  double a = pos * inv_freq;
-  a -= two_pi * rint(a / two_pi);
-  sincosf((float)a, &s, &c);
+  double a = pos * inv_freq * 0.15915494309189533576888376337251;
+  a -= rint(a);
+  sincospif((float)(2.0 * a), &s, &c);
 }
 
 __device__ __forceinline__ float block_sum256(float v, float* red) {
@@ -329,11 +330,13 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(const LatentParams p
     for (int u = 0; u < 2; ++u) {
       const int row = (wave + 8 * u) * 8 + lrow;
       const long s = s0 + row < s_end ? s0 + row : s_end - 1;
+      const uint16_t *crow = cc + s * p.kv_rank, *rrow = rc + s * p.rot - p.kv_rank;
       const int lc = ((lane & 7) ^ tile_swz(row)) * 8;
-      for (int c0 = 0; c0 < p.kp; c0 += 64) {
-        const int c = c0 + lc < width ? c0 + lc : 0;
-        load_lds16(c < p.kv_rank ? cc + s * p.kv_rank + c : rc + s * p.rot + (c - p.kv_rank),
-                   &cl[((c0 >> 6) * kDecKeys + (wave + 8 * u) * 8) * 64]);
+#pragma unroll
+      for (int cb = 0; cb < KC / 2; ++cb) {
+        if (cb * 64 >= p.kp) break;
+        const int c = cb * 64 + lc < width ? cb * 64 + lc : 0;
+        load_lds16((c < p.kv_rank ? crow : rrow) + c, &cl[(cb * kDecKeys + (wave + 8 * u) * 8) * 64]);
       }
     }
     wait_loads<0>();
@@ -402,17 +405,15 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(const LatentParams p
     }
   }
   if (h0 + i16 < p.heads) {
-    float* dst = p.part + (((long)tok * p.heads + h0 + i16) * p.splits + split) * (p.kv_rank + 2);
+    const long at = ((long)tok * p.heads + h0 + i16) * p.splits + split;
 #pragma unroll
-    for (int j = 0; j < NT; ++j)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) {
-        const int c = 16 * (wave + 8 * j) + 4 * g + r;
-        if (c < p.kv_rank) dst[c] = acc[j][r];
-      }
+    for (int j = 0; j < NT; ++j) {
+      const int c = 16 * (wave + 8 * j) + 4 * g;  // (kv_rank is a multiple of 8)
+      if (c < p.kv_rank) *(f32x4*)&p.part[at * p.kv_rank + c] = acc[j];
+    }
     if (wave == 0 && g == 0) {
-      dst[p.kv_rank] = m;
-      dst[p.kv_rank + 1] = l;
+      p.part_ml[at * 2] = m;
+      p.part_ml[at * 2 + 1] = l;
     }
   }
 }
@@ -425,11 +426,11 @@ __global__ void __launch_bounds__(256) latent_output_kernel(const LatentParams p
   __shared__ float ws[kMaxSplits];
   float* o = (float*)la_smem;  // kv_rank
   const int h = blockIdx.x, tok = blockIdx.z, t = threadIdx.x;
-  const long stride = p.kv_rank + 2;
-  const float* part = p.part + ((long)tok * p.heads + h) * p.splits * stride;
+  const long at = ((long)tok * p.heads + h) * p.splits;
+  const float* part = p.part + at * p.kv_rank;
   if (t < kWave) {  // the splits' shares, one per lane
     const bool in = t < p.splits;
-    const float mm = in ? part[t * stride + p.kv_rank] : -1e30f, ll = in ? part[t * stride + p.kv_rank + 1] : 0.f;
+    const float mm = in ? p.part_ml[(at + t) * 2] : -1e30f, ll = in ? p.part_ml[(at + t) * 2 + 1] : 0.f;
     const float e = exp2f(mm - wave_max(mm));
     const float l = wave_sum(e * ll);
     if (in) ws[t] = ll > 0.f ? e / l : 0.f;
@@ -438,7 +439,7 @@ __global__ void __launch_bounds__(256) latent_output_kernel(const LatentParams p
   for (int r = t; r < p.kv_rank; r += 256) {
     float a = 0.f;
 #pragma unroll 8
-    for (int s = 0; s < p.splits; ++s) a = fmaf(ws[s], part[s * stride + r], a);
+    for (int s = 0; s < p.splits; ++s) a = fmaf(ws[s], part[(long)s * p.kv_rank + r], a);
     o[r] = a;
   }
   __syncthreads();
@@ -800,6 +801,7 @@ extern "C" int mui_latent_attention(mui_stream_t stream, int dtype, int route, c
   latent_split(batch, t, heads, span, &p.splits, &p.split_keys);
   p.q_abs = scratch;
   p.part = (float*)((char*)scratch + ((size_t)batch * t * heads * p.kp * 2 + 255) / 256 * 256);
+  p.part_ml = p.part + (size_t)batch * t * heads * p.splits * kv_rank;
   if (dtype == MUI_DTYPE_F16) return launch_latent_decode<F16>(s, p);
   if (dtype == MUI_DTYPE_BF16) return launch_latent_decode<BF16>(s, p);
   return MUI_ERR_INVALID_ARG;

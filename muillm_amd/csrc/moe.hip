@@ -18,8 +18,8 @@
 //   tile 16   up to 16 pairs of an expert: 16 gate + 16 up rows (or 32 rows) per workgroup, K dealt out to
 //             its four waves, operands straight from global memory in matrix order. Decode and short
 //             prompts: every chosen expert's weights are streamed once.
-//   tile 128 / 256   as many pairs x as many rows, waves of 64 x 64, both operands through swizzled LDS
-//             stages filled by LDS-direct loads.
+//   tile 128 / 256   as many pairs x as many rows, both operands through swizzled LDS stages filled by
+//             LDS-direct loads; waves of 64 x 64, or of 128 x 64 with operands read a half step ahead.
 // fp32 models and sizes that are no multiple of 8 take a plain one-wave-per-output kernel.
 #include "skinny.cuh"
 
@@ -89,7 +89,7 @@ __global__ void __launch_bounds__(256) linear_f32_rows_kernel(const typename T::
 // routing
 // ---------------------------------------------------------------------------------------
 constexpr int kMaxRouter = 1024;   // router outputs
-constexpr int kRouteThreads = 1024;
+constexpr int kRouteThreads = 1024;  // at most; few tokens take fewer
 constexpr int kRouterPerLane = kMaxRouter / kWave;
 
 // one token by one wave
@@ -176,17 +176,17 @@ __global__ void __launch_bounds__(kRouteThreads) moe_group_kernel(const float* l
                                                                   float* weight, int32_t* pairs, MoeTile* tiles) {
   __shared__ int count[kMaxRouter], cursor[kMaxRouter], first_tile[kMaxRouter];
   __shared__ int n_tiles_s;
-  const int t = threadIdx.x;
+  const int t = threadIdx.x, nt_threads = blockDim.x;
   const int n_pairs = tokens * top;
-  for (int e = t; e < n_experts; e += kRouteThreads) count[e] = 0;
+  for (int e = t; e < n_experts; e += nt_threads) count[e] = 0;
   if constexpr (ROUTE) {
-    for (int tk = t >> 6; tk < tokens; tk += kRouteThreads / kWave)
+    for (int tk = t >> 6; tk < tokens; tk += nt_threads / kWave)
       route_token<T>(logits + (long)tk * n_out, corr, n_out, top, t & (kWave - 1), expert + (long)tk * top,
                      weight + (long)tk * top);
     __threadfence_block();
   }
   __syncthreads();
-  for (int i = t; i < n_pairs; i += kRouteThreads) {
+  for (int i = t; i < n_pairs; i += nt_threads) {
     const int e = expert[i];
     if (e < n_experts) atomicAdd(&count[e], 1);
   }
@@ -214,17 +214,17 @@ __global__ void __launch_bounds__(kRouteThreads) moe_group_kernel(const float* l
   }
   __syncthreads();
   const int n_tiles = n_tiles_s;
-  for (int e = t; e < n_experts; e += kRouteThreads) {
+  for (int e = t; e < n_experts; e += nt_threads) {
     const int c = count[e], base = cursor[e], ft = first_tile[e];
     for (int i = 0; i * tile_pairs < c && ft + i < max_tiles; ++i) {
       const int left = c - i * tile_pairs;
       tiles[1 + ft + i] = MoeTile{e, base + i * tile_pairs, left < tile_pairs ? left : tile_pairs, 0};
     }
   }
-  for (int i = n_tiles + t; i < max_tiles; i += kRouteThreads) tiles[1 + i] = MoeTile{0, 0, 0, 0};
+  for (int i = n_tiles + t; i < max_tiles; i += nt_threads) tiles[1 + i] = MoeTile{0, 0, 0, 0};
   if (t == 0) tiles[0] = MoeTile{0, 0, n_tiles, 0};
   __syncthreads();  // cursors are read above before they move
-  for (int i = t; i < n_pairs; i += kRouteThreads) {
+  for (int i = t; i < n_pairs; i += nt_threads) {
     const int e = expert[i];
     if (e < n_experts) pairs[atomicAdd(&cursor[e], 1)] = i;
   }
@@ -523,6 +523,171 @@ __global__ void __launch_bounds__(64 * NWR * NWT, NWR * NWT == 4 ? 2 : 1) moe_ti
   }
 }
 
+// 256 rows x 256 pairs on eight waves of 128 x 64 (a quarter less LDS traffic per product than waves of 64 x 64,
+// which is what bounds those), k a multiple of 64. A wave holds two sets of operands: the LDS reads of one
+// half of a k-step are in flight while the other half is multiplied, and the one barrier per step has a
+// half's multiplications behind it.
+template <typename T, int EPI>
+__global__ void __launch_bounds__(512) moe_pipe_kernel(const MoeGemmParams p) {
+  constexpr int NW = 8, TILE = 256, OUT = EPI == MOE_GATEUP ? TILE / 2 : TILE, WR = 8, WT = 4;
+  typedef uint16_t Stage[TILE * kMgK];
+  Stage* w_lds = (Stage*)moe_smem;
+  Stage* x_lds = (Stage*)(moe_smem + 2 * sizeof(Stage));
+  __shared__ int prow[TILE];
+  constexpr int SUP = 2;
+  const int n_tiles = p.tiles[0].count;
+  const int r_tiles = (p.n + OUT - 1) / OUT;
+  const int total = ((n_tiles + SUP - 1) / SUP) * SUP * r_tiles;
+  const int share = (total + 7) / 8;
+  const int slot = blockIdx.x >> 3, id = (blockIdx.x & 7) * share + slot;
+  if (slot >= share || id >= total) return;
+  const int sup = id / (SUP * r_tiles), in_sup = id - sup * SUP * r_tiles;
+  const int ti = sup * SUP + in_sup % SUP;
+  if (ti >= n_tiles) return;
+  const MoeTile tile = p.tiles[1 + ti];
+  const int o0 = (in_sup / SUP) * OUT;
+
+  const int t = threadIdx.x, lane = t & (kWave - 1), wave = __builtin_amdgcn_readfirstlane(t >> 6);
+  // SIMD i runs waves i and i + 4, which are 128 pairs apart: a tile of few pairs leaves every SIMD its share
+  const int wr = wave & 1, wt = wave >> 1;
+  if (t < TILE) prow[t] = p.pairs[tile.first + (t < tile.count ? t : 0)];
+  __syncthreads();
+  // wave instruction q covers tile rows (q NW + wave) * 8 ..: 32-bit offsets from bases that are the same for
+  // the wave (gate and up rows change at multiples of 64)
+  const int sr = lane >> 3, sc = lane & 7;
+  const int chunk = (sc ^ (((wave * 8 + sr) >> 1) & 7)) * 8;
+  const uint16_t* wbase[4];
+  unsigned woff[4], xoff[4];
+  const long eb = (long)tile.expert * p.expert_stride;
+#pragma unroll
+  for (int q = 0; q < 4; ++q) {
+    const int r0 = (q * NW + wave) * 8, r = r0 + sr;
+    int o;
+    if constexpr (EPI == MOE_GATEUP) {  // a wave's 128 rows: 64 gate rows, the 64 up rows of the same outputs
+      o = o0 + (r >> 7) * 64 + (r & 63);
+      wbase[q] = ((r0 & 64) ? p.w1 : p.w0) + eb;
+    } else {
+      o = o0 + r;
+      wbase[q] = p.w0 + eb;
+    }
+    o = o < p.n ? o : p.n - 1;
+    woff[q] = (unsigned)o * (unsigned)p.k + chunk;
+    const int pr = prow[r];
+    xoff[q] = (unsigned)(EPI == MOE_GATEUP ? pr / p.top : pr) * (unsigned)p.k + chunk;
+  }
+  auto dma = [&](int s, int buf) {
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      unsigned off = woff[q];
+      asm volatile("" : "+v"(off));  // (kept as a 32-bit offset from a scalar base)
+      load_lds16(wbase[q] + s * kMgK + off, &w_lds[buf][(q * NW + wave) * 8 * kMgK]);
+    }
+#pragma unroll
+    for (int q = 0; q < 4; ++q) {
+      unsigned off = xoff[q];
+      asm volatile("" : "+v"(off));
+      load_lds16(p.x + s * kMgK + off, &x_lds[buf][(q * NW + wave) * 8 * kMgK]);
+    }
+  };
+  f32x4 acc[WR][WT];
+#pragma unroll
+  for (int i = 0; i < WR; ++i)
+#pragma unroll
+    for (int j = 0; j < WT; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+  const int r16 = lane & 15, lg = lane >> 4, lsw = (r16 >> 1) & 7;
+  const int a_base = (wr * 128 + r16) * kMgK, b_base = (wt * 64 + r16) * kMgK;
+  u32x4 a[2][WR], b[2][WT];
+  auto read = [&](int buf, int kk, int set) {
+    const int c = ((kk * 4 + lg) ^ lsw) * 8;
+#pragma unroll
+    for (int j = 0; j < WT; ++j) b[set][j] = *(const u32x4*)&x_lds[buf][b_base + j * 16 * kMgK + c];
+#pragma unroll
+    for (int i = 0; i < WR; ++i) a[set][i] = *(const u32x4*)&w_lds[buf][a_base + i * 16 * kMgK + c];
+  };
+  auto multiply = [&](int set) {
+#pragma unroll
+    for (int i = 0; i < WR; ++i)
+#pragma unroll
+      for (int j = 0; j < WT; ++j) acc[i][j] = mfma16x16x32<T>(a[set][i], b[set][j], acc[i][j]);
+  };
+  const int steps = p.k / kMgK;
+  dma(0, 0);
+  wait_loads<0>();
+  __syncthreads();
+  dma(steps > 1 ? 1 : 0, 1);
+  // Loads past the last step repeat it, into a stage nobody reads any more: no branches in the loop.
+  if (wt * 64 < tile.count) {
+    read(0, 0, 0);
+    for (int s = 0; s < steps; ++s) {
+      const int buf = s & 1;
+      read(buf, 1, 1);
+      multiply(0);
+      // issue order of the half: two matrix instructions, an LDS read, ...
+#pragma unroll
+      for (int i = 0; i < WR + WT; ++i) {
+        __builtin_amdgcn_sched_group_barrier(0x008, 2, 0);
+        __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+      }
+      __builtin_amdgcn_sched_group_barrier(0x008, WR * WT - 2 * (WR + WT), 0);
+      wait_loads<0>();  // step s + 1 has landed
+      __syncthreads();  // ... for everybody, and everybody has read step s
+      dma(s + 2 < steps ? s + 2 : steps - 1, buf);
+      read(buf ^ 1, 0, 0);
+      multiply(1);
+      // ... a matrix instruction and a load, eight times, then two matrix instructions and a read
+#pragma unroll
+      for (int i = 0; i < 8; ++i) {
+        __builtin_amdgcn_sched_group_barrier(0x008, 1, 0);
+        __builtin_amdgcn_sched_group_barrier(0x010, 1, 0);
+      }
+#pragma unroll
+      for (int i = 0; i < WR + WT; ++i) {
+        __builtin_amdgcn_sched_group_barrier(0x008, 2, 0);
+        __builtin_amdgcn_sched_group_barrier(0x100, 1, 0);
+      }
+    }
+  } else {  // none of this wave's pairs exist: it only keeps the loads going
+    for (int s = 0; s < steps; ++s) {
+      wait_loads<0>();
+      __syncthreads();
+      dma(s + 2 < steps ? s + 2 : steps - 1, s & 1);
+    }
+  }
+  wait_loads<0>();  // no load is still on its way into LDS when the workgroup ends
+  const bool n4 = (p.n & 3) == 0;
+  auto store4 = [&](uint16_t* yr, int o, const float (&v)[4]) {
+    if (n4 && o + 4 <= p.n) {
+      *(u32x2*)&yr[o] = u32x2{T::pack2(v[0], v[1]), T::pack2(v[2], v[3])};
+    } else {
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (o + r < p.n) yr[o + r] = T::pack(v[r]);
+    }
+  };
+#pragma unroll
+  for (int j = 0; j < WT; ++j) {
+    const int c = wt * 64 + j * 16 + r16;
+    if (c >= tile.count) continue;
+    uint16_t* yr = (uint16_t*)p.y + (long)prow[c] * p.n;
+    float v[4];
+    if constexpr (EPI == MOE_GATEUP) {
+#pragma unroll
+      for (int i = 0; i < WR / 2; ++i) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] = moe_act(acc[i][j][r], acc[i + WR / 2][j][r], p.limit);
+        store4(yr, o0 + wr * 64 + i * 16 + 4 * lg, v);
+      }
+    } else {
+#pragma unroll
+      for (int i = 0; i < WR; ++i) {
+#pragma unroll
+        for (int r = 0; r < 4; ++r) v[r] = acc[i][j][r];
+        store4(yr, o0 + wr * 128 + i * 16 + 4 * lg, v);
+      }
+    }
+  }
+}
+
 // one wave per output of a pair: fp32 storage, and sizes that are no multiple of 8
 template <typename T, int EPI>
 __global__ void __launch_bounds__(256) moe_rows_kernel(const typename T::storage* w0, const typename T::storage* w1,
@@ -590,7 +755,16 @@ static int launch_moe_product(hipStream_t s, const MoeGemmParams& p, const int32
     }
     if (((uintptr_t)p.y & 7) != 0) return MUI_ERR_ALIGNMENT;
     if (tile_pairs == 128) return launch_moe_tile<T, EPI, 2, 2>(s, p);
-    if (tile_pairs == 256) return launch_moe_tile<T, EPI, 4, 4>(s, p);
+    if (tile_pairs == 256) {
+      const long xrows = EPI == MOE_GATEUP ? p.tokens : (long)p.tokens * p.top;
+      if (p.k % kMgK == 0 && (long)p.n * p.k < (1L << 30) && xrows * p.k < (1L << 30)) {
+        const long total = (long)ceil_div(p.max_tiles, 2) * 2 * ceil_div(p.n, EPI == MOE_GATEUP ? 128 : 256);
+        if (total > (1L << 30)) return MUI_ERR_UNSUPPORTED;
+        return launch_with_lds(moe_pipe_kernel<T, EPI>, dim3((unsigned)((total + 7) / 8 * 8)), dim3(512),
+                               (size_t)4 * 256 * kMgK * 2, s, p);
+      }
+      return launch_moe_tile<T, EPI, 4, 4>(s, p);
+    }
     return MUI_ERR_INVALID_ARG;
   }
   return MUI_ERR_UNSUPPORTED;
@@ -634,7 +808,7 @@ static int launch_route(hipStream_t s, const float* logits, const void* corr, in
                        top, tokens, expert, weight);
   if (!tile_pairs) return launch_status();
   if (one)
-    hipLaunchKernelGGL((moe_group_kernel<T, true>), dim3(1), dim3(kRouteThreads), 0, s, logits, (const S*)corr, n_out,
+    hipLaunchKernelGGL((moe_group_kernel<T, true>), dim3(1), dim3(tokens <= 4 ? 256 : kRouteThreads), 0, s, logits, (const S*)corr, n_out,
                        n_experts, top, tokens, tile_pairs, max_tiles, expert, weight, pairs, tiles);
   else
     hipLaunchKernelGGL((moe_group_kernel<T, false>), dim3(1), dim3(kRouteThreads), 0, s, logits, (const S*)corr, n_out,
@@ -662,11 +836,12 @@ extern "C" int mui_linear_f32(mui_stream_t stream, int dtype, const void* weight
 
 extern "C" int mui_moe_tile_pairs(int dtype, int tokens, int top, int n_experts, int width, int ff) {
   if (dtype == MUI_DTYPE_F32 || width % 8 || ff % 8 || n_experts < 1) return 0;
-  // wide tiles once the experts have enough pairs each to fill a good part of one; of the two widths the one
-  // whose tiles cost less (a 256-pair tile about 1.3 times as much as a 128-pair one)
+  // 16-pair tiles stream an expert's weights once per tile; from about a dozen pairs per expert on a wide tile
+  // is cheaper even half empty. Of the two widths the one whose tiles cost less (a 256-pair tile about one
+  // and a half times as much as a 128-pair one).
   const long per = (long)tokens * top / n_experts;
-  if (per < 40) return 16;
-  return 13 * ((per + 255) / 256) < 10 * ((per + 127) / 128) ? 256 : 128;
+  if (per < 12) return 16;
+  return 15 * ((per + 255) / 256) < 10 * ((per + 127) / 128) ? 256 : 128;
 }
 
 extern "C" int mui_moe_max_tiles(int tokens, int top, int n_experts, int tile_pairs) {

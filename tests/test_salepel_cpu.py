@@ -137,7 +137,7 @@ def test_argument_checks_need_no_gpu():
     assert lib.mui_mlstm(None, 1, None, None, None, 8, None, 1.0, 1.0, None, None, None, None, None, None, None, 1, 1, 1, 8, 8) == -1
     assert lib.mui_moe_tile_pairs(2, 100, 2, 4, 64, 64) == 0 and lib.mui_moe_tile_pairs(1, 4, 2, 4, 64, 63) == 0
     assert lib.mui_moe_tile_pairs(1, 4, 2, 4, 64, 64) == 16 and lib.mui_moe_tile_pairs(1, 4000, 2, 4, 64, 64) == 256
-    assert lib.mui_moe_tile_pairs(1, 100, 2, 4, 64, 64) == 128
+    assert lib.mui_moe_tile_pairs(1, 100, 2, 4, 64, 64) == 128 and lib.mui_moe_tile_pairs(1, 20, 2, 4, 64, 64) == 16
     # enough tiles whatever the routing: every expert may leave one tile part empty
     for tokens, top, experts, tile in ((1, 3, 5, 16), (100, 2, 3, 16), (1000, 4, 60, 128)):
         n = lib.mui_moe_max_tiles(tokens, top, experts, tile)
