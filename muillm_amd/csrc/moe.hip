@@ -95,7 +95,7 @@ constexpr int kRouterPerLane = kMaxRouter / kWave;
 // one token by one wave
 template <typename T>
 __device__ __forceinline__ void route_token(const float* lg, const typename T::storage* corr, int n_out, int top,
-                                            int lane, int32_t* expert, float* weight) {
+                                            int lane, int32_t* expert, float* weight, int* expert_lds = nullptr) {
   float s[kRouterPerLane], choice[kRouterPerLane];
   float mx = -INFINITY;
 #pragma unroll
@@ -154,6 +154,7 @@ __device__ __forceinline__ void route_token(const float* lg, const typename T::s
     if (lane == 0) {
       expert[j] = bi;
       weight[j] = bs;
+      if (expert_lds) expert_lds[j] = bi;
     }
   }
 }
@@ -169,6 +170,7 @@ __global__ void __launch_bounds__(256) moe_route_kernel(const float* logits, con
 
 // One workgroup: (ROUTE: the routing of all tokens, then) count per expert, cut into tiles, scatter.
 // tiles[0].count = number of tiles, tiles[1 + i] the i-th tile; unused entries up to max_tiles get count 0.
+constexpr int kChosen = 1024;
 template <typename T, bool ROUTE>
 __global__ void __launch_bounds__(kRouteThreads) moe_group_kernel(const float* logits, const typename T::storage* corr,
                                                                   int n_out, int n_experts, int top, int tokens,
@@ -176,18 +178,23 @@ __global__ void __launch_bounds__(kRouteThreads) moe_group_kernel(const float* l
                                                                   float* weight, int32_t* pairs, MoeTile* tiles) {
   __shared__ int count[kMaxRouter], cursor[kMaxRouter], first_tile[kMaxRouter];
   __shared__ int n_tiles_s;
+  __shared__ int chosen[ROUTE ? kChosen : 1];  // the routing's result without the way through memory
   const int t = threadIdx.x, nt_threads = blockDim.x;
   const int n_pairs = tokens * top;
   for (int e = t; e < n_experts; e += nt_threads) count[e] = 0;
   if constexpr (ROUTE) {
     for (int tk = t >> 6; tk < tokens; tk += nt_threads / kWave)
       route_token<T>(logits + (long)tk * n_out, corr, n_out, top, t & (kWave - 1), expert + (long)tk * top,
-                     weight + (long)tk * top);
+                     weight + (long)tk * top, n_pairs <= kChosen ? chosen + tk * top : nullptr);
     __threadfence_block();
   }
+  auto expert_of = [&](int i) {
+    if constexpr (ROUTE) return n_pairs <= kChosen ? chosen[i] : expert[i];
+    else return expert[i];
+  };
   __syncthreads();
   for (int i = t; i < n_pairs; i += nt_threads) {
-    const int e = expert[i];
+    const int e = expert_of(i);
     if (e < n_experts) atomicAdd(&count[e], 1);
   }
   __syncthreads();
@@ -225,7 +232,7 @@ __global__ void __launch_bounds__(kRouteThreads) moe_group_kernel(const float* l
   if (t == 0) tiles[0] = MoeTile{0, 0, n_tiles, 0};
   __syncthreads();  // cursors are read above before they move
   for (int i = t; i < n_pairs; i += nt_threads) {
-    const int e = expert[i];
+    const int e = expert_of(i);
     if (e < n_experts) pairs[atomicAdd(&cursor[e], 1)] = i;
   }
 }
