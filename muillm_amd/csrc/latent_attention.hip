@@ -135,6 +135,31 @@ __device__ __forceinline__ float rotated_q(const typename T::storage* qh, const 
   return j < half ? u * c - v * s : v * c + u * s;
 }
 
+// elements e0 .. e0 + 7 of the same, rounded and packed; vec: dim a multiple of 8 and rot of 16, whole chunks by
+// 128-bit loads
+template <typename T>
+__device__ __forceinline__ u32x4 rotated_q8(const uint16_t* qh, const float* cs, int dim, int rot, int e0, bool vec) {
+  const u32x4 zero = {0u, 0u, 0u, 0u};
+  if (vec) {
+    if (e0 < dim) return ld16(qh + e0);
+    if (e0 >= dim + rot) return zero;
+    const int half = rot >> 1, j = e0 - dim, i = j < half ? j : j - half;
+    float u[8], v[8], c[8], s[8], o[8];
+    unpack8<T>(ld16(qh + dim + i), u);
+    unpack8<T>(ld16(qh + dim + half + i), v);
+    load8<F32>(cs + i, c);
+    load8<F32>(cs + half + i, s);
+#pragma unroll
+    for (int k = 0; k < 8; ++k) o[k] = j < half ? u[k] * c[k] - v[k] * s[k] : v[k] * c[k] + u[k] * s[k];
+    return pack8<T>(o);
+  }
+  uint32_t w[8];
+#pragma unroll
+  for (int k = 0; k < 8; ++k)
+    w[k] = e0 + k < dim + rot ? T::pack(rotated_q<T>(qh, cs, dim, rot, e0 + k)) : (uint16_t)0;
+  return u32x4{w[0] | (w[1] << 16), w[2] | (w[3] << 16), w[4] | (w[5] << 16), w[6] | (w[7] << 16)};
+}
+
 // first and last visible slot of token tok (of batch row b)
 __device__ __forceinline__ void visible(const LatentParams& p, int tok, int b, long& lo, long& hi) {
   hi = p.cache_position[tok - b * p.t];
@@ -461,41 +486,28 @@ __global__ void __launch_bounds__(256) latent_output_kernel(const LatentParams p
 }
 
 // ---------------------------------------------------------------------------------------
-// prefill: grid (heads, tiles of 128 queries, longest first) of one batch row; four waves of 32 queries, two
+// prefill: grid (heads, tiles of 32 NW queries, longest first) of one batch row; NW waves of 32 queries, two or more
 // workgroups per CU. LDS holds two stages of 64 keys and one of their values: while block s is multiplied with
 // the queries, its values and the keys of block s + 1 are on their way (LDS-direct loads, no registers).
 // ---------------------------------------------------------------------------------------
-template <typename T, int DKC, int DVT>
-__global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(const LatentParams p) {
-  static_assert(DKC % 2 == 0 && DVT % 4 == 0, "tiles of 64 columns");
-  constexpr int QT = 128, KG = DKC / 2, VG = DVT / 4;  // queries per workgroup, blocks of 64 columns
-  constexpr int KSTAGE = KG * 64 * 64, VSTAGE = VG * 64 * 64;
-  uint16_t* smem = (uint16_t*)la_smem;  // first the queries, [KG][QT][64], then K, K', V
+template <int DKC, int DVT, int NW>
+constexpr size_t latent_prefill_lds() {  // K stage, then (the queries, before the loop | second K stage, V)
+  constexpr size_t k = (size_t)64 * DKC * 32 * 2, v = (size_t)64 * DVT * 16 * 2, q = (size_t)32 * NW * DKC * 32 * 2;
+  return k + (q > k + v ? q : k + v);
+}
+template <typename T, int DKC, int DVT, int NW>
+__global__ void __launch_bounds__(64 * NW, DKC > 6 ? 1 : 2) latent_prefill_kernel(const LatentParams p) {
+  static_assert(DKC % 2 == 0 && DVT % 4 == 0 && (NW == 2 || NW == 4), "tiles of 64 columns");
+  constexpr int QT = 32 * NW, KG = DKC / 2, VG = DVT / 4;  // queries per workgroup, blocks of 64 columns
+  constexpr int RB = 8 / NW, RSTEP = 8 * NW;               // blocks of eight rows per wave, rows between them
+  constexpr int KSTAGE = KG * 64 * 64;
+  uint16_t* smem = (uint16_t*)la_smem;
   uint16_t* vl = smem + 2 * KSTAGE;
+  uint16_t* ql = smem + KSTAGE;  // [KG][QT][64], until the loop starts
   const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), g = lane >> 4, i16 = lane & 15;
   const int h = blockIdx.x, qt0 = ((int)gridDim.y - 1 - (int)blockIdx.y) * QT;
   const int hd = p.dim + p.rot, dk = hd;
   const long first_row = p.row_start ? p.row_start[p.b0] : 0;
-  // queries: rotated, rounded, through LDS into operand registers (column i16, k-chunk g)
-  for (int c = t; c < QT * DKC * 4; c += 256) {
-    const int r = c / (DKC * 4), e0 = (c - r * DKC * 4) * 8;
-    uint16_t v[8];
-    const int tq = qt0 + r;
-    const long tok = (long)p.b0 * p.t + (tq < p.t ? tq : p.t - 1);
-    const uint16_t* qh = (const uint16_t*)p.q + (tok * p.heads + h) * hd;
-#pragma unroll
-    for (int j = 0; j < 8; ++j)
-      v[j] = e0 + j < dk ? T::pack(rotated_q<T>(qh, p.cos_sin + tok * p.rot, p.dim, p.rot, e0 + j)) : (uint16_t)0;
-    *(u32x4*)&smem[tile_at<QT>(r, e0)] = u32x4{(uint32_t)v[0] | ((uint32_t)v[1] << 16), (uint32_t)v[2] | ((uint32_t)v[3] << 16),
-                                               (uint32_t)v[4] | ((uint32_t)v[5] << 16), (uint32_t)v[6] | ((uint32_t)v[7] << 16)};
-  }
-  __syncthreads();
-  u32x4 q[2][DKC];
-#pragma unroll
-  for (int qt = 0; qt < 2; ++qt)
-#pragma unroll
-    for (int c = 0; c < DKC; ++c) q[qt][c] = *(const u32x4*)&smem[tile_at<QT>(wave * 32 + qt * 16 + i16, c * 32 + 8 * g)];
-  __syncthreads();
   f32x4 acc[2][DVT];
   float m[2] = {-1e30f, -1e30f}, l[2] = {0.f, 0.f};
 #pragma unroll
@@ -515,24 +527,24 @@ __global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(co
   const uint16_t* rc = (const uint16_t*)p.r_cache + p.b0 * p.r_batch + lo * p.rot;
   const int n_keys = hi >= lo ? (int)(hi - lo + 1) : 0;
   const bool vec = p.dim % 8 == 0 && p.rot % 8 == 0 && p.vdim % 8 == 0;  // 16-byte chunks stay aligned
-  // Wave w delivers rows 8 w .. and 32 + 8 w .. of a block (their swizzles agree). Rows past the last key
+  // Wave w delivers rows 8 w .., 8 (w + NW) .., ... of a block (their swizzles agree). Rows past the last key
   // repeat it (masked), columns past a key's end repeat its start (the queries hold zeros there), columns
   // past a value's end are never stored.
   const int lrow = wave * 8 + (lane >> 3), lc = ((lane & 7) ^ tile_swz(lrow)) * 8;
   auto load_k = [&](int s0, uint16_t* dst) {
     if (vec) {
 #pragma unroll
-      for (int u = 0; u < 2; ++u) {
-        const long row = s0 + lrow + 32 * u < n_keys ? s0 + lrow + 32 * u : n_keys - 1;
+      for (int u = 0; u < RB; ++u) {
+        const long row = s0 + lrow + RSTEP * u < n_keys ? s0 + lrow + RSTEP * u : n_keys - 1;
 #pragma unroll
         for (int cg = 0; cg < KG; ++cg) {
           const int c = cg * 64 + lc < dk ? cg * 64 + lc : 0;
           load_lds16(c < p.dim ? kbase + row * kvp + c : rc + row * p.rot + (c - p.dim),
-                     &dst[(cg * 64 + wave * 8 + 32 * u) * 64]);
+                     &dst[(cg * 64 + wave * 8 + RSTEP * u) * 64]);
         }
       }
     } else {
-      for (int c = t; c < 64 * DKC * 32; c += 256) {
+      for (int c = t; c < 64 * DKC * 32; c += 64 * NW) {
         const int r = c / (DKC * 32), e = c - r * DKC * 32;
         const long row = s0 + r < n_keys ? s0 + r : n_keys - 1;
         dst[tile_at<64>(r, e)] = e < p.dim ? kbase[row * kvp + e] : (e < dk ? rc[row * p.rot + e - p.dim] : (uint16_t)0);
@@ -542,23 +554,38 @@ __global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(co
   auto load_v = [&](int s0) {
     if (vec) {
 #pragma unroll
-      for (int u = 0; u < 2; ++u) {
-        const long row = s0 + lrow + 32 * u < n_keys ? s0 + lrow + 32 * u : n_keys - 1;
+      for (int u = 0; u < RB; ++u) {
+        const long row = s0 + lrow + RSTEP * u < n_keys ? s0 + lrow + RSTEP * u : n_keys - 1;
 #pragma unroll
         for (int cg = 0; cg < VG; ++cg)
-          load_lds16(vbase + row * kvp + (cg * 64 + lc < p.vdim ? cg * 64 + lc : 0), &vl[(cg * 64 + wave * 8 + 32 * u) * 64]);
+          load_lds16(vbase + row * kvp + (cg * 64 + lc < p.vdim ? cg * 64 + lc : 0), &vl[(cg * 64 + wave * 8 + RSTEP * u) * 64]);
       }
     } else {
-      for (int c = t; c < 64 * DVT * 16; c += 256) {
+      for (int c = t; c < 64 * DVT * 16; c += 64 * NW) {
         const int r = c / (DVT * 16), e = c - r * DVT * 16;
         const long row = s0 + r < n_keys ? s0 + r : n_keys - 1;
         vl[tile_at<64>(r, e)] = e < p.vdim ? vbase[row * kvp + e] : (uint16_t)0;
       }
     }
   };
+  if (n_keys > 0) load_k(0, smem);
+  // queries: rotated, rounded, through LDS into operand registers (column i16, k-chunk g)
+  const bool qvec = p.dim % 8 == 0 && p.rot % 16 == 0;
+#pragma unroll 4
+  for (int c = t; c < QT * DKC * 4; c += 64 * NW) {
+    const int r = c / (DKC * 4), e0 = (c - r * DKC * 4) * 8;
+    const long tok = (long)p.b0 * p.t + (qt0 + r < p.t ? qt0 + r : p.t - 1);
+    *(u32x4*)&ql[tile_at<QT>(r, e0)] =
+        rotated_q8<T>((const uint16_t*)p.q + (tok * p.heads + h) * hd, p.cos_sin + tok * p.rot, p.dim, p.rot, e0, qvec);
+  }
+  __syncthreads();
+  u32x4 q[2][DKC];
+#pragma unroll
+  for (int qt = 0; qt < 2; ++qt)
+#pragma unroll
+    for (int c = 0; c < DKC; ++c) q[qt][c] = *(const u32x4*)&ql[tile_at<QT>(wave * 32 + qt * 16 + i16, c * 32 + 8 * g)];
   // this wave's queries, as positions counted from lo
   const int wq0 = (int)((long)p.q_first + qt0 + wave * 32 - lo), wq1 = wq0 + 31;
-  if (n_keys > 0) load_k(0, smem);
   for (int s0 = 0, buf = 0; s0 < n_keys; s0 += 64, buf ^= 1) {
     const uint16_t* kl = smem + buf * KSTAGE;
     const bool more = s0 + 64 < n_keys;
@@ -634,7 +661,7 @@ __global__ void __launch_bounds__(256, DKC > 6 ? 1 : 2) latent_prefill_kernel(co
       }
     }
     // the values were requested before the next keys
-    if (more) wait_loads<2 * KG>();
+    if (more) wait_loads<RB * KG>();
     else wait_loads<0>();
     __syncthreads();
     if (mine) {
@@ -697,12 +724,19 @@ static int launch_latent_decode(hipStream_t s, const LatentParams& p) {
                          (size_t)p.kv_rank * 4, s, p);
 }
 
+template <typename T, int DKC, int DVT, int NW>
+static int launch_latent_prefill_w(hipStream_t s, const LatentParams& p) {
+  const int tiles = ceil_div(p.t, 32 * NW);
+  if (tiles > 65535) return MUI_ERR_UNSUPPORTED;
+  return launch_with_lds(latent_prefill_kernel<T, DKC, DVT, NW>, dim3(p.heads, tiles), dim3(64 * NW),
+                         latent_prefill_lds<DKC, DVT, NW>(), s, p);
+}
+
 template <typename T, int DKC, int DVT>
 static int launch_latent_prefill_t(hipStream_t s, const LatentParams& p) {
-  constexpr size_t kv = (size_t)(2 * DKC * 32 + DVT * 16) * 64 * 2, q = (size_t)128 * DKC * 32 * 2;
-  const int tiles = ceil_div(p.t, 128);
-  if (tiles > 65535) return MUI_ERR_UNSUPPORTED;
-  return launch_with_lds(latent_prefill_kernel<T, DKC, DVT>, dim3(p.heads, tiles), dim3(256), kv > q ? kv : q, s, p);
+  // short prompts: half as many queries per workgroup, so that there are workgroups for every CU
+  if (p.heads * ceil_div(p.t, 128) <= device_cus()) return launch_latent_prefill_w<T, DKC, DVT, 2>(s, p);
+  return launch_latent_prefill_w<T, DKC, DVT, 4>(s, p);
 }
 
 static bool prefill_covers(int dk, int vdim) { return dk <= 256 && vdim <= 256; }

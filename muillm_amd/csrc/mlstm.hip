@@ -172,17 +172,37 @@ __device__ __forceinline__ void chunk_gates(const MlstmParams& p, int b, int h, 
 constexpr int kPitchRow = 68;  // tiles read [row][k]: 16 rows x 4 consecutive k in 64 different banks
 constexpr int kPitchCol = 80;  // tiles read [k][column]: 4 rows x 16 consecutive columns likewise
 
-// a 64 x 64 tile of a 16-bit or fp32 token-major matrix into LDS, rows past `rows` and columns past `cols` zero
+// a 64 x 64 tile of a 16-bit or fp32 token-major matrix into LDS, rows past `rows` and columns past `cols` zero;
+// four consecutive columns per thread and access where the rows allow it
 template <typename T>
 __device__ __forceinline__ void load_tile(float* dst, int pitch, const typename T::storage* src, long src_pitch, int rows,
                                           int cols, float scale) {
-  for (int c = threadIdx.x; c < 64 * 16; c += 256) {
-    const int r = c >> 4, k = (c & 15) * 4;
-    float v[4];
+  typedef typename T::storage S;
+  const int r0 = threadIdx.x >> 4, k = (threadIdx.x & 15) * 4;
+  f32x4 v[4];
+  if (((uintptr_t)src & (4 * sizeof(S) - 1)) == 0 && (src_pitch & 3) == 0 && (cols >= 64 || (cols & 3) == 0)) {
 #pragma unroll
-    for (int j = 0; j < 4; ++j) v[j] = r < rows && k + j < cols ? T::one(src[(long)r * src_pitch + k + j]) * scale : 0.f;
-    *(f32x4*)&dst[r * pitch + k] = f32x4{v[0], v[1], v[2], v[3]};
+    for (int i = 0; i < 4; ++i) {  // (clamped, not branched around)
+      const bool live = r0 + 16 * i < rows && k < cols;
+      const S* at = src + (live ? (long)(r0 + 16 * i) * src_pitch + k : 0);
+      if constexpr (T::kDtype == MUI_DTYPE_F32) {
+        v[i] = __builtin_bit_cast(f32x4, ld16(at));
+      } else {
+        const u32x2 w = ld8(at);
+        v[i] = f32x4{T::lo(w.x), T::hi(w.x), T::lo(w.y), T::hi(w.y)};
+      }
+#pragma unroll
+      for (int j = 0; j < 4; ++j) v[i][j] = live ? v[i][j] * scale : 0.f;
+    }
+  } else {
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        v[i][j] = r0 + 16 * i < rows && k + j < cols ? T::one(src[(long)(r0 + 16 * i) * src_pitch + k + j]) * scale : 0.f;
   }
+#pragma unroll
+  for (int i = 0; i < 4; ++i) *(f32x4*)&dst[(r0 + 16 * i) * pitch + k] = v[i];
 }
 
 __device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) {

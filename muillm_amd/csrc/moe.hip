@@ -844,11 +844,11 @@ extern "C" int mui_linear_f32(mui_stream_t stream, int dtype, const void* weight
 extern "C" int mui_moe_tile_pairs(int dtype, int tokens, int top, int n_experts, int width, int ff) {
   if (dtype == MUI_DTYPE_F32 || width % 8 || ff % 8 || n_experts < 1) return 0;
   // 16-pair tiles stream an expert's weights once per tile; from about a dozen pairs per expert on a wide tile
-  // is cheaper even half empty. Of the two widths the one whose tiles cost less (a 256-pair tile about one
-  // and a half times as much as a 128-pair one).
+  // is cheaper even half empty. Of the two widths the one whose tiles cost less (a 256-pair tile, rarely full,
+  // about 1.3 times as much as a 128-pair one).
   const long per = (long)tokens * top / n_experts;
   if (per < 12) return 16;
-  return 15 * ((per + 255) / 256) < 10 * ((per + 127) / 128) ? 256 : 128;
+  return 13 * ((per + 255) / 256) < 10 * ((per + 127) / 128) ? 256 : 128;
 }
 
 extern "C" int mui_moe_max_tiles(int tokens, int top, int n_experts, int tile_pairs) {
