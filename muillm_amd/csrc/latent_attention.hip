@@ -309,31 +309,32 @@ __device__ __forceinline__ int tile_at(int row, int col) {  // in elements
   return ((col >> 6) * ROWS + row) * 64 + ((((col >> 3) & 7) ^ tile_swz(row)) << 3) + (col & 7);
 }
 
-// Grid (splits, head groups of 16, tokens); eight waves, 128 keys per block, all of a block's rows requested at
-// once.
-//   scores: wave w takes keys 16 w ..: A = key rows, B = the 16 heads' queries (registers); lane (g, i) ends up
-//           with head i, keys 16 w + 4 g + r
+// Splits of token tok that hold visible keys: the grid covers the largest span, the rest leave at once
+__device__ __forceinline__ int live_splits(const LatentParams& p, long lo, long hi) {
+  return hi < lo ? 0 : (int)((hi - lo) / p.split_keys) + 1;
+}
+
+// Grid (splits, groups of 16 HT heads, tokens); eight waves, 64 keys per block; the queries and all of a block's
+// rows are requested at once.
+//   scores: wave w takes keys 16 (w % 4) .. and head tile w / 4: A = key rows, B = the 16 heads' queries; lane
+//           (g, i) ends up with head i, keys 16 (w % 4) + 4 g + r
 //   values: O^T[rank, head] += C^T P^T, the latent rows read back transposed; wave w owns the rank
-//           tiles w, w + 8, ...; contraction slots of lane group g: keys 4 g + r and 16 + 4 g + r of 32
-constexpr int kDecKeys = 128;
-constexpr int kMaxDecodeWidth = 576;  // kv_rank + rot, rounded up to 64: 128 rows of it fit into LDS
-template <typename T, int NT>  // kv_rank <= 128 NT
-__global__ void __launch_bounds__(512) latent_decode_kernel(const LatentParams p) {
-  constexpr int KC = 4 * NT + 2;  // query chunks of 32 (kv_rank + rot <= 128 NT + 64)
-  __shared__ float mred[8][16], lred[8][16];
-  __shared__ __align__(16) uint16_t pl[16][kDecKeys + 8];
-  uint16_t* cl = (uint16_t*)la_smem;  // [kp / 64][128][64]
+//           tiles w, w + 8, ... of all head tiles; contraction slots of lane group g: keys 4 g + r and
+//           16 + 4 g + r of 32
+constexpr int kDecKeys = 64, kDecThreads = 512;
+constexpr int kMaxDecodeWidth = 576;  // kv_rank + rot, rounded up to 64
+template <typename T, int NT, int HT>  // kv_rank <= 128 NT
+__global__ void __launch_bounds__(kDecThreads) latent_decode_kernel(const LatentParams p) {
+  constexpr int KG = 2 * NT + 1, HEADS = 16 * HT;  // blocks of 64 columns (kv_rank + rot <= 128 NT + 64)
+  __shared__ float mred[4][HEADS], lred[4][HEADS];
+  __shared__ __align__(16) uint16_t pl[HEADS][kDecKeys + 8];
+  uint16_t* cl = (uint16_t*)la_smem;    // [kp / 64][64 keys][64]
+  uint16_t* ql = cl + kDecKeys * p.kp;  // [kp / 64][HEADS][64]
   const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), g = lane >> 4, i16 = lane & 15;
-  const int split = blockIdx.x, h0 = blockIdx.y * 16, tok = blockIdx.z, b = tok / p.t;
-  u32x4 q[KC];
-  {
-    const int hh = h0 + i16 < p.heads ? h0 + i16 : p.heads - 1;
-    const uint16_t* src = (const uint16_t*)p.q_abs + ((long)tok * p.heads + hh) * p.kp + 8 * g;
-#pragma unroll
-    for (int c = 0; c < KC; ++c) q[c] = ld16(src + (c * 32 < p.kp ? c * 32 : 0));
-  }
+  const int split = blockIdx.x, h0 = blockIdx.y * HEADS, tok = blockIdx.z, b = tok / p.t;
   long lo, hi;
   visible(p, tok, b, lo, hi);
+  if (split >= live_splits(p, lo, hi)) return;  // uniform for the workgroup
   const long s_begin = lo + (long)split * p.split_keys;
   long s_end = s_begin + p.split_keys;  // exclusive
   s_end = s_end < hi + 1 ? s_end : hi + 1;
@@ -341,33 +342,51 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(const LatentParams p
   const uint16_t* rc = (const uint16_t*)p.r_cache + b * p.r_batch;
   const bool rot8 = p.rot % 8 == 0;
   const int lrow = lane >> 3;
+  {  // the heads' queries: eight rows per instruction, the instructions dealt out to the waves
+    constexpr int QB = HEADS / 8;
+    const int qb = wave % QB, row = qb * 8 + lrow, hh = h0 + row < p.heads ? h0 + row : p.heads - 1;
+    const uint16_t* src = (const uint16_t*)p.q_abs + ((long)tok * p.heads + hh) * p.kp + ((lane & 7) ^ tile_swz(row)) * 8;
+    for (int cb = wave / QB; cb * 64 < p.kp; cb += 8 / QB) load_lds16(src + cb * 64, &ql[(cb * HEADS + qb * 8) * 64]);
+  }
   const int width = p.kv_rank + (rot8 ? p.rot : 0);  // columns that are loaded
-  f32x4 acc[NT];
+  f32x4 acc[NT][HT];
+  float m[HT], l[HT];
 #pragma unroll
-  for (int j = 0; j < NT; ++j) acc[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-  float m = -1e30f, l = 0.f;
+  for (int h = 0; h < HT; ++h) {
+    m[h] = -1e30f;
+    l[h] = 0.f;
+#pragma unroll
+    for (int j = 0; j < NT; ++j) acc[j][h] = f32x4{0.f, 0.f, 0.f, 0.f};
+  }
   const float sc = p.scale * 1.4426950408889634f;
+  const int kt = wave & 3, ht = wave >> 2;  // key tile and head tile of this wave's scores
+  // operand addresses: only the block of columns and multiples of 16 rows change, by constants
+  const int krow = 16 * kt + i16, kswz = tile_swz(krow);
+  const uint16_t *ka = cl + krow * 64 + ((g ^ kswz) << 3), *kb = cl + krow * 64 + (((4 + g) ^ kswz) << 3);
+  const int qrow = 16 * (ht < HT ? ht : 0) + i16, qswz = tile_swz(qrow);
+  const uint16_t *qa = ql + qrow * 64 + ((g ^ qswz) << 3), *qb = ql + qrow * 64 + (((4 + g) ^ qswz) << 3);
+  const int vrow = 4 * g + (i16 >> 2);
+  const uint16_t* va = cl + ((wave >> 2) * kDecKeys + vrow) * 64 + (((2 * (wave & 3) + ((i16 & 3) >> 1)) ^ tile_swz(vrow)) << 3) + 4 * (i16 & 1);
   for (long s0 = s_begin; s0 < s_end; s0 += kDecKeys) {
     __syncthreads();  // the previous block is done with
-    // wave w delivers rows 8 w .. and 64 + 8 w ..; rows past the split repeat its last one (their scores
-    // are masked), columns past the rows' end repeat their start (the queries hold zeros there)
-#pragma unroll
-    for (int u = 0; u < 2; ++u) {
-      const int row = (wave + 8 * u) * 8 + lrow;
+    // wave w delivers rows 8 w ..; rows past the split repeat its last one (their scores are masked), columns
+    // past the rows' end repeat their start (the queries hold zeros there)
+    {
+      const int row = wave * 8 + lrow;
       const long s = s0 + row < s_end ? s0 + row : s_end - 1;
       const uint16_t *crow = cc + s * p.kv_rank, *rrow = rc + s * p.rot - p.kv_rank;
       const int lc = ((lane & 7) ^ tile_swz(row)) * 8;
 #pragma unroll
-      for (int cb = 0; cb < KC / 2; ++cb) {
+      for (int cb = 0; cb < KG; ++cb) {
         if (cb * 64 >= p.kp) break;
         const int c = cb * 64 + lc < width ? cb * 64 + lc : 0;
-        load_lds16((c < p.kv_rank ? crow : rrow) + c, &cl[(cb * kDecKeys + (wave + 8 * u) * 8) * 64]);
+        load_lds16((c < p.kv_rank ? crow : rrow) + c, &cl[(cb * kDecKeys + wave * 8) * 64]);
       }
     }
     wait_loads<0>();
     if (!rot8) {  // the rotated part element by element
       __syncthreads();
-      for (int c = t; c < kDecKeys * p.rot; c += 512) {
+      for (int c = t; c < kDecKeys * p.rot; c += kDecThreads) {
         const int r = c / p.rot, e = c - r * p.rot;
         const long s = s0 + r < s_end ? s0 + r : s_end - 1;
         cl[tile_at<kDecKeys>(r, p.kv_rank + e)] = rc[s * p.rot + e];
@@ -375,70 +394,86 @@ __global__ void __launch_bounds__(512) latent_decode_kernel(const LatentParams p
     }
     __syncthreads();
     f32x4 s4 = {0.f, 0.f, 0.f, 0.f}, s5 = {0.f, 0.f, 0.f, 0.f};
+    if (ht < HT) {
 #pragma unroll
-    for (int c = 0; c < KC; c += 2) {
-      if (c * 32 < p.kp) {  // (kp is a multiple of 64)
-        s4 = mfma16x16x32<T>(*(const u32x4*)&cl[tile_at<kDecKeys>(16 * wave + i16, c * 32 + 8 * g)], q[c], s4);
-        s5 = mfma16x16x32<T>(*(const u32x4*)&cl[tile_at<kDecKeys>(16 * wave + i16, c * 32 + 32 + 8 * g)], q[c + 1], s5);
+      for (int cb = 0; cb < KG; ++cb) {
+        if (cb * 64 < p.kp) {
+          s4 = mfma16x16x32<T>(*(const u32x4*)(ka + cb * kDecKeys * 64), *(const u32x4*)(qa + cb * HEADS * 64), s4);
+          s5 = mfma16x16x32<T>(*(const u32x4*)(kb + cb * kDecKeys * 64), *(const u32x4*)(qb + cb * HEADS * 64), s5);
+        }
       }
+      float mx = -INFINITY;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        s4[r] = s0 + 16 * kt + 4 * g + r < s_end ? (s4[r] + s5[r]) * sc : -INFINITY;
+        mx = fmaxf(mx, s4[r]);
+      }
+      mx = fmaxf(mx, __shfl_xor(mx, 16));
+      mx = fmaxf(mx, __shfl_xor(mx, 32));
+      if (g == 0) mred[kt][16 * ht + i16] = mx;
     }
-    float mx = -INFINITY;
+    __syncthreads();
+    float keep[HT];
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      s4[r] = s0 + 16 * wave + 4 * g + r < s_end ? (s4[r] + s5[r]) * sc : -INFINITY;
-      mx = fmaxf(mx, s4[r]);
+    for (int h = 0; h < HT; ++h) {
+      float mn = m[h];
+#pragma unroll
+      for (int w = 0; w < 4; ++w) mn = fmaxf(mn, mred[w][16 * h + i16]);
+      keep[h] = exp2f(m[h] - mn);
+      m[h] = mn;
     }
-    mx = fmaxf(mx, __shfl_xor(mx, 16));
-    mx = fmaxf(mx, __shfl_xor(mx, 32));
-    if (g == 0) mred[wave][i16] = mx;
+    if (ht < HT) {
+      const float mn = HT == 2 && ht ? m[HT - 1] : m[0];
+      float e[4], sum = 0.f;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) { e[r] = exp2f(s4[r] - mn); sum += e[r]; }
+      *(u32x2*)&pl[16 * ht + i16][16 * kt + 4 * g] = u32x2{T::pack2(e[0], e[1]), T::pack2(e[2], e[3])};
+      sum += __shfl_xor(sum, 16);
+      sum += __shfl_xor(sum, 32);
+      if (g == 0) lred[kt][16 * ht + i16] = sum;
+    }
     __syncthreads();
-    float mn = m;
 #pragma unroll
-    for (int w = 0; w < 8; ++w) mn = fmaxf(mn, mred[w][i16]);
-    const float keep = exp2f(m - mn);
-    m = mn;
-    float e[4], sum = 0.f;
+    for (int h = 0; h < HT; ++h) {
+      l[h] = l[h] * keep[h] + ((lred[0][16 * h + i16] + lred[1][16 * h + i16]) + (lred[2][16 * h + i16] + lred[3][16 * h + i16]));
 #pragma unroll
-    for (int r = 0; r < 4; ++r) { e[r] = exp2f(s4[r] - mn); sum += e[r]; }
-    *(u32x2*)&pl[i16][16 * wave + 4 * g] = u32x2{T::pack2(e[0], e[1]), T::pack2(e[2], e[3])};
-    sum += __shfl_xor(sum, 16);
-    sum += __shfl_xor(sum, 32);
-    if (g == 0) lred[wave][i16] = sum;
-    __syncthreads();
-    sum = 0.f;
+      for (int j = 0; j < NT; ++j)
 #pragma unroll
-    for (int w = 0; w < 8; ++w) sum += lred[w][i16];
-    l = l * keep + sum;
-#pragma unroll
-    for (int j = 0; j < NT; ++j)
-#pragma unroll
-      for (int r = 0; r < 4; ++r) acc[j][r] *= keep;
+        for (int r = 0; r < 4; ++r) acc[j][h][r] *= keep[h];
+    }
 #pragma unroll
     for (int kk = 0; kk < kDecKeys / 32; ++kk) {
-      const u32x2 plo = *(const u32x2*)&pl[i16][32 * kk + 4 * g], phi = *(const u32x2*)&pl[i16][32 * kk + 16 + 4 * g];
-      const u32x4 pb = {plo.x, plo.y, phi.x, phi.y};
+      u32x4 pb[HT];
+#pragma unroll
+      for (int h = 0; h < HT; ++h) {
+        const u32x2 plo = *(const u32x2*)&pl[16 * h + i16][32 * kk + 4 * g], phi = *(const u32x2*)&pl[16 * h + i16][32 * kk + 16 + 4 * g];
+        pb[h] = u32x4{plo.x, plo.y, phi.x, phi.y};
+      }
 #pragma unroll
       for (int j = 0; j < NT; ++j) {
-        const int col = 16 * (wave + 8 * j);
-        if (col < p.kv_rank) {  // uniform; a last tile may reach into the rotated part: never stored
-          const int row = 32 * kk + 4 * g + (i16 >> 2);
-          const u32x2 a0 = lds_read_tr16(&cl[tile_at<kDecKeys>(row, col + 4 * (i16 & 3))]);
-          const u32x2 a1 = lds_read_tr16(&cl[tile_at<kDecKeys>(row + 16, col + 4 * (i16 & 3))]);
-          acc[j] = mfma16x16x32<T>(u32x4{a0.x, a0.y, a1.x, a1.y}, pb, acc[j]);
+        if (16 * (wave + 8 * j) < p.kv_rank) {  // uniform; a last tile may reach into the rotated part: never stored
+          const u32x2 a0 = lds_read_tr16(va + (2 * j * kDecKeys + 32 * kk) * 64);
+          const u32x2 a1 = lds_read_tr16(va + (2 * j * kDecKeys + 32 * kk + 16) * 64);
+          const u32x4 a = {a0.x, a0.y, a1.x, a1.y};
+#pragma unroll
+          for (int h = 0; h < HT; ++h) acc[j][h] = mfma16x16x32<T>(a, pb[h], acc[j][h]);
         }
       }
     }
   }
-  if (h0 + i16 < p.heads) {
-    const long at = ((long)tok * p.heads + h0 + i16) * p.splits + split;
+#pragma unroll
+  for (int h = 0; h < HT; ++h) {
+    const int hh = h0 + 16 * h + i16;
+    if (hh >= p.heads) continue;
+    const long at = ((long)tok * p.heads + hh) * p.splits + split;
 #pragma unroll
     for (int j = 0; j < NT; ++j) {
       const int c = 16 * (wave + 8 * j) + 4 * g;  // (kv_rank is a multiple of 8)
-      if (c < p.kv_rank) *(f32x4*)&p.part[at * p.kv_rank + c] = acc[j];
+      if (c < p.kv_rank) *(f32x4*)&p.part[at * p.kv_rank + c] = acc[j][h];
     }
     if (wave == 0 && g == 0) {
-      p.part_ml[at * 2] = m;
-      p.part_ml[at * 2 + 1] = l;
+      p.part_ml[at * 2] = m[h];
+      p.part_ml[at * 2 + 1] = l[h];
     }
   }
 }
@@ -453,18 +488,26 @@ __global__ void __launch_bounds__(256) latent_output_kernel(const LatentParams p
   const int h = blockIdx.x, tok = blockIdx.z, t = threadIdx.x;
   const long at = ((long)tok * p.heads + h) * p.splits;
   const float* part = p.part + at * p.kv_rank;
+  long lo, hi;
+  visible(p, tok, tok / p.t, lo, hi);
+  const int live = live_splits(p, lo, hi);
   if (t < kWave) {  // the splits' shares, one per lane
-    const bool in = t < p.splits;
+    const bool in = t < live;
     const float mm = in ? p.part_ml[(at + t) * 2] : -1e30f, ll = in ? p.part_ml[(at + t) * 2 + 1] : 0.f;
     const float e = exp2f(mm - wave_max(mm));
-    const float l = wave_sum(e * ll);
-    if (in) ws[t] = ll > 0.f ? e / l : 0.f;
+    ws[t] = in ? e / wave_sum(e * ll) : 0.f;
   }
   __syncthreads();
+  // splits past the live ones repeat the last one with a share of zero: sixteen loads in flight
   for (int r = t; r < p.kv_rank; r += 256) {
     float a = 0.f;
-#pragma unroll 8
-    for (int s = 0; s < p.splits; ++s) a = fmaf(ws[s], part[(long)s * p.kv_rank + r], a);
+    for (int s0 = 0; s0 < live; s0 += 16) {
+      float v[16];
+#pragma unroll
+      for (int u = 0; u < 16; ++u) v[u] = part[(long)(s0 + u < live ? s0 + u : live - 1) * p.kv_rank + r];
+#pragma unroll
+      for (int u = 0; u < 16; ++u) a = fmaf(ws[s0 + u], v[u], a);
+    }
     o[r] = a;
   }
   __syncthreads();
@@ -707,18 +750,22 @@ static int launch_latent_plain(hipStream_t s, const LatentParams& p) {
   return launch_with_lds(latent_plain_kernel<T>, dim3(p.heads, p.batch * p.t), dim3(256), lds, s, p);
 }
 
+template <typename T, int HT>
+static int launch_latent_decode_h(hipStream_t s, const LatentParams& p) {
+  const dim3 grid(p.splits, ceil_div(p.heads, 16 * HT), p.batch * p.t), block(kDecThreads);
+  const size_t lds = (size_t)(kDecKeys + 16 * HT) * p.kp * 2;
+  if (p.kp <= 192 && p.kv_rank <= 128) return launch_with_lds(latent_decode_kernel<T, 1, HT>, grid, block, lds, s, p);
+  if (p.kp <= 320 && p.kv_rank <= 256) return launch_with_lds(latent_decode_kernel<T, 2, HT>, grid, block, lds, s, p);
+  return launch_with_lds(latent_decode_kernel<T, 4, HT>, grid, block, lds, s, p);
+}
+
 template <typename T>
 static int launch_latent_decode(hipStream_t s, const LatentParams& p) {
   const int tokens = p.batch * p.t;
   if (tokens > 65535 || p.kp > kMaxDecodeWidth) return MUI_ERR_UNSUPPORTED;
   hipLaunchKernelGGL((latent_absorb_kernel<T>), dim3(p.heads, ceil_div(p.kv_rank, 64), ceil_div(tokens, kAbsTok)),
                      dim3(256), 0, s, p);
-  const dim3 grid(p.splits, ceil_div(p.heads, 16), tokens);
-  const size_t lds = (size_t)kDecKeys * p.kp * 2;
-  int st;
-  if (p.kp <= 192 && p.kv_rank <= 128) st = launch_with_lds(latent_decode_kernel<T, 1>, grid, dim3(512), lds, s, p);
-  else if (p.kp <= 320 && p.kv_rank <= 256) st = launch_with_lds(latent_decode_kernel<T, 2>, grid, dim3(512), lds, s, p);
-  else st = launch_with_lds(latent_decode_kernel<T, 4>, grid, dim3(512), lds, s, p);
+  const int st = p.heads > 16 ? launch_latent_decode_h<T, 2>(s, p) : launch_latent_decode_h<T, 1>(s, p);
   if (st != MUI_OK) return st;
   return launch_with_lds(latent_output_kernel<T>, dim3(p.heads, ceil_div(p.vdim, 32), tokens), dim3(256),
                          (size_t)p.kv_rank * 4, s, p);
@@ -783,7 +830,7 @@ static int latent_kp(int kv_rank, int rot_dim) { return (kv_rank + rot_dim + 63)
 
 // keys per split and number of splits of the decode kernel for spans of up to `span` keys
 static void latent_split(int batch, int t, int heads, int span, int* splits, int* split_keys) {
-  const int groups = batch * t * ceil_div(heads, 16);
+  const int groups = batch * t * ceil_div(heads, heads > 16 ? 32 : 16);
   int want = device_cus() * 2 / (groups > 0 ? groups : 1);
   want = want < 1 ? 1 : (want > kMaxSplits ? kMaxSplits : want);
   const int blocks = ceil_div(span, kDecKeys);
