@@ -18,6 +18,9 @@ the dominant kernel (the fused gate/up GEMV: half of all bytes streamed per toke
 live with HIP events over cold (distinct) weight buffers, a `cpu_baseline` object (the
 reference's PyTorch fallback path in fp16 on this box's host cores, bounded sample), and a
 `kernels` table (GB/s per fused kernel family, informational).
+
+`--salepel` times the Salepel decoder (latent attention, matrix memory, mixture of experts) beside a
+Llama-shaped model of equal width and active MLP size instead, and prints one JSON line of its own.
 """
 
 import argparse

@@ -15,7 +15,7 @@ _HI = torch.float64
 
 
 def rms(x: torch.Tensor, eps: float) -> torch.Tensor:
-    """Last dimension divided by its root mean square (eps inside the root)."""
+    """x scaled to unit RMS over the last dimension; eps is added to the mean square."""
     x = x.to(_HI)
     return x / torch.sqrt((x * x).mean(-1, keepdim=True) + eps)
 
