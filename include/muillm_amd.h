@@ -30,7 +30,7 @@ extern "C" {
 
 /* bumped whenever a struct below changes layout or an entry point changes its arguments;
  * mui_abi_version() returns the value the library was built with */
-#define MUI_ABI_VERSION 3
+#define MUI_ABI_VERSION 4
 
 /* status codes (reference: TORCH_CHECK exceptions, csrc/linear/linear.cu:72-74;
  * muillm_error_t, csrc/base.h:4-7) */
@@ -132,6 +132,11 @@ int mui_rmsnorm(mui_stream_t stream, int dtype, const void* weights, const void*
 int mui_gateup_silu(mui_stream_t stream, int dtype, const void* gate, const void* up,
                     long gu_pitch, const void* x, const void* norm_weights, float epsilon,
                     void* h, int n_inter, int k_in, int tokens);
+
+/* The same with biases on the two products, silu(G xn + gate_bias) * (U xn + up_bias), both [n_inter] or both NULL. */
+int mui_gateup_silu_bias(mui_stream_t stream, int dtype, const void* gate, const void* up, long gu_pitch,
+                         const void* x, const void* norm_weights, float epsilon, const void* gate_bias,
+                         const void* up_bias, void* h, int n_inter, int k_in, int tokens);
 
 /* Activation step of the unfused MLP route for prompts longer than MUI_MAX_TOKENS tokens
  * (muillm/modules/gateupdownmlp.py:343-359: two matmuls, SiLU, multiply): with the gate and up
@@ -518,27 +523,27 @@ int mui_embedding(mui_stream_t stream, int dtype, const void* table, long row_pi
                   const void* ids, int ids_are_int32, void* out, int n_tokens, int dim, int vocab);
 
 /* ------------------------------------------------------------------------------------
- * Decoders with an fp32 residual stream and a norm on both sides of every sublayer, latent
- * attention, recurrent (matrix-memory) layers and mixtures of experts. No counterpart in the
- * reference. Every entry point of this section also takes MUI_DTYPE_F32: activations and weights are
+ * Decoders with an fp32 residual stream and norms around every sublayer, latent attention or
+ * grouped-query attention with sinks, recurrent layers (matrix memory, delta rule) and mixtures of
+ * experts. No counterpart in the reference. Every entry point of this section also takes MUI_DTYPE_F32: activations and weights are
  * then fp32 ("activations' type" below is the type `dtype` names).
  * ---------------------------------------------------------------------------------- */
 
-/* Between two sublayers, per row of k elements:
- *   x = residual_in + (post_gain ? post_gain * y * rsqrt(mean((y_scale y)^2) + epsilon) * y_scale : y_scale * y)
- *   residual_out = x;   h = next_gain * x * rsqrt(mean(x^2) + epsilon)
+/* Between two sublayers, per row of k elements, with y' = y_scale y:
+ *   x = residual_in + (post_gain ? branch_scale * post_gain * y' * rsqrt(mean(y'^2) + epsilon) : y')
+ *   residual_out = x;   h = next_scale * (next_gain ? next_gain * x * rsqrt(mean(x^2) + epsilon) : x)
  * residual_in (NULL: 0) and residual_out (may be residual_in) are fp32 [rows, k]; y, the gains and h are
- * in the activations' type; next_gain and h are both NULL or both given. Any k. */
+ * in the activations' type; h may be NULL where next_gain is. Any k. */
 int mui_residual_norm(mui_stream_t stream, int dtype, const float* residual_in, const void* y, float y_scale,
-                      const void* post_gain, const void* next_gain, float epsilon, float* residual_out,
-                      void* h, int rows, int k);
+                      const void* post_gain, float branch_scale, const void* next_gain, float next_scale,
+                      float epsilon, float* residual_out, void* h, int rows, int k);
 
 /* The same with y[r] = sum_j weight[r, j] * (expert[r, j] < n_experts ? pair_out[r * top + j] : identity_in[r]):
  * the end of a mixture of experts (mui_moe_down's output, the block's own input for identity experts). */
 int mui_moe_residual_norm(mui_stream_t stream, int dtype, const float* residual_in, const void* pair_out,
                           const void* identity_in, const int32_t* expert, const float* weight, int n_experts,
-                          int top, const void* post_gain, const void* next_gain, float epsilon,
-                          float* residual_out, void* h, int rows, int k);
+                          int top, const void* post_gain, float branch_scale, const void* next_gain,
+                          float next_scale, float epsilon, float* residual_out, void* h, int rows, int k);
 
 /* y[t, n] = W[n, :] . x[t, :] + bias[n] with fp32 outputs: router logits, recurrence gates. W [n_out, k_in],
  * x [tokens, k_in] and bias [n_out] (may be NULL) in the activations' type. Any sizes. */
@@ -634,6 +639,74 @@ int mui_mlstm(mui_stream_t stream, int dtype, const void* q, const void* k, cons
 /* y[tok, h, :] = o[tok, h, :] * rsqrt(mean over the head + epsilon) * gain[h, :] * sigmoid(gate[tok, h, :]) */
 int mui_mlstm_output(mui_stream_t stream, int dtype, const float* o, const void* gain, const void* gate,
                      long gate_pitch, float epsilon, void* y, int tokens, int heads, int dv);
+
+/* x[tok, :] = scale * table[id, :] + bigram[(previous id * mul_prev + id * mul_cur) mod buckets, :], row number
+ * `buckets` (the last) for the first token of a sequence (cache_position[t] <= row_start[b], NULL: 0). ids
+ * [batch, t] are clamped to [0, vocab); the id in front of a row's first token is prev[b], which becomes the
+ * row's last id. x fp32, h the same rounded to the activations' type, [batch * t, width]. */
+int mui_bigram_embedding(mui_stream_t stream, int dtype, const int64_t* ids, int64_t* prev,
+                         const int64_t* cache_position, const int64_t* row_start, const void* table,
+                         const void* bigram, float scale, long mul_prev, long mul_cur, int buckets, float* x,
+                         void* h, int batch, int t, int width, int vocab);
+
+/* Grouped-query attention over cached rows, in front of the scores: per token, from a projection's output row
+ * (q at 0, k and v at their offsets, rows `pitch` elements apart)
+ *   q_out = rotate(q_gain * rmsnorm(q)), the norm over all heads * dim values at once; k likewise into
+ *   k_cache[b, slot], v as it is into v_cache[b, slot]
+ * A gain that is NULL skips its norm. rotate: the first rot_dims dimensions of every head, pairs (2 i, 2 i + 1),
+ * angle (slot - row_start[b]) * inv_freq[i]. slot = cache_position[t]; slots outside [0, max_cache_len) are
+ * skipped. Caches [batch, max_cache_len, kv_heads * dim | kv_heads * vdim]. */
+int mui_hybrid_prepare(mui_stream_t stream, int dtype, const void* proj, long pitch, long k_offset, long v_offset,
+                       const void* q_gain, const void* k_gain, float epsilon, const double* inv_freq, int rot_dims,
+                       const int64_t* cache_position, const int64_t* row_start, void* q_out, void* k_cache,
+                       long k_batch_stride, void* v_cache, long v_batch_stride, int batch, int t, int heads,
+                       int kv_heads, int dim, int vdim, int max_cache_len);
+
+/* Which kernels serve a call of `tokens` per batch row: PLAIN (fp32, sizes that are no multiple of 8 or above 256),
+ * DECODE, PREFILL. */
+#define MUI_HYBRID_PLAIN 0
+#define MUI_HYBRID_DECODE 1
+#define MUI_HYBRID_PREFILL 2
+int mui_hybrid_attention_route(int dtype, int tokens, int dim, int vdim);
+size_t mui_hybrid_decode_scratch_bytes(int batch, int t, int heads, int kv_heads, int vdim, int span);
+
+/* out[tok, h, :] = sigmoid(gate[tok, h, :]) * sum_s p_s v_s, p = softmax over the visible slots of
+ * c((q[tok, h] . k_s) * scale), c(x) = softcap * tanh(x / softcap), or x where softcap is 0. The query in slot
+ * cache_position[t] (consecutive) sees row_start[b] <= s <= slot, where window > 0 only those with
+ * s > slot - window or s < row_start[b] + keep_first. gate (rows gate_pitch apart) may be NULL. The caches
+ * already hold the new rows. DECODE: span = the largest number of visible keys (window + keep_first, or the
+ * cache's capacity), scratch mui_hybrid_decode_scratch_bytes() bytes, 16-byte aligned. */
+int mui_hybrid_attention(mui_stream_t stream, int dtype, int route, const void* q, const void* k_cache,
+                         long k_batch_stride, const void* v_cache, long v_batch_stride, const void* gate,
+                         long gate_pitch, const int64_t* cache_position, const int64_t* row_start, float scale,
+                         float softcap, int window, int keep_first, void* scratch, int span, void* out, int batch,
+                         int t, int heads, int kv_heads, int dim, int vdim, int max_cache_len);
+
+/* Gated delta rule with one decay per head and key channel, over t tokens per batch row, from and to the state
+ * S [batch, heads, dk, dv] (fp32; zero: a fresh sequence); value head h uses query / key head
+ * h / (heads / kv_heads):
+ *   q, k, v = silu(conv(.)) of the projection's columns at their offsets (a causal convolution per channel over
+ *     `taps` tokens, conv [channels q | k | v, taps], the last column meets the current token)
+ *   q <- q_scale q / sqrt(|q|^2 + 1e-6), k <- k / sqrt(|k|^2 + 1e-6);  beta = sigmoid(b)
+ *   decay = exp(-exp(a_log[h]) softplus(a2 a + dt_bias)),  a: `ra` columns, a2 [heads * dk, ra]
+ *   S <- decay S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+ *   y[tok, h, :] = o * rsqrt(mean(o^2) + epsilon) * gain * sigmoid(g2 g),  g: `rg` columns, g2 [heads * dv, rg]
+ * ring [batch, mui_channel_delta_ring_rows(taps), channels] (activations' type) keeps the convolutions' last inputs;
+ * its rows in front of a sequence's first token are never read. Tokens with cache_position[t] < row_start[b]
+ * leave the state alone. At most mui_channel_delta_max_tokens(dk, taps) tokens a call; workspace:
+ * mui_channel_delta_workspace_bytes() bytes (0 up to MUI_MAX_TOKENS tokens), 16-byte aligned. */
+typedef struct mui_channel_delta {
+  const void *conv, *a2, *dt_bias, *a_log, *g2, *gain; /* activations' type */
+  int heads, kv_heads, dk, dv, ra, rg, taps;
+  int q_offset, k_offset, v_offset, a_offset, g_offset, b_offset;
+  float q_scale, epsilon;
+} mui_channel_delta_t;
+int mui_channel_delta_ring_rows(int taps);
+int mui_channel_delta_max_tokens(int dk, int taps);
+size_t mui_channel_delta_workspace_bytes(int batch, int t, int heads, int dk, int dv);
+int mui_channel_delta(mui_stream_t stream, int dtype, const mui_channel_delta_t* layer, const void* proj, long pitch,
+                      float* state, void* ring, const int64_t* cache_position, const int64_t* row_start, void* y,
+                      void* workspace, int batch, int t);
 
 #ifdef __cplusplus
 }

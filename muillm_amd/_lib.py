@@ -23,6 +23,7 @@ MUI_DTYPE_BF16 = 1
 MUI_DTYPE_F32 = 2
 MUI_MAX_TOKENS = 16
 MUI_LATENT_PLAIN, MUI_LATENT_DECODE, MUI_LATENT_PREFILL = 0, 1, 2
+MUI_HYBRID_PLAIN, MUI_HYBRID_DECODE, MUI_HYBRID_PREFILL = 0, 1, 2
 
 
 class MuiDeviceInfo(ctypes.Structure):
@@ -56,6 +57,7 @@ _SIGNATURES = {
     "mui_linear_workspace_bytes": (ctypes.c_size_t, []),
     "mui_rmsnorm": (c_int, [_P, c_int, _P, _P, c_float, _P, c_int, c_int]),
     "mui_gateup_silu": (c_int, [_P, c_int, _P, _P, c_long, _P, _P, c_float, _P, c_int, c_int, c_int]),
+    "mui_gateup_silu_bias": (c_int, [_P, c_int, _P, _P, c_long, _P, _P, c_float, _P, _P, _P, c_int, c_int, c_int]),
     "mui_silu_mul_interleaved": (c_int, [_P, c_int, _P, _P, c_long, c_int]),
     "mui_int8_linear": (c_int, [_P, c_int, _P, c_long, _P, _P, _P, c_float, _P, _P, _P, c_int, c_int, c_int]),
     "mui_int8_gateup_silu": (c_int, [_P, c_int, _P, _P, c_long, _P, _P, c_long, _P, _P, c_float, _P, c_int, c_int, c_int]),
@@ -97,9 +99,9 @@ _SIGNATURES = {
     "mui_embedding": (c_int, [_P, c_int, _P, c_long, _P, c_int, _P, c_int, c_int, c_int]),
     "mui_decoder_stack_workspace_bytes": (ctypes.c_size_t, [_P, c_int, c_int]),
     "mui_decoder_stack_step": (c_int, [_P, _P, c_int, _P, _P, _P, c_long, _P, c_int, _P, c_long, c_int, _P]),
-    "mui_residual_norm": (c_int, [_P, c_int, _P, _P, c_float, _P, _P, c_float, _P, _P, c_int, c_int]),
-    "mui_moe_residual_norm": (c_int, [_P, c_int, _P, _P, _P, _P, _P, c_int, c_int, _P, _P, c_float, _P, _P, c_int,
-                                      c_int]),
+    "mui_residual_norm": (c_int, [_P, c_int, _P, _P, c_float, _P, c_float, _P, c_float, c_float, _P, _P, c_int, c_int]),
+    "mui_moe_residual_norm": (c_int, [_P, c_int, _P, _P, _P, _P, _P, c_int, c_int, _P, c_float, _P, c_float, c_float, _P, _P,
+                                      c_int, c_int]),
     "mui_linear_f32": (c_int, [_P, c_int, _P, _P, _P, _P, c_int, c_int, c_int]),
     "mui_moe_tile_pairs": (c_int, [c_int, c_int, c_int, c_int, c_int, c_int]),
     "mui_moe_max_tiles": (c_int, [c_int, c_int, c_int, c_int]),
@@ -120,6 +122,18 @@ _SIGNATURES = {
     "mui_mlstm": (c_int, [_P, c_int, _P, _P, _P, c_long, _P, c_float, c_float, _P, _P, _P, _P, _P, _P, _P, c_int,
                           c_int, c_int, c_int, c_int]),
     "mui_mlstm_output": (c_int, [_P, c_int, _P, _P, _P, c_long, c_float, _P, c_int, c_int, c_int]),
+    "mui_bigram_embedding": (c_int, [_P, c_int, _P, _P, _P, _P, _P, _P, c_float, c_long, c_long, c_int, _P, _P, c_int, c_int,
+                                     c_int, c_int]),
+    "mui_hybrid_prepare": (c_int, [_P, c_int, _P, c_long, c_long, c_long, _P, _P, c_float, _P, c_int, _P, _P, _P, _P, c_long,
+                                   _P, c_long, c_int, c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mui_hybrid_attention_route": (c_int, [c_int, c_int, c_int, c_int]),
+    "mui_hybrid_decode_scratch_bytes": (ctypes.c_size_t, [c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mui_hybrid_attention": (c_int, [_P, c_int, c_int, _P, _P, c_long, _P, c_long, _P, c_long, _P, _P, c_float, c_float, c_int,
+                                     c_int, _P, c_int, _P, c_int, c_int, c_int, c_int, c_int, c_int, c_int]),
+    "mui_channel_delta_ring_rows": (c_int, [c_int]),
+    "mui_channel_delta_max_tokens": (c_int, [c_int, c_int]),
+    "mui_channel_delta_workspace_bytes": (ctypes.c_size_t, [c_int, c_int, c_int, c_int, c_int]),
+    "mui_channel_delta": (c_int, [_P, c_int, _P, _P, c_long, _P, _P, _P, _P, _P, _P, c_int, c_int]),
     "mui_probe_read": (c_int, [_P, _P, ctypes.c_uint64, _P]),
     "mui_tune_lock": (c_int, []),
     "mui_tune_gemv": (c_int, [c_int, c_int]),
@@ -155,7 +169,15 @@ class MuiDecoderStackDesc(ctypes.Structure):
                 ("cache_token_stride", c_long), ("max_cache_len", c_int)]
 
 
-MUI_ABI_VERSION = 3  # MUI_ABI_VERSION of the public header: layout of the structs above
+class MuiChannelDeltaDesc(ctypes.Structure):
+    """struct mui_channel_delta of the public header."""
+    _fields_ = ([(n, _P) for n in ("conv", "a2", "dt_bias", "a_log", "g2", "gain")]
+                + [(n, c_int) for n in ("heads", "kv_heads", "dk", "dv", "ra", "rg", "taps", "q_offset", "k_offset", "v_offset",
+                                        "a_offset", "g_offset", "b_offset")]
+                + [("q_scale", c_float), ("epsilon", c_float)])
+
+
+MUI_ABI_VERSION = 4  # MUI_ABI_VERSION of the public header: layout of the structs above
 
 _lib: Optional[ctypes.CDLL] = None
 

@@ -1,0 +1,917 @@
+// Gated delta rule with one decay per head and key channel, per head:
+//   S <- g_t * S (rows), u_t = beta_t (v_t - S^T k_t), S <- S + k_t u_t^T, o_t = S^T q_t
+// q, k, v come from a projection through a short causal convolution per channel and silu; q and k are unit vectors
+// per (query / key) head, q scaled by q_scale; beta = sigmoid(b); g = exp(-exp(A_log) softplus(A2 a + dt_bias)), a a
+// low-rank projection; the result is normed per head, times a gain, times sigmoid(G2 g) of another one.
+// S and everything that enters it stays in fp32; only the projections arrive in the activations' type.
+//
+//   step    (few tokens) one workgroup per head and batch row does all of it, S in registers.
+//   chunks  (prompts) 64 tokens at a time, in sub-chunks of 16. With G_t the product of the decays of a chunk up to t,
+//             A_ts = sum_d k_t k_s (G_t / G_s),  (1 + diag(beta) A) U = diag(beta) (V - (G * K) S_in)   (A strictly lower)
+//             O = (G * Q) S_in + A^qk U,  S_out = G_end * S_in + ((G_end / G) * K)^T U
+//           No quotient is ever formed: rows are multiplied by the decays since the start of their sub-chunk,
+//           columns by the decays up to the end of theirs, whole sub-chunks in between are a factor of their own,
+//           and pairs inside a sub-chunk carry a running product. Strong decays underflow to the zero they mean.
+//           1. prepare: convolutions, norms, decays, A, and W, U0 from U = U0 - W S_in, all chunks at once
+//           2. scan: one workgroup per head and 16 value columns walks the chunks, S in accumulators
+//           3. output: norm, gain, gate; the last inputs of the convolutions for the next call
+//           All products with S or U are v_mfma_f32_16x16x4_f32.
+// The last taps - 1 inputs of the convolutions are kept in a ring of rows by slot. Tokens in front of a row's
+// first slot (left padding) leave the state alone and are zeros to the convolutions.
+#include "hybrid.cuh"
+
+namespace mui {
+
+constexpr int kDChunk = 64, kDSub = 16;
+constexpr float kUnitEps = 1e-6f;
+
+struct DeltaParams {
+  const void* proj;  // [tokens, pitch]; q | k | v | a | g | b at the offsets below
+  long pitch;
+  int q_off, k_off, v_off, a_off, g_off, b_off;
+  const void* conv;  // [channels, taps], channels q | k | v
+  const void* a2;    // [heads * dk, ra]
+  const void* dt_bias;  // [heads * dk]
+  const void* a_log;    // [heads]
+  const void* g2;    // [heads * dv, rg]
+  const void* gain;  // [dv]
+  float q_scale, eps;
+  float* s;          // [batch, heads, dk, dv]
+  void* ring;        // [batch, ring_rows, channels]
+  const int64_t* cache_position;  // [t], consecutive slots
+  const int64_t* row_start;       // [batch] or null
+  void* y;           // [tokens, heads * dv]
+  int batch, t, heads, kv_heads, dk, dv, ra, rg, taps, ring_rows, channels;
+  bool vec;  // the low-rank operands may be read 16 bytes at a time (where their rank is a multiple of 8)
+  // chunks
+  float *qe, *w, *kd, *gc, *aqk, *u0, *o;  // per (batch, head, chunk); o [tokens, heads, dv]
+  int chunks, dkp, dvp;
+};
+
+template <typename T>
+struct DeltaRow {  // one batch row
+  typedef typename T::storage S;
+  const S* proj;
+  const S* ring;
+  long p0, start;  // slot of token 0, first slot of the row
+  __device__ __forceinline__ DeltaRow(const DeltaParams& p, int b)
+      : proj((const S*)p.proj + (long)b * p.t * p.pitch), ring((const S*)p.ring + (long)b * p.ring_rows * p.channels),
+        p0(p.cache_position[0]), start(p.row_start ? p.row_start[b] : 0) {}
+  __device__ __forceinline__ bool live(int tok) const { return p0 + tok >= start; }
+  // input of channel c (column `col` of the projection) at token tok, which may lie in front of this call
+  __device__ __forceinline__ float raw(const DeltaParams& p, int tok, int col, int c) const {
+    const long slot = p0 + tok;
+    if (slot < start || slot < 0) return 0.f;
+    return T::one(tok >= 0 ? proj[(long)tok * p.pitch + col] : ring[(long)((uint32_t)slot % (uint32_t)p.ring_rows) * p.channels + c]);
+  }
+  // convolution and silu
+  __device__ __forceinline__ float conv(const DeltaParams& p, int tok, int col, int c) const {
+    const S* w = (const S*)p.conv + (long)c * p.taps;
+    float a = 0.f;
+    for (int j = p.taps - 1; j >= 0; --j) a = fmaf(T::one(w[p.taps - 1 - j]), raw(p, tok - j, col, c), a);
+    return a / (1.f + expf(-a));
+  }
+};
+
+__device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
+__device__ __forceinline__ float sigm(float z) { return 1.f / (1.f + expf(-z)); }
+
+// the last taps - 1 inputs of the call into the ring; head h writes its value channels, the first head of a group
+// its query and key channels
+template <typename T>
+__device__ __forceinline__ void keep_inputs(const DeltaParams& p, int b, int h, int t, int nt) {
+  typedef typename T::storage S;
+  const int share = p.heads / p.kv_heads, kvh = h / share, nq = p.kv_heads * p.dk;
+  const bool first = h % share == 0;
+  const int from = p.t - (p.taps - 1) > 0 ? p.t - (p.taps - 1) : 0;
+  const int per = (first ? 2 * p.dk : 0) + p.dv;
+  const long p0 = p.cache_position[0];
+  S* ring = (S*)p.ring + (long)b * p.ring_rows * p.channels;
+  for (int i = t; i < per * (p.t - from); i += nt) {
+    const int tok = from + i / per;
+    int e = i % per, c, col;
+    if (e < p.dv) {
+      c = 2 * nq + h * p.dv + e;
+      col = p.v_off + h * p.dv + e;
+    } else {
+      e -= p.dv;
+      const int k = e >= p.dk;
+      c = k * nq + kvh * p.dk + (e - k * p.dk);
+      col = (k ? p.k_off : p.q_off) + kvh * p.dk + (e - k * p.dk);
+    }
+    ring[(long)((uint32_t)(p0 + tok) % (uint32_t)p.ring_rows) * p.channels + c] = ((const S*)p.proj)[((long)b * p.t + tok) * p.pitch + col];
+  }
+}
+
+// ---------------------------------------------------------------------------------------
+// step: grid (heads, batch), 512 threads; thread = (four columns, rows rg, rg + RG, ..)
+// ---------------------------------------------------------------------------------------
+extern __shared__ __align__(16) unsigned char cd_smem[];
+constexpr int kStepThreads = 512;
+
+// out[row] = f(sum_k W[row, k] x[k]) for rows of a low-rank second factor; eight threads per row, x in LDS
+template <typename T, typename F>
+__device__ __forceinline__ void low_rank_rows(const typename T::storage* w, const float* x, int rows, int r, bool vec, F f) {
+  const int t = threadIdx.x, sub = t & 7;
+  for (int row0 = 0; row0 < rows; row0 += kStepThreads / 8) {
+    const int row = row0 + (t >> 3);
+    const typename T::storage* wr = w + (long)(row < rows ? row : rows - 1) * r;
+    float a = 0.f;
+    if (vec) {
+#pragma unroll 2
+      for (int c = sub * 8; c < r; c += 64) {
+        float fw[8];
+        load8<T>(wr + c, fw);
+#pragma unroll
+        for (int i = 0; i < 8; ++i) a = fmaf(fw[i], x[c + i], a);
+      }
+    } else {
+      for (int c = sub; c < r; c += 8) a = fmaf(T::one(wr[c]), x[c], a);
+    }
+    a += dpp_f32<kDppXor1>(a);
+    a += dpp_f32<kDppXor2>(a);
+    a += dpp_f32<kDppHalfMirror>(a);
+    if (sub == 0 && row < rows) f(row, a);
+  }
+}
+
+template <typename T, int NR>  // NR rows of S per thread in registers; 0: S stays in memory
+__global__ void __launch_bounds__(kStepThreads) delta_step_kernel(const DeltaParams p, int cgp) {
+  typedef typename T::storage S;
+  __shared__ float red[8][4];
+  const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
+  const int h = blockIdx.x, b = blockIdx.y, share = p.heads / p.kv_heads, kvh = h / share, nq = p.kv_heads * p.dk;
+  const int parts = cgp <= 64 ? 8 : kStepThreads / cgp, cols = 4 * cgp;
+  float* qs = (float*)cd_smem;     // dk
+  float* ks = qs + p.dk;           // dk
+  float* gs = ks + p.dk;           // dk: decays
+  float* vs = gs + p.dk;           // dv; later u
+  float* og = vs + p.dv;           // dv: output gate
+  float* av = og + p.dv;           // max(ra, rg)
+  float* part = av + (p.ra > p.rg ? p.ra : p.rg) + ((4 - ((3 * p.dk + 2 * p.dv + (p.ra > p.rg ? p.ra : p.rg)) & 3)) & 3);  // [2][parts][cols]
+  const DeltaRow<T> row(p, b);
+  const int cg = t & (cgp - 1), rg = t / cgp, RG = kStepThreads / cgp, c0 = cg * 4;
+  float* st = p.s + ((long)b * p.heads + h) * p.dk * p.dv;
+  const bool v4 = p.dv % 4 == 0;
+  const float neg_a = -expf(T::one(((const S*)p.a_log)[h]));
+  const bool vec_a = p.ra % 8 == 0 && p.vec, vec_g = p.rg % 8 == 0 && p.vec;
+  f32x4 sreg[NR > 0 ? NR : 1];
+  auto load_s = [&](int d) {
+    f32x4 x = {0.f, 0.f, 0.f, 0.f};
+    if (d < p.dk && c0 < p.dv) {
+      if (v4) {
+        x = *(const f32x4*)(st + (long)d * p.dv + c0);
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (c0 + j < p.dv) x[j] = st[(long)d * p.dv + c0 + j];
+      }
+    }
+    return x;
+  };
+  auto store_s = [&](int d, f32x4 x) {
+    if (d < p.dk && c0 < p.dv) {
+      if (v4) {
+        *(f32x4*)(st + (long)d * p.dv + c0) = x;
+      } else {
+#pragma unroll
+        for (int j = 0; j < 4; ++j)
+          if (c0 + j < p.dv) st[(long)d * p.dv + c0 + j] = x[j];
+      }
+    }
+  };
+  if constexpr (NR > 0) {
+#pragma unroll
+    for (int i = 0; i < NR; ++i) sreg[i] = load_s(rg + RG * i);
+  }
+  for (int tok = 0; tok < p.t; ++tok) {
+    S* yrow = (S*)p.y + (((long)b * p.t + tok) * p.heads + h) * p.dv;
+    if (!row.live(tok)) {  // uniform for the workgroup
+      for (int i = t; i < p.dv; i += kStepThreads) yrow[i] = T::pack(0.f);
+      continue;
+    }
+    const S* pr = row.proj + (long)tok * p.pitch;
+    // inputs of the recurrence
+    float qq = 0.f, kk = 0.f, qk = 0.f;
+    for (int d = t; d < p.dk; d += kStepThreads) {
+      const int c = kvh * p.dk + d;
+      const float x = row.conv(p, tok, p.q_off + c, c), y = row.conv(p, tok, p.k_off + c, nq + c);
+      qs[d] = x;
+      ks[d] = y;
+      qq = fmaf(x, x, qq);
+      kk = fmaf(y, y, kk);
+      qk = fmaf(x, y, qk);
+    }
+    for (int e = kStepThreads - 1 - t; e < p.dv; e += kStepThreads) {  // (from the other end: dk threads are busy above)
+      const int c = h * p.dv + e;
+      vs[e] = row.conv(p, tok, p.v_off + c, 2 * nq + c);
+    }
+    for (int i = t; i < p.ra; i += kStepThreads) av[i] = T::one(pr[p.a_off + i]);
+    qq = wave_sum(qq);
+    kk = wave_sum(kk);
+    qk = wave_sum(qk);
+    if (lane == 0) {
+      red[wave][0] = qq;
+      red[wave][1] = kk;
+      red[wave][2] = qk;
+    }
+    __syncthreads();
+    low_rank_rows<T>((const S*)p.a2 + (long)h * p.dk * p.ra, av, p.dk, p.ra, vec_a, [&](int d, float z) {
+      gs[d] = expf(neg_a * softplus_f32(z + T::one(((const S*)p.dt_bias)[h * p.dk + d])));
+    });
+    qq = kk = qk = 0.f;
+#pragma unroll
+    for (int w = 0; w < 8; ++w) {
+      qq += red[w][0];
+      kk += red[w][1];
+      qk += red[w][2];
+    }
+    const float rq = p.q_scale / sqrtf(qq + kUnitEps), rk = 1.f / sqrtf(kk + kUnitEps);
+    __syncthreads();
+    for (int i = t; i < p.rg; i += kStepThreads) av[i] = T::one(pr[p.g_off + i]);
+    // decayed S against k and q
+    f32x4 pk = {0.f, 0.f, 0.f, 0.f}, pq = pk;
+    auto sweep = [&](f32x4& x, int d) {
+      const float g = gs[d], k = ks[d] * rk, q = qs[d] * rq;
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        x[j] *= g;
+        pk[j] = fmaf(x[j], k, pk[j]);
+        pq[j] = fmaf(x[j], q, pq[j]);
+      }
+    };
+    if constexpr (NR > 0) {
+#pragma unroll
+      for (int i = 0; i < NR; ++i)
+        if (rg + RG * i < p.dk) sweep(sreg[i], rg + RG * i);
+    } else {
+      for (int d = rg; d < p.dk; d += RG) {
+        f32x4 x = load_s(d);
+        sweep(x, d);
+      }
+    }
+    for (int o = cgp; o < 64; o <<= 1)
+#pragma unroll
+      for (int j = 0; j < 4; ++j) {
+        pk[j] += __shfl_xor(pk[j], o);
+        pq[j] += __shfl_xor(pq[j], o);
+      }
+    if (lane < cgp) {
+      const int pi = cgp <= 64 ? wave : rg;
+      *(f32x4*)&part[pi * cols + c0] = pk;
+      *(f32x4*)&part[(parts + pi) * cols + c0] = pq;
+    }
+    __syncthreads();
+    low_rank_rows<T>((const S*)p.g2 + (long)h * p.dv * p.rg, av, p.dv, p.rg, vec_g, [&](int e, float z) { og[e] = sigm(z); });
+    const float beta = sigm(T::one(pr[p.b_off + h]));
+    const float dot = qk * rq * rk;
+    float ss = 0.f;
+    for (int e = t; e < p.dv; e += kStepThreads) {
+      float a = 0.f, o = 0.f;
+      for (int i = 0; i < parts; ++i) {
+        a += part[i * cols + e];
+        o += part[(parts + i) * cols + e];
+      }
+      const float u = beta * (vs[e] - a);
+      o = fmaf(dot, u, o);
+      vs[e] = u;
+      part[e] = o;  // (this thread's column of the sums just read)
+      ss = fmaf(o, o, ss);
+    }
+    ss = wave_sum(ss);
+    if (lane == 0) red[wave][3] = ss;
+    __syncthreads();
+    auto write = [&](f32x4& x, int d) {
+      const float k = ks[d] * rk;
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (c0 + j < p.dv) x[j] = fmaf(k, vs[c0 + j], x[j]);
+    };
+    if constexpr (NR > 0) {
+#pragma unroll
+      for (int i = 0; i < NR; ++i)
+        if (rg + RG * i < p.dk) write(sreg[i], rg + RG * i);
+    } else {
+      for (int d = rg; d < p.dk; d += RG) {
+        f32x4 x = load_s(d);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) x[j] *= gs[d];
+        write(x, d);
+        store_s(d, x);
+      }
+    }
+    ss = 0.f;
+#pragma unroll
+    for (int w = 0; w < 8; ++w) ss += red[w][3];
+    const float rs = 1.f / sqrtf(ss / (float)p.dv + p.eps);
+    for (int e = t; e < p.dv; e += kStepThreads) yrow[e] = T::pack(part[e] * rs * T::one(((const S*)p.gain)[e]) * og[e]);
+    __syncthreads();  // everything in LDS is free
+  }
+  if constexpr (NR > 0) {
+#pragma unroll
+    for (int i = 0; i < NR; ++i) store_s(rg + RG * i, sreg[i]);
+  }
+  keep_inputs<T>(p, b, h, t, kStepThreads);
+}
+
+// ---------------------------------------------------------------------------------------
+// chunks
+// ---------------------------------------------------------------------------------------
+// 16 x 16 tile of X W^T over r: lane's row of X and of W (row lane % 16 each); D: column W row lane % 16, rows X 4 (lane / 16) + r
+template <typename T>
+__device__ __forceinline__ f32x4 low_rank_tile(const typename T::storage* x, const typename T::storage* w, int r, bool vec) {
+  const int g = (threadIdx.x & 63) >> 4;
+  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+  if constexpr (T::kDtype == MUI_DTYPE_F32) {
+    for (int k = 0; k < r; k += 4) {
+      const int e = k + g;
+      acc = mfma_f32(e < r ? x[e] : 0.f, e < r ? w[e] : 0.f, acc);
+    }
+  } else {
+    for (int k = 0; k < r; k += 32) {
+      const int e = k + 8 * g;
+      u32x4 a, b;
+      if (vec) {
+        const u32x4 zero = {0u, 0u, 0u, 0u};
+        a = ld16(x + (e < r ? e : 0));
+        b = ld16(w + (e < r ? e : 0));
+        a = e < r ? a : zero;
+        b = e < r ? b : zero;
+      } else {
+        uint32_t aw[4], bw[4];
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+          const int e0 = e + 2 * i, e1 = e0 + 1;
+          aw[i] = (e0 < r ? (uint32_t)x[e0] : 0u) | ((e1 < r ? (uint32_t)x[e1] : 0u) << 16);
+          bw[i] = (e0 < r ? (uint32_t)w[e0] : 0u) | ((e1 < r ? (uint32_t)w[e1] : 0u) << 16);
+        }
+        a = u32x4{aw[0], aw[1], aw[2], aw[3]};
+        b = u32x4{bw[0], bw[1], bw[2], bw[3]};
+      }
+      acc = mfma16x16x32<T>(a, b, acc);
+    }
+  }
+  return acc;
+}
+
+// 16 consecutive tokens of a convolved channel, from token tok0 >= 0 (may reach past the call: zeros). x: the TAPS - 1
+// inputs in front of tok0 on entry, those in front of tok0 + 16 on return. TAPS >= p.taps: older ones weigh zero.
+template <typename T, int TAPS>
+struct ConvTaps {
+  float w[TAPS], x[TAPS - 1 > 0 ? TAPS - 1 : 1];
+  __device__ __forceinline__ void start(const DeltaParams& p, const DeltaRow<T>& row, int tok0, int col, int c) {
+    typedef typename T::storage S;
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) {
+      const int i = j - (TAPS - p.taps);
+      const float v = T::one(((const S*)p.conv)[(long)c * p.taps + (i > 0 ? i : 0)]);
+      w[j] = i >= 0 ? v : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) {
+      const int tok = tok0 - (TAPS - 1) + j;
+      const long slot = row.p0 + tok;
+      const bool on = slot >= row.start && slot >= 0 && j >= TAPS - p.taps;
+      const long ring_row = (long)((uint32_t)(slot > 0 ? slot : 0) % (uint32_t)p.ring_rows);
+      // (sub-chunks behind the call's last token read that one: their outputs are zero anyway)
+      const S* src = tok >= 0 ? row.proj + (long)(tok < p.t ? tok : p.t - 1) * p.pitch + col : row.ring + ring_row * p.channels + c;
+      const float v = T::one(*src);
+      x[j] = on ? v : 0.f;
+    }
+  }
+  __device__ __forceinline__ void run(const DeltaParams& p, const DeltaRow<T>& row, int tok0, int col, float (&y)[16]) {
+    typedef typename T::storage S;
+    // live tokens of the sixteen: first <= i < last (in vector registers: sixteen scalar conditions would spill)
+    const long lead = row.start - row.p0;
+    int first = (int)(lead > 0 ? (lead < p.t ? lead : p.t) : 0) - tok0, last = p.t - tok0;
+    asm volatile("" : "+v"(first), "+v"(last));
+    float z[16 + TAPS - 1];
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) z[j] = x[j];
+    const S* src = row.proj + (long)(tok0 < p.t ? tok0 : p.t - 1) * p.pitch + col;
+    const int pitch = (int)p.pitch;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      const float v = T::one(src[(unsigned)((i < last ? i : 0) * pitch)]);
+      z[TAPS - 1 + i] = i >= first && i < last ? v : 0.f;
+    }
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      float a = 0.f;
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) a = fmaf(w[j], z[i + j], a);
+      a /= 1.f + expf(-a);
+      y[i] = i >= first && i < last ? a : 0.f;
+    }
+#pragma unroll
+    for (int j = 0; j < TAPS - 1; ++j) x[j] = z[16 + j];
+  }
+};
+
+// 1. grid (chunks, heads, batch); wave w owns sub-chunk w, lane = channel of a block of 64 (NB blocks: dk <= 64 NB)
+constexpr int kDPitch = 68;  // 16 rows x 4 consecutive k in 64 different banks
+template <typename T, int NB, int TAPS>
+__global__ void __launch_bounds__(256, NB > 2 ? 1 : 2) delta_prepare_kernel(const DeltaParams p) {
+  typedef typename T::storage S;
+  constexpr int DKP = 64 * NB;  // = p.dkp
+  float* qh = (float*)cd_smem;              // [64][kDPitch]: q times the decays since the start of its sub-chunk
+  float* kh = qh + kDChunk * kDPitch;       // the same of k
+  float* ke = kh + kDChunk * kDPitch;       // k times the decays up to the end of its sub-chunk
+  float* lm = ke + kDChunk * kDPitch;       // [64][kDPitch]: beta_t A_ts
+  __shared__ float gm[4][64 * NB], bt[kDChunk];
+  const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), g4 = lane >> 4, i16 = lane & 15;
+  const int chunk = blockIdx.x, h = blockIdx.y, b = blockIdx.z, kvh = h / (p.heads / p.kv_heads), nq = p.kv_heads * p.dk;
+  const long bhc = ((long)b * p.heads + h) * p.chunks + chunk;
+  const DeltaRow<T> row(p, b);
+  const int tok0 = chunk * kDChunk + wave * kDSub;  // of this wave
+  float* qe_out = p.qe + bhc * kDChunk * DKP;
+  float* w_out = p.w + bhc * kDChunk * DKP;
+  float* kd_out = p.kd + bhc * kDChunk * DKP;
+  float* aqk_out = p.aqk + bhc * kDChunk * kDChunk;
+
+  // q, k and decays of this wave's 16 tokens, channel `lane` of every block
+  float q[NB][16], k[NB][16], g[NB][16];
+#pragma unroll
+  for (int nb = 0; nb < NB; ++nb) {
+    const int d = nb * 64 + lane, c = kvh * p.dk + (d < p.dk ? d : 0);
+    ConvTaps<T, TAPS> cv;
+    cv.start(p, row, tok0, p.q_off + c, c);
+    cv.run(p, row, tok0, p.q_off + c, q[nb]);
+    cv.start(p, row, tok0, p.k_off + c, nq + c);
+    cv.run(p, row, tok0, p.k_off + c, k[nb]);
+    if (d >= p.dk) {
+#pragma unroll
+      for (int i = 0; i < 16; ++i) q[nb][i] = k[nb][i] = 0.f;
+    }
+  }
+  {
+    const float neg_a = -expf(T::one(((const S*)p.a_log)[h]));
+    const bool vec = p.ra % 8 == 0 && p.vec;
+    const int tk = tok0 + i16 < p.t ? tok0 + i16 : p.t - 1;
+    const S* x = row.proj + (long)tk * p.pitch + p.a_off;
+    float* z = qh + wave * kDSub * kDPitch;  // this wave's rows
+#pragma unroll
+    for (int nb = 0; nb < NB; ++nb) {
+#pragma unroll 1
+      for (int ct = 0; ct < 4; ++ct) {
+        const int d = nb * 64 + ct * 16 + i16, dc = h * p.dk + (d < p.dk ? d : 0);
+        const f32x4 v = low_rank_tile<T>(x, (const S*)p.a2 + (long)dc * p.ra, p.ra, vec);
+        const float bias = T::one(((const S*)p.dt_bias)[dc]);
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          const int tr = tok0 + 4 * g4 + r;
+          const float e = expf(neg_a * softplus_f32(v[r] + bias));
+          z[(4 * g4 + r) * kDPitch + ct * 16 + i16] = tr < p.t && row.live(tr) ? e : 1.f;
+        }
+      }
+      __builtin_amdgcn_wave_barrier();
+#pragma unroll
+      for (int i = 0; i < 16; ++i) g[nb][i] = z[i * kDPitch + lane];
+      __builtin_amdgcn_wave_barrier();
+    }
+  }
+  if (t < kDChunk) {
+    const int tk = chunk * kDChunk + t;
+    bt[t] = tk < p.t && row.live(tk) ? sigm(T::one(row.proj[(long)tk * p.pitch + p.b_off + h])) : 0.f;
+  }
+  // unit vectors
+#pragma unroll
+  for (int i = 0; i < 16; ++i) {
+    float sq = 0.f, sk = 0.f;
+#pragma unroll
+    for (int nb = 0; nb < NB; ++nb) {
+      sq = fmaf(q[nb][i], q[nb][i], sq);
+      sk = fmaf(k[nb][i], k[nb][i], sk);
+    }
+    const float rq = p.q_scale / sqrtf(wave_sum(sq) + kUnitEps), rk = 1.f / sqrtf(wave_sum(sk) + kUnitEps);
+#pragma unroll
+    for (int nb = 0; nb < NB; ++nb) {
+      q[nb][i] *= rq;
+      k[nb][i] *= rk;
+    }
+  }
+#pragma unroll
+  for (int nb = 0; nb < NB; ++nb) {
+    float a = 1.f;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) a *= g[nb][i];
+    gm[wave][nb * 64 + lane] = a;
+  }
+  __syncthreads();  // bt, gm
+  // pairs inside this wave's sub-chunk: k_s times a running product of decays, against k_t and q_t
+#pragma unroll
+  for (int s = 0; s < 16; ++s) {
+    float w[NB], vk[16], vq[16];
+#pragma unroll
+    for (int nb = 0; nb < NB; ++nb) w[nb] = k[nb][s];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      vk[i] = vq[i] = 0.f;
+      if (i >= s) {
+#pragma unroll
+        for (int nb = 0; nb < NB; ++nb) {
+          if (i > s) {
+            w[nb] *= g[nb][i];
+            vk[i] = fmaf(w[nb], k[nb][i], vk[i]);
+          }
+          vq[i] = fmaf(w[nb], q[nb][i], vq[i]);
+        }
+      }
+    }
+    row16_reduce_scatter<16>(vk, lane);  // lane i of a row of 16 lanes: token i
+    row16_reduce_scatter<16>(vq, lane);
+    float a = vk[0], c = vq[0];
+    a += __shfl_xor(a, 16);
+    c += __shfl_xor(c, 16);
+    a += __shfl_xor(a, 32);
+    c += __shfl_xor(c, 32);
+    if (g4 == 0) {
+      const int tr = wave * kDSub + i16, sc = wave * kDSub + s;
+      lm[tr * kDPitch + sc] = a * bt[tr];  // zero on and above the diagonal
+      aqk_out[tr * kDChunk + sc] = c;      // zero above it
+    }
+  }
+  // pairs of different sub-chunks (row I, column J < I): (3,0) (3,1) | (3,2) (2,0) | (2,1) | (1,0)
+  const int pi[2] = {wave < 2 ? 3 : (wave == 2 ? 2 : 1), wave == 0 ? 3 : 2}, pj[2] = {wave == 1 ? 2 : (wave == 2 ? 1 : 0), wave == 0 ? 1 : 0};
+  f32x4 akk[2], aqk[2];
+#pragma unroll
+  for (int u = 0; u < 2; ++u) akk[u] = aqk[u] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int nb = 0; nb < NB; ++nb) {
+    const int d = nb * 64 + lane;
+    float before = 1.f, after = 1.f;  // whole sub-chunks in front of and behind this one
+    for (int m = 0; m < 4; ++m) {
+      if (m < wave) before *= gm[m][d];
+      if (m > wave) after *= gm[m][d];
+    }
+    float kd[16];
+    float a = 1.f;
+#pragma unroll
+    for (int i = 15; i >= 0; --i) {
+      const float e = k[nb][i] * a;
+      ke[(wave * kDSub + i) * kDPitch + lane] = e;
+      kd[i] = e * after;
+      a *= g[nb][i];
+    }
+    a = 1.f;
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      a *= g[nb][i];
+      const float x = q[nb][i] * a, y = k[nb][i] * a;
+      const int tr = wave * kDSub + i;
+      qh[tr * kDPitch + lane] = x;
+      kh[tr * kDPitch + lane] = y;
+      qe_out[tr * DKP + d] = x * before;
+      w_out[tr * DKP + d] = y * before;  // (solved in place below)
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      *(f32x4*)&kd_out[(long)d * kDChunk + wave * kDSub + 4 * i] = f32x4{kd[4 * i], kd[4 * i + 1], kd[4 * i + 2], kd[4 * i + 3]};
+    if (wave == 3) p.gc[bhc * DKP + d] = before * gm[3][d];
+    __syncthreads();
+#pragma unroll
+    for (int u = 0; u < 2; ++u) {
+      if (u == 1 && wave > 1) continue;
+      const int I = pi[u], J = pj[u];
+#pragma unroll 4
+      for (int k0 = 0; k0 < 64; k0 += 4) {
+        float e = ke[(J * kDSub + i16) * kDPitch + k0 + g4];
+        for (int m = J + 1; m < I; ++m) e *= gm[m][nb * 64 + k0 + g4];
+        akk[u] = mfma_f32(kh[(I * kDSub + i16) * kDPitch + k0 + g4], e, akk[u]);
+        aqk[u] = mfma_f32(qh[(I * kDSub + i16) * kDPitch + k0 + g4], e, aqk[u]);
+      }
+    }
+    __syncthreads();
+  }
+#pragma unroll
+  for (int u = 0; u < 2; ++u) {
+    if (u == 1 && wave > 1) continue;
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int tr = pi[u] * kDSub + 4 * g4 + r, sc = pj[u] * kDSub + i16;
+      lm[tr * kDPitch + sc] = akk[u][r] * bt[tr];
+      aqk_out[tr * kDChunk + sc] = aqk[u][r];
+    }
+  }
+  __syncthreads();  // lm, and w_out as seen by this workgroup
+  // x_t = beta_t rhs_t - sum_{s < t} lm_ts x_s, one column per thread: W from the decayed keys, U0 from the values
+  // (which pass through their place in memory: short code instead of 64 convolutions in a row)
+#pragma unroll 1
+  for (int c = t; c < DKP + p.dvp; c += 256) {
+    const bool is_w = c < DKP;  // (a multiple of 64: uniform for the wave)
+    float* wcol = w_out + c;
+    float* ucol = p.u0 + (bhc * p.dvp + (is_w ? 0 : c - DKP)) * kDChunk;
+    float x[kDChunk];
+    if (is_w) {
+#pragma unroll
+      for (int i = 0; i < kDChunk; ++i) x[i] = wcol[i * DKP];
+    } else {
+      const int v = c - DKP, ch = h * p.dv + (v < p.dv ? v : 0);
+      ConvTaps<T, TAPS> cv;
+      cv.start(p, row, chunk * kDChunk, p.v_off + ch, 2 * nq + ch);
+#pragma unroll 1
+      for (int i = 0; i < kDChunk; i += 16) {
+        float y[16];
+        cv.run(p, row, chunk * kDChunk + i, p.v_off + ch, y);
+#pragma unroll
+        for (int j = 0; j < 16; j += 4) *(f32x4*)(ucol + i + j) = v < p.dv ? f32x4{y[j], y[j + 1], y[j + 2], y[j + 3]} : f32x4{0.f, 0.f, 0.f, 0.f};
+      }
+#pragma unroll
+      for (int i = 0; i < kDChunk; i += 4) {
+        const f32x4 y = *(const f32x4*)(ucol + i);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) x[i + j] = y[j];
+      }
+    }
+#pragma unroll
+    for (int i = 0; i < kDChunk; ++i) {
+      float a = x[i] * bt[i], a2 = 0.f;
+#pragma unroll
+      for (int s = 0; s + 4 <= i; s += 4) {
+        const f32x4 l = *(const f32x4*)&lm[i * kDPitch + s];
+        a = fmaf(-l[0], x[s], a);
+        a2 = fmaf(-l[1], x[s + 1], a2);
+        a = fmaf(-l[2], x[s + 2], a);
+        a2 = fmaf(-l[3], x[s + 3], a2);
+      }
+#pragma unroll
+      for (int s = i & ~3; s < i; ++s) a = fmaf(-lm[i * kDPitch + s], x[s], a);
+      x[i] = a + a2;
+      if (i % 4 == 3) asm volatile("" ::: "memory");  // the matrix is read row by row, not all of it ahead
+    }
+    if (is_w) {
+#pragma unroll
+      for (int i = 0; i < kDChunk; ++i) wcol[i * DKP] = x[i];
+    } else {
+#pragma unroll
+      for (int i = 0; i < kDChunk; i += 4) *(f32x4*)(ucol + i) = f32x4{x[i], x[i + 1], x[i + 2], x[i + 3]};
+    }
+  }
+}
+
+// 2. grid (heads * slices of 16 value columns, batch); wave w owns key rows 16 NT w .. of S (dkp = 64 NT). The slices
+// of a head are `heads` workgroups apart: one XCD's L2 serves them all where the heads are a multiple of 8.
+// An accumulator tile (rows 4 g + r, column lane % 16) is the B operand of the next product as it stands, with
+// the contraction dealt out as 4 g + r.
+template <int NT>
+__global__ void __launch_bounds__(256, 1) delta_scan_kernel(const DeltaParams p) {
+  __shared__ __align__(16) f32x4 xu[2][4][4][64], xo[2][4][4][64];  // [buffer][wave][row tile][lane]
+  const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), g = lane >> 4, i16 = lane & 15;
+  const int h = blockIdx.x % p.heads, c0 = (blockIdx.x / p.heads) * 16, b = blockIdx.y;
+  const long bh = (long)b * p.heads + h;
+  const int d0 = wave * NT * 16;
+  float* st = p.s + bh * p.dk * p.dv;
+  const bool col = c0 + i16 < p.dv;
+  f32x4 s[NT];
+#pragma unroll
+  for (int i = 0; i < NT; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = d0 + 16 * i + 4 * g + r;
+      s[i][r] = d < p.dk && col ? st[(long)d * p.dv + c0 + i16] : 0.f;
+    }
+  f32x4 w[4][NT], q[4][NT], kd[4][NT], gc[NT], aq[4], u0[4];
+  auto load_wq = [&](int c) {
+    const float* wp = p.w + (bh * p.chunks + c) * kDChunk * p.dkp + (long)i16 * p.dkp + d0 + 4 * g;
+    const float* qp = p.qe + (bh * p.chunks + c) * kDChunk * p.dkp + (long)i16 * p.dkp + d0 + 4 * g;
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt)
+#pragma unroll
+      for (int i = 0; i < NT; ++i) {
+        w[rt][i] = *(const f32x4*)(wp + (long)16 * rt * p.dkp + 16 * i);
+        q[rt][i] = *(const f32x4*)(qp + (long)16 * rt * p.dkp + 16 * i);
+      }
+  };
+  auto load_u = [&](int c) {
+    const float* up = p.u0 + ((bh * p.chunks + c) * p.dvp + c0 + i16) * kDChunk + 4 * g;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) u0[j] = *(const f32x4*)(up + 16 * j);
+  };
+  auto load_a = [&](int c) {
+    const float* ap = p.aqk + (bh * p.chunks + c) * kDChunk * kDChunk + (long)(16 * wave + i16) * kDChunk + 4 * g;
+#pragma unroll
+    for (int j = 0; j < 4; ++j) aq[j] = *(const f32x4*)(ap + 16 * (j <= wave ? j : wave));
+  };
+  auto load_k = [&](int c) {
+    const float* kp = p.kd + ((bh * p.chunks + c) * p.dkp + d0 + i16) * kDChunk + 4 * g;
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) kd[j][i] = *(const f32x4*)(kp + (long)16 * i * kDChunk + 16 * j);
+      gc[i] = *(const f32x4*)(p.gc + (bh * p.chunks + c) * p.dkp + d0 + 16 * i + 4 * g);
+    }
+  };
+  load_wq(0);
+  load_u(0);
+  load_a(0);
+  load_k(0);
+  for (int c = 0; c < p.chunks; ++c) {
+    const int buf = c & 1, next = c + 1 < p.chunks ? c + 1 : c;
+    // this wave's key rows of W S and Q S
+#pragma unroll
+    for (int rt = 0; rt < 4; ++rt) {
+      f32x4 a = {0.f, 0.f, 0.f, 0.f}, o = a;
+#pragma unroll
+      for (int i = 0; i < NT; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          a = mfma_f32(w[rt][i][r], s[i][r], a);
+          o = mfma_f32(q[rt][i][r], s[i][r], o);
+        }
+      xu[buf][wave][rt][lane] = a;
+      xo[buf][wave][rt][lane] = o;
+    }
+    load_wq(next);
+    __syncthreads();
+    f32x4 u[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const f32x4 a = xu[buf][0][j][lane], b4 = xu[buf][1][j][lane], c4 = xu[buf][2][j][lane], d4 = xu[buf][3][j][lane];
+#pragma unroll
+      for (int r = 0; r < 4; ++r) u[j][r] = u0[j][r] - ((a[r] + b4[r]) + (c4[r] + d4[r]));
+    }
+    load_u(next);
+    {
+      const f32x4 a = xo[buf][0][wave][lane], b4 = xo[buf][1][wave][lane], c4 = xo[buf][2][wave][lane], d4 = xo[buf][3][wave][lane];
+      f32x4 o;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[r] = (a[r] + b4[r]) + (c4[r] + d4[r]);
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (j <= wave)
+#pragma unroll
+          for (int r = 0; r < 4; ++r) o = mfma_f32(aq[j][r], u[j][r], o);
+      const int tk = c * kDChunk + 16 * wave + 4 * g;
+      float* dst = p.o + (((long)b * p.t + tk) * p.heads + h) * p.dv + c0 + i16;
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (tk + r < p.t && col) dst[(long)r * p.heads * p.dv] = o[r];
+    }
+    load_a(next);
+#pragma unroll
+    for (int i = 0; i < NT; ++i) {
+#pragma unroll
+      for (int r = 0; r < 4; ++r) s[i][r] *= gc[i][r];
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) s[i] = mfma_f32(kd[j][i][r], u[j][r], s[i]);
+    }
+    load_k(next);
+  }
+#pragma unroll
+  for (int i = 0; i < NT; ++i)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int d = d0 + 16 * i + 4 * g + r;
+      if (d < p.dk && col) st[(long)d * p.dv + c0 + i16] = s[i][r];
+    }
+}
+
+// 3. grid (chunks, heads, batch); wave w takes tokens 16 w .. of the chunk
+template <typename T>
+__global__ void __launch_bounds__(256) delta_output_kernel(const DeltaParams p) {
+  typedef typename T::storage S;
+  const int t = threadIdx.x, lane = t & 63, wave = t >> 6, g = lane >> 4, i16 = lane & 15;
+  const int chunk = blockIdx.x, h = blockIdx.y, b = blockIdx.z;
+  const int tok0 = chunk * kDChunk + wave * kDSub;
+  if (chunk == p.chunks - 1) keep_inputs<T>(p, b, h, t, 256);
+  if (tok0 >= p.t) return;
+  const bool vec = p.rg % 8 == 0 && p.vec;
+  const int tk = tok0 + i16 < p.t ? tok0 + i16 : p.t - 1;
+  const S* x = (const S*)p.proj + ((long)b * p.t + tk) * p.pitch + p.g_off;
+  long at[4];  // rows of this lane
+  float ss[4] = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int r = 0; r < 4; ++r) {
+    const int tr = tok0 + 4 * g + r < p.t ? tok0 + 4 * g + r : p.t - 1;
+    at[r] = (((long)b * p.t + tr) * p.heads + h) * p.dv;
+  }
+  for (int c = i16; c < p.dv; c += 16)
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const float o = p.o[at[r] + c];
+      ss[r] = fmaf(o, o, ss[r]);
+    }
+#pragma unroll
+  for (int r = 0; r < 4; ++r) ss[r] = 1.f / sqrtf(row16_sum(ss[r]) / (float)p.dv + p.eps);
+  for (int c0 = 0; c0 < p.dv; c0 += 16) {
+    const int c = c0 + i16, cc = c < p.dv ? c : p.dv - 1;
+    const f32x4 z = low_rank_tile<T>(x, (const S*)p.g2 + ((long)h * p.dv + cc) * p.rg, p.rg, vec);
+    const float gain = T::one(((const S*)p.gain)[cc]);
+#pragma unroll
+    for (int r = 0; r < 4; ++r)
+      if (c < p.dv && tok0 + 4 * g + r < p.t) ((S*)p.y)[at[r] + c] = T::pack(p.o[at[r] + c] * ss[r] * gain * sigm(z[r]));
+  }
+}
+
+// ---------------------------------------------------------------------------------------
+// launchers
+// ---------------------------------------------------------------------------------------
+// what the chunk kernels cover
+constexpr int kMaxDeltaKey = 256, kMaxDeltaTaps = 8;
+static bool delta_chunked(int dk, int taps) { return dk <= kMaxDeltaKey && taps <= kMaxDeltaTaps; }
+static int delta_dkp(int dk) { return dk <= 64 ? 64 : (dk <= 128 ? 128 : 256); }
+
+template <typename T>
+static int launch_delta_step(hipStream_t s, const DeltaParams& p) {
+  int cgp = 16;
+  while (cgp * 4 < p.dv) cgp <<= 1;
+  if (cgp > kStepThreads) return MUI_ERR_UNSUPPORTED;
+  const int rows = ceil_div(p.dk, kStepThreads / cgp), parts = cgp <= 64 ? 8 : kStepThreads / cgp;
+  const size_t lds = ((size_t)3 * p.dk + 2 * p.dv + (p.ra > p.rg ? p.ra : p.rg) + 4 + (size_t)2 * parts * 4 * cgp) * 4;
+  const dim3 grid(p.heads, p.batch), block(kStepThreads);
+  auto launch = [&](auto kernel) {
+    if (lds > 160 * 1024) return (int)MUI_ERR_UNSUPPORTED;
+    if (lds > 48 * 1024 && hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
+      return (int)MUI_ERR_LAUNCH;
+    hipLaunchKernelGGL(kernel, grid, block, lds, s, p, cgp);
+    return launch_status();
+  };
+  if (rows <= 4) return launch(delta_step_kernel<T, 4>);
+  if (rows <= 8) return launch(delta_step_kernel<T, 8>);
+  if (rows <= 16) return launch(delta_step_kernel<T, 16>);
+  if (rows <= 32) return launch(delta_step_kernel<T, 32>);
+  return launch(delta_step_kernel<T, 0>);
+}
+
+template <typename T, int NB>
+static int launch_delta_chunks(hipStream_t s, const DeltaParams& p) {
+  if (p.heads > 65535 || p.batch > 65535) return MUI_ERR_UNSUPPORTED;
+  const size_t lds = (size_t)4 * kDChunk * kDPitch * 4;
+  const dim3 grid(p.chunks, p.heads, p.batch), block(256);
+  const int st = p.taps <= 4 ? launch_with_lds(delta_prepare_kernel<T, NB, 4>, grid, block, lds, s, p)
+                             : launch_with_lds(delta_prepare_kernel<T, NB, kMaxDeltaTaps>, grid, block, lds, s, p);
+  if (st != MUI_OK) return st;
+  hipLaunchKernelGGL((delta_scan_kernel<NB>), dim3(p.heads * (p.dvp / 16), p.batch), block, 0, s, p);
+  hipLaunchKernelGGL((delta_output_kernel<T>), grid, block, 0, s, p);
+  return launch_status();
+}
+
+template <typename T>
+static int launch_delta(hipStream_t s, const DeltaParams& p) {
+  if (p.chunks == 0) return launch_delta_step<T>(s, p);
+  if (p.dkp <= 64) return launch_delta_chunks<T, 1>(s, p);
+  if (p.dkp <= 128) return launch_delta_chunks<T, 2>(s, p);
+  return launch_delta_chunks<T, 4>(s, p);
+}
+
+// floats per (batch row, head, chunk) of the workspace, o apart
+static size_t delta_unit(int dkp, int dvp) { return (size_t)kDChunk * (3 * dkp + dvp + kDChunk) + dkp; }
+
+}  // namespace mui
+
+using namespace mui;
+
+extern "C" int mui_channel_delta_max_tokens(int dk, int taps) { return delta_chunked(dk, taps) ? (1 << 30) : MUI_MAX_TOKENS; }
+
+extern "C" int mui_channel_delta_ring_rows(int taps) { return taps - 1 + MUI_MAX_TOKENS; }
+
+extern "C" size_t mui_channel_delta_workspace_bytes(int batch, int t, int heads, int dk, int dv) {
+  if (batch < 1 || t <= MUI_MAX_TOKENS || heads < 1 || dk < 1 || dk > kMaxDeltaKey || dv < 1) return 0;
+  const int dkp = delta_dkp(dk), dvp = ceil_div(dv, 16) * 16;
+  return ((size_t)batch * heads * ceil_div(t, kDChunk) * delta_unit(dkp, dvp) + (size_t)batch * t * heads * dv) * 4;
+}
+
+extern "C" int mui_channel_delta(mui_stream_t stream, int dtype, const mui_channel_delta_t* d, const void* proj, long pitch,
+                                 float* state, void* ring, const int64_t* cache_position, const int64_t* row_start, void* y,
+                                 void* workspace, int batch, int t) {
+  MUI_CHECK_ARG(d && proj && state && ring && cache_position && y && batch > 0 && t > 0);
+  MUI_CHECK_ARG(d->conv && d->a2 && d->dt_bias && d->a_log && d->g2 && d->gain);
+  MUI_CHECK_ARG(d->heads > 0 && d->kv_heads > 0 && d->heads % d->kv_heads == 0 && d->dk > 0 && d->dv > 0 && d->ra > 0 && d->rg > 0 &&
+                d->taps > 0);
+  const long nq = (long)d->kv_heads * d->dk, nv = (long)d->heads * d->dv;
+  MUI_CHECK_ARG(d->q_offset >= 0 && d->k_offset >= 0 && d->v_offset >= 0 && d->a_offset >= 0 && d->g_offset >= 0 && d->b_offset >= 0);
+  MUI_CHECK_ARG(pitch >= d->q_offset + nq && pitch >= d->k_offset + nq && pitch >= d->v_offset + nv && pitch >= d->a_offset + d->ra &&
+                pitch >= d->g_offset + d->rg && pitch >= d->b_offset + d->heads);
+  if (batch > 65535 || !aligned16(state) || (long)batch * t * d->heads > (1L << 31) - 1) return MUI_ERR_UNSUPPORTED;
+  DeltaParams p = {};
+  p.proj = proj; p.pitch = pitch; p.q_off = d->q_offset; p.k_off = d->k_offset; p.v_off = d->v_offset; p.a_off = d->a_offset;
+  p.g_off = d->g_offset; p.b_off = d->b_offset; p.conv = d->conv; p.a2 = d->a2; p.dt_bias = d->dt_bias; p.a_log = d->a_log;
+  p.g2 = d->g2; p.gain = d->gain; p.q_scale = d->q_scale; p.eps = d->epsilon; p.s = state; p.ring = ring;
+  p.cache_position = cache_position; p.row_start = row_start; p.y = y; p.batch = batch; p.t = t; p.heads = d->heads;
+  p.kv_heads = d->kv_heads; p.dk = d->dk; p.dv = d->dv; p.ra = d->ra; p.rg = d->rg; p.taps = d->taps;
+  p.vec = aligned16(proj) && aligned16(d->a2) && aligned16(d->g2) && pitch % 8 == 0 && d->a_offset % 8 == 0 && d->g_offset % 8 == 0;
+  p.ring_rows = mui_channel_delta_ring_rows(d->taps); p.channels = (int)(2 * nq + nv);
+  if (t > MUI_MAX_TOKENS) {
+    if (!delta_chunked(d->dk, d->taps)) return MUI_ERR_UNSUPPORTED;
+    MUI_CHECK_ARG(workspace);
+    if (!aligned16(workspace)) return MUI_ERR_ALIGNMENT;
+    p.chunks = ceil_div(t, kDChunk);
+    p.dkp = delta_dkp(d->dk);
+    p.dvp = ceil_div(d->dv, 16) * 16;
+    const size_t units = (size_t)batch * d->heads * p.chunks;
+    p.qe = (float*)workspace;
+    p.w = p.qe + units * kDChunk * p.dkp;
+    p.kd = p.w + units * kDChunk * p.dkp;
+    p.u0 = p.kd + units * kDChunk * p.dkp;
+    p.aqk = p.u0 + units * kDChunk * p.dvp;
+    p.gc = p.aqk + units * kDChunk * kDChunk;
+    p.o = p.gc + units * p.dkp;
+  }
+  hipStream_t s = (hipStream_t)stream;
+  if (dtype == MUI_DTYPE_F16) return launch_delta<F16>(s, p);
+  if (dtype == MUI_DTYPE_BF16) return launch_delta<BF16>(s, p);
+  if (dtype == MUI_DTYPE_F32) return launch_delta<F32>(s, p);
+  return MUI_ERR_INVALID_ARG;
+}

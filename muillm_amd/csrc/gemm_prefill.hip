@@ -775,7 +775,12 @@ __device__ __forceinline__ void prefill_gemm_tile(const PrefillGemmParams& p, co
             for (int e = 0; e < 4; ++e) {
               const int oe = ow0 + 16 * i + 4 * ag + e;
               if constexpr (EPI == SK_GATEUP) {
-                v[e] = gateup_f32(acc[i][j][e], acc[i + OT][j][e]);
+                float g = acc[i][j][e], u = acc[i + OT][j][e];
+                if (p.add_bias) {
+                  g += T::one(p.add_bias[oe]);
+                  u += T::one(p.mul_bias[oe]);
+                }
+                v[e] = gateup_f32(g, u);
               } else {
                 float r = acc[i][j][e];
                 if (p.mul_bias) r *= T::one(p.mul_bias[oe]);
@@ -854,6 +859,10 @@ __device__ __forceinline__ void prefill_gemm_tile(const PrefillGemmParams& p, co
           if constexpr (WF == WF_I8_CHANNEL) {
             g *= T::one(p.s0[(long)oe * p.s_pitch]);
             u *= T::one(p.s1[(long)oe * p.s_pitch]);
+          }
+          if (p.add_bias) {
+            g += T::one(p.add_bias[oe]);
+            u += T::one(p.mul_bias[oe]);
           }
           v[e] = gateup_f32(g, u);
         } else {
@@ -1144,6 +1153,10 @@ static int launch_prefill_t(hipStream_t s, const PrefillGemmParams& p) {
           b.w0 += (long)a.n * p.pitch;
           b.w1 += (long)a.n * p.pitch;
           b.y += a.n;
+          if (p.add_bias) {
+            b.add_bias += a.n;
+            b.mul_bias += a.n;
+          }
           int st = g_prefill_stages3_big ? launch_prefill_cfg<T, WF, EPI, 4, 8, 4, 2, 1, 64, 3, true>(s, a)
                                          : launch_prefill_cfg<T, WF, EPI, 4, 8, 4, 2, 1, 64, 2, true>(s, a);
           if (st == MUI_OK) st = g_prefill_stages3 ? launch_prefill_cfg<T, WF, EPI, 4, 4, 2, 4, 1, 64, 3, true>(s, b)

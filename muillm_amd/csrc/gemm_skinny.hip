@@ -176,6 +176,10 @@ __global__ void __launch_bounds__(kSkThreads) gemm_skinny_kernel(const SkinnyPar
           gt *= T::one(p.s0[(long)n * p.s_pitch]);
           up *= T::one(p.s1[(long)n * p.s_pitch]);
         }
+        if (p.add_bias) {
+          gt += T::one(p.add_bias[n]);
+          up += T::one(p.mul_bias[n]);
+        }
         v = silu_f32(gt) * up;
       } else {
         v = total(i) * rs;
@@ -312,6 +316,10 @@ __global__ void __launch_bounds__(kSkThreads) gemm_skinny_bstat_kernel(const Ski
           if constexpr (WF == WF_I8_CHANNEL) {
             gt *= T::one(p.s0[(long)n * p.s_pitch]);
             up *= T::one(p.s1[(long)n * p.s_pitch]);
+          }
+          if (p.add_bias) {
+            gt += T::one(p.add_bias[n]);
+            up += T::one(p.mul_bias[n]);
           }
           v = silu_f32(gt) * up;
         } else {

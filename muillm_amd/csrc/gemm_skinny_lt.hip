@@ -269,6 +269,10 @@ __global__ void __launch_bounds__(kLtThreads) gemm_skinny_lt_kernel(
           gt *= T::one((uint16_t)ex.sc0);
           up *= T::one((uint16_t)ex.sc1);
         }
+        if (p.add_bias) {
+          gt += T::one(p.add_bias[nn]);
+          up += T::one(p.mul_bias[nn]);
+        }
         v = silu_f32(gt) * up;
       } else {
         v = v0 * ep_rs;

@@ -189,6 +189,10 @@ __global__ void __launch_bounds__(kWideThreads) gemm_wide_kernel(const WideParam
         g *= T::one(p.s0[(long)o * p.s_pitch]);
         u *= T::one(p.s1[(long)o * p.s_pitch]);
       }
+      if (p.add_bias) {
+        g += T::one(p.add_bias[o]);
+        u += T::one(p.mul_bias[o]);
+      }
       v = silu_f32(g) * u;
     } else {
       v = total(r);

@@ -96,13 +96,13 @@ __global__ void __launch_bounds__(kThreads) gemv_kernel(const uint16_t* a_w0, co
 
   // epilogue operands (biases, residual) of a row group are fetched together with its
   // weights, one group ahead, so no dependent global load sits behind the final barrier
-  float e_mb = 1.f, e_ab = 0.f, e_res = 0.f;
+  float e_mb = EPI == EPI_LINEAR ? 1.f : 0.f, e_ab = 0.f, e_res = 0.f;
   auto issue_epi = [&](int rg) {
-    if constexpr (EPI == EPI_LINEAR) {
+    if (EPI == EPI_LINEAR || p.add_bias) {  // (gate/up: the biases of the up and of the gate rows)
       if (t < OUT) {
         int n = rg * OUT + t;
         n = n < p.n ? n : p.n - 1;
-        e_mb = p.mul_bias ? T::one(p.mul_bias[n]) : 1.f;
+        e_mb = p.mul_bias ? T::one(p.mul_bias[n]) : e_mb;
         e_ab = p.add_bias ? T::one(p.add_bias[n]) : 0.f;
         e_res = p.residual ? T::one(p.residual[n]) : 0.f;
       }
@@ -192,7 +192,7 @@ __global__ void __launch_bounds__(kThreads) gemv_kernel(const uint16_t* a_w0, co
           const int rg_ = 2 * t, ru_ = 2 * t + 1;
           const float g = ((red[buf][0][rg_] + red[buf][1][rg_]) + (red[buf][2][rg_] + red[buf][3][rg_])) * rs;
           const float u = ((red[buf][0][ru_] + red[buf][1][ru_]) + (red[buf][2][ru_] + red[buf][3][ru_])) * rs;
-          v = silu_f32(g) * u;
+          v = silu_f32(g + c_ab) * (u + c_mb);
         } else {
           v = ((red[buf][0][t] + red[buf][1][t]) + (red[buf][2][t] + red[buf][3][t])) * rs;
           v = fmaf(v, c_mb, c_ab) + c_res;
@@ -396,7 +396,14 @@ extern "C" int mui_linear_ws(mui_stream_t stream, int dtype, const void* weights
 extern "C" int mui_gateup_silu(mui_stream_t stream, int dtype, const void* gate, const void* up,
                                long gu_pitch, const void* x, const void* norm_weights,
                                float epsilon, void* h, int n_inter, int k_in, int tokens) {
-  MUI_CHECK_ARG(gate && up && x && h);
+  return mui_gateup_silu_bias(stream, dtype, gate, up, gu_pitch, x, norm_weights, epsilon, nullptr, nullptr, h, n_inter,
+                              k_in, tokens);
+}
+
+extern "C" int mui_gateup_silu_bias(mui_stream_t stream, int dtype, const void* gate, const void* up, long gu_pitch,
+                                    const void* x, const void* norm_weights, float epsilon, const void* gate_bias,
+                                    const void* up_bias, void* h, int n_inter, int k_in, int tokens) {
+  MUI_CHECK_ARG(gate && up && x && h && (gate_bias == nullptr) == (up_bias == nullptr));
   MUI_CHECK_ARG(n_inter > 0 && k_in > 0 && tokens > 0);
   MUI_CHECK_ARG(dtype == MUI_DTYPE_F16 || dtype == MUI_DTYPE_BF16);
   if (gu_pitch < k_in) return MUI_ERR_INVALID_ARG;
@@ -411,6 +418,7 @@ extern "C" int mui_gateup_silu(mui_stream_t stream, int dtype, const void* gate,
     sp.w0 = gate; sp.w1 = up; sp.pitch = gu_pitch; sp.x = (const uint16_t*)x;
     sp.gamma = (const uint16_t*)norm_weights; sp.y = (uint16_t*)h; sp.n = n_inter; sp.k = k_in;
     sp.tokens = tokens; sp.eps = epsilon;
+    sp.add_bias = (const uint16_t*)gate_bias; sp.mul_bias = (const uint16_t*)up_bias;
     return launch_prefill_gemm(s, dtype, WF_16BIT, SK_GATEUP, sp);
   }
   // bf16 has no mixed-precision fma: a single bf16 token takes the packed-dot kernel here too
@@ -426,6 +434,8 @@ extern "C" int mui_gateup_silu(mui_stream_t stream, int dtype, const void* gate,
     sp.k = k_in;
     sp.tokens = tokens;
     sp.eps = epsilon;
+    sp.add_bias = (const uint16_t*)gate_bias;
+    sp.mul_bias = (const uint16_t*)up_bias;
     if (tokens <= g_multi_max_tokens) {
       const int st = launch_gemv_multi(s, dtype, SK_GATEUP, sp);
       if (st != MUI_ERR_UNSUPPORTED) return st;
@@ -440,7 +450,9 @@ extern "C" int mui_gateup_silu(mui_stream_t stream, int dtype, const void* gate,
     p.pitch = gu_pitch;
     p.x = (const uint16_t*)x + (long)tkn * k_in;
     p.gamma = (const uint16_t*)norm_weights;
-    p.mul_bias = p.add_bias = p.residual = nullptr;
+    p.add_bias = (const uint16_t*)gate_bias;
+    p.mul_bias = (const uint16_t*)up_bias;
+    p.residual = nullptr;
     p.y = (uint16_t*)h + (long)tkn * n_inter;
     p.n = n_inter;
     p.k = k_in;

@@ -216,7 +216,13 @@ __global__ void __launch_bounds__(kMtThreads) gemv_multi_kernel(
           for (int i = 1; i < TOK; ++i) rsv = (tk == i) ? rs[i] : rsv;
           float v;
           if constexpr (EPI == SK_GATEUP) {
-            v = silu_f32(v0 * rsv) * (v1 * rsv);
+            v0 *= rsv;
+            v1 *= rsv;
+            if (add_bias) {
+              v0 += T::one(add_bias[row]);
+              v1 += T::one(mul_bias[row]);
+            }
+            v = silu_f32(v0) * v1;
           } else {
             v = v0 * rsv;
             if (mul_bias) v *= T::one(mul_bias[row]);
@@ -268,7 +274,13 @@ __global__ void __launch_bounds__(kMtThreads) gemv_multi_kernel(
           for (int i = 1; i < TOK; ++i) rsv = (tk == i) ? rs[i] : rsv;
           float v;
           if constexpr (EPI == SK_GATEUP) {
-            v = silu_f32(v0 * rsv) * (v1 * rsv);
+            v0 *= rsv;
+            v1 *= rsv;
+            if (add_bias) {
+              v0 += T::one(add_bias[row]);
+              v1 += T::one(mul_bias[row]);
+            }
+            v = silu_f32(v0) * v1;
           } else {
             v = v0 * rsv;
             if (mul_bias) v *= T::one(mul_bias[row]);

@@ -36,6 +36,51 @@ __global__ void __launch_bounds__(256) embedding_kernel(const uint16_t* table, l
 }
 
 // ---------------------------------------------------------------------------------------
+// token embedding plus bigram embedding: x = scale * table[id] + bigram[(prev * mul_prev + id * mul_cur) mod buckets],
+// the last row (number `buckets`) for the first token of a sequence; x in fp32 and, rounded, as the first
+// sublayer's input. One workgroup per token; the one of a row's first token reads and replaces prev[row].
+// ---------------------------------------------------------------------------------------
+struct BigramParams {
+  const int64_t* ids; int64_t* prev; const int64_t* cache_position; const int64_t* row_start;
+  const void *table, *bigram; float* x; void* h;
+  long mul_prev, mul_cur; float scale; int t, width, vocab, buckets;
+};
+
+template <typename T>
+__global__ void __launch_bounds__(256) bigram_embedding_kernel(const BigramParams p) {
+  typedef typename T::storage S;
+  const int tok = blockIdx.x, b = tok / p.t, tt = tok - b * p.t;
+  auto clamped = [&](long id) { return id < 0 ? 0L : (id >= p.vocab ? (long)p.vocab - 1 : id); };
+  const long id = clamped(p.ids[tok]), last = clamped(tt > 0 ? p.ids[tok - 1] : p.prev[b]);
+  const bool first = p.cache_position[tt] <= (p.row_start ? p.row_start[b] : 0);
+  const long row = first ? p.buckets : (last * p.mul_prev + id * p.mul_cur) % p.buckets;
+  if (tt == 0) {
+    __syncthreads();  // every thread has read prev[b]
+    if (threadIdx.x == 0) p.prev[b] = p.ids[tok + p.t - 1];
+  }
+  const S *e = (const S*)p.table + id * p.width, *g = (const S*)p.bigram + row * p.width;
+  float* x = p.x + (long)tok * p.width;
+  S* h = (S*)p.h + (long)tok * p.width;
+  if ((p.width & 7) == 0 && (((uintptr_t)p.table | (uintptr_t)p.bigram | (uintptr_t)p.x | (uintptr_t)p.h) & 15u) == 0) {
+    for (int c = threadIdx.x * 8; c < p.width; c += 256 * 8) {
+      float a[8], u[8];
+      load8<T>(e + c, a);
+      load8<T>(g + c, u);
+#pragma unroll
+      for (int i = 0; i < 8; ++i) a[i] = fmaf(a[i], p.scale, u[i]);
+      store8<F32>(x + c, a);
+      store8<T>(h + c, a);
+    }
+  } else {
+    for (int c = threadIdx.x; c < p.width; c += 256) {
+      const float a = fmaf(T::one(e[c]), p.scale, T::one(g[c]));
+      x[c] = a;
+      h[c] = T::pack(a);
+    }
+  }
+}
+
+// ---------------------------------------------------------------------------------------
 // Philox4x32-10 (Salmon et al., "Parallel random numbers: as easy as 1, 2, 3", SC'11)
 // ---------------------------------------------------------------------------------------
 struct Philox4 { uint32_t x, y, z, w; };
@@ -169,5 +214,21 @@ extern "C" int mui_sample_advance(mui_stream_t stream, int dtype, const void* lo
     hipLaunchKernelGGL((sample_advance_kernel<BF16>), dim3(rows), dim3(kSampleThreads), 0, s, p);
   else
     return MUI_ERR_INVALID_ARG;
+  return launch_status();
+}
+
+extern "C" int mui_bigram_embedding(mui_stream_t stream, int dtype, const int64_t* ids, int64_t* prev,
+                                    const int64_t* cache_position, const int64_t* row_start, const void* table,
+                                    const void* bigram, float scale, long mul_prev, long mul_cur, int buckets, float* x,
+                                    void* h, int batch, int t, int width, int vocab) {
+  MUI_CHECK_ARG(ids && prev && cache_position && table && bigram && x && h && batch > 0 && t > 0 && width > 0 && vocab > 0);
+  MUI_CHECK_ARG(buckets > 0 && mul_prev >= 0 && mul_cur >= 0 && (long)batch * t < (1L << 31));
+  const BigramParams p = {ids, prev, cache_position, row_start, table, bigram, x, h, mul_prev, mul_cur, scale, t, width, vocab, buckets};
+  const dim3 grid(batch * t), block(256);
+  hipStream_t s = (hipStream_t)stream;
+  if (dtype == MUI_DTYPE_F16) hipLaunchKernelGGL((bigram_embedding_kernel<F16>), grid, block, 0, s, p);
+  else if (dtype == MUI_DTYPE_BF16) hipLaunchKernelGGL((bigram_embedding_kernel<BF16>), grid, block, 0, s, p);
+  else if (dtype == MUI_DTYPE_F32) hipLaunchKernelGGL((bigram_embedding_kernel<F32>), grid, block, 0, s, p);
+  else return MUI_ERR_INVALID_ARG;
   return launch_status();
 }

@@ -16,7 +16,7 @@
 //
 // Positions: a token's slot in the cache minus its row's first slot (left-padded batches). Angles are
 // formed and reduced in double precision and rounded to fp32 once: no table, no longest sequence.
-#include "skinny.cuh"
+#include "hybrid.cuh"
 
 namespace mui {
 
@@ -49,21 +49,6 @@ struct LatentParams {
   const void* kv;    // prefill: [keys, heads * (dim + vdim)], key row 0 = slot kv_first
   int kv_first, kv_rows, q_first, b0;
 };
-
-// cos and sin of pos * inv_freq: the angle in turns, its whole turns dropped in double precision, rounded once
-__device__ __forceinline__ void rope_angle(double pos, double inv_freq, float& c, float& s) {
-  double a = pos * inv_freq * 0.15915494309189533576888376337251;
-  a -= rint(a);
-  sincospif((float)(2.0 * a), &s, &c);
-}
-
-__device__ __forceinline__ float block_sum256(float v, float* red) {
-  v = wave_sum(v);
-  __syncthreads();
-  if ((threadIdx.x & (kWave - 1)) == 0) red[threadIdx.x >> 6] = v;
-  __syncthreads();
-  return (red[0] + red[1]) + (red[2] + red[3]);
-}
 
 // ---------------------------------------------------------------------------------------
 // prepare: one workgroup per token
@@ -298,15 +283,6 @@ __global__ void __launch_bounds__(256) latent_absorb_kernel(const LatentParams p
                      : (uint16_t)0;
     }
   }
-}
-
-// LDS tiles filled by LDS-direct loads: blocks of 64 columns, in a block rows of 128 bytes whose 16-byte chunk c
-// lives at chunk c ^ ((row >> 1) & 7) (16 rows of one logical chunk fall into 64 different banks). A wave
-// instruction delivers eight rows of one block.
-__device__ __forceinline__ int tile_swz(int row) { return (row >> 1) & 7; }
-template <int ROWS>
-__device__ __forceinline__ int tile_at(int row, int col) {  // in elements
-  return ((col >> 6) * ROWS + row) * 64 + ((((col >> 3) & 7) ^ tile_swz(row)) << 3) + (col & 7);
 }
 
 // Splits of token tok that hold visible keys: the grid covers the largest span, the rest leave at once

@@ -17,7 +17,7 @@
 //           D: column lane % 16, rows 4 (lane / 16) + r).
 //   output  a head's o divided by its root mean square, times a gain, times sigmoid of the output gate.
 // Tokens in front of a row's first slot (left padding) leave the state alone.
-#include "common.cuh"
+#include "hybrid.cuh"
 
 namespace mui {
 
@@ -203,10 +203,6 @@ __device__ __forceinline__ void load_tile(float* dst, int pitch, const typename 
   }
 #pragma unroll
   for (int i = 0; i < 4; ++i) *(f32x4*)&dst[(r0 + 16 * i) * pitch + k] = v[i];
-}
-
-__device__ __forceinline__ f32x4 mfma_f32(float a, float b, f32x4 c) {
-  return __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, 0, 0, 0);
 }
 
 // 1. contribution of a chunk: grid (chunks, heads * dk tiles * dv tiles, batch)

@@ -1,8 +1,8 @@
 // The boundary between two sublayers of a decoder whose residual stream is fp32 and whose sublayers
 // are normalised on both sides (a norm on the sublayer's output before it joins the residual, a
 // norm on the residual before the next sublayer):
-//   x <- x + post_gain * y * rsqrt(mean(y^2) + eps)
-//   h  = next_gain * x * rsqrt(mean(x^2) + eps)
+//   x <- x + branch_scale * post_gain * y * rsqrt(mean(y^2) + eps)
+//   h  = next_scale * next_gain * x * rsqrt(mean(x^2) + eps), or next_scale * x without a gain
 // in one launch: y is read once, x is read and written once, h leaves in the activations' type. The
 // first sublayer's input takes the same kernel without a post norm (x = scale * embedding row).
 // Where the sublayer is a mixture of experts, y is summed up on the fly from the chosen experts'
@@ -18,10 +18,12 @@ struct ResidualNormParams {
   const void* y;             // [rows, k] (dense sublayer output), activations' type
   float y_scale;
   const void* post_gain;  // [k] or null: y joins the residual as y_scale * y
-  const void* next_gain;  // [k] or null: no h
+  float branch_scale;     // on the normed y
+  const void* next_gain;  // [k] or null: h is the sum itself
+  float next_scale;
   float eps;
   float* residual_out;  // [rows, k], may be residual_in
-  void* h;              // [rows, k]
+  void* h;              // [rows, k] or null
   int k;
   // mixture of experts: y[r] = sum_j weight[r, j] * (expert[r, j] < n_experts ? pairs[r * top + j] : identity[r])
   const void* pairs;
@@ -107,7 +109,7 @@ __global__ void __launch_bounds__(kRnThreads) residual_norm_vec_kernel(const Res
         float g[8];
         load8<T>((const S*)p.post_gain + (c << 3), g);
 #pragma unroll
-        for (int i = 0; i < 8; ++i) x[j][i] = fmaf(g[i], y[j][i] * rs, x[j][i]);
+        for (int i = 0; i < 8; ++i) x[j][i] = fmaf(g[i] * p.branch_scale, y[j][i] * rs, x[j][i]);
       }
     }
   } else {
@@ -126,14 +128,19 @@ __global__ void __launch_bounds__(kRnThreads) residual_norm_vec_kernel(const Res
       for (int i = 0; i < 8; ++i) ss = fmaf(x[j][i], x[j][i], ss);
     }
   }
-  if (!p.next_gain) return;
-  const float rs = rsqrtf(rn_block_sum(ss, red) / (float)p.k + p.eps);
+  if (!p.h) return;
+  const float rs = p.next_gain ? rsqrtf(rn_block_sum(ss, red) / (float)p.k + p.eps) * p.next_scale : p.next_scale;
 #pragma unroll
   for (int j = 0; j < CH; ++j) {
     const int c = t + kRnThreads * j;
     if (c < kc) {
       float g[8], o[8];
-      load8<T>((const S*)p.next_gain + (c << 3), g);
+      if (p.next_gain) {
+        load8<T>((const S*)p.next_gain + (c << 3), g);
+      } else {
+#pragma unroll
+        for (int i = 0; i < 8; ++i) g[i] = 1.f;
+      }
 #pragma unroll
       for (int i = 0; i < 8; ++i) o[i] = g[i] * (x[j][i] * rs);
       store8<T>((S*)p.h + base + (c << 3), o);
@@ -175,14 +182,14 @@ __global__ void __launch_bounds__(kRnThreads) residual_norm_any_kernel(const Res
   for (int i = t; i < p.k; i += kRnThreads) {
     float x = p.residual_in ? p.residual_in[base + i] : 0.f;
     const float y = y_at(i);
-    x = p.post_gain ? fmaf(T::one(((const S*)p.post_gain)[i]), y * rs, x) : x + y;
+    x = p.post_gain ? fmaf(T::one(((const S*)p.post_gain)[i]) * p.branch_scale, y * rs, x) : x + y;
     p.residual_out[base + i] = x;
     ss = fmaf(x, x, ss);
   }
-  if (!p.next_gain) return;
-  rs = rsqrtf(rn_block_sum(ss, red) / (float)p.k + p.eps);
+  if (!p.h) return;
+  rs = p.next_gain ? rsqrtf(rn_block_sum(ss, red) / (float)p.k + p.eps) * p.next_scale : p.next_scale;
   for (int i = t; i < p.k; i += kRnThreads)
-    ((S*)p.h)[base + i] = T::pack(T::one(((const S*)p.next_gain)[i]) * (p.residual_out[base + i] * rs));
+    ((S*)p.h)[base + i] = T::pack((p.next_gain ? T::one(((const S*)p.next_gain)[i]) : 1.f) * (p.residual_out[base + i] * rs));
 }
 
 template <typename T, bool MOE>
@@ -217,25 +224,24 @@ static int dispatch_residual_norm(mui_stream_t stream, int dtype, const Residual
 using namespace mui;
 
 extern "C" int mui_residual_norm(mui_stream_t stream, int dtype, const float* residual_in, const void* y, float y_scale,
-                                 const void* post_gain, const void* next_gain, float epsilon, float* residual_out,
-                                 void* h, int rows, int k) {
-  MUI_CHECK_ARG(y && residual_out && rows > 0 && k > 0);
-  MUI_CHECK_ARG((next_gain == nullptr) == (h == nullptr));
+                                 const void* post_gain, float branch_scale, const void* next_gain, float next_scale,
+                                 float epsilon, float* residual_out, void* h, int rows, int k) {
+  MUI_CHECK_ARG(y && residual_out && rows > 0 && k > 0 && (h || !next_gain));
   ResidualNormParams p = {};
   p.residual_in = residual_in; p.y = y; p.y_scale = y_scale; p.post_gain = post_gain; p.next_gain = next_gain;
-  p.eps = epsilon; p.residual_out = residual_out; p.h = h; p.k = k;
+  p.branch_scale = branch_scale; p.next_scale = next_scale; p.eps = epsilon; p.residual_out = residual_out; p.h = h; p.k = k;
   return dispatch_residual_norm<false>(stream, dtype, p, rows);
 }
 
 extern "C" int mui_moe_residual_norm(mui_stream_t stream, int dtype, const float* residual_in, const void* pair_out,
                                      const void* identity_in, const int32_t* expert, const float* weight, int n_experts,
-                                     int top, const void* post_gain, const void* next_gain, float epsilon,
-                                     float* residual_out, void* h, int rows, int k) {
+                                     int top, const void* post_gain, float branch_scale, const void* next_gain,
+                                     float next_scale, float epsilon, float* residual_out, void* h, int rows, int k) {
   MUI_CHECK_ARG(pair_out && identity_in && expert && weight && residual_out && rows > 0 && k > 0);
-  MUI_CHECK_ARG(n_experts >= 0 && top > 0 && (next_gain == nullptr) == (h == nullptr));
+  MUI_CHECK_ARG(n_experts >= 0 && top > 0 && (h || !next_gain));
   ResidualNormParams p = {};
   p.residual_in = residual_in; p.y_scale = 1.f; p.post_gain = post_gain; p.next_gain = next_gain;
-  p.eps = epsilon; p.residual_out = residual_out; p.h = h; p.k = k;
+  p.branch_scale = branch_scale; p.next_scale = next_scale; p.eps = epsilon; p.residual_out = residual_out; p.h = h; p.k = k;
   p.pairs = pair_out; p.identity = identity_in; p.expert = expert; p.weight = weight; p.n_experts = n_experts; p.top = top;
   return dispatch_residual_norm<true>(stream, dtype, p, rows);
 }

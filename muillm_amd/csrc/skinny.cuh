@@ -19,8 +19,8 @@ struct SkinnyParams {
   const uint16_t* x;    // [tokens, k], token rows x_pitch elements apart (0: k)
   long x_pitch;         // honoured by the 1..4-token kernels (their K-segment calls); others need 0
   const uint16_t* gamma;
-  const uint16_t* mul_bias;
-  const uint16_t* add_bias;
+  const uint16_t* mul_bias;  // gate/up: the up rows' bias (both biases or none)
+  const uint16_t* add_bias;  // gate/up: the gate rows' bias
   const uint16_t* residual;  // [tokens, n]
   uint16_t* y;               // [tokens, n]
   int n;       // outputs (weight rows, or gate/up pairs)

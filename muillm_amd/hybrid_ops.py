@@ -1,10 +1,11 @@
-"""Operators of the sandwich-norm / latent-attention / recurrent / mixture-of-experts section of the C ABI
+"""Operators of the section of the C ABI for hybrid decoders (norms around sublayers, attention, recurrences, experts)
 (include/muillm_amd.h), in the manner of muillm_ext.py: validate, allocate outputs with torch, hand raw
 pointers and the current stream to the library. Activations and weights are fp16, bf16 or fp32 tensors of
 one dtype; the residual stream, router logits, recurrence gates and state are fp32."""
 
 from __future__ import annotations
 
+import ctypes
 from dataclasses import dataclass
 from typing import List, Optional, Tuple
 
@@ -69,10 +70,12 @@ class MoEOutput:
 
 
 def residual_norm(residual: Optional[torch.Tensor], y, post_gain: Optional[torch.Tensor],
-                  next_gain: Optional[torch.Tensor], eps: float, y_scale: float = 1.0) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
-    """(residual + norm_post(y), norm_next of that): the boundary between two sublayers. residual fp32
-    [..., width] or None (zero), updated in place; y a tensor [..., width] or a MoEOutput; a gain that is
-    None skips its norm (no second result without next_gain)."""
+                  next_gain: Optional[torch.Tensor], eps: float, y_scale: float = 1.0, branch_scale: float = 1.0,
+                  next_scale: float = 1.0, emit: bool = False) -> Tuple[torch.Tensor, Optional[torch.Tensor]]:
+    """(residual + branch_scale norm_post(y), next_scale norm_next of that): the boundary between two sublayers.
+    residual fp32 [..., width] or None (zero), updated in place; y a tensor [..., width] or a MoEOutput; a gain
+    that is None skips its norm: without post_gain y_scale * y joins as it is, without next_gain the second
+    result is the (scaled) sum itself, rounded, where emit asks for it, and None otherwise."""
     moe = isinstance(y, MoEOutput)
     src = y.identity if moe else y
     width = src.shape[-1]
@@ -87,7 +90,7 @@ def residual_norm(residual: Optional[torch.Tensor], y, post_gain: Optional[torch
         raise RuntimeError("residual and sublayer output differ in size")
     _operand(post_gain, "post_gain", src, (width,))
     _operand(next_gain, "next_gain", src, (width,))
-    h = None if next_gain is None else torch.empty_like(src)
+    h = torch.empty_like(src) if emit or next_gain is not None else None
     if rows == 0:
         return out, h
     lib, code = _lib.load(), dtype_code(src.dtype)
@@ -98,12 +101,12 @@ def residual_norm(residual: Optional[torch.Tensor], y, post_gain: Optional[torch
         _operand(y.weight, "weight", src, (rows, top), torch.float32)
         check(lib.mui_moe_residual_norm(_stream(src), code, _ptr(residual), y.pairs.data_ptr(), src.data_ptr(),
                                         y.expert.data_ptr(), y.weight.data_ptr(), y.n_experts, top, _ptr(post_gain),
-                                        _ptr(next_gain), float(eps), out.data_ptr(), _ptr(h), rows, width),
-              "mui_moe_residual_norm")
+                                        float(branch_scale), _ptr(next_gain), float(next_scale), float(eps), out.data_ptr(),
+                                        _ptr(h), rows, width), "mui_moe_residual_norm")
     else:
         check(lib.mui_residual_norm(_stream(src), code, _ptr(residual), src.data_ptr(), float(y_scale), _ptr(post_gain),
-                                    _ptr(next_gain), float(eps), out.data_ptr(), _ptr(h), rows, width),
-              "mui_residual_norm")
+                                    float(branch_scale), _ptr(next_gain), float(next_scale), float(eps), out.data_ptr(), _ptr(h),
+                                    rows, width), "mui_residual_norm")
     return out, h
 
 
@@ -320,4 +323,172 @@ def mlstm_output(o: torch.Tensor, gain: torch.Tensor, gate: torch.Tensor, eps: f
     check(_lib.load().mui_mlstm_output(_stream(gate), dtype_code(gate.dtype), o.data_ptr(), gain.data_ptr(),
                                        gate.data_ptr(), gate.stride(1), float(eps), y.data_ptr(), b * t, heads, dv),
           "mui_mlstm_output")
+    return y
+
+
+# --------------------------------------------------------------------------------------
+# token plus bigram embedding
+# --------------------------------------------------------------------------------------
+def bigram_embedding(ids: torch.Tensor, prev: torch.Tensor, cache_position: torch.Tensor, row_start: Optional[torch.Tensor],
+                     table: torch.Tensor, bigram: torch.Tensor, scale: float, mul_prev: int, mul_cur: int):
+    """(x fp32, h in the table's dtype) [B, T, width]: scale * table row + bigram row of (previous, current) token; prev
+    int64 [B'] holds the ids in front of this call's first tokens and takes its last ones. bigram [buckets + 1, width]."""
+    b, t = ids.shape
+    vocab, width = table.shape
+    ids = ids.to(torch.int64).contiguous()
+    _operand(table, "table", table)
+    _operand(bigram, "bigram", table, (bigram.shape[0], width))
+    _operand(ids, "ids", table, None, torch.int64)
+    _operand(prev, "prev", table, None, torch.int64)
+    _positions(cache_position, row_start, table, b, t)
+    if b > prev.numel():
+        raise RuntimeError("more batch rows than the state has")
+    x = torch.empty((b, t, width), dtype=torch.float32, device=table.device)
+    h = torch.empty((b, t, width), dtype=table.dtype, device=table.device)
+    check(_lib.load().mui_bigram_embedding(_stream(table), dtype_code(table.dtype), ids.data_ptr(), prev.data_ptr(),
+                                           cache_position.data_ptr(), _ptr(row_start), table.data_ptr(), bigram.data_ptr(),
+                                           float(scale), mul_prev, mul_cur, bigram.shape[0] - 1, x.data_ptr(), h.data_ptr(),
+                                           b, t, width, vocab), "mui_bigram_embedding")
+    return x, h
+
+
+# --------------------------------------------------------------------------------------
+# grouped-query attention over cached rows
+# --------------------------------------------------------------------------------------
+def hybrid_prepare(proj: torch.Tensor, heads: int, kv_heads: int, dim: int, vdim: int, q_gain: Optional[torch.Tensor],
+                   k_gain: Optional[torch.Tensor], eps: float, inv_freq: torch.Tensor, cache_position: torch.Tensor,
+                   row_start: Optional[torch.Tensor], k_cache: torch.Tensor, v_cache: torch.Tensor) -> torch.Tensor:
+    """Normed and rotated queries [B, T, heads * dim]; keys and values go to their cache slots. proj [B, T, .] starts
+    with q | k | v; caches [B', capacity, kv_heads * dim | kv_heads * vdim]; inv_freq double [rotated dims / 2]."""
+    b, t, pitch = proj.shape
+    nq, nk, nv = heads * dim, kv_heads * dim, kv_heads * vdim
+    if pitch < nq + nk + nv:
+        raise RuntimeError("the projection has too few columns")
+    _operand(proj, "proj", proj)
+    _operand(q_gain, "q_gain", proj, (nq,))
+    _operand(k_gain, "k_gain", proj, (nk,))
+    _operand(inv_freq, "inv_freq", proj, None, torch.float64)
+    _operand(k_cache, "k_cache", proj, (k_cache.shape[0], k_cache.shape[1], nk))
+    _operand(v_cache, "v_cache", proj, (k_cache.shape[0], k_cache.shape[1], nv))
+    _positions(cache_position, row_start, proj, b, t)
+    if b > k_cache.shape[0]:
+        raise RuntimeError("more batch rows than the cache has")
+    q = torch.empty((b, t, nq), dtype=proj.dtype, device=proj.device)
+    check(_lib.load().mui_hybrid_prepare(_stream(proj), dtype_code(proj.dtype), proj.data_ptr(), pitch, nq, nq + nk, _ptr(q_gain),
+                                         _ptr(k_gain), float(eps), inv_freq.data_ptr(), 2 * inv_freq.numel(),
+                                         cache_position.data_ptr(), _ptr(row_start), q.data_ptr(), k_cache.data_ptr(),
+                                         k_cache.stride(0), v_cache.data_ptr(), v_cache.stride(0), b, t, heads, kv_heads, dim,
+                                         vdim, k_cache.shape[1]), "mui_hybrid_prepare")
+    return q
+
+
+def hybrid_route(dtype: torch.dtype, tokens: int, dim: int, vdim: int) -> int:
+    return _lib.load().mui_hybrid_attention_route(dtype_code(dtype), tokens, dim, vdim)
+
+
+def hybrid_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, gate: Optional[torch.Tensor],
+                     cache_position: torch.Tensor, row_start: Optional[torch.Tensor], heads: int, kv_heads: int, scale: float,
+                     softcap: float = 0.0, window: int = 0, keep_first: int = 0, route: Optional[int] = None) -> torch.Tensor:
+    """[B, T, heads * vdim]: attention of q [B, T, heads * dim] over the caches, which hold the new tokens already, times
+    sigmoid(gate); gate: a column slice [B, T, heads * vdim] of a projection's output, or None."""
+    b, t = q.shape[0], q.shape[1]
+    cap, dim, vdim = k_cache.shape[1], k_cache.shape[2] // kv_heads, v_cache.shape[2] // kv_heads
+    _operand(q, "q", q, (b, t, heads * dim))
+    _operand(k_cache, "k_cache", q, (k_cache.shape[0], cap, kv_heads * dim))
+    _operand(v_cache, "v_cache", q, (k_cache.shape[0], cap, kv_heads * vdim))
+    _positions(cache_position, row_start, q, b, t)
+    if b > k_cache.shape[0]:
+        raise RuntimeError("more batch rows than the cache has")
+    pitch = 0
+    if gate is not None:
+        pitch = gate.stride(1)
+        if not gate.is_cuda or gate.dtype != q.dtype or tuple(gate.shape) != (b, t, heads * vdim) or gate.stride(2) != 1 or \
+                (b > 1 and gate.stride(0) != t * pitch):
+            raise RuntimeError("gate must be a slice of a contiguous [B, T, .] projection output")
+    lib = _lib.load()
+    if route is None:
+        route = hybrid_route(q.dtype, t, dim, vdim)
+    if route != _lib.MUI_HYBRID_PLAIN and gate is not None and (pitch % 4 or gate.data_ptr() % 8):
+        route = _lib.MUI_HYBRID_PLAIN
+    out = torch.empty((b, t, heads * vdim), dtype=q.dtype, device=q.device)
+    span = min(window + keep_first, cap) if window > 0 else cap
+    scratch = None
+    if route == _lib.MUI_HYBRID_DECODE:
+        nbytes = lib.mui_hybrid_decode_scratch_bytes(b, t, heads, kv_heads, vdim, span)
+        scratch = torch.empty(nbytes, dtype=torch.uint8, device=q.device) if nbytes else None
+    check(lib.mui_hybrid_attention(_stream(q), dtype_code(q.dtype), route, q.data_ptr(), k_cache.data_ptr(), k_cache.stride(0),
+                                   v_cache.data_ptr(), v_cache.stride(0), _ptr(gate), pitch, cache_position.data_ptr(),
+                                   _ptr(row_start), float(scale), float(softcap), window, keep_first, _ptr(scratch), span,
+                                   out.data_ptr(), b, t, heads, kv_heads, dim, vdim, cap), "mui_hybrid_attention")
+    return out
+
+
+# --------------------------------------------------------------------------------------
+# gated delta rule
+# --------------------------------------------------------------------------------------
+DELTA_SEGMENT = 4096  # tokens per call: bounds the workspace of a long prompt
+
+
+@dataclass
+class ChannelDelta:
+    """One layer's constants and parameters; offsets: columns of q, k, v, a, g, b in the projection's output."""
+    heads: int
+    kv_heads: int
+    dk: int
+    dv: int
+    offsets: Tuple[int, int, int, int, int, int]
+    conv: torch.Tensor     # [2 kv_heads dk + heads dv, taps]
+    a2: torch.Tensor       # [heads * dk, ra]
+    dt_bias: torch.Tensor  # [heads * dk]
+    a_log: torch.Tensor    # [heads]
+    g2: torch.Tensor       # [heads * dv, rg]
+    gain: torch.Tensor     # [dv]
+    eps: float
+
+    @property
+    def channels(self) -> int:
+        return 2 * self.kv_heads * self.dk + self.heads * self.dv
+
+    @property
+    def ring_rows(self) -> int:
+        return _lib.load().mui_channel_delta_ring_rows(self.conv.shape[1])
+
+    def descriptor(self) -> "_lib.MuiChannelDeltaDesc":
+        ptrs = [x.data_ptr() for x in (self.conv, self.a2, self.dt_bias, self.a_log, self.g2, self.gain)]
+        return _lib.MuiChannelDeltaDesc(*ptrs, self.heads, self.kv_heads, self.dk, self.dv, self.a2.shape[1], self.g2.shape[1],
+                                        self.conv.shape[1], *self.offsets, self.dk ** -0.5, self.eps)
+
+
+def channel_delta(layer: ChannelDelta, proj: torch.Tensor, state: torch.Tensor, ring: torch.Tensor,
+                  cache_position: torch.Tensor, row_start: Optional[torch.Tensor]) -> torch.Tensor:
+    """y [B, T, heads * dv] of the projection's output proj [B, T, .]; advances state fp32 [B', heads, dk, dv] and the ring
+    of the convolutions' inputs [B', ring_rows, channels] in place."""
+    b, t, pitch = proj.shape
+    c = layer
+    _operand(proj, "proj", proj)
+    _operand(c.conv, "conv", proj, (c.channels, c.conv.shape[1]))
+    _operand(c.a2, "a2", proj, (c.heads * c.dk, c.a2.shape[1]))
+    _operand(c.dt_bias, "dt_bias", proj, (c.heads * c.dk,))
+    _operand(c.a_log, "a_log", proj, (c.heads,))
+    _operand(c.g2, "g2", proj, (c.heads * c.dv, c.g2.shape[1]))
+    _operand(c.gain, "gain", proj, (c.dv,))
+    _operand(state, "state", proj, (state.shape[0], c.heads, c.dk, c.dv), torch.float32)
+    _operand(ring, "ring", proj, (state.shape[0], c.ring_rows, c.channels))
+    _positions(cache_position, row_start, proj, b, t)
+    if b > state.shape[0]:
+        raise RuntimeError("more batch rows than the state has")
+    lib = _lib.load()
+    most = min(DELTA_SEGMENT, lib.mui_channel_delta_max_tokens(c.dk, c.conv.shape[1]))
+    if t > most and b > 1:  # (the kernels address a whole batch by one token count)
+        return torch.cat([channel_delta(layer, proj[i:i + 1], state[i:i + 1], ring[i:i + 1], cache_position,
+                                        None if row_start is None else row_start[i:i + 1]) for i in range(b)])
+    y = torch.empty((b, t, c.heads * c.dv), dtype=proj.dtype, device=proj.device)
+    desc = c.descriptor()
+    for t0 in range(0, t, most):
+        tn = min(most, t - t0)
+        nbytes = lib.mui_channel_delta_workspace_bytes(b, tn, c.heads, c.dk, c.dv) if tn > _lib.MUI_MAX_TOKENS else 0
+        ws = torch.empty(nbytes, dtype=torch.uint8, device=proj.device) if nbytes else None
+        check(lib.mui_channel_delta(_stream(proj), dtype_code(proj.dtype), ctypes.byref(desc), proj[:, t0:].data_ptr(), pitch, state.data_ptr(),
+                                    ring.data_ptr(), cache_position[t0:].data_ptr(), _ptr(row_start), y[:, t0:].data_ptr(),
+                                    _ptr(ws), b, tn), "mui_channel_delta")
     return y

@@ -33,15 +33,15 @@ def apply_rotary_pos_emb(q, k, cos, sin, unsqueeze_dim: int = 1):
     return (q * cos) + (rotate_half(q) * sin), (k * cos) + (rotate_half(k) * sin)
 
 
-def _default_inv_freq(theta: float, dim: int, device=None) -> torch.Tensor:
-    return 1.0 / (theta ** (torch.arange(0, dim, 2, dtype=torch.int64, device=device).to(torch.float32) / dim))
+def _default_inv_freq(theta: float, dim: int, device=None, dtype: torch.dtype = torch.float32) -> torch.Tensor:
+    return 1.0 / (theta ** (torch.arange(0, dim, 2, dtype=torch.int64, device=device).to(dtype) / dim))
 
 
 def compute_rope_inv_freq(rope_type: str, theta: float, dim: int, scaling: Optional[Dict[str, Any]] = None,
-                          device=None) -> Tuple[torch.Tensor, float]:
-    """(inv_freq [dim/2] fp32, attention_scaling) for the supported rope types, restating the
+                          device=None, dtype: torch.dtype = torch.float32) -> Tuple[torch.Tensor, float]:
+    """(inv_freq [dim/2] in `dtype`, attention_scaling) for the supported rope types, restating the
     published HuggingFace ROPE_INIT_FUNCTIONS formulas."""
-    inv_freq = _default_inv_freq(theta, dim, device)
+    inv_freq = _default_inv_freq(theta, dim, device, dtype)
     if rope_type in (None, "default"):
         return inv_freq, 1.0
     if rope_type == "linear":

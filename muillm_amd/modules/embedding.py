@@ -1,14 +1,15 @@
 """MuiEmbedding -- muillm/modules/embedding.py:13-140 of the reference: an nn.Embedding whose
 forward is a gather kernel for 16-bit tables on the GPU (int32 or int64 ids), so that the
 lookup of a decode step is a plain kernel launch that a HIP graph can replay."""
-from typing import Optional, Union
+from typing import Optional, Tuple, Union
 
 import torch
 import torch.nn as nn
 
-from .. import muillm_ext
+from .. import hybrid_ops, muillm_ext
 from ..engineconfig import MuiEngineConfig
 from ..replacement.replacementcontext import MuiReplacementContext
+from .kvcache.hybridcache import MuiRecurrentState
 from .module import MuiModule
 
 
@@ -74,3 +75,24 @@ class MuiEmbedding(MuiModule, nn.Module):
         if self.dispatchable and self.cpp_module is not None and input.is_cuda and input.dtype in (torch.int32, torch.int64):
             return _MuiEmbedding.apply(self.cpp_module, input)
         return nn.functional.embedding(input, self.weight, self.padding_idx)
+
+
+class MuiBigramEmbedding(MuiModule):
+    """Token embedding (scaled) plus an embedding of the pair (previous token, token), hashed into `buckets` rows; one
+    more row, the last, serves a sequence's first token. The previous token is a state of its own, kept per batch row in
+    the cache. Yields the fp32 residual stream and its rounded copy."""
+
+    def __init__(self, engine_config: MuiEngineConfig, num_embeddings: int, embedding_dim: int, scale: float, buckets: int,
+                 mul_prev: int, mul_cur: int, device=None, dtype=None):
+        super().__init__(engine_config=engine_config)
+        kw = dict(device=device, dtype=dtype)
+        self.scale, self.mul_prev, self.mul_cur = scale, mul_prev, mul_cur
+        self.weight = nn.Parameter(torch.empty(num_embeddings, embedding_dim, **kw), requires_grad=False)
+        self.bigram = nn.Parameter(torch.empty(buckets + 1, embedding_dim, **kw), requires_grad=False)
+
+    def new_state(self, batch: int, capacity: int, device, dtype) -> MuiRecurrentState:
+        return MuiRecurrentState(torch.zeros(batch, dtype=torch.int64, device=device))
+
+    def forward(self, input: torch.Tensor, cache, cache_position: torch.Tensor) -> Tuple[torch.Tensor, torch.Tensor]:
+        return hybrid_ops.bigram_embedding(input, cache.front.values[0], cache_position, cache.row_start, self.weight, self.bigram,
+                                           self.scale, self.mul_prev, self.mul_cur)

@@ -36,9 +36,9 @@ class _MuiGateUpSiLUMethod(Enum):
 class _MuiGateUpSiLU(torch.autograd.Function):
     @staticmethod
     def forward(ctx, engine, inputs, norm_weights, variance_epsilon, gate_weights, up_weights,
-                down_weights, residual):
+                down_weights, residual, biases):
         return muillm_ext.muillm_gateupsilu_forward(
-            engine, norm_weights, variance_epsilon, gate_weights, up_weights, down_weights, residual, inputs)
+            engine, norm_weights, variance_epsilon, gate_weights, up_weights, down_weights, residual, inputs, biases)
 
     @staticmethod
     def backward(ctx, grad_output):
@@ -48,9 +48,9 @@ class _MuiGateUpSiLU(torch.autograd.Function):
 class _MuiGateUpSiLUSplit(torch.autograd.Function):
     @staticmethod
     def forward(ctx, engine, inputs, norm_weights, variance_epsilon, gate_weights, up_weights,
-                down_weights, residual):
+                down_weights, residual, biases):
         return muillm_ext.muillm_gateupsilu_split_forward(
-            engine, norm_weights, variance_epsilon, gate_weights, up_weights, down_weights, residual, inputs)
+            engine, norm_weights, variance_epsilon, gate_weights, up_weights, down_weights, residual, inputs, biases)
 
     @staticmethod
     def backward(ctx, grad_output):
@@ -60,7 +60,7 @@ class _MuiGateUpSiLUSplit(torch.autograd.Function):
 class MuiGateUpDownMLP(MuiModule):
     def __init__(self, engine_config: MuiEngineConfig, hidden_size: int, intermediate_size: int,
                  activation_function: nn.Module, variance_epsilon: float = 0.0, normalize: bool = False,
-                 device=None, dtype=None) -> None:
+                 device=None, dtype=None, bias: bool = False) -> None:
         super().__init__(engine_config=engine_config)
         self.cpp_engine = engine_config.cpp_engine
         self.hidden_size = hidden_size
@@ -68,9 +68,9 @@ class MuiGateUpDownMLP(MuiModule):
         self.normalize = normalize
         self.variance_epsilon = variance_epsilon
         self.norm_weights = nn.Parameter(torch.ones(hidden_size, dtype=dtype, device=device)) if normalize else None
-        self.gate_proj = MuiLinear(engine_config, hidden_size, intermediate_size, bias=False, device=device, dtype=dtype)
-        self.up_proj = MuiLinear(engine_config, hidden_size, intermediate_size, bias=False, device=device, dtype=dtype)
-        self.down_proj = MuiLinear(engine_config, intermediate_size, hidden_size, bias=False, device=device, dtype=dtype)
+        self.gate_proj = MuiLinear(engine_config, hidden_size, intermediate_size, bias=bias, device=device, dtype=dtype)
+        self.up_proj = MuiLinear(engine_config, hidden_size, intermediate_size, bias=bias, device=device, dtype=dtype)
+        self.down_proj = MuiLinear(engine_config, intermediate_size, hidden_size, bias=bias, device=device, dtype=dtype)
         self.activation_function = activation_function
         self._check_dispatchable()
         self.method = _MuiGateUpSiLUMethod.GATEUPSILU_FUSED
@@ -146,7 +146,7 @@ class MuiGateUpDownMLP(MuiModule):
             engine_config=engine_config, hidden_size=prev_module.gate_proj.in_features,
             intermediate_size=prev_module.up_proj.out_features, activation_function=activation_function,
             variance_epsilon=variance_epsilon, normalize=normalize,
-            dtype=prev_module.gate_proj.weight.dtype, device=device)
+            dtype=prev_module.gate_proj.weight.dtype, device=device, bias=prev_module.gate_proj.bias is not None)
         new_module.copy_module(prev_module=prev_module, norm_weights=norm_weights, device=device)
 
         if not isinstance(prev_module, MuiGateUpDownMLP):
@@ -197,6 +197,12 @@ class MuiGateUpDownMLP(MuiModule):
             output = output + residual
         return output
 
+    def _biases(self):
+        """(gate, up, down) biases for the fused kernels, or None."""
+        if self.gate_proj.bias is None:
+            return None
+        return self.gate_proj.bias, self.up_proj.bias, self.down_proj.bias
+
     def _kernel_ok(self, input: Tensor) -> bool:
         return (self.dispatchable and muillm_ext.kernel_dispatchable(input)
                 and isinstance(self.gate_proj, MuiLinear) and isinstance(self.up_proj, MuiLinear))
@@ -204,13 +210,13 @@ class MuiGateUpDownMLP(MuiModule):
     def _forward_fused(self, input: Tensor, residual: Optional[Tensor] = None) -> Tensor:
         if self._kernel_ok(input):
             return _MuiGateUpSiLU.apply(self.cpp_engine, input, self.norm_weights, self.variance_epsilon,
-                                        self.gate_proj.weight, self.up_proj.weight, self.down_proj.weight, residual)
+                                        self.gate_proj.weight, self.up_proj.weight, self.down_proj.weight, residual, self._biases())
         return self._forward_unfused(input=input, residual=residual)
 
     def _forward_split(self, input: Tensor, residual: Optional[Tensor] = None) -> Tensor:
         if self._kernel_ok(input):
             return _MuiGateUpSiLUSplit.apply(self.cpp_engine, input, self.norm_weights, self.variance_epsilon,
-                                             self.gate_proj.weight, self.up_proj.weight, self.down_proj.weight, residual)
+                                             self.gate_proj.weight, self.up_proj.weight, self.down_proj.weight, residual, self._biases())
         return self._forward_unfused(input=input, residual=residual)
 
     def forward(self, input: Tensor, residual: Optional[Tensor] = None) -> Tensor:

@@ -1,43 +1,71 @@
-"""Cache of a decoder whose layers keep different things: a latent row per token, a recurrent state, or
-nothing of their own (a layer that attends over another layer's rows).
+"""Cache of a decoder whose layers keep different things: rows per token (keys and values, or a latent row), a
+recurrent state, or nothing of their own (a layer that attends over another layer's rows).
 
 Every mixer makes its own layer state (`new_state`); the cache holds them in layer order and gives the
 decode loop what MuiStaticCache gives it: capacity (a power of two, grown on demand), the count of seen
 tokens, reset for the next sequence. Rows of a batch advance together; a left-padded row starts at
 row_start[b], keys in front of it are never seen and recurrent states pass over it."""
-from typing import List, Optional
+from typing import List, Optional, Sequence
 
 import torch
 
 from .cache_utils import MuiCache, _next_pow2
 
 
-class MuiLatentState:
-    """Latent rows c [B, capacity, kv_rank] and rotated key parts r [B, capacity, rot] of one layer."""
+class MuiRowState:
+    """Tensors [B, capacity, width] with one row per token."""
 
-    def __init__(self, batch: int, capacity: int, kv_rank: int, rot_dim: int, device, dtype):
-        self.c = torch.zeros((batch, capacity, kv_rank), dtype=dtype, device=device)
-        self.r = torch.zeros((batch, capacity, rot_dim), dtype=dtype, device=device)
+    def __init__(self, batch: int, capacity: int, widths: Sequence[int], device, dtype):
+        self.rows = [torch.zeros((batch, capacity, w), dtype=dtype, device=device) for w in widths]
 
     def tensors(self) -> List[torch.Tensor]:
-        return [self.c, self.r]
+        return list(self.rows)
 
     def recurrent(self) -> List[torch.Tensor]:
         return []
 
     def grow(self, capacity: int) -> None:
-        for name in ("c", "r"):
-            old = getattr(self, name)
-            new = torch.zeros((old.shape[0], capacity, old.shape[2]), dtype=old.dtype, device=old.device)
-            new[:, :old.shape[1]] = old
-            setattr(self, name, new)
+        for i, old in enumerate(self.rows):
+            self.rows[i] = torch.zeros((old.shape[0], capacity, old.shape[2]), dtype=old.dtype, device=old.device)
+            self.rows[i][:, :old.shape[1]] = old
 
     def reset(self) -> None:
         pass  # rows behind the count of seen tokens are never read before they are written again
 
 
+class MuiLatentState(MuiRowState):
+    """Latent rows c [B, capacity, kv_rank] and rotated key parts r [B, capacity, rot] of one layer."""
+
+    def __init__(self, batch: int, capacity: int, kv_rank: int, rot_dim: int, device, dtype):
+        super().__init__(batch, capacity, (kv_rank, rot_dim), device, dtype)
+
+    @property
+    def c(self) -> torch.Tensor:
+        return self.rows[0]
+
+    @property
+    def r(self) -> torch.Tensor:
+        return self.rows[1]
+
+
+class MuiKeyValueState(MuiRowState):
+    """Keys [B, capacity, kv_heads * dim] (rotated) and values [B, capacity, kv_heads * vdim] of one layer."""
+
+    def __init__(self, batch: int, capacity: int, kv_heads: int, dim: int, vdim: int, device, dtype):
+        super().__init__(batch, capacity, (kv_heads * dim, kv_heads * vdim), device, dtype)
+
+    @property
+    def k(self) -> torch.Tensor:
+        return self.rows[0]
+
+    @property
+    def v(self) -> torch.Tensor:
+        return self.rows[1]
+
+
 class MuiRecurrentState:
-    """fp32 tensors of fixed size that every token rewrites; a fresh sequence starts from zero."""
+    """Tensors of fixed size that every token rewrites (memories in fp32, the last inputs of a short convolution,
+    the last token); a fresh sequence starts from zero."""
 
     def __init__(self, *tensors: torch.Tensor):
         self.values = tuple(tensors)
@@ -57,12 +85,14 @@ class MuiRecurrentState:
 
 
 class MuiHybridCache(MuiCache):
-    def __init__(self, engine_config, mixers, max_batch_size: int, max_cache_len: int, device, dtype: torch.dtype):
+    def __init__(self, engine_config, mixers, max_batch_size: int, max_cache_len: int, device, dtype: torch.dtype, front=None):
+        """front: what stands in front of the layers and keeps a state of its own (an embedding that looks back)."""
         self.engine_config = engine_config
         self.max_batch_size = max_batch_size
         self.max_cache_len = _next_pow2(max_cache_len)
         self.device, self.dtype = device, dtype
         self.layers = [m.new_state(max_batch_size, self.max_cache_len, device, dtype) for m in mixers]
+        self.front = None if front is None else front.new_state(max_batch_size, self.max_cache_len, device, dtype)
         self.row_start: Optional[torch.Tensor] = None
         self._seen_tokens = 0
         # True while a captured decode step runs: positions are read from device memory only
@@ -73,7 +103,7 @@ class MuiHybridCache(MuiCache):
         return len(self.layers)
 
     def _states(self):
-        return [s for s in self.layers if s is not None]
+        return [s for s in self.layers + [self.front] if s is not None]
 
     def tensors(self) -> List[torch.Tensor]:
         out = [t for s in self._states() for t in s.tensors()]

@@ -80,7 +80,8 @@ class MuiGraphDecoder:
         # loads at the head of every step)
         table = getattr(getattr(getattr(self.lm, "model", None), "embed_tokens", None), "weight", None)
         self._embed_table = None
-        if (not self.do_sample and table is not None and table.is_cuda and table.dim() == 2 and table.stride(1) == 1
+        if (not self.do_sample and table is not None and getattr(self.lm, "takes_embeddings", True)
+                and table.is_cuda and table.dim() == 2 and table.stride(1) == 1
                 and table.dtype in (torch.float16, torch.bfloat16)):
             self._embed_table = table
             self.hidden = torch.zeros((batch, 1, table.shape[1]), dtype=table.dtype, device=device)

@@ -4,13 +4,16 @@ Folders with a HuggingFace config (`architectures`) go through transformers and 
 replacement; native designs (`architecture`) are built directly."""
 import json
 import os
-from typing import Callable, Dict
+from typing import Callable, Dict, Type
 
 import torch
 
 from ...engineconfig import MuiEngineConfig
+from .native import MuiNativeForCausalLM
 from .salepel.config import ARCHITECTURE as SALEPEL
 from .salepel.model import MuiSalepelForCausalLM
+from .zufadra.config import ARCHITECTURE as ZUFADRA
+from .zufadra.model import MuiZufadraForCausalLM
 
 
 def _load_hf(path: str, dtype, device, engine_config: MuiEngineConfig):
@@ -22,14 +25,18 @@ def _load_hf(path: str, dtype, device, engine_config: MuiEngineConfig):
     return init_engine(model, device=device, engine_config=engine_config)
 
 
-def _load_salepel(path: str, dtype, device, engine_config: MuiEngineConfig):
-    return MuiSalepelForCausalLM.from_pretrained(path, dtype=dtype, device=device, engine_config=engine_config)
+def _native(cls: Type[MuiNativeForCausalLM]) -> Callable:
+    def load(path: str, dtype, device, engine_config: MuiEngineConfig):
+        return cls.from_pretrained(path, dtype=dtype, device=device, engine_config=engine_config)
+
+    return load
 
 
 MODEL_LOADERS: Dict[str, Callable] = {
     "LlamaForCausalLM": _load_hf,
     "MistralForCausalLM": _load_hf,
-    SALEPEL: _load_salepel,
+    SALEPEL: _native(MuiSalepelForCausalLM),
+    ZUFADRA: _native(MuiZufadraForCausalLM),
 }
 
 

@@ -2,25 +2,15 @@
 a key that this build does not know is reported."""
 import json
 import os
-import warnings
 from dataclasses import dataclass, field
 from typing import Any, Dict, List, Optional, Union
 
 from ...attention.latentattention import MuiLatentAttentionConfig
 from ...moe import MuiMoEConfig
 from ...recurrent.mlstm import MuiMLstmConfig
+from ..nativeconfig import take_section
 
 ARCHITECTURE = "Salepel"
-
-
-def _take(section: Dict[str, Any], where: str, required, optional=()) -> Dict[str, Any]:
-    missing = sorted(set(required) - set(section))
-    if missing:
-        raise ValueError(f"{where}: missing keys {missing}")
-    unknown = sorted(set(section) - set(required) - set(optional))
-    if unknown:
-        warnings.warn(f"{where}: unknown keys {unknown} are ignored")
-    return section
 
 
 @dataclass
@@ -30,9 +20,9 @@ class MuiSalepelLayerConfig:
 
 
 def _latent_attention(mx: Dict[str, Any], where: str) -> MuiLatentAttentionConfig:
-    _take(mx, where, ("dim", "heads", "kv_rank", "mask", "q_rank", "rot", "rot_dim", "scale", "vdim"), ("kv_from",))
-    mask = _take(mx["mask"], where + ".mask", ("size",))
-    rot = _take(mx["rot"], where + ".rot", ("base", "dims"))
+    take_section(mx, where, ("dim", "heads", "kv_rank", "mask", "q_rank", "rot", "rot_dim", "scale", "vdim"), ("kv_from",))
+    mask = take_section(mx["mask"], where + ".mask", ("size",))
+    rot = take_section(mx["rot"], where + ".rot", ("base", "dims"))
     if rot["dims"] != mx["rot_dim"]:
         raise ValueError(f"{where}: rot.dims {rot['dims']} is not rot_dim {mx['rot_dim']}")
     if mask["size"] < 1:
@@ -43,7 +33,7 @@ def _latent_attention(mx: Dict[str, Any], where: str) -> MuiLatentAttentionConfi
 
 
 def _mlstm(mx: Dict[str, Any], where: str) -> MuiMLstmConfig:
-    _take(mx, where, ("dim", "gate_cap", "heads", "vdim"))
+    take_section(mx, where, ("dim", "gate_cap", "heads", "vdim"))
     return MuiMLstmConfig(heads=mx["heads"], dim=mx["dim"], vdim=mx["vdim"], gate_cap=float(mx["gate_cap"]))
 
 
@@ -53,11 +43,11 @@ _MIXERS = {"latent_attention": _latent_attention, "mlstm": _mlstm}
 def _mlp(ff: Optional[Dict[str, Any]], where: str) -> Optional[MuiMoEConfig]:
     if ff is None:
         return None
-    _take(ff, where, ("kind", "expert", "router"))
+    take_section(ff, where, ("kind", "expert", "router"))
     if ff["kind"] != "moe":
         raise ValueError(f"{where}: unknown feed-forward {ff['kind']!r}")
-    expert = _take(ff["expert"], where + ".expert", ("ff", "limit"))
-    router = _take(ff["router"], where + ".router", ("experts", "top"), ("identity",))
+    expert = take_section(ff["expert"], where + ".expert", ("ff", "limit"))
+    router = take_section(ff["router"], where + ".router", ("experts", "top"), ("identity",))
     return MuiMoEConfig(experts=router["experts"], identity=router.get("identity", 0), top=router["top"], ff=expert["ff"],
                         limit=float(expert["limit"]))
 
@@ -91,22 +81,25 @@ class MuiSalepelConfig:
     def num_hidden_layers(self) -> int:
         return len(self.layers)
 
+    def with_tensor_shapes(self, shapes) -> "MuiSalepelConfig":
+        return self  # the configuration says every size
+
     @staticmethod
     def from_dict(cfg: Dict[str, Any]) -> "MuiSalepelConfig":
-        _take(cfg, "config", ("architecture", "embedding", "layers", "norm", "vocab", "width"))
+        take_section(cfg, "config", ("architecture", "embedding", "layers", "norm", "vocab", "width"))
         if cfg["architecture"] != ARCHITECTURE:
             raise ValueError(f"architecture {cfg['architecture']!r} is not {ARCHITECTURE}")
         layers = []
         for i, layer in enumerate(cfg["layers"]):
             where = f"layers[{i}]"
-            _take(layer, where, ("type", "mixer"), ("mlp",))
+            take_section(layer, where, ("type", "mixer"), ("mlp",))
             if layer["type"] not in _MIXERS:
                 raise ValueError(f"{where}: unknown mixer {layer['type']!r}")
             layers.append(MuiSalepelLayerConfig(_MIXERS[layer["type"]](layer["mixer"], where + ".mixer"),
                                                 _mlp(layer.get("mlp"), where + ".mlp")))
         return MuiSalepelConfig(vocab_size=cfg["vocab"], hidden_size=cfg["width"],
-                                rms_norm_eps=float(_take(cfg["norm"], "norm", ("eps",))["eps"]),
-                                embedding_scale=float(_take(cfg["embedding"], "embedding", ("scale",))["scale"]), layers=layers)
+                                rms_norm_eps=float(take_section(cfg["norm"], "norm", ("eps",))["eps"]),
+                                embedding_scale=float(take_section(cfg["embedding"], "embedding", ("scale",))["scale"]), layers=layers)
 
     @staticmethod
     def from_pretrained(path: str) -> "MuiSalepelConfig":

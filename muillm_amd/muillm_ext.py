@@ -311,8 +311,8 @@ def muillm_linear_module_forward(module: MuiLinearModuleHandle, inputs: torch.Te
 # --------------------------------------------------------------------------------------
 # Gate/Up/Down MLP  (csrc/module.cpp:182,215; csrc/ffn/gateup.cu:88-391)
 # --------------------------------------------------------------------------------------
-def mui_gateup_silu(norm_weights, epsilon, gate_weights, up_weights, x) -> torch.Tensor:
-    """h = silu(G xn) * (U xn) for 1..MUI_MAX_TOKENS tokens; gate/up may be views into one
+def mui_gateup_silu(norm_weights, epsilon, gate_weights, up_weights, x, gate_bias=None, up_bias=None) -> torch.Tensor:
+    """h = silu(G xn + gate_bias) * (U xn + up_bias) for any number of tokens; gate/up may be views into one
     interleaved [N, 2, K] buffer (common row pitch)."""
     n, k = gate_weights.shape
     if up_weights.shape != gate_weights.shape:
@@ -325,6 +325,11 @@ def mui_gateup_silu(norm_weights, epsilon, gate_weights, up_weights, x) -> torch
             (norm_weights is not None and (norm_weights.dtype != x.dtype or norm_weights.numel() != k)):
         raise RuntimeError("mui_gateup_silu: weights and norm weights must have the activations' dtype "
                            "(norm weights: one value per input feature)")
+    if (gate_bias is None) != (up_bias is None):
+        raise RuntimeError("gate and up biases come together")
+    for bias in (gate_bias, up_bias):
+        if bias is not None and (bias.dtype != x.dtype or bias.device != x.device or bias.numel() != n or not bias.is_contiguous()):
+            raise RuntimeError(f"gate and up biases must be {x.dtype} vectors of {n} elements on {x.device}")
     x = x.contiguous()
     x, norm_weights = _norm_first(x, norm_weights, epsilon, FUSED_CHUNK_MAX_TOKENS)
     tokens = _num_tokens(x)
@@ -332,9 +337,9 @@ def mui_gateup_silu(norm_weights, epsilon, gate_weights, up_weights, x) -> torch
     lib, stream, code, esz = _lib.load(), _stream(x), _dtype_code(x), x.element_size()
     for off, cnt in _token_calls(tokens, FUSED_CHUNK_MAX_TOKENS):
         check(
-            lib.mui_gateup_silu(
+            lib.mui_gateup_silu_bias(
                 stream, code, gate_weights.data_ptr(), up_weights.data_ptr(), pitch,
-                x.data_ptr() + off * k * esz, _ptr(norm_weights), float(epsilon),
+                x.data_ptr() + off * k * esz, _ptr(norm_weights), float(epsilon), _ptr(gate_bias), _ptr(up_bias),
                 h.data_ptr() + off * n * esz, n, k, cnt,
             ),
             "mui_gateup_silu",
@@ -354,21 +359,23 @@ def mui_silu_mul_interleaved(gate_up: torch.Tensor) -> torch.Tensor:
 
 
 def muillm_gateupsilu_forward(engine, norm_weights, epsilon, gate_weights, up_weights, down_weights,
-                              residual, x) -> torch.Tensor:
-    """out = Wd (silu(Wg xn) * (Wu xn)) + residual, argument order of csrc/module.cpp:182."""
+                              residual, x, biases=None) -> torch.Tensor:
+    """out = Wd (silu(Wg xn) * (Wu xn)) + residual, argument order of csrc/module.cpp:182. biases: (gate, up, down)
+    vectors added to the three products, or None."""
     if not (kernel_dispatchable(x) and gate_weights.dtype == x.dtype):
         raise RuntimeError("muillm_gateupsilu_forward needs fp16 / bf16 CUDA tensors with k % 8 == 0")
-    h = mui_gateup_silu(norm_weights, epsilon, gate_weights, up_weights, x)
-    return muillm_linear_forward(engine, h, down_weights, residual=residual)
+    gate_bias, up_bias, down_bias = biases or (None, None, None)
+    h = mui_gateup_silu(norm_weights, epsilon, gate_weights, up_weights, x, gate_bias, up_bias)
+    return muillm_linear_forward(engine, h, down_weights, add_bias=down_bias, residual=residual)
 
 
 def muillm_gateupsilu_split_forward(engine, norm_weights, epsilon, gate_weights, up_weights,
-                                    down_weights, residual, x) -> torch.Tensor:
+                                    down_weights, residual, x, biases=None) -> torch.Tensor:
     """The reference's split-K variant (csrc/module.cpp:215) exists to create more blocks on
     MI300; the gfx950 kernel already sizes its grid to the CU count, so both names run the
     same path."""
     return muillm_gateupsilu_forward(engine, norm_weights, epsilon, gate_weights, up_weights,
-                                     down_weights, residual, x)
+                                     down_weights, residual, x, biases)
 
 
 # --------------------------------------------------------------------------------------

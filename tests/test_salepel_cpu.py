@@ -132,7 +132,7 @@ def test_argument_checks_need_no_gpu():
     from muillm_amd import _lib
 
     lib = _lib.load()
-    assert lib.mui_residual_norm(None, 1, None, None, 1.0, None, None, 0.0, None, None, 1, 8) == -1
+    assert lib.mui_residual_norm(None, 1, None, None, 1.0, None, 1.0, None, 1.0, 0.0, None, None, 1, 8) == -1
     assert lib.mui_moe_route(None, 1, None, None, 4, 0, 2, 1, 0, None, None, None, None) == -1
     assert lib.mui_mlstm(None, 1, None, None, None, 8, None, 1.0, 1.0, None, None, None, None, None, None, None, 1, 1, 1, 8, 8) == -1
     assert lib.mui_moe_tile_pairs(2, 100, 2, 4, 64, 64) == 0 and lib.mui_moe_tile_pairs(1, 4, 2, 4, 64, 63) == 0
