@@ -19,8 +19,9 @@ live with HIP events over cold (distinct) weight buffers, a `cpu_baseline` objec
 reference's PyTorch fallback path in fp16 on this box's host cores, bounded sample), and a
 `kernels` table (GB/s per fused kernel family, informational).
 
-`--salepel` times the Salepel decoder (latent attention, matrix memory, mixture of experts) beside a
-Llama-shaped model of equal width and active MLP size instead, and prints one JSON line of its own.
+`--salepel` (latent attention, matrix memory, mixture of experts) and `--zufadra` (windowed attention with sinks, gated
+delta rule) time those decoders beside a Llama-shaped model of equal width and active MLP size instead, and print one
+JSON line of their own.
 """
 
 import argparse
@@ -1158,15 +1159,21 @@ def _cpu_model():
 
 
 # --------------------------------------------------------------------------------------
-# the Salepel decoder beside the Llama-shaped one
+# the hybrid decoders beside the Llama-shaped one
 # --------------------------------------------------------------------------------------
-# layer sizes of real models' order; the Llama-shaped twin has the same width and, as its MLP, as many
-# features as a token's chosen experts have together
-SALEPEL_SIZES = {
-    "width4096": dict(width=4096, heads=32, q_rank=1536, window=4096, lstm_heads=8, experts=64, identity=8, top=8, ff=1792),
-    "width2048": dict(width=2048, heads=16, q_rank=768, window=1024, lstm_heads=4, experts=64, identity=8, top=6, ff=1408),
+# Layer sizes of real models' order, eight layers. The Llama-shaped twin has the same width, heads of 128, four
+# query heads per KV head, and an MLP of `twin_ff` features (Salepel: as many as a token's chosen experts have together).
+HYBRID_VOCAB = 32768
+HYBRID_SIZES = {
+    "salepel": {
+        "width4096": dict(width=4096, heads=32, q_rank=1536, window=4096, lstm_heads=8, experts=64, identity=8, top=8, ff=1792, twin_ff=14336),
+        "width2048": dict(width=2048, heads=16, q_rank=768, window=1024, lstm_heads=4, experts=64, identity=8, top=6, ff=1408, twin_ff=8448),
+    },
+    "zufadra": {
+        "width4096": dict(width=4096, heads=32, kv_heads=8, window=4096, keep_first=64, rank=128, ff=14336, twin_ff=14336),
+        "width2048": dict(width=2048, heads=16, kv_heads=4, window=1024, keep_first=64, rank=128, ff=8192, twin_ff=8192),
+    },
 }
-SALEPEL_VOCAB = 32768
 
 
 def _salepel_config(z):
@@ -1184,40 +1191,57 @@ def _salepel_config(z):
     mem = MuiMLstmConfig(heads=z["lstm_heads"], dim=256, vdim=512, gate_cap=15.0)
     ff = MuiMoEConfig(experts=z["experts"], identity=z["identity"], top=z["top"], ff=z["ff"], limit=7.0)
     mixers = [latent(), latent(0), latent(), mem, latent(), latent(4), latent(), mem]
-    return MuiSalepelConfig(vocab_size=SALEPEL_VOCAB, hidden_size=z["width"], rms_norm_eps=1e-5, embedding_scale=1.0,
+    return MuiSalepelConfig(vocab_size=HYBRID_VOCAB, hidden_size=z["width"], rms_norm_eps=1e-5, embedding_scale=1.0,
                             layers=[MuiSalepelLayerConfig(m, ff) for m in mixers])
 
 
-def _salepel_models(z, which=("salepel", "llama")):
+def _zufadra_config(z):
+    """Eight layers, a delta rule and windowed attention in turn, a dense feed-forward in each."""
+    from muillm_amd.modules.attention.hybridattention import MuiHybridAttentionConfig
+    from muillm_amd.modules.models.zufadra.config import MuiBigramConfig, MuiZufadraConfig, MuiZufadraLayerConfig
+    from muillm_amd.modules.recurrent.channeldelta import MuiChannelDeltaConfig
+
+    att = MuiHybridAttentionConfig(heads=z["heads"], kv_heads=z["kv_heads"], dim=128, vdim=128, scale=128 ** -0.5, rot_dims=64,
+                                   softcap=30.0, window=z["window"], keep_first=z["keep_first"])
+    mem = MuiChannelDeltaConfig(heads=z["heads"], kv_heads=z["heads"], dim=128, vdim=128, taps=4, decay_rank=z["rank"],
+                                gate_rank=z["rank"])
+    return MuiZufadraConfig(vocab_size=HYBRID_VOCAB, hidden_size=z["width"], rms_norm_eps=1e-5, embedding_scale=1.0, residual_mult=1.0,
+                            logit_scale=1.0, bigram=MuiBigramConfig(32003, 1009, 31),
+                            layers=[MuiZufadraLayerConfig(m, z["ff"]) for m in (mem, att) * 4])
+
+
+def _hybrid_models(design, z, which):
     import torch
 
     from muillm_amd.engineconfig import MuiEngineConfig
     from muillm_amd.modules.models.llama.model import MuiDecoderConfig, MuiLlamaForCausalLM
     from muillm_amd.modules.models.salepel.model import MuiSalepelForCausalLM
+    from muillm_amd.modules.models.zufadra.model import MuiZufadraForCausalLM
 
     for name in which:
-        if name == "salepel":
-            yield name, MuiSalepelForCausalLM.from_config(MuiEngineConfig(), _salepel_config(z), dtype=torch.bfloat16)
-        else:
-            cfg = MuiDecoderConfig(hidden_size=z["width"], intermediate_size=z["top"] * z["ff"], num_hidden_layers=8,
+        if name == "llama":
+            cfg = MuiDecoderConfig(hidden_size=z["width"], intermediate_size=z["twin_ff"], num_hidden_layers=8,
                                    num_attention_heads=z["width"] // 128, num_key_value_heads=z["width"] // 512,
-                                   vocab_size=SALEPEL_VOCAB, max_position_embeddings=8192)
+                                   vocab_size=HYBRID_VOCAB, max_position_embeddings=8192)
             yield name, MuiLlamaForCausalLM.from_config(MuiEngineConfig(), cfg, dtype=torch.bfloat16, device="cuda", seed=0)
+        else:
+            cls, config = {"salepel": (MuiSalepelForCausalLM, _salepel_config), "zufadra": (MuiZufadraForCausalLM, _zufadra_config)}[design]
+            yield name, cls.from_config(MuiEngineConfig(), config(z), dtype=torch.bfloat16)
 
 
-def bench_salepel(steps=64, sizes=None):
-    """Prefill and decode throughput of both models at every size; prints one JSON line."""
+def bench_hybrid(design, steps=64, sizes=None):
+    """Prefill and decode throughput of the design and its twin at every size; prints one JSON line."""
     import torch
 
     out = {}
-    for size, z in SALEPEL_SIZES.items():
+    for size, z in HYBRID_SIZES[design].items():
         if sizes and size not in sizes:
             continue
         out[size] = {}
-        for name, lm in _salepel_models(z):
+        for name, lm in _hybrid_models(design, z, (design, "llama")):
             r = out[size][name] = {}
             for tokens in (512, 2048, 4096):
-                ids = torch.randint(0, SALEPEL_VOCAB, (1, tokens), generator=torch.Generator().manual_seed(1)).to("cuda")
+                ids = torch.randint(0, HYBRID_VOCAB, (1, tokens), generator=torch.Generator().manual_seed(1)).to("cuda")
                 with torch.no_grad():
                     us = _event_time_us(lambda i: lm(input_ids=ids, num_logits_to_keep=1), 5, 2)
                 r[f"prefill_{tokens}_tokens_ms"] = round(us / 1e3, 3)
@@ -1229,17 +1253,17 @@ def bench_salepel(steps=64, sizes=None):
             _progress(f"{size} {name}: {r}")
             del lm
             torch.cuda.empty_cache()
-    print(json.dumps({"salepel": out, "dtype": "bf16", "layers": 8, "data": "random weights and tokens"}))
+    print(json.dumps({design: out, "dtype": "bf16", "layers": 8, "data": "random weights and tokens"}))
 
 
-def trace_salepel(spec):
+def trace_hybrid(design, spec):
     """SIZE:MODEL:prefill=TOKENS or SIZE:MODEL:decode=BATCH -- a few passes for rocprofv3 --kernel-trace."""
     import torch
 
     size, name, what = spec.split(":")
     mode, n = what.split("=")
-    (_, lm), = _salepel_models(SALEPEL_SIZES[size], (name,))
-    ids = torch.randint(0, SALEPEL_VOCAB, (1 if mode == "prefill" else int(n), int(n) if mode == "prefill" else 2048)).to("cuda")
+    (_, lm), = _hybrid_models(design, HYBRID_SIZES[design][size], (name,))
+    ids = torch.randint(0, HYBRID_VOCAB, (1 if mode == "prefill" else int(n), int(n) if mode == "prefill" else 2048)).to("cuda")
     with torch.no_grad():
         if mode == "prefill":
             for _ in range(4):
@@ -1250,7 +1274,7 @@ def trace_salepel(spec):
             for _ in range(32):
                 lm(input_ids=ids[:, :1], past_key_values=cache)
     torch.cuda.synchronize()
-    print("traced", spec)
+    print("traced", design, spec)
 
 
 def main():
@@ -1311,10 +1335,13 @@ def main():
     ap.add_argument("--pmc-probe-prompt", action="store_true",
                     help="launch the gate/up prompt GEMM (2048 tokens) and prompt attention (4096) three times and exit "
                          "(for rocprofv3 --pmc)")
-    ap.add_argument("--salepel", nargs="?", const="", default=None, metavar="SIZES",
-                    help="prefill and decode throughput of the Salepel decoder beside the Llama-shaped model at equal size, and exit")
-    ap.add_argument("--trace-salepel", default=None, metavar="SIZE:MODEL:MODE=N",
-                    help="a few passes of one of those models (MODE prefill=TOKENS or decode=BATCH) for rocprofv3 --kernel-trace, and exit")
+    for design in HYBRID_SIZES:
+        ap.add_argument(f"--{design}", nargs="?", const="", default=None, metavar="SIZES",
+                        help=f"prefill and decode throughput of the {design.capitalize()} decoder beside the Llama-shaped model at "
+                             "equal size, and exit")
+        ap.add_argument(f"--trace-{design}", default=None, metavar="SIZE:MODEL:MODE=N",
+                        help="a few passes of one of those models (MODE prefill=TOKENS or decode=BATCH) for rocprofv3 "
+                             "--kernel-trace, and exit")
     args = ap.parse_args()
     if args.gpus != 1:
         print("bench.py: this build drives exactly one GPU (no tensor parallelism, no collectives); "
@@ -1327,12 +1354,14 @@ def main():
     from muillm_amd.modules.models.llama.model import MuiDecoderConfig, MuiLlamaForCausalLM
 
     assert torch.cuda.is_available(), "bench.py needs a GPU"
-    if args.salepel is not None:
-        bench_salepel(sizes=[v for v in args.salepel.split(",") if v])
-        return
-    if args.trace_salepel:
-        trace_salepel(args.trace_salepel)
-        return
+    for design in HYBRID_SIZES:
+        sizes, spec = getattr(args, design), getattr(args, "trace_" + design)
+        if sizes is not None:
+            bench_hybrid(design, sizes=[v for v in sizes.split(",") if v])
+            return
+        if spec:
+            trace_hybrid(design, spec)
+            return
     if args.pmc_probe:
         pmc_probe()
         return
