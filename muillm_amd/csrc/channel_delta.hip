@@ -48,33 +48,64 @@ struct DeltaParams {
   int chunks, dkp, dvp;
 };
 
+// Each is a few fp32 operations around the hardware's exp2, log2 and reciprocal (1 ulp).
+constexpr float kLog2E = 1.4426950408889634f;
+__device__ __forceinline__ float sigm(float z) { return __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-kLog2E * z)); }
+__device__ __forceinline__ float silu(float z) { return z * sigm(z); }
+// exp(neg_a softplus(z)), softplus(z) = max(z, 0) + log(1 + u), u = exp(-|z|); the logarithm of w = 1 + u is scaled by
+// u / (w - 1), which makes good what the sum lost
+__device__ __forceinline__ float decay_of(float neg_a, float z) {
+  const float u = __builtin_amdgcn_exp2f(-kLog2E * fabsf(z)), w = 1.f + u, d = w - 1.f;
+  const float l = d > 0.f ? __builtin_amdgcn_logf(w) * (u * __builtin_amdgcn_rcpf(d)) : u * kLog2E;
+  return __builtin_amdgcn_exp2f(neg_a * fmaf(fmaxf(z, 0.f), kLog2E, l));
+}
+
 template <typename T>
 struct DeltaRow {  // one batch row
   typedef typename T::storage S;
   const S* proj;
   const S* ring;
   long p0, start;  // slot of token 0, first slot of the row
+  int ring0;       // ring row of token 0
   __device__ __forceinline__ DeltaRow(const DeltaParams& p, int b)
       : proj((const S*)p.proj + (long)b * p.t * p.pitch), ring((const S*)p.ring + (long)b * p.ring_rows * p.channels),
-        p0(p.cache_position[0]), start(p.row_start ? p.row_start[b] : 0) {}
+        p0(p.cache_position[0]), start(p.row_start ? p.row_start[b] : 0), ring0((int)((uint32_t)p0 % (uint32_t)p.ring_rows)) {}
+  // ring row of token tok, -ring_rows <= tok < 0
+  __device__ __forceinline__ int ring_row(const DeltaParams& p, int tok) const { return ring0 + tok + (ring0 + tok < 0 ? p.ring_rows : 0); }
   __device__ __forceinline__ bool live(int tok) const { return p0 + tok >= start; }
   // input of channel c (column `col` of the projection) at token tok, which may lie in front of this call
   __device__ __forceinline__ float raw(const DeltaParams& p, int tok, int col, int c) const {
     const long slot = p0 + tok;
     if (slot < start || slot < 0) return 0.f;
-    return T::one(tok >= 0 ? proj[(long)tok * p.pitch + col] : ring[(long)((uint32_t)slot % (uint32_t)p.ring_rows) * p.channels + c]);
+    return T::one(tok >= 0 ? proj[(long)tok * p.pitch + col] : ring[(long)ring_row(p, tok) * p.channels + c]);
   }
   // convolution and silu
   __device__ __forceinline__ float conv(const DeltaParams& p, int tok, int col, int c) const {
     const S* w = (const S*)p.conv + (long)c * p.taps;
     float a = 0.f;
     for (int j = p.taps - 1; j >= 0; --j) a = fmaf(T::one(w[p.taps - 1 - j]), raw(p, tok - j, col, c), a);
-    return a / (1.f + expf(-a));
+    return silu(a);
+  }
+  // the same for up to four taps, all operands requested at once (taps that are not there, or inputs in front of the
+  // sequence, read something valid and count as zero)
+  __device__ __forceinline__ float conv4(const DeltaParams& p, int tok, int col, int c) const {
+    const S* w = (const S*)p.conv + (long)c * p.taps;
+    float x[4], a = 0.f;
+    S f[4];
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+      const S* src = tok >= j ? proj + (long)(tok - j) * p.pitch + col : ring + (long)ring_row(p, tok - j) * p.channels + c;
+      x[j] = T::one(*src);
+      f[j] = w[j < p.taps ? p.taps - 1 - j : 0];
+    }
+#pragma unroll
+    for (int j = 3; j >= 0; --j) {
+      const bool on = j < p.taps && p0 + tok - j >= (start > 0 ? start : 0);
+      a = on ? fmaf(T::one(f[j]), x[j], a) : a;
+    }
+    return silu(a);
   }
 };
-
-__device__ __forceinline__ float softplus_f32(float z) { return fmaxf(z, 0.f) + log1pf(expf(-fabsf(z))); }
-__device__ __forceinline__ float sigm(float z) { return 1.f / (1.f + expf(-z)); }
 
 // the last taps - 1 inputs of the call into the ring; head h writes its value channels, the first head of a group
 // its query and key channels
@@ -135,56 +166,119 @@ __device__ __forceinline__ void low_rank_rows(const typename T::storage* w, cons
   }
 }
 
-template <typename T, int NR>  // NR rows of S per thread in registers; 0: S stays in memory
+// The same with the matrix in registers: up to kLowRankHeld vectors of 8 per thread (16-bit types), requested before x is known.
+constexpr int kLowRankHeld = 4;
+template <typename T>
+struct LowRankHeld {
+  u32x4 w[kLowRankHeld];
+  int rows, iters;  // iters: vectors of a row per thread
+  __device__ __forceinline__ void load(int t, const typename T::storage* m, int n, int r) {
+    const int sub = t & 7;
+    rows = n;
+    iters = (r + 63) / 64;
+    int row = t >> 3, c = sub * 8;
+#pragma unroll
+    for (int i = 0; i < kLowRankHeld; ++i) {
+      w[i] = ld16(m + (row < n ? row : n - 1) * r + (c < r ? c : 0));
+      if (c >= r) w[i] = u32x4{0u, 0u, 0u, 0u};
+      step(t, row, c);
+    }
+  }
+  template <typename F>
+  __device__ __forceinline__ void run(int t, const float* x, int r, F f) const {
+    const int sub = t & 7;
+    float a = 0.f;
+    int row = t >> 3, c = sub * 8;
+#pragma unroll
+    for (int i = 0; i < kLowRankHeld; ++i) {
+      const float* xc = x + (c < r ? c : 0);
+#pragma unroll
+      for (int j = 0; j < 4; ++j) a = fmaf(T::hi(w[i][j]), xc[2 * j + 1], fmaf(T::lo(w[i][j]), xc[2 * j], a));
+      const int at = row;
+      if (step(t, row, c)) {  // uniform for the workgroup
+        a += dpp_f32<kDppXor1>(a);
+        a += dpp_f32<kDppXor2>(a);
+        a += dpp_f32<kDppHalfMirror>(a);
+        if (sub == 0 && at < rows) f(at, a);
+        a = 0.f;
+      }
+    }
+  }
+  // the next vector; true at the end of a row
+  __device__ __forceinline__ bool step(int t, int& row, int& c) const {
+    c += 64;
+    if (c < iters * 64) return false;
+    c = (t & 7) * 8;
+    row += 64;
+    return true;
+  }
+};
+
+// NR > 0: NR rows of S per thread in registers, for the sizes that delta_step_held names. 0: every size, S stays in memory.
+template <typename T, int NR>
 __global__ void __launch_bounds__(kStepThreads) delta_step_kernel(const DeltaParams p, int cgp) {
   typedef typename T::storage S;
   __shared__ float red[8][4];
-  const int t = threadIdx.x, lane = t & 63, wave = t >> 6;
+  int t = threadIdx.x;
+  const int lane = t & 63, wave = t >> 6;
   const int h = blockIdx.x, b = blockIdx.y, share = p.heads / p.kv_heads, kvh = h / share, nq = p.kv_heads * p.dk;
   const int parts = cgp <= 64 ? 8 : kStepThreads / cgp, cols = 4 * cgp;
-  float* qs = (float*)cd_smem;     // dk
-  float* ks = qs + p.dk;           // dk
-  float* gs = ks + p.dk;           // dk: decays
-  float* vs = gs + p.dk;           // dv; later u
-  float* og = vs + p.dv;           // dv: output gate
-  float* av = og + p.dv;           // max(ra, rg)
-  float* part = av + (p.ra > p.rg ? p.ra : p.rg) + ((4 - ((3 * p.dk + 2 * p.dv + (p.ra > p.rg ? p.ra : p.rg)) & 3)) & 3);  // [2][parts][cols]
+  // rows and columns past a head's end are zeros
+  const int dkp = NR > 0 ? NR * (kStepThreads / cgp) : p.dk;
+  float* qs = (float*)cd_smem;  // dkp
+  float* ks = qs + dkp;         // dkp
+  float* gs = ks + dkp;         // dkp: first the decays' biases, then the decays
+  float* vs = gs + dkp;         // cols; later u
+  float* og = vs + cols;        // dv: gain, then gain times output gate
+  float* gz = og + p.dv;        // dv: output gate before its sigmoid
+  float* av = gz + p.dv;        // ra
+  float* gv = av + p.ra;        // rg
+  float* part = gv + p.rg + ((4 - ((3 * dkp + 2 * p.dv + p.ra + p.rg) & 3)) & 3);  // [2][parts][cols]
   const DeltaRow<T> row(p, b);
   const int cg = t & (cgp - 1), rg = t / cgp, RG = kStepThreads / cgp, c0 = cg * 4;
   float* st = p.s + ((long)b * p.heads + h) * p.dk * p.dv;
-  const bool v4 = p.dv % 4 == 0;
   const float neg_a = -expf(T::one(((const S*)p.a_log)[h]));
-  const bool vec_a = p.ra % 8 == 0 && p.vec, vec_g = p.rg % 8 == 0 && p.vec;
   f32x4 sreg[NR > 0 ? NR : 1];
   auto load_s = [&](int d) {
     f32x4 x = {0.f, 0.f, 0.f, 0.f};
-    if (d < p.dk && c0 < p.dv) {
-      if (v4) {
-        x = *(const f32x4*)(st + (long)d * p.dv + c0);
-      } else {
+    const bool in = d < p.dk && c0 < p.dv;
+    if constexpr (NR > 0) {  // dv is a multiple of 4
+      const f32x4 y = *(const f32x4*)(st + (in ? d * p.dv + c0 : 0));
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-          if (c0 + j < p.dv) x[j] = st[(long)d * p.dv + c0 + j];
-      }
+      for (int j = 0; j < 4; ++j) x[j] = in ? y[j] : 0.f;
+    } else {
+#pragma unroll
+      for (int j = 0; j < 4; ++j)
+        if (in && c0 + j < p.dv) x[j] = st[d * p.dv + c0 + j];
     }
     return x;
   };
   auto store_s = [&](int d, f32x4 x) {
-    if (d < p.dk && c0 < p.dv) {
-      if (v4) {
-        *(f32x4*)(st + (long)d * p.dv + c0) = x;
-      } else {
+    if (d >= p.dk || c0 >= p.dv) return;
+    if constexpr (NR > 0) {
+      *(f32x4*)(st + d * p.dv + c0) = x;
+    } else {
 #pragma unroll
-        for (int j = 0; j < 4; ++j)
-          if (c0 + j < p.dv) st[(long)d * p.dv + c0 + j] = x[j];
-      }
+      for (int j = 0; j < 4; ++j)
+        if (c0 + j < p.dv) st[d * p.dv + c0 + j] = x[j];
     }
   };
+  const S *a2 = (const S*)p.a2 + (long)h * p.dk * p.ra, *g2 = (const S*)p.g2 + (long)h * p.dv * p.rg;
+  LowRankHeld<T> held_a, held_g;
   if constexpr (NR > 0) {
+    held_a.load(t, a2, p.dk, p.ra);
+    held_g.load(t, g2, p.dv, p.rg);
 #pragma unroll
     for (int i = 0; i < NR; ++i) sreg[i] = load_s(rg + RG * i);
   }
+  auto conv = [&](int tok, int col, int c) {
+    if constexpr (NR > 0) return row.conv4(p, tok, col, c);
+    else return row.conv(p, tok, col, c);
+  };
+  for (int i = p.dk + t; i < dkp; i += kStepThreads) qs[i] = ks[i] = gs[i] = 0.f;
+  for (int i = p.dv + t; i < cols; i += kStepThreads) vs[i] = 0.f;
   for (int tok = 0; tok < p.t; ++tok) {
+    asm volatile("" : "+v"(t));  // (one token is the rule: addresses kept from token to token would only cost registers)
     S* yrow = (S*)p.y + (((long)b * p.t + tok) * p.heads + h) * p.dv;
     if (!row.live(tok)) {  // uniform for the workgroup
       for (int i = t; i < p.dv; i += kStepThreads) yrow[i] = T::pack(0.f);
@@ -195,18 +289,22 @@ __global__ void __launch_bounds__(kStepThreads) delta_step_kernel(const DeltaPar
     float qq = 0.f, kk = 0.f, qk = 0.f;
     for (int d = t; d < p.dk; d += kStepThreads) {
       const int c = kvh * p.dk + d;
-      const float x = row.conv(p, tok, p.q_off + c, c), y = row.conv(p, tok, p.k_off + c, nq + c);
+      const float x = conv(tok, p.q_off + c, c), y = conv(tok, p.k_off + c, nq + c);
       qs[d] = x;
       ks[d] = y;
+      gs[d] = T::one(((const S*)p.dt_bias)[h * p.dk + d]);
       qq = fmaf(x, x, qq);
       kk = fmaf(y, y, kk);
       qk = fmaf(x, y, qk);
     }
     for (int e = kStepThreads - 1 - t; e < p.dv; e += kStepThreads) {  // (from the other end: dk threads are busy above)
       const int c = h * p.dv + e;
-      vs[e] = row.conv(p, tok, p.v_off + c, 2 * nq + c);
+      vs[e] = conv(tok, p.v_off + c, 2 * nq + c);
+      og[e] = T::one(((const S*)p.gain)[e]);
     }
     for (int i = t; i < p.ra; i += kStepThreads) av[i] = T::one(pr[p.a_off + i]);
+    for (int i = kStepThreads - 1 - t; i < p.rg; i += kStepThreads) gv[i] = T::one(pr[p.g_off + i]);
+    const float beta = sigm(T::one(pr[p.b_off + h]));
     qq = wave_sum(qq);
     kk = wave_sum(kk);
     qk = wave_sum(qk);
@@ -216,9 +314,15 @@ __global__ void __launch_bounds__(kStepThreads) delta_step_kernel(const DeltaPar
       red[wave][2] = qk;
     }
     __syncthreads();
-    low_rank_rows<T>((const S*)p.a2 + (long)h * p.dk * p.ra, av, p.dk, p.ra, vec_a, [&](int d, float z) {
-      gs[d] = expf(neg_a * softplus_f32(z + T::one(((const S*)p.dt_bias)[h * p.dk + d])));
-    });
+    auto decay = [&](int d, float z) { gs[d] += z; };
+    auto open = [&](int e, float z) { gz[e] = z; };
+    if constexpr (NR > 0) {
+      held_a.run(t, av, p.ra, decay);
+      held_g.run(t, gv, p.rg, open);
+    } else {
+      low_rank_rows<T>(a2, av, p.dk, p.ra, p.ra % 8 == 0 && p.vec, decay);
+      low_rank_rows<T>(g2, gv, p.dv, p.rg, p.rg % 8 == 0 && p.vec, open);
+    }
     qq = kk = qk = 0.f;
 #pragma unroll
     for (int w = 0; w < 8; ++w) {
@@ -228,7 +332,9 @@ __global__ void __launch_bounds__(kStepThreads) delta_step_kernel(const DeltaPar
     }
     const float rq = p.q_scale / sqrtf(qq + kUnitEps), rk = 1.f / sqrtf(kk + kUnitEps);
     __syncthreads();
-    for (int i = t; i < p.rg; i += kStepThreads) av[i] = T::one(pr[p.g_off + i]);
+    for (int d = t; d < p.dk; d += kStepThreads) gs[d] = decay_of(neg_a, gs[d]);
+    for (int e = kStepThreads - 1 - t; e < p.dv; e += kStepThreads) og[e] *= sigm(gz[e]);
+    __syncthreads();
     // decayed S against k and q
     f32x4 pk = {0.f, 0.f, 0.f, 0.f}, pq = pk;
     auto sweep = [&](f32x4& x, int d) {
@@ -242,8 +348,10 @@ __global__ void __launch_bounds__(kStepThreads) delta_step_kernel(const DeltaPar
     };
     if constexpr (NR > 0) {
 #pragma unroll
-      for (int i = 0; i < NR; ++i)
-        if (rg + RG * i < p.dk) sweep(sreg[i], rg + RG * i);
+      for (int i = 0; i < NR; ++i) {
+        sweep(sreg[i], rg + RG * i);
+        if (i % 4 == 3) asm volatile("" ::: "memory");  // (LDS reads of four rows ahead are enough)
+      }
     } else {
       for (int d = rg; d < p.dk; d += RG) {
         f32x4 x = load_s(d);
@@ -262,8 +370,6 @@ __global__ void __launch_bounds__(kStepThreads) delta_step_kernel(const DeltaPar
       *(f32x4*)&part[(parts + pi) * cols + c0] = pq;
     }
     __syncthreads();
-    low_rank_rows<T>((const S*)p.g2 + (long)h * p.dv * p.rg, av, p.dv, p.rg, vec_g, [&](int e, float z) { og[e] = sigm(z); });
-    const float beta = sigm(T::one(pr[p.b_off + h]));
     const float dot = qk * rq * rk;
     float ss = 0.f;
     for (int e = t; e < p.dv; e += kStepThreads) {
@@ -281,16 +387,18 @@ __global__ void __launch_bounds__(kStepThreads) delta_step_kernel(const DeltaPar
     ss = wave_sum(ss);
     if (lane == 0) red[wave][3] = ss;
     __syncthreads();
+    const f32x4 u = {vs[c0], vs[c0 + 1], vs[c0 + 2], vs[c0 + 3]};
     auto write = [&](f32x4& x, int d) {
       const float k = ks[d] * rk;
 #pragma unroll
-      for (int j = 0; j < 4; ++j)
-        if (c0 + j < p.dv) x[j] = fmaf(k, vs[c0 + j], x[j]);
+      for (int j = 0; j < 4; ++j) x[j] = fmaf(k, u[j], x[j]);
     };
     if constexpr (NR > 0) {
 #pragma unroll
-      for (int i = 0; i < NR; ++i)
-        if (rg + RG * i < p.dk) write(sreg[i], rg + RG * i);
+      for (int i = 0; i < NR; ++i) {
+        write(sreg[i], rg + RG * i);
+        if (i % 4 == 3) asm volatile("" ::: "memory");
+      }
     } else {
       for (int d = rg; d < p.dk; d += RG) {
         f32x4 x = load_s(d);
@@ -304,7 +412,7 @@ __global__ void __launch_bounds__(kStepThreads) delta_step_kernel(const DeltaPar
 #pragma unroll
     for (int w = 0; w < 8; ++w) ss += red[w][3];
     const float rs = 1.f / sqrtf(ss / (float)p.dv + p.eps);
-    for (int e = t; e < p.dv; e += kStepThreads) yrow[e] = T::pack(part[e] * rs * T::one(((const S*)p.gain)[e]) * og[e]);
+    for (int e = t; e < p.dv; e += kStepThreads) yrow[e] = T::pack(part[e] * rs * og[e]);
     __syncthreads();  // everything in LDS is free
   }
   if constexpr (NR > 0) {
@@ -317,41 +425,54 @@ __global__ void __launch_bounds__(kStepThreads) delta_step_kernel(const DeltaPar
 // ---------------------------------------------------------------------------------------
 // chunks
 // ---------------------------------------------------------------------------------------
-// 16 x 16 tile of X W^T over r: lane's row of X and of W (row lane % 16 each); D: column W row lane % 16, rows X 4 (lane / 16) + r
-template <typename T>
-__device__ __forceinline__ f32x4 low_rank_tile(const typename T::storage* x, const typename T::storage* w, int r, bool vec) {
+// N 16 x 16 tiles of X W^T over r: lane's row of X and of each tile's W (row lane % 16 each); D: column W row lane % 16,
+// rows X 4 (lane / 16) + r
+template <typename T, int N>
+__device__ __forceinline__ void low_rank_tiles(const typename T::storage* x, const typename T::storage* const (&w)[N], int r, bool vec, f32x4 (&acc)[N]) {
   const int g = (threadIdx.x & 63) >> 4;
-  f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+  for (int n = 0; n < N; ++n) acc[n] = f32x4{0.f, 0.f, 0.f, 0.f};
   if constexpr (T::kDtype == MUI_DTYPE_F32) {
     for (int k = 0; k < r; k += 4) {
-      const int e = k + g;
-      acc = mfma_f32(e < r ? x[e] : 0.f, e < r ? w[e] : 0.f, acc);
+      const int e = k + g < r ? k + g : 0;
+      const float a = k + g < r ? x[e] : 0.f;
+#pragma unroll
+      for (int n = 0; n < N; ++n) acc[n] = mfma_f32(a, w[n][e], acc[n]);
+    }
+  } else if (vec) {
+    for (int k = 0; k < r; k += 64) {
+      u32x4 a[2], b[2][N];
+#pragma unroll
+      for (int u = 0; u < 2; ++u) {
+        const int e = k + 32 * u + 8 * g, c = e < r ? e : 0;
+        a[u] = ld16(x + c);
+        if (e >= r) a[u] = u32x4{0u, 0u, 0u, 0u};
+#pragma unroll
+        for (int n = 0; n < N; ++n) b[u][n] = ld16(w[n] + c);
+      }
+#pragma unroll
+      for (int u = 0; u < 2; ++u)
+#pragma unroll
+        for (int n = 0; n < N; ++n) acc[n] = mfma16x16x32<T>(a[u], b[u][n], acc[n]);
     }
   } else {
+#pragma unroll 1
     for (int k = 0; k < r; k += 32) {
       const int e = k + 8 * g;
-      u32x4 a, b;
-      if (vec) {
-        const u32x4 zero = {0u, 0u, 0u, 0u};
-        a = ld16(x + (e < r ? e : 0));
-        b = ld16(w + (e < r ? e : 0));
-        a = e < r ? a : zero;
-        b = e < r ? b : zero;
-      } else {
-        uint32_t aw[4], bw[4];
+      auto words = [&](const typename T::storage* m) {
+        u32x4 v;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
           const int e0 = e + 2 * i, e1 = e0 + 1;
-          aw[i] = (e0 < r ? (uint32_t)x[e0] : 0u) | ((e1 < r ? (uint32_t)x[e1] : 0u) << 16);
-          bw[i] = (e0 < r ? (uint32_t)w[e0] : 0u) | ((e1 < r ? (uint32_t)w[e1] : 0u) << 16);
+          v[i] = (e0 < r ? (uint32_t)m[e0] : 0u) | ((e1 < r ? (uint32_t)m[e1] : 0u) << 16);
         }
-        a = u32x4{aw[0], aw[1], aw[2], aw[3]};
-        b = u32x4{bw[0], bw[1], bw[2], bw[3]};
-      }
-      acc = mfma16x16x32<T>(a, b, acc);
+        return v;
+      };
+      const u32x4 a = words(x);
+#pragma unroll
+      for (int n = 0; n < N; ++n) acc[n] = mfma16x16x32<T>(a, words(w[n]), acc[n]);
     }
   }
-  return acc;
 }
 
 // 16 consecutive tokens of a convolved channel, from token tok0 >= 0 (may reach past the call: zeros). x: the TAPS - 1
@@ -372,9 +493,8 @@ struct ConvTaps {
       const int tok = tok0 - (TAPS - 1) + j;
       const long slot = row.p0 + tok;
       const bool on = slot >= row.start && slot >= 0 && j >= TAPS - p.taps;
-      const long ring_row = (long)((uint32_t)(slot > 0 ? slot : 0) % (uint32_t)p.ring_rows);
       // (sub-chunks behind the call's last token read that one: their outputs are zero anyway)
-      const S* src = tok >= 0 ? row.proj + (long)(tok < p.t ? tok : p.t - 1) * p.pitch + col : row.ring + ring_row * p.channels + c;
+      const S* src = tok >= 0 ? row.proj + (long)(tok < p.t ? tok : p.t - 1) * p.pitch + col : row.ring + (long)row.ring_row(p, tok) * p.channels + c;
       const float v = T::one(*src);
       x[j] = on ? v : 0.f;
     }
@@ -400,8 +520,7 @@ struct ConvTaps {
       float a = 0.f;
 #pragma unroll
       for (int j = 0; j < TAPS; ++j) a = fmaf(w[j], z[i + j], a);
-      a /= 1.f + expf(-a);
-      y[i] = i >= first && i < last ? a : 0.f;
+      y[i] = i >= first && i < last ? silu(a) : 0.f;
     }
 #pragma unroll
     for (int j = 0; j < TAPS - 1; ++j) x[j] = z[16 + j];
@@ -410,6 +529,7 @@ struct ConvTaps {
 
 // 1. grid (chunks, heads, batch); wave w owns sub-chunk w, lane = channel of a block of 64 (NB blocks: dk <= 64 NB)
 constexpr int kDPitch = 68;  // 16 rows x 4 consecutive k in 64 different banks
+constexpr int kDInvPitch = 20;
 template <typename T, int NB, int TAPS>
 __global__ void __launch_bounds__(256, NB > 2 ? 1 : 2) delta_prepare_kernel(const DeltaParams p) {
   typedef typename T::storage S;
@@ -417,7 +537,7 @@ __global__ void __launch_bounds__(256, NB > 2 ? 1 : 2) delta_prepare_kernel(cons
   float* qh = (float*)cd_smem;              // [64][kDPitch]: q times the decays since the start of its sub-chunk
   float* kh = qh + kDChunk * kDPitch;       // the same of k
   float* ke = kh + kDChunk * kDPitch;       // k times the decays up to the end of its sub-chunk
-  float* lm = ke + kDChunk * kDPitch;       // [64][kDPitch]: beta_t A_ts
+  float* lm = ke + kDChunk * kDPitch;       // [64][kDPitch]: -beta_t A_ts
   __shared__ float gm[4][64 * NB], bt[kDChunk];
   const int t = threadIdx.x, lane = t & 63, wave = __builtin_amdgcn_readfirstlane(t >> 6), g4 = lane >> 4, i16 = lane & 15;
   const int chunk = blockIdx.x, h = blockIdx.y, b = blockIdx.z, kvh = h / (p.heads / p.kv_heads), nq = p.kv_heads * p.dk;
@@ -452,18 +572,24 @@ __global__ void __launch_bounds__(256, NB > 2 ? 1 : 2) delta_prepare_kernel(cons
     float* z = qh + wave * kDSub * kDPitch;  // this wave's rows
 #pragma unroll
     for (int nb = 0; nb < NB; ++nb) {
-#pragma unroll 1
+      const S* wr[4];
+      float bias[4];
+      f32x4 v[4];
+#pragma unroll
       for (int ct = 0; ct < 4; ++ct) {
         const int d = nb * 64 + ct * 16 + i16, dc = h * p.dk + (d < p.dk ? d : 0);
-        const f32x4 v = low_rank_tile<T>(x, (const S*)p.a2 + (long)dc * p.ra, p.ra, vec);
-        const float bias = T::one(((const S*)p.dt_bias)[dc]);
+        wr[ct] = (const S*)p.a2 + (long)dc * p.ra;
+        bias[ct] = T::one(((const S*)p.dt_bias)[dc]);
+      }
+      low_rank_tiles<T, 4>(x, wr, p.ra, vec, v);
+#pragma unroll
+      for (int ct = 0; ct < 4; ++ct)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           const int tr = tok0 + 4 * g4 + r;
-          const float e = expf(neg_a * softplus_f32(v[r] + bias));
+          const float e = decay_of(neg_a, v[ct][r] + bias[ct]);
           z[(4 * g4 + r) * kDPitch + ct * 16 + i16] = tr < p.t && row.live(tr) ? e : 1.f;
         }
-      }
       __builtin_amdgcn_wave_barrier();
 #pragma unroll
       for (int i = 0; i < 16; ++i) g[nb][i] = z[i * kDPitch + lane];
@@ -527,7 +653,7 @@ __global__ void __launch_bounds__(256, NB > 2 ? 1 : 2) delta_prepare_kernel(cons
     c += __shfl_xor(c, 32);
     if (g4 == 0) {
       const int tr = wave * kDSub + i16, sc = wave * kDSub + s;
-      lm[tr * kDPitch + sc] = a * bt[tr];  // zero on and above the diagonal
+      lm[tr * kDPitch + sc] = -a * bt[tr];  // zero on and above the diagonal
       aqk_out[tr * kDChunk + sc] = c;      // zero above it
     }
   }
@@ -589,63 +715,116 @@ __global__ void __launch_bounds__(256, NB > 2 ? 1 : 2) delta_prepare_kernel(cons
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int tr = pi[u] * kDSub + 4 * g4 + r, sc = pj[u] * kDSub + i16;
-      lm[tr * kDPitch + sc] = akk[u][r] * bt[tr];
+      lm[tr * kDPitch + sc] = -akk[u][r] * bt[tr];
       aqk_out[tr * kDChunk + sc] = aqk[u][r];
     }
   }
   __syncthreads();  // lm, and w_out as seen by this workgroup
-  // x_t = beta_t rhs_t - sum_{s < t} lm_ts x_s, one column per thread: W from the decayed keys, U0 from the values
-  // (which pass through their place in memory: short code instead of 64 convolutions in a row)
+  // X = (1 + L)^-1 diag(beta) R by blocks of 16 rows, X_I = D_I^-1 (beta_I R_I - sum_{J < I} L_IJ X_J): W from the decayed
+  // keys, U0 from the values. First the inverses of the diagonal blocks, one per wave, one column per lane.
+  float* dinv = qh;  // [64][kDInvPitch]
+  {
+    float x[16];
+#pragma unroll
+    for (int i = 0; i < 16; ++i) {
+      x[i] = i == i16 ? 1.f : 0.f;
+#pragma unroll
+      for (int s = 0; s < i; ++s) x[i] = fmaf(lm[(wave * kDSub + i) * kDPitch + wave * kDSub + s], x[s], x[i]);
+    }
+    if (g4 == 0)
+#pragma unroll
+      for (int i = 0; i < 16; ++i) dinv[(wave * kDSub + i) * kDInvPitch + i16] = x[i];
+  }
+  __syncthreads();
+  f32x4 lo[6], di[4], be[4];
+#pragma unroll
+  for (int I = 0; I < 4; ++I) {
+    di[I] = *(const f32x4*)&dinv[(I * kDSub + i16) * kDInvPitch + 4 * g4];
+#pragma unroll
+    for (int r = 0; r < 4; ++r) be[I][r] = bt[I * kDSub + 4 * g4 + r];
+#pragma unroll
+    for (int J = 0; J < I; ++J) lo[I * (I - 1) / 2 + J] = *(const f32x4*)&lm[(I * kDSub + i16) * kDPitch + J * kDSub + 4 * g4];
+  }
+  // columns in the layout of accumulators: an accumulator is the next product's right operand with the contraction
+  // dealt out as 4 g + r
+  auto solve = [&](auto& x) {
+    constexpr int N = sizeof(x) / sizeof(x[0]);
+#pragma unroll
+    for (int I = 0; I < 4; ++I) {
+      f32x4 c[N];
+#pragma unroll
+      for (int n = 0; n < N; ++n) c[n] = x[n][I] * be[I];
+#pragma unroll
+      for (int J = 0; J < I; ++J)
+#pragma unroll
+        for (int r = 0; r < 4; ++r)
+#pragma unroll
+          for (int n = 0; n < N; ++n) c[n] = mfma_f32(lo[I * (I - 1) / 2 + J][r], x[n][J][r], c[n]);
+#pragma unroll
+      for (int n = 0; n < N; ++n) x[n][I] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+#pragma unroll
+        for (int n = 0; n < N; ++n) x[n][I] = mfma_f32(di[I][r], c[n][r], x[n][I]);
+    }
+  };
+  {
+    f32x4 x[NB][4];
+    float* wp = w_out + (4 * g4) * DKP + wave * 16 + i16;
+#pragma unroll
+    for (int n = 0; n < NB; ++n)
+#pragma unroll
+      for (int I = 0; I < 4; ++I)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) x[n][I][r] = wp[(I * kDSub + r) * DKP + n * 64];
+    solve(x);
+#pragma unroll
+    for (int n = 0; n < NB; ++n)
+#pragma unroll
+      for (int I = 0; I < 4; ++I)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) wp[(I * kDSub + r) * DKP + n * 64] = x[n][I][r];
+  }
+  const int lead = row.start > row.p0 ? (row.start - row.p0 < p.t ? (int)(row.start - row.p0) : p.t) : -(int)(row.p0 - (row.start > 0 ? row.start : 0));
 #pragma unroll 1
-  for (int c = t; c < DKP + p.dvp; c += 256) {
-    const bool is_w = c < DKP;  // (a multiple of 64: uniform for the wave)
-    float* wcol = w_out + c;
-    float* ucol = p.u0 + (bhc * p.dvp + (is_w ? 0 : c - DKP)) * kDChunk;
-    float x[kDChunk];
-    if (is_w) {
+  for (int v0 = wave * 16; v0 < p.dvp; v0 += 128) {  // columns v0 .. and v0 + 64 ..
+    f32x4 x[2][4];
 #pragma unroll
-      for (int i = 0; i < kDChunk; ++i) x[i] = wcol[i * DKP];
-    } else {
-      const int v = c - DKP, ch = h * p.dv + (v < p.dv ? v : 0);
-      ConvTaps<T, TAPS> cv;
-      cv.start(p, row, chunk * kDChunk, p.v_off + ch, 2 * nq + ch);
-#pragma unroll 1
-      for (int i = 0; i < kDChunk; i += 16) {
-        float y[16];
-        cv.run(p, row, chunk * kDChunk + i, p.v_off + ch, y);
+    for (int n = 0; n < 2; ++n) {
+      const int v = v0 + 64 * n + i16, ch = h * p.dv + (v < p.dv ? v : 0);
+      float w[TAPS];
 #pragma unroll
-        for (int j = 0; j < 16; j += 4) *(f32x4*)(ucol + i + j) = v < p.dv ? f32x4{y[j], y[j + 1], y[j + 2], y[j + 3]} : f32x4{0.f, 0.f, 0.f, 0.f};
+      for (int j = 0; j < TAPS; ++j) {
+        const int i = j - (TAPS - p.taps);
+        const float f = T::one(((const S*)p.conv)[(long)(2 * nq + ch) * p.taps + (i > 0 ? i : 0)]);
+        w[j] = i >= 0 && v < p.dv ? f : 0.f;
       }
 #pragma unroll
-      for (int i = 0; i < kDChunk; i += 4) {
-        const f32x4 y = *(const f32x4*)(ucol + i);
+      for (int I = 0; I < 4; ++I) {
+        float z[TAPS + 3];
 #pragma unroll
-        for (int j = 0; j < 4; ++j) x[i + j] = y[j];
+        for (int j = 0; j < TAPS + 3; ++j) {
+          const int tok = chunk * kDChunk + I * kDSub + 4 * g4 - (TAPS - 1) + j;
+          const S* src = row.proj + (tok < 0 ? 0 : (tok < p.t ? tok : p.t - 1)) * p.pitch + p.v_off + ch;
+          if (chunk == 0 && I == 0 && tok < 0) src = row.ring + (long)row.ring_row(p, tok) * p.channels + 2 * nq + ch;
+          const float f = T::one(*src);
+          z[j] = tok >= lead && tok < p.t && j >= TAPS - p.taps ? f : 0.f;  // (older ring rows hold anything)
+        }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+          float a = 0.f;
+#pragma unroll
+          for (int j = 0; j < TAPS; ++j) a = fmaf(w[j], z[r + j], a);
+          x[n][I][r] = silu(a);
+        }
       }
     }
+    solve(x);
 #pragma unroll
-    for (int i = 0; i < kDChunk; ++i) {
-      float a = x[i] * bt[i], a2 = 0.f;
+    for (int n = 0; n < 2; ++n)
+      if (v0 + 64 * n < p.dvp)
 #pragma unroll
-      for (int s = 0; s + 4 <= i; s += 4) {
-        const f32x4 l = *(const f32x4*)&lm[i * kDPitch + s];
-        a = fmaf(-l[0], x[s], a);
-        a2 = fmaf(-l[1], x[s + 1], a2);
-        a = fmaf(-l[2], x[s + 2], a);
-        a2 = fmaf(-l[3], x[s + 3], a2);
-      }
-#pragma unroll
-      for (int s = i & ~3; s < i; ++s) a = fmaf(-lm[i * kDPitch + s], x[s], a);
-      x[i] = a + a2;
-      if (i % 4 == 3) asm volatile("" ::: "memory");  // the matrix is read row by row, not all of it ahead
-    }
-    if (is_w) {
-#pragma unroll
-      for (int i = 0; i < kDChunk; ++i) wcol[i * DKP] = x[i];
-    } else {
-#pragma unroll
-      for (int i = 0; i < kDChunk; i += 4) *(f32x4*)(ucol + i) = f32x4{x[i], x[i + 1], x[i + 2], x[i + 3]};
-    }
+        for (int I = 0; I < 4; ++I) *(f32x4*)(p.u0 + (bhc * p.dvp + v0 + 64 * n + i16) * kDChunk + I * kDSub + 4 * g4) = x[n][I];
   }
 }
 
@@ -787,21 +966,38 @@ __global__ void __launch_bounds__(256) delta_output_kernel(const DeltaParams p) 
     const int tr = tok0 + 4 * g + r < p.t ? tok0 + 4 * g + r : p.t - 1;
     at[r] = (((long)b * p.t + tr) * p.heads + h) * p.dv;
   }
-  for (int c = i16; c < p.dv; c += 16)
+  for (int c0 = 0; c0 < p.dv; c0 += 64)
 #pragma unroll
-    for (int r = 0; r < 4; ++r) {
-      const float o = p.o[at[r] + c];
-      ss[r] = fmaf(o, o, ss[r]);
+    for (int n = 0; n < 4; ++n) {
+      const int c = c0 + 16 * n + i16;
+#pragma unroll
+      for (int r = 0; r < 4; ++r) {
+        const float o = p.o[at[r] + (c < p.dv ? c : 0)];
+        ss[r] = c < p.dv ? fmaf(o, o, ss[r]) : ss[r];
+      }
     }
 #pragma unroll
   for (int r = 0; r < 4; ++r) ss[r] = 1.f / sqrtf(row16_sum(ss[r]) / (float)p.dv + p.eps);
-  for (int c0 = 0; c0 < p.dv; c0 += 16) {
-    const int c = c0 + i16, cc = c < p.dv ? c : p.dv - 1;
-    const f32x4 z = low_rank_tile<T>(x, (const S*)p.g2 + ((long)h * p.dv + cc) * p.rg, p.rg, vec);
-    const float gain = T::one(((const S*)p.gain)[cc]);
+  for (int c0 = 0; c0 < p.dv; c0 += 64) {
+    const S* wr[4];
+    float gain[4], o[4][4];
+    f32x4 z[4];
 #pragma unroll
-    for (int r = 0; r < 4; ++r)
-      if (c < p.dv && tok0 + 4 * g + r < p.t) ((S*)p.y)[at[r] + c] = T::pack(p.o[at[r] + c] * ss[r] * gain * sigm(z[r]));
+    for (int n = 0; n < 4; ++n) {
+      const int c = c0 + 16 * n + i16, cc = c < p.dv ? c : p.dv - 1;
+      wr[n] = (const S*)p.g2 + ((long)h * p.dv + cc) * p.rg;
+      gain[n] = T::one(((const S*)p.gain)[cc]);
+#pragma unroll
+      for (int r = 0; r < 4; ++r) o[n][r] = p.o[at[r] + cc];
+    }
+    low_rank_tiles<T, 4>(x, wr, p.rg, vec, z);
+#pragma unroll
+    for (int n = 0; n < 4; ++n) {
+      const int c = c0 + 16 * n + i16;
+#pragma unroll
+      for (int r = 0; r < 4; ++r)
+        if (c < p.dv && tok0 + 4 * g + r < p.t) ((S*)p.y)[at[r] + c] = T::pack(o[n][r] * ss[r] * gain[n] * sigm(z[n][r]));
+    }
   }
 }
 
@@ -813,26 +1009,36 @@ constexpr int kMaxDeltaKey = 256, kMaxDeltaTaps = 8;
 static bool delta_chunked(int dk, int taps) { return dk <= kMaxDeltaKey && taps <= kMaxDeltaTaps; }
 static int delta_dkp(int dk) { return dk <= 64 ? 64 : (dk <= 128 ? 128 : 256); }
 
+// sizes whose operands the step kernel may keep in registers
+static bool delta_step_held(const DeltaParams& p) {
+  auto fits = [](int rows, int r) { return r % 8 == 0 && ceil_div(rows, 64) * ceil_div(r, 64) <= kLowRankHeld; };
+  return p.vec && p.dv % 4 == 0 && p.taps <= 4 && fits(p.dk, p.ra) && fits(p.dv, p.rg);
+}
+
 template <typename T>
 static int launch_delta_step(hipStream_t s, const DeltaParams& p) {
   int cgp = 16;
   while (cgp * 4 < p.dv) cgp <<= 1;
-  if (cgp > kStepThreads) return MUI_ERR_UNSUPPORTED;
+  if (cgp > kStepThreads || (long)p.dk * p.dv > (1L << 30)) return MUI_ERR_UNSUPPORTED;
   const int rows = ceil_div(p.dk, kStepThreads / cgp), parts = cgp <= 64 ? 8 : kStepThreads / cgp;
-  const size_t lds = ((size_t)3 * p.dk + 2 * p.dv + (p.ra > p.rg ? p.ra : p.rg) + 4 + (size_t)2 * parts * 4 * cgp) * 4;
   const dim3 grid(p.heads, p.batch), block(kStepThreads);
-  auto launch = [&](auto kernel) {
+  auto launch = [&](auto kernel, int nr) {
+    const size_t dkp = nr > 0 ? (size_t)nr * (kStepThreads / cgp) : p.dk;
+    const size_t lds = (3 * dkp + 4 * cgp + 2 * p.dv + p.ra + p.rg + 4 + (size_t)2 * parts * 4 * cgp) * 4;
     if (lds > 160 * 1024) return (int)MUI_ERR_UNSUPPORTED;
     if (lds > 48 * 1024 && hipFuncSetAttribute((const void*)kernel, hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds) != hipSuccess)
       return (int)MUI_ERR_LAUNCH;
     hipLaunchKernelGGL(kernel, grid, block, lds, s, p, cgp);
     return launch_status();
   };
-  if (rows <= 4) return launch(delta_step_kernel<T, 4>);
-  if (rows <= 8) return launch(delta_step_kernel<T, 8>);
-  if (rows <= 16) return launch(delta_step_kernel<T, 16>);
-  if (rows <= 32) return launch(delta_step_kernel<T, 32>);
-  return launch(delta_step_kernel<T, 0>);
+  if constexpr (T::kDtype != MUI_DTYPE_F32) {
+    if (delta_step_held(p)) {
+      if (rows <= 4) return launch(delta_step_kernel<T, 4>, 4);
+      if (rows <= 8) return launch(delta_step_kernel<T, 8>, 8);
+      if (rows <= 16) return launch(delta_step_kernel<T, 16>, 16);
+    }
+  }
+  return launch(delta_step_kernel<T, 0>, 0);
 }
 
 template <typename T, int NB>
