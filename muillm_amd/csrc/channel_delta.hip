@@ -440,10 +440,10 @@ __device__ __forceinline__ void low_rank_tiles(const typename T::storage* x, con
       for (int n = 0; n < N; ++n) acc[n] = mfma_f32(a, w[n][e], acc[n]);
     }
   } else if (vec) {
-    for (int k = 0; k < r; k += 64) {
-      u32x4 a[2], b[2][N];
+    for (int k = 0; k < r; k += 128) {
+      u32x4 a[4], b[4][N];
 #pragma unroll
-      for (int u = 0; u < 2; ++u) {
+      for (int u = 0; u < 4; ++u) {
         const int e = k + 32 * u + 8 * g, c = e < r ? e : 0;
         a[u] = ld16(x + c);
         if (e >= r) a[u] = u32x4{0u, 0u, 0u, 0u};
@@ -451,7 +451,7 @@ __device__ __forceinline__ void low_rank_tiles(const typename T::storage* x, con
         for (int n = 0; n < N; ++n) b[u][n] = ld16(w[n] + c);
       }
 #pragma unroll
-      for (int u = 0; u < 2; ++u)
+      for (int u = 0; u < 4; ++u)
 #pragma unroll
         for (int n = 0; n < N; ++n) acc[n] = mfma16x16x32<T>(a[u], b[u][n], acc[n]);
     }
@@ -475,63 +475,61 @@ __device__ __forceinline__ void low_rank_tiles(const typename T::storage* x, con
   }
 }
 
-// 16 consecutive tokens of a convolved channel, from token tok0 >= 0 (may reach past the call: zeros). x: the TAPS - 1
-// inputs in front of tok0 on entry, those in front of tok0 + 16 on return. TAPS >= p.taps: older ones weigh zero.
+// 16 consecutive tokens of a convolved channel, from token tok0 >= 0 (uniform for the wave); TAPS >= p.taps: older ones
+// weigh zero. Tokens behind the call read its last one: nothing that reaches a result depends on them (beta is zero there).
 template <typename T, int TAPS>
-struct ConvTaps {
-  float w[TAPS], x[TAPS - 1 > 0 ? TAPS - 1 : 1];
-  __device__ __forceinline__ void start(const DeltaParams& p, const DeltaRow<T>& row, int tok0, int col, int c) {
-    typedef typename T::storage S;
+struct ConvRun {
+  typedef typename T::storage S;
+  S w[TAPS], x[TAPS + 15];
+  // column `col` of the projection and channel `c` of lane 0's channel, `lane`: this one's offset
+  __device__ __forceinline__ void load(const DeltaParams& p, const DeltaRow<T>& row, int tok0, int col, int c, int lane) {
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) {
       const int i = j - (TAPS - p.taps);
-      const float v = T::one(((const S*)p.conv)[(long)c * p.taps + (i > 0 ? i : 0)]);
-      w[j] = i >= 0 ? v : 0.f;
+      w[j] = ((const S*)p.conv)[(long)(c + lane) * p.taps + (i > 0 ? i : 0)];
     }
 #pragma unroll
-    for (int j = 0; j < TAPS - 1; ++j) {
+    for (int j = 0; j < TAPS + 15; ++j) {
       const int tok = tok0 - (TAPS - 1) + j;
-      const long slot = row.p0 + tok;
-      const bool on = slot >= row.start && slot >= 0 && j >= TAPS - p.taps;
-      // (sub-chunks behind the call's last token read that one: their outputs are zero anyway)
-      const S* src = tok >= 0 ? row.proj + (long)(tok < p.t ? tok : p.t - 1) * p.pitch + col : row.ring + (long)row.ring_row(p, tok) * p.channels + c;
-      const float v = T::one(*src);
-      x[j] = on ? v : 0.f;
+      const S* src = tok >= 0 ? row.proj + (tok < p.t ? tok : p.t - 1) * p.pitch + col : row.ring + (long)row.ring_row(p, tok) * p.channels + c;
+      x[j] = src[lane];
     }
   }
-  __device__ __forceinline__ void run(const DeltaParams& p, const DeltaRow<T>& row, int tok0, int col, float (&y)[16]) {
-    typedef typename T::storage S;
-    // live tokens of the sixteen: first <= i < last (in vector registers: sixteen scalar conditions would spill)
-    const long lead = row.start - row.p0;
-    int first = (int)(lead > 0 ? (lead < p.t ? lead : p.t) : 0) - tok0, last = p.t - tok0;
-    asm volatile("" : "+v"(first), "+v"(last));
-    float z[16 + TAPS - 1];
+  // lead: the first token whose input counts (delta_lead)
+  __device__ __forceinline__ void run(const DeltaParams& p, int tok0, int lead, float (&y)[16]) const {
+    float f[TAPS], z[TAPS + 15];
 #pragma unroll
-    for (int j = 0; j < TAPS - 1; ++j) z[j] = x[j];
-    const S* src = row.proj + (long)(tok0 < p.t ? tok0 : p.t - 1) * p.pitch + col;
-    const int pitch = (int)p.pitch;
+    for (int j = 0; j < TAPS; ++j) f[j] = j >= TAPS - p.taps ? T::one(w[j]) : 0.f;
 #pragma unroll
-    for (int i = 0; i < 16; ++i) {
-      const float v = T::one(src[(unsigned)((i < last ? i : 0) * pitch)]);
-      z[TAPS - 1 + i] = i >= first && i < last ? v : 0.f;
+    for (int j = 0; j < TAPS + 15; ++j) z[j] = T::one(x[j]);
+    if (tok0 - (TAPS - 1) < lead) {
+      int first = lead - (tok0 - (TAPS - 1));
+      asm volatile("" : "+v"(first));  // (compared in vector registers: so many scalar conditions would spill)
+#pragma unroll
+      for (int j = 0; j < TAPS + 15; ++j) z[j] = j >= first ? z[j] : 0.f;
     }
 #pragma unroll
     for (int i = 0; i < 16; ++i) {
       float a = 0.f;
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) a = fmaf(w[j], z[i + j], a);
-      y[i] = i >= first && i < last ? silu(a) : 0.f;
+      for (int j = 0; j < TAPS; ++j) a = fmaf(f[j], z[i + j], a);
+      y[i] = silu(a);
     }
-#pragma unroll
-    for (int j = 0; j < TAPS - 1; ++j) x[j] = z[16 + j];
   }
 };
+
+// the first token (from this call's start; negative: in the ring) that a convolution may see
+template <typename T>
+__device__ __forceinline__ int delta_lead(const DeltaParams& p, const DeltaRow<T>& row) {
+  const long lead = (row.start > 0 ? row.start : 0) - row.p0;
+  return lead < 1 - p.taps ? 1 - p.taps : (lead < p.t ? (int)lead : p.t);
+}
 
 // 1. grid (chunks, heads, batch); wave w owns sub-chunk w, lane = channel of a block of 64 (NB blocks: dk <= 64 NB)
 constexpr int kDPitch = 68;  // 16 rows x 4 consecutive k in 64 different banks
 constexpr int kDInvPitch = 20;
 template <typename T, int NB, int TAPS>
-__global__ void __launch_bounds__(256, NB > 2 ? 1 : 2) delta_prepare_kernel(const DeltaParams p) {
+__global__ void __launch_bounds__(256, NB > 2 || TAPS > 4 ? 1 : 2) delta_prepare_kernel(const DeltaParams p) {
   typedef typename T::storage S;
   constexpr int DKP = 64 * NB;  // = p.dkp
   float* qh = (float*)cd_smem;              // [64][kDPitch]: q times the decays since the start of its sub-chunk
@@ -551,17 +549,24 @@ __global__ void __launch_bounds__(256, NB > 2 ? 1 : 2) delta_prepare_kernel(cons
 
   // q, k and decays of this wave's 16 tokens, channel `lane` of every block
   float q[NB][16], k[NB][16], g[NB][16];
+  const int lead = delta_lead<T>(p, row);
+  {
+    ConvRun<T, TAPS> cq[NB], ck[NB];
 #pragma unroll
-  for (int nb = 0; nb < NB; ++nb) {
-    const int d = nb * 64 + lane, c = kvh * p.dk + (d < p.dk ? d : 0);
-    ConvTaps<T, TAPS> cv;
-    cv.start(p, row, tok0, p.q_off + c, c);
-    cv.run(p, row, tok0, p.q_off + c, q[nb]);
-    cv.start(p, row, tok0, p.k_off + c, nq + c);
-    cv.run(p, row, tok0, p.k_off + c, k[nb]);
-    if (d >= p.dk) {
+    for (int nb = 0; nb < NB; ++nb) {
+      const int c = kvh * p.dk, d = nb * 64 + lane < p.dk ? nb * 64 + lane : 0;
+      cq[nb].load(p, row, tok0, p.q_off + c, c, d);
+      ck[nb].load(p, row, tok0, p.k_off + c, nq + c, d);
+    }
+    asm volatile("" ::: "memory");  // all of it is requested before the first use
 #pragma unroll
-      for (int i = 0; i < 16; ++i) q[nb][i] = k[nb][i] = 0.f;
+    for (int nb = 0; nb < NB; ++nb) {
+      cq[nb].run(p, tok0, lead, q[nb]);
+      ck[nb].run(p, tok0, lead, k[nb]);
+      if (nb * 64 + lane >= p.dk) {
+#pragma unroll
+        for (int i = 0; i < 16; ++i) q[nb][i] = k[nb][i] = 0.f;
+      }
     }
   }
   {
@@ -719,6 +724,29 @@ __global__ void __launch_bounds__(256, NB > 2 ? 1 : 2) delta_prepare_kernel(cons
       aqk_out[tr * kDChunk + sc] = aqk[u][r];
     }
   }
+  // the values' inputs in front of their convolution (columns v0 + i16 and v0 + 64 + i16, rows 4 g .. of every sub-chunk)
+  S vw[2][TAPS], vx[2][4][TAPS + 3];
+  auto load_v = [&](int v0) {
+#pragma unroll
+    for (int n = 0; n < 2; ++n) {
+      const int v = v0 + 64 * n + i16, ch = h * p.dv + (v < p.dv ? v : 0);
+#pragma unroll
+      for (int j = 0; j < TAPS; ++j) {
+        const int i = j - (TAPS - p.taps);
+        vw[n][j] = ((const S*)p.conv)[(long)(2 * nq + ch) * p.taps + (i > 0 ? i : 0)];
+      }
+#pragma unroll
+      for (int I = 0; I < 4; ++I)
+#pragma unroll
+        for (int j = 0; j < TAPS + 3; ++j) {
+          const int tok = chunk * kDChunk + I * kDSub + 4 * g4 - (TAPS - 1) + j;
+          const S* src = row.proj + (tok < 0 ? 0 : (tok < p.t ? tok : p.t - 1)) * p.pitch + p.v_off + ch;
+          if (chunk == 0 && I == 0 && tok < 0) src = row.ring + (long)row.ring_row(p, tok) * p.channels + 2 * nq + ch;
+          vx[n][I][j] = *src;
+        }
+    }
+  };
+  if (wave * 16 < p.dvp) load_v(wave * 16);
   __syncthreads();  // lm, and w_out as seen by this workgroup
   // X = (1 + L)^-1 diag(beta) R by blocks of 16 rows, X_I = D_I^-1 (beta_I R_I - sum_{J < I} L_IJ X_J): W from the decayed
   // keys, U0 from the values. First the inverses of the diagonal blocks, one per wave, one column per lane.
@@ -785,36 +813,25 @@ __global__ void __launch_bounds__(256, NB > 2 ? 1 : 2) delta_prepare_kernel(cons
 #pragma unroll
         for (int r = 0; r < 4; ++r) wp[(I * kDSub + r) * DKP + n * 64] = x[n][I][r];
   }
-  const int lead = row.start > row.p0 ? (row.start - row.p0 < p.t ? (int)(row.start - row.p0) : p.t) : -(int)(row.p0 - (row.start > 0 ? row.start : 0));
 #pragma unroll 1
   for (int v0 = wave * 16; v0 < p.dvp; v0 += 128) {  // columns v0 .. and v0 + 64 ..
     f32x4 x[2][4];
+    if (v0 != wave * 16) load_v(v0);
 #pragma unroll
     for (int n = 0; n < 2; ++n) {
-      const int v = v0 + 64 * n + i16, ch = h * p.dv + (v < p.dv ? v : 0);
-      float w[TAPS];
+      float f[TAPS];
 #pragma unroll
-      for (int j = 0; j < TAPS; ++j) {
-        const int i = j - (TAPS - p.taps);
-        const float f = T::one(((const S*)p.conv)[(long)(2 * nq + ch) * p.taps + (i > 0 ? i : 0)]);
-        w[j] = i >= 0 && v < p.dv ? f : 0.f;
-      }
+      for (int j = 0; j < TAPS; ++j) f[j] = j >= TAPS - p.taps && v0 + 64 * n + i16 < p.dv ? T::one(vw[n][j]) : 0.f;
 #pragma unroll
       for (int I = 0; I < 4; ++I) {
         float z[TAPS + 3];
 #pragma unroll
-        for (int j = 0; j < TAPS + 3; ++j) {
-          const int tok = chunk * kDChunk + I * kDSub + 4 * g4 - (TAPS - 1) + j;
-          const S* src = row.proj + (tok < 0 ? 0 : (tok < p.t ? tok : p.t - 1)) * p.pitch + p.v_off + ch;
-          if (chunk == 0 && I == 0 && tok < 0) src = row.ring + (long)row.ring_row(p, tok) * p.channels + 2 * nq + ch;
-          const float f = T::one(*src);
-          z[j] = tok >= lead && tok < p.t && j >= TAPS - p.taps ? f : 0.f;  // (older ring rows hold anything)
-        }
+        for (int j = 0; j < TAPS + 3; ++j) z[j] = chunk * kDChunk + I * kDSub + 4 * g4 - (TAPS - 1) + j >= lead ? T::one(vx[n][I][j]) : 0.f;
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
           float a = 0.f;
 #pragma unroll
-          for (int j = 0; j < TAPS; ++j) a = fmaf(w[j], z[r + j], a);
+          for (int j = 0; j < TAPS; ++j) a = fmaf(f[j], z[r + j], a);
           x[n][I][r] = silu(a);
         }
       }
@@ -847,7 +864,9 @@ __global__ void __launch_bounds__(256, 1) delta_scan_kernel(const DeltaParams p)
 #pragma unroll
     for (int r = 0; r < 4; ++r) {
       const int d = d0 + 16 * i + 4 * g + r;
-      s[i][r] = d < p.dk && col ? st[(long)d * p.dv + c0 + i16] : 0.f;
+      const bool in = d < p.dk && col;
+      const float x = st[in ? (long)d * p.dv + c0 + i16 : 0];
+      s[i][r] = in ? x : 0.f;
     }
   f32x4 w[4][NT], q[4][NT], kd[4][NT], gc[NT], aq[4], u0[4];
   auto load_wq = [&](int c) {
@@ -880,10 +899,13 @@ __global__ void __launch_bounds__(256, 1) delta_scan_kernel(const DeltaParams p)
       gc[i] = *(const f32x4*)(p.gc + (bh * p.chunks + c) * p.dkp + d0 + 16 * i + 4 * g);
     }
   };
+  // (what the next chunk needs is requested as soon as its registers are free, and stays there)
+  auto stay = [] { asm volatile("" ::: "memory"); };
   load_wq(0);
   load_u(0);
   load_a(0);
   load_k(0);
+  stay();
   for (int c = 0; c < p.chunks; ++c) {
     const int buf = c & 1, next = c + 1 < p.chunks ? c + 1 : c;
     // this wave's key rows of W S and Q S
@@ -901,6 +923,7 @@ __global__ void __launch_bounds__(256, 1) delta_scan_kernel(const DeltaParams p)
       xo[buf][wave][rt][lane] = o;
     }
     load_wq(next);
+    stay();
     __syncthreads();
     f32x4 u[4];
 #pragma unroll
@@ -910,6 +933,7 @@ __global__ void __launch_bounds__(256, 1) delta_scan_kernel(const DeltaParams p)
       for (int r = 0; r < 4; ++r) u[j][r] = u0[j][r] - ((a[r] + b4[r]) + (c4[r] + d4[r]));
     }
     load_u(next);
+    stay();
     {
       const f32x4 a = xo[buf][0][wave][lane], b4 = xo[buf][1][wave][lane], c4 = xo[buf][2][wave][lane], d4 = xo[buf][3][wave][lane];
       f32x4 o;
@@ -927,6 +951,7 @@ __global__ void __launch_bounds__(256, 1) delta_scan_kernel(const DeltaParams p)
         if (tk + r < p.t && col) dst[(long)r * p.heads * p.dv] = o[r];
     }
     load_a(next);
+    stay();
 #pragma unroll
     for (int i = 0; i < NT; ++i) {
 #pragma unroll
@@ -937,6 +962,7 @@ __global__ void __launch_bounds__(256, 1) delta_scan_kernel(const DeltaParams p)
         for (int r = 0; r < 4; ++r) s[i] = mfma_f32(kd[j][i][r], u[j][r], s[i]);
     }
     load_k(next);
+    stay();
   }
 #pragma unroll
   for (int i = 0; i < NT; ++i)
