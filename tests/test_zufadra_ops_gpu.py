@@ -294,8 +294,11 @@ class _Delta:
 # y is normed per head, which magnifies what is small; S is compared on its own
 Y_REL = {torch.float32: 1e-4, torch.bfloat16: 1e-2, torch.float16: 2e-3}
 
+# (heads, kv_heads, dk, dv, taps[, ranks])
 DELTA = [(4, 2, 40, 56, 3), (2, 2, 64, 64, 4), (3, 1, 24, 20, 1), (2, 1, 130, 33, 2), (1, 1, 256, 40, 4), (2, 2, 12, 13, 5), (2, 1, 64, 300, 8),
-         (1, 1, 264, 16, 4), (2, 1, 16, 16, 9), (2, 2, 128, 128, 4), (1, 1, 200, 72, 6)]
+         (1, 1, 264, 16, 4), (2, 1, 16, 16, 9), (2, 2, 128, 128, 4), (1, 1, 200, 72, 6),
+         # ranks (of the decay and of the gate) that fill the registers of the step kernel, exceed them, are no multiple of 8
+         (2, 2, 128, 128, 4, 128, 128), (1, 1, 128, 256, 4, 64, 24), (2, 1, 48, 72, 4, 200, 13), (2, 1, 100, 40, 2, 72, 136)]
 
 
 @pytest.mark.parametrize("dtype", DTYPES)
